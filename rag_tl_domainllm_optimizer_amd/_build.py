@@ -64,6 +64,9 @@ def kernel_flags(debug: bool = False):
     return [
         "-x", "hip", f"--offload-arch={ARCH}", *opt, "-fPIC", "-std=c++17", "-munsafe-fp-atomics",
         "-I", os.path.join(CSRC, "include"), "-Wno-unused-result",
+        # no packed fp32 arithmetic (v_pk_add / mul / fma_f32): hipcc forms it from ordinary float code
+        # at -O3, and some forms have returned wrong results on MI355X without an error
+        "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     ]
 
 

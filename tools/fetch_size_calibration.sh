@@ -8,7 +8,7 @@ set -o pipefail
 R=$PWD
 out=$R/gpurun_out/fetch_cal
 mkdir -p $out
-hipcc --offload-arch=gfx950 -O3 -o /tmp/hbm_pattern $R/tools/microbench/hbm_pattern.hip || exit 1
+hipcc --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -O3 -o /tmp/hbm_pattern $R/tools/microbench/hbm_pattern.hip || exit 1
 cd /tmp && export TMPDIR=/tmp
 rm -rf /tmp/fsc
 timeout -s KILL 120 rocprofv3 --pmc FETCH_SIZE -f csv -d /tmp/fsc -o run -- /tmp/hbm_pattern > $out/run.log 2>&1 || exit $?

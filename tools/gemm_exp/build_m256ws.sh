@@ -8,7 +8,7 @@ OUT=tools/gemm_exp/run
 SRC=tools/gemm_exp/src
 mkdir -p "$OUT" "$SRC"
 H=/opt/rocm/bin/hipcc
-F="-O3 --offload-arch=gfx950 -std=c++17 -munsafe-fp-atomics -Icsrc/include -Wno-unused-result"
+F="-O3 --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops -std=c++17 -munsafe-fp-atomics -Icsrc/include -Wno-unused-result"
 $H $F -c csrc/kernels/gemm_big.hip -o $SRC/gb.o &
 $H $F -c tools/gemm_exp/m256_main.cpp -o $SRC/m256_main.o &
 $H -O2 -std=c++17 -Icsrc/include -c csrc/host/tuning.cpp -o $SRC/tuning.o &
@@ -20,7 +20,7 @@ done
 wait
 for v in $VARIANTS; do
   IFS=: read xs ws nt <<<"$v"
-  $H --offload-arch=gfx950 $SRC/m256ws_x${xs}w${ws}n${nt}.o $SRC/gb.o $SRC/m256_main.o $SRC/tuning.o \
+  $H --offload-arch=gfx950 -Xclang -target-feature -Xclang -packed-fp32-ops $SRC/m256ws_x${xs}w${ws}n${nt}.o $SRC/gb.o $SRC/m256_main.o $SRC/tuning.o \
     -o $OUT/gemm_m256ws_x${xs}w${ws}n${nt}
 done
 ls $OUT
