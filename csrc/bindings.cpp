@@ -18,6 +18,14 @@
 #include "rt_tuning.h"
 
 extern "C" {
+int rt_gemm_nt_glu(const void*, long, const void*, long, const void*, long, const void*, long, int, const void*, void*,
+                   long, int, int, int, int, int, float*, unsigned*, const void*, long, float, int, const float*,
+                   hipStream_t);
+int rt_gemm_big_glu(int, int, const void*, long, const void*, long, const void*, long, const void*, long, int,
+                    const void*, void*, long, void*, long, const void*, long, int, int, int, int, int, int, const void*,
+                    int, const float*, hipStream_t);
+int rt_gemm_splitk_reduce_glu(const float*, int, int, int, const void*, int, const void*, long, void*, long,
+                              const float*, hipStream_t);
 int rt_gemm_nt(const void*, long, const void*, long, const void*, long, const void*, long, int, const void*, void*,
                long, int, int, int, int, int, float*, unsigned*, const void*, long, float, int, hipStream_t);
 int rt_shuffle_decode_weight(const void*, void*, long, long, hipStream_t);
@@ -170,6 +178,17 @@ void check_rc(int rc, const char* what) {
 #define CHECK_ALIGN16(t)                                                                             \
   TORCH_CHECK(reinterpret_cast<uintptr_t>((t).data_ptr()) % 16 == 0, #t " must be 16-byte aligned")
 
+// {limit, alpha, offset} of a gated linear unit (empty: silu(g) * u)
+struct GluArg {
+  float v[3];
+  bool on;
+  explicit GluArg(const std::vector<double>& g) : v{0, 0, 0}, on(!g.empty()) {
+    TORCH_CHECK(g.empty() || g.size() == 3, "glu: {limit, alpha, offset} expected");
+    for (size_t i = 0; i < g.size(); ++i) v[i] = (float)g[i];
+  }
+  const float* ptr() const { return on ? v : nullptr; }
+};
+
 const void* opt_ptr(const optional<Tensor>& t) { return t.has_value() && t->defined() ? t->data_ptr() : nullptr; }
 
 // Split-K workspace of the decode GEMM (fp32 slabs + self-resetting arrival tickets), one per
@@ -211,7 +230,7 @@ std::vector<int64_t> decode_ws_dirty_tickets() {
 // ---------------------------------------------------------------------------------------------
 Tensor gemm(const Tensor& a, const Tensor& w, const optional<Tensor>& u, const optional<Tensor>& ub,
             const optional<Tensor>& bias, int64_t act, bool out_f32, optional<Tensor> out,
-            const optional<Tensor>& residual, double norm_eps, bool w_shuffled) {
+            const optional<Tensor>& residual, double norm_eps, bool w_shuffled, const std::vector<double>& glu) {
   CHECK_CUDA(a); CHECK_CUDA(w); CHECK_BF16(a); CHECK_BF16(w); CHECK_ROWS(a); CHECK_ROWS(w);
   if (w_shuffled)
     TORCH_CHECK(a.size(0) <= 64 && w.size(0) % 16 == 0 && w.is_contiguous(),
@@ -264,11 +283,11 @@ Tensor gemm(const Tensor& a, const Tensor& w, const optional<Tensor>& u, const o
     tickets = (unsigned*)ws.tickets.data_ptr<int>();
     TORCH_CHECK((N + 63) / 64 <= ws.tickets.numel(), "gemm: N too large for the decode workspace");
   }
-  check_rc(rt_gemm_nt(a.data_ptr(), a.stride(0), w.data_ptr(), w.stride(0), opt_ptr(u), Rp ? u->stride(0) : 0,
+  check_rc(rt_gemm_nt_glu(a.data_ptr(), a.stride(0), w.data_ptr(), w.stride(0), opt_ptr(u), Rp ? u->stride(0) : 0,
                       opt_ptr(ub), Rp ? ub->stride(0) : 0, Rp, opt_ptr(bias), c.data_ptr(), c.stride(0), (int)M,
                       (int)N, (int)K, (int)act, out_f32 ? 1 : 0, slabs, tickets,
                       has_res ? residual->data_ptr() : nullptr, has_res ? residual->stride(0) : 0, (float)norm_eps,
-                      w_shuffled ? 1 : 0, st),
+                      w_shuffled ? 1 : 0, GluArg(glu).ptr(), st),
            "gemm");
   return c;
 }
@@ -322,7 +341,7 @@ const Tensor& zero_page(const Tensor& like) {
 Tensor gemm_big(const Tensor& a, const Tensor& b, int64_t layout_a, int64_t layout_b, const optional<Tensor>& a2,
                 const optional<Tensor>& b2, const optional<Tensor>& bias, int64_t act, int64_t out_mode,
                 int64_t nsplit, optional<Tensor> out, const optional<Tensor>& out2, const optional<Tensor>& residual,
-                int64_t bn) {
+                int64_t bn, const std::vector<double>& glu) {
   CHECK_CUDA(a); CHECK_CUDA(b); CHECK_BF16(a); CHECK_BF16(b); CHECK_ROWS(a); CHECK_ROWS(b);
   CHECK_ALIGN16(a); CHECK_ALIGN16(b);
   TORCH_CHECK(a.stride(0) % 8 == 0 && b.stride(0) % 8 == 0, "gemm_big: row strides must be multiples of 8");
@@ -419,12 +438,12 @@ Tensor gemm_big(const Tensor& a, const Tensor& b, int64_t layout_a, int64_t layo
     CHECK_ALIGN16(*residual);
   }
   if (M == 0 || N == 0) return c;
-  check_rc(rt_gemm_big((int)layout_a, (int)layout_b, a.data_ptr(), a.stride(0), b.data_ptr(), b.stride(0),
+  check_rc(rt_gemm_big_glu((int)layout_a, (int)layout_b, a.data_ptr(), a.stride(0), b.data_ptr(), b.stride(0),
                        ext ? a2->data_ptr() : nullptr, ext ? a2->stride(0) : 0, ext ? b2->data_ptr() : nullptr,
                        ext ? b2->stride(0) : 0, (int)K2, opt_ptr(bias), c.data_ptr(), c.stride(0), c2, ldc2,
                        has_r ? residual->data_ptr() : nullptr, has_r ? residual->stride(0) : 0, (int)M,
                        (int)N, (int)K, (int)act, (int)out_mode, (int)nsplit, zero_page(a).data_ptr(), (int)bn,
-                       cur_stream()),
+                       GluArg(glu).ptr(), cur_stream()),
            "gemm_big");
   return c;
 }
@@ -514,7 +533,8 @@ Tensor gemm_small(const Tensor& a, const Tensor& b, int64_t layout_a, int64_t la
 // K split over `nsplit` workgroup rows into fp32 slabs (workspace `slabs`, >= nsplit*M*N floats),
 // then one reduce kernel with the epilogue (bias, act / SwiGLU pairing, residual).
 Tensor gemm_splitk(const Tensor& a, const Tensor& w, int64_t nsplit, Tensor slabs, const optional<Tensor>& bias,
-                   int64_t act, optional<Tensor> out, const optional<Tensor>& residual, int64_t bn) {
+                   int64_t act, optional<Tensor> out, const optional<Tensor>& residual, int64_t bn,
+                   const std::vector<double>& glu) {
   CHECK_CUDA(a); CHECK_BF16(a); CHECK_BF16(w); CHECK_ROWS(a); CHECK_ROWS(w); CHECK_F32(slabs);
   CHECK_ALIGN16(a); CHECK_ALIGN16(w);
   const int64_t M = a.size(0), K = a.size(1), N = w.size(0);
@@ -544,9 +564,9 @@ Tensor gemm_splitk(const Tensor& a, const Tensor& w, int64_t nsplit, Tensor slab
                        nullptr, slabs.data_ptr(), N, nullptr, 0, nullptr, 0, (int)M, (int)N, (int)K, 0, 3,
                        (int)nsplit, zero_page(a).data_ptr(), (int)bn, cur_stream()),
            "gemm_splitk");
-  check_rc(rt_gemm_splitk_reduce(slabs.data_ptr<float>(), (int)nsplit, (int)M, (int)N, opt_ptr(bias), (int)act,
+  check_rc(rt_gemm_splitk_reduce_glu(slabs.data_ptr<float>(), (int)nsplit, (int)M, (int)N, opt_ptr(bias), (int)act,
                                  has_r ? residual->data_ptr() : nullptr, has_r ? residual->stride(0) : 0, c.data_ptr(),
-                                 c.stride(0), cur_stream()),
+                                 c.stride(0), GluArg(glu).ptr(), cur_stream()),
            "gemm_splitk_reduce");
   return c;
 }
@@ -1317,13 +1337,16 @@ void decode_update(const Tensor& tok, Tensor out_tokens, const optional<Tensor>&
 
 }  // namespace
 
+void bind_layered(py::module_& m);  // csrc/host/bind_layered.cpp
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  bind_layered(m);
   m.doc() = "gfx950 (MI355X) HIP kernels + native host runtime";
   m.def("decode_ws_dirty_tickets", &decode_ws_dirty_tickets, "per decode workspace: tickets not at zero");
   m.def("gemm", &gemm, "bf16 MFMA GEMM C = act(rstd(A) A W^T + U UB^T + bias) + R", py::arg("a"), py::arg("w"),
         py::arg("u") = py::none(), py::arg("ub") = py::none(), py::arg("bias") = py::none(), py::arg("act") = 0,
         py::arg("out_f32") = false, py::arg("out") = py::none(), py::arg("residual") = py::none(),
-        py::arg("norm_eps") = 0.0, py::arg("w_shuffled") = false);
+        py::arg("norm_eps") = 0.0, py::arg("w_shuffled") = false, py::arg("glu") = std::vector<double>());
   m.def("rows_scatter", &rows_scatter, "varlen: out[r] = src[inv[r]] (zeros where inv[r] < 0)", py::arg("src"),
         py::arg("inv"), py::arg("R"));
   m.def("shuffle_decode_weight", &shuffle_decode_weight, "W [N, K] -> tile-ordered decode image (gemm w_shuffled=True)",
@@ -1351,14 +1374,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("a"), py::arg("b"), py::arg("layout_a"), py::arg("layout_b"), py::arg("a2") = py::none(),
         py::arg("b2") = py::none(), py::arg("bias") = py::none(), py::arg("act") = 0, py::arg("out_mode") = 0,
         py::arg("nsplit") = 1, py::arg("out") = py::none(), py::arg("out2") = py::none(),
-        py::arg("residual") = py::none(), py::arg("bn") = 0);
+        py::arg("residual") = py::none(), py::arg("bn") = 0, py::arg("glu") = std::vector<double>());
   m.def("gemm_rope", &gemm_rope, "NT GEMM with the rotary embedding of the q / k heads in the epilogue", py::arg("a"),
         py::arg("w"), py::arg("u") = py::none(), py::arg("ub") = py::none(), py::arg("bias") = py::none(),
         py::arg("pos"), py::arg("cos"), py::arg("sin"), py::arg("rope_cols"), py::arg("head_dim"),
         py::arg("out") = py::none(), py::arg("bn") = 0);
   m.def("gemm_splitk", &gemm_splitk, "small-M NT GEMM: split-K fp32 slabs + fused reduce epilogue", py::arg("a"),
         py::arg("w"), py::arg("nsplit"), py::arg("slabs"), py::arg("bias") = py::none(), py::arg("act") = 0,
-        py::arg("out") = py::none(), py::arg("residual") = py::none(), py::arg("bn") = 256);
+        py::arg("out") = py::none(), py::arg("residual") = py::none(), py::arg("bn") = 256, py::arg("glu") = std::vector<double>());
   m.def("gemm_small", &gemm_small, "64x64-tile GEMM for narrow (LoRA) products", py::arg("a"), py::arg("b"),
         py::arg("layout_a"), py::arg("layout_b"), py::arg("out_mode") = 0, py::arg("nsplit") = 1,
         py::arg("out") = py::none(), py::arg("bm") = 64);

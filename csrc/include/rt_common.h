@@ -258,7 +258,7 @@ __device__ __forceinline__ uint2 f32x8_to_fp8(const float* v, float inv) {
 // slab order from slab 0 (bitwise equal to a rolled `for q` loop). The loads of the first 8 slabs
 // are issued unconditionally (indices clamped to ns - 1, the surplus ones hit cache) before the
 // first add: ONE L2/MALL round trip, where a rolled loop with a runtime trip count waits for every
-// slab's loads in turn (docs/DESIGN.md 'A rolled reduction loop ... Unroll it').
+// slab's loads in turn.
 __device__ __forceinline__ void sum_slabs8(const float* p, long stride, int ns, float (&out)[8]) {
   float4 lo[8], hi[8];
 #pragma unroll
@@ -280,6 +280,17 @@ __device__ __forceinline__ void sum_slabs8(const float* p, long stride, int ns, 
     out[0] += a.x; out[1] += a.y; out[2] += a.z; out[3] += a.w;
     out[4] += b.x; out[5] += b.y; out[6] += b.z; out[7] += b.w;
   }
+}
+
+// Gated linear unit: f(g, u) = g' * sigmoid(alpha * g') * (u' + offset) with g' = min(g, limit) and
+// u' = clamp(u, -limit, limit). The default is SwiGLU (silu(g) * u, unclamped).
+struct GluP {
+  float limit = INFINITY, alpha = 1.f, offset = 0.f;
+};
+__device__ __forceinline__ float glu(float g, float u, const GluP& p) {
+  g = g > p.limit ? p.limit : g;  // a NaN stays a NaN
+  u = u > p.limit ? p.limit : (u < -p.limit ? -p.limit : u);
+  return g / (1.f + __expf(-(p.alpha * g))) * (u + p.offset);
 }
 
 __device__ __forceinline__ float wave_sum(float v) {

@@ -64,6 +64,7 @@ struct GemmArgs {
   // decode kernel only: B is in the MFMA-fragment order of shuffle_decode_weight (each 16-row x
   // 64-k tile = 2 KiB contiguous, one 1-KiB run per load instruction) instead of row-major
   int wshuf;
+  GluP glu;  // ACT_SWIGLU: the gated linear unit of the epilogue (default silu(g) * u)
 };
 
 typedef __attribute__((address_space(3))) void lds_void;
@@ -333,7 +334,7 @@ __global__ __launch_bounds__(256, 2) void gemm_decode_kernel(GemmArgs p, float* 
       const int row = e / 32, c = e % 32;
       if (row >= p.M) continue;
       const float gt = red[row * LDR + c], up = red[row * LDR + c + 32];
-      const float y = gt / (1.f + __expf(-gt)) * up;
+      const float y = glu(gt, up, p.glu);
       if constexpr (OUT_F32) ((float*)p.C)[(long)row * p.ldc + cg * 32 + c] = y;
       else ((bf16_t*)p.C)[(long)row * p.ldc + cg * 32 + c] = f2bf(y);
     }
@@ -526,7 +527,7 @@ __global__ __launch_bounds__(64 * NW) void gemv16_kernel(GemmArgs p) {
       float up = uu * rs;
       if constexpr (W8) { y *= p.sb[col]; up *= p.sb[F + col]; }
       if (p.bias) { y += bf2f(p.bias[col]); up += bf2f(p.bias[F + col]); }
-      y = y / (1.f + __expf(-y)) * up;
+      y = glu(y, up, p.glu);
     } else {
       if constexpr (W8) y *= p.sb[col];
       if (p.bias) y += bf2f(p.bias[col]);
@@ -624,7 +625,7 @@ __device__ __forceinline__ void m64_finish(const GemmArgs& p, f32x4 (&acc)[4], f
         const int row = wid * 16 + fq * 4 + r;
         if (row >= p.M) continue;
         const float gt = acc[j][r] * sg + bg, up = acc[j + 2][r] * su + bu;
-        const float y = gt / (1.f + __expf(-gt)) * up;
+        const float y = glu(gt, up, p.glu);
         if constexpr (OUT_F32) ((float*)p.C)[(long)row * p.ldc + col] = y;
         else ((bf16_t*)p.C)[(long)row * p.ldc + col] = f2bf(y);
       }
@@ -965,7 +966,7 @@ __global__ __launch_bounds__(512, 1) void gemm_w8_wide_kernel(GemmArgs p, float*
       for (int r = 0; r < 4; ++r) {
         float gt = acc[rr][0][r] * rs * sgv[r], up = acc[rr][1][r] * rs * suv[r];
         if (p.bias) { gt += bf2f(p.bias[col + r]); up += bf2f(p.bias[F + col + r]); }
-        y[r] = gt / (1.f + __expf(-gt)) * up;
+        y[r] = glu(gt, up, p.glu);
       }
       if constexpr (OUT_F32) *(float4*)((float*)p.C + (long)row * p.ldc + col) = make_float4(y[0], y[1], y[2], y[3]);
       else *(uint2*)((bf16_t*)p.C + (long)row * p.ldc + col) = make_uint2(pack2bf(y[0], y[1]), pack2bf(y[2], y[3]));
@@ -1040,7 +1041,7 @@ __global__ __launch_bounds__(256) void wide_reduce_kernel(GemmArgs p, const floa
     if (pair) {
       float gt = gv[r] * rs * (p.sb ? p.sb[col + r] : 1.f), up = uv[r] * rs * (p.sb ? p.sb[F + col + r] : 1.f);
       if (p.bias) { gt += bf2f(p.bias[col + r]); up += bf2f(p.bias[F + col + r]); }
-      y[r] = gt / (1.f + __expf(-gt)) * up;
+      y[r] = glu(gt, up, p.glu);
     } else {
       float v = gv[r] * rs * (p.sb ? p.sb[col + r] : 1.f);
       if (p.bias) v += bf2f(p.bias[col + r]);
@@ -1149,10 +1150,12 @@ static int decode_depth(int MT, long blocks) {
 }
 
 
-extern "C" int rt_gemm_nt(const void* A, long lda, const void* B, long ldb, const void* U, long ldu,
+// glu_p: {limit, alpha, offset} of the ACT_SWIGLU epilogue (host pointer; null = silu(g) * u)
+extern "C" int rt_gemm_nt_glu(const void* A, long lda, const void* B, long ldb, const void* U, long ldu,
                           const void* UB, long ldub, int Rp, const void* bias, void* C, long ldc, int M,
                           int N, int K, int act, int out_f32, float* slabs, unsigned* tickets,
-                          const void* R, long ldr, float norm_eps, int wshuf, hipStream_t stream) {
+                          const void* R, long ldr, float norm_eps, int wshuf, const float* glu_p,
+                              hipStream_t stream) {
   GemmArgs p;
   p.A = (const bf16_t*)A; p.lda = lda;
   p.B = (const bf16_t*)B; p.ldb = ldb;
@@ -1164,6 +1167,7 @@ extern "C" int rt_gemm_nt(const void* A, long lda, const void* B, long ldb, cons
   p.M = M; p.N = N; p.K = K; p.act = act;
   p.sa = nullptr; p.sb = nullptr;
   p.R = (const bf16_t*)R; p.ldr = ldr; p.norm_eps = norm_eps; p.wshuf = wshuf;
+  if (glu_p) { p.glu.limit = glu_p[0]; p.glu.alpha = glu_p[1]; p.glu.offset = glu_p[2]; }
   if (M <= 0 || N <= 0) return 0;
   if (wshuf && (M > 64 || N % 16 != 0 || K % 64 != 0)) return -4;  // shuffled weights: decode kernel only
   if (act == ACT_SWIGLU && (M > 64 || N % 64 != 0 || (U && UB))) return -2;
@@ -1232,6 +1236,14 @@ extern "C" int rt_gemm_nt(const void* A, long lda, const void* B, long ldb, cons
   }
   RT_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int rt_gemm_nt(const void* A, long lda, const void* B, long ldb, const void* U, long ldu,
+                          const void* UB, long ldub, int Rp, const void* bias, void* C, long ldc, int M,
+                          int N, int K, int act, int out_f32, float* slabs, unsigned* tickets,
+                          const void* R, long ldr, float norm_eps, int wshuf, hipStream_t stream) {
+  return rt_gemm_nt_glu(A, lda, B, ldb, U, ldu, UB, ldub, Rp, bias, C, ldc, M, N, K, act, out_f32, slabs, tickets, R,
+                        ldr, norm_eps, wshuf, nullptr, stream);
 }
 
 extern "C" int rt_gemm_big_fp8(const void*, long, const float*, const void*, long, const float*, const void*, void*,

@@ -89,6 +89,13 @@ struct Args {
   const float* rope_cos;
   const float* rope_sin;
   int rope_cols, rope_d;
+  // GRP: row tiles {group, first row, end row, -}, their device-side count, sorted row -> A row, and the
+  // weight elements per group
+  const int4* grp_tiles;
+  const int* grp_n;
+  const int* row_map;
+  long b_stride;
+  GluP glu;  // E_SWIGLU: the gated linear unit of the epilogue (default silu(g) * u)
 };
 
 __device__ __forceinline__ int row_swz(int row) { return (row >> 1) & 7; }
@@ -133,7 +140,13 @@ __device__ __forceinline__ void wait_granules(int n) {
 // each wave owns 2 B fragments instead of 4 (columns 64 (wc >> 1) + 16 (wc & 1) + 32 s): used for
 // M = 256 decode GEMMs (twice the workgroups, no split-K on the widest weights) and for the last,
 // partial wave of tiles of a large GEMM (rt_gemm_big_planned).
-template <int LA, int LB, int OUT, int EPI, int BN, bool F8 = false>
+//
+// GRP (grouped NT product, mixture-of-experts feed-forwards): the M rows are sorted by group; row tile
+// i is p.grp_tiles[i] = {group, first row, end row} and multiplies that group's weight (p.B + group *
+// b_stride). Tiles never straddle a group; their number (*p.grp_n) is only known on the device, so the
+// grid covers the upper bound and surplus workgroups leave at once. p.row_map (optional) gives the
+// row of A behind each sorted row: the gather of the routed tokens rides on the LDS-DMA addresses.
+template <int LA, int LB, int OUT, int EPI, int BN, bool F8 = false, bool GRP = false>
 __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
   static_assert(BN == 256 || BN == 128, "BN");
   static_assert(!F8 || (LA == ROW && LB == ROW && (OUT == O_BF16 || OUT == O_F32_SLAB)),
@@ -142,9 +155,10 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
   __shared__ __attribute__((aligned(16))) char smem[2 * BUF];  // the only __shared__ object
 
 
-  const int tiles_m = (p.M + 255) / 256;
+  const int tiles_m = GRP ? *p.grp_n : (p.M + 255) / 256;
   const int tiles_n = EPI == E_SWIGLU ? p.N / BN : (p.N + BN - 1) / BN;
   const int nwg = tiles_m * tiles_n;
+  if (GRP && (int)blockIdx.x >= nwg) return;
   // ---- K-steps ----
   const int nk1 = (p.K + 63) / 64;
   const int nk2 = p.A2 ? (p.K2 + 63) / 64 : 0;
@@ -164,7 +178,9 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
   const int gsz = min(tiles_m - first_m, GM);
   const int tm = first_m + (bid % gsz);
   const int tn = (bid % (GM * tiles_n)) / gsz;
-  const int m0 = tm * 256, n0 = tn * BN;
+  const int m0 = GRP ? p.grp_tiles[tm].y : tm * 256, n0 = tn * BN;
+  const int Mv = GRP ? p.grp_tiles[tm].z : p.M;  // end of the tile's valid rows
+  const bf16_t* const Bp = GRP ? p.B + (long)p.grp_tiles[tm].x * p.b_stride : p.B;
   const int Fh = p.N / 2;  // E_SWIGLU: gate rows [0, F), up rows [F, 2F)
   constexpr int HALF = BN / 2;  // E_SWIGLU: tile columns [0, HALF) gate, [HALF, BN) up
 
@@ -192,7 +208,10 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
       const int row = rb + (lane >> 3);
       const int kc = (lane & 7) ^ row_swz(row);
       int grow;
-      if (op == 0) grow = min(m0 + row, p.M - 1);
+      if (op == 0) {
+        grow = min(m0 + row, Mv - 1);
+        if (GRP && p.row_map) grow = p.row_map[grow];
+      }
       // SwiGLU: tile rows [0, HALF) are gate rows, [HALF, BN) the matching up rows — for the weight
       // and for its K-extension (LoRA UB rows follow the weight's row order)
       else if (EPI == E_SWIGLU) grow = row < HALF ? tn * HALF + row : Fh + tn * HALF + row - HALF;
@@ -203,7 +222,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
     const int blk = op == 0 ? (o >> 3) * 4 + s * 2 + ((o >> 2) & 1) : (o >> 2) * 2 + s;
     const int kr = (o & 3) * 16 + (lane >> 2);
     const int ch = (lane & 3) ^ kmaj_swz(kr);
-    const int col = min((op == 0 ? m0 : n0) + blk * 32 + ch * 8, (op == 0 ? p.M : p.N) - 8);
+    const int col = min((op == 0 ? m0 : n0) + blk * 32 + ch * 8, (op == 0 ? Mv : p.N) - 8);
     kin = kr;
     return (uint32_t)kr * (uint32_t)ld + (uint32_t)col;
   };
@@ -224,7 +243,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
     if (t < nk1) {
       const int k0 = t * 64;
       const long adv = ((op ? LB : LA) == ROW) ? (long)k0 : (long)k0 * (op ? p.ldb : p.lda);
-      const bf16_t* base = (op ? p.B : p.A) + adv;
+      const bf16_t* base = (op ? Bp : p.A) + adv;
       if (k0 + 64 <= p.K) {
 #pragma unroll
         for (int j = 0; j < (op ? NB : 2); ++j)
@@ -372,7 +391,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
     auto stage_fast = [&](int g, int u) {
       const int op = g >> 1;
       const long adv = ((op ? LB : LA) == ROW) ? (long)u * 64 : (long)u * 64 * (op ? p.ldb : p.lda);
-      const bf16_t* base = (op ? p.B : p.A) + adv;
+      const bf16_t* base = (op ? Bp : p.A) + adv;
       char* img = smem + (u & 1) * BUF;
 #pragma unroll
       for (int j = 0; j < (op ? NB : 2); ++j)
@@ -441,7 +460,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int row = m0 + wr * 128 + i * 16 + fq * 4 + r;
-          if (row < p.M && col < p.N)
+          if (row < Mv && col < p.N)
             __hip_atomic_fetch_add(C + (long)row * p.ldc + col, acc[i][j][r], __ATOMIC_RELAXED, __HIP_MEMORY_SCOPE_AGENT);
         }
     }
@@ -467,7 +486,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
 #pragma unroll
       for (int i = 0; i < 8; ++i) {
         const int row = m0 + wr * 128 + i * 16 + frow;
-        if (row < p.M && col < p.N) {
+        if (row < Mv && col < p.N) {
           const float sr = F8 ? p.sa[row] : 1.f;
           float4 v;
           v.x = act_fn((F8 ? acc[i][j][0] * (sr * sc[0]) : acc[i][j][0]) + bv[0], EPI);
@@ -509,7 +528,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           // F8: per-token activation scale of this fragment row (x the column's weight scale)
-          const float srow = F8 ? p.sa[min(m0 + hh * 128 + i * 16 + frow, p.M - 1)] : 1.f;
+          const float srow = F8 ? p.sa[min(m0 + hh * 128 + i * 16 + frow, Mv - 1)] : 1.f;
 #pragma unroll
           for (int j = 0; j < 2 * NB; ++j) {
             const int row = i * 16 + frow, col = col_of(j) + fq * 4;
@@ -534,13 +553,13 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
         for (int pass = 0; pass < 128 * CH / 512; ++pass) {
           const int row = pass * (512 / CH) + tid / CH;
           const int grow = m0 + hh * 128 + row;
-          if (grow < p.M) {
+          if (grow < Mv) {
             const uint4 g4 = ld16(row, cc), u4 = ld16(row, CH + cc);
             float g[8], u[8], f[8];
             unpack8(g4, g);
             unpack8(u4, u);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) f[e] = g[e] / (1.f + __expf(-g[e])) * u[e];
+            for (int e = 0; e < 8; ++e) f[e] = glu(g[e], u[e], p.glu);
             const int fcol = tn * HALF + cc * 8;
             *(uint4*)(Cf + (long)grow * p.ldc + fcol) = pack8(f);
             if (p.C2) {
@@ -558,7 +577,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
         for (int pass = 0; pass < 128 * CH / 512; ++pass) {
           const int row = pass * (512 / CH) + tid / CH;
           const int grow = m0 + hh * 128 + row, gcol = n0 + cc * 8;
-          if (grow < p.M && gcol < F) {
+          if (grow < Mv && gcol < F) {
             float d[8], g[8], u[8], dg[8], du[8];
             unpack8(ld16(row, cc), d);
             unpack8(*(const uint4*)(p.R + (long)grow * p.ldr + gcol), g);
@@ -582,7 +601,7 @@ __global__ __launch_bounds__(512, 2) void gemm_big_kernel(Args p) {
         for (int pass = 0; pass < 128 * CH / 512; ++pass) {
           const int row = pass * (512 / CH) + tid / CH;
           const int grow = m0 + hh * 128 + row, gcol = n0 + cc * 8;
-          if (grow < p.M && gcol < p.N) {
+          if (grow < Mv && gcol < p.N) {
             uint4 v = ld16(row, cc);
             if constexpr (EPI == E_ROPE) {
               if (gcol < p.rope_cols) {
@@ -797,7 +816,7 @@ __global__ __launch_bounds__(256, 2) void gemm_small_kernel(Args p) {
 __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restrict__ slabs, int nsplit, int M, int N,
                                                             const bf16_t* __restrict__ bias, int act,
                                                             const bf16_t* __restrict__ R, long ldr,
-                                                            bf16_t* __restrict__ C, long ldc) {
+                                                            bf16_t* __restrict__ C, long ldc, GluP gp) {
   const bool swiglu = act == E_SWIGLU;
   const int Nout = swiglu ? N / 2 : N;
   const int cpr = Nout / 8;
@@ -814,7 +833,7 @@ __global__ __launch_bounds__(256) void splitk_reduce_kernel(const float* __restr
 #pragma unroll
     for (int q = 0; q < 8; ++q) {
       const float g = bf2f(f2bf(a[q])), u = bf2f(f2bf(b[q]));
-      y[q] = g / (1.f + __expf(-g)) * u;
+      y[q] = glu(g, u, gp);
     }
   } else {
     float bb[8] = {0, 0, 0, 0, 0, 0, 0, 0}, rr[8] = {0, 0, 0, 0, 0, 0, 0, 0};
@@ -922,10 +941,11 @@ static int gemm_big_planned(const Args& p, int layout_a, int layout_b, int act, 
 // (e.g. M = 9632 tokens x N = 4096: 608 tiles = 2.4 waves of 256 CUs -> 512 tiles + 192 half tiles).
 // Requirements (checked): KMAJ operands have M / N % 8 == 0 and 16-B aligned rows; ROW operands
 // 16-B aligned rows; K, K2 % 8 == 0; E_SWIGLU: ROW/ROW, bf16 out, N % 256 == 0.
-extern "C" int rt_gemm_big(int layout_a, int layout_b, const void* A, long lda, const void* B, long ldb,
+extern "C" int rt_gemm_big_glu(int layout_a, int layout_b, const void* A, long lda, const void* B, long ldb,
                            const void* A2, long lda2, const void* B2, long ldb2, int K2, const void* bias,
                            void* C, long ldc, void* C2, long ldc2, const void* R, long ldr, int M, int N, int K,
-                           int act, int out, int nsplit, const void* zpage, int bn, hipStream_t stream) {
+                           int act, int out, int nsplit, const void* zpage, int bn, const float* glu_p,
+                               hipStream_t stream) {
   if (M <= 0 || N <= 0) return 0;
   if (act == E_ROPE) return -5;  // rt_gemm_big_rope (the rotary tables are its arguments)
   // a ROW operand reads 8-element k-chunks: its reduction length must be a multiple of 8
@@ -958,7 +978,16 @@ extern "C" int rt_gemm_big(int layout_a, int layout_b, const void* A, long lda, 
   p.R = (const bf16_t*)R; p.ldr = ldr;
   p.M = M; p.N = N; p.K = K; p.act = act; p.nsplit = nsplit; p.zpage = (const bf16_t*)zpage;
   p.group_m = tuning().gemm_group_m;
+  if (glu_p) { p.glu.limit = glu_p[0]; p.glu.alpha = glu_p[1]; p.glu.offset = glu_p[2]; }
   return gemm_big_planned(p, layout_a, layout_b, act, out, bn, stream);
+}
+
+extern "C" int rt_gemm_big(int layout_a, int layout_b, const void* A, long lda, const void* B, long ldb,
+                           const void* A2, long lda2, const void* B2, long ldb2, int K2, const void* bias,
+                           void* C, long ldc, void* C2, long ldc2, const void* R, long ldr, int M, int N, int K,
+                           int act, int out, int nsplit, const void* zpage, int bn, hipStream_t stream) {
+  return rt_gemm_big_glu(layout_a, layout_b, A, lda, B, ldb, A2, lda2, B2, ldb2, K2, bias, C, ldc, C2, ldc2, R, ldr, M,
+                         N, K, act, out, nsplit, zpage, bn, nullptr, stream);
 }
 
 // bn = 0: the wave planner over validated arguments p
@@ -1001,6 +1030,31 @@ static int gemm_big_planned(const Args& p, int layout_a, int layout_b, int act, 
   if (p.R) q.R = p.R + r0 * ldr;
   if (p.rope_pos) q.rope_pos = p.rope_pos + r0;
   return launch_gemm_big(q, layout_a, layout_b, act, out, 128, stream);
+}
+
+// Grouped NT product C[r] = epi(A[row_map[r]] B_g^T) over rows sorted by group g (see GRP above): bf16 out,
+// act 0 or E_SWIGLU (each group's weight = [gate; up]; N % (2 * bn / 2) == 0). tiles: int4 [max_tiles]
+// {group, first row, end row, -}, n_tiles: device count (<= max_tiles). bn: 256 or 128.
+extern "C" int rt_gemm_grouped(const void* A, long lda, const int* row_map, const void* B, long b_stride, long ldb,
+                               void* C, long ldc, const void* tiles, const int* n_tiles, int max_tiles, int N, int K,
+                               int act, const float* glu_p, const void* zpage, int bn, hipStream_t stream) {
+  if (max_tiles <= 0 || N <= 0) return 0;
+  if (K % 8 || N % 8 || ldc % 8 || !zpage || !tiles || !n_tiles || (bn != 128 && bn != 256)) return -1;
+  if (act != E_NONE && (act != E_SWIGLU || N % bn)) return -3;
+  Args p{};
+  p.A = (const bf16_t*)A; p.lda = lda; p.B = (const bf16_t*)B; p.ldb = ldb;
+  p.C = C; p.ldc = ldc; p.M = 0; p.N = N; p.K = K; p.act = act; p.nsplit = 1; p.zpage = (const bf16_t*)zpage;
+  p.group_m = tuning().gemm_group_m;
+  p.grp_tiles = (const int4*)tiles; p.grp_n = n_tiles; p.row_map = row_map; p.b_stride = b_stride;
+  if (glu_p) { p.glu.limit = glu_p[0]; p.glu.alpha = glu_p[1]; p.glu.offset = glu_p[2]; }
+  const int tiles_n = act == E_SWIGLU ? N / bn : (N + bn - 1) / bn;
+  dim3 grid(max_tiles * tiles_n), block(512);
+#define GG(E, BN) hipLaunchKernelGGL((gemm_big_kernel<ROW, ROW, O_BF16, E, BN, false, true>), grid, block, 0, stream, p)
+  if (act == E_SWIGLU) { if (bn == 256) GG(E_SWIGLU, 256); else GG(E_SWIGLU, 128); }
+  else { if (bn == 256) GG(E_NONE, 256); else GG(E_NONE, 128); }
+#undef GG
+  RT_LAUNCH_CHECK();
+  return 0;
 }
 
 // NT GEMM + rotary epilogue (E_ROPE): C = rope(A B^T (+ A2 B2^T) + bias) for a fused qkv
@@ -1115,15 +1169,23 @@ extern "C" int rt_gemm_big_fp8_slabs(const void* A, long lda, const float* sa, c
   return 0;
 }
 
-extern "C" int rt_gemm_splitk_reduce(const float* slabs, int nsplit, int M, int N, const void* bias, int act,
-                                     const void* R, long ldr, void* C, long ldc, hipStream_t stream) {
+extern "C" int rt_gemm_splitk_reduce_glu(const float* slabs, int nsplit, int M, int N, const void* bias, int act,
+                                         const void* R, long ldr, void* C, long ldc, const float* glu_p,
+                                         hipStream_t stream) {
+  GluP gp;
+  if (glu_p) { gp.limit = glu_p[0]; gp.alpha = glu_p[1]; gp.offset = glu_p[2]; }
   const int Nout = act == E_SWIGLU ? N / 2 : N;
   if (Nout % 8 || M <= 0) return M <= 0 ? 0 : -1;
   const long work = (long)M * (Nout / 8);
   hipLaunchKernelGGL(splitk_reduce_kernel, dim3((unsigned)((work + 255) / 256)), dim3(256), 0, stream, slabs, nsplit,
-                     M, N, (const bf16_t*)bias, act, (const bf16_t*)R, ldr, (bf16_t*)C, ldc);
+                     M, N, (const bf16_t*)bias, act, (const bf16_t*)R, ldr, (bf16_t*)C, ldc, gp);
   RT_LAUNCH_CHECK();
   return 0;
+}
+
+extern "C" int rt_gemm_splitk_reduce(const float* slabs, int nsplit, int M, int N, const void* bias, int act,
+                                     const void* R, long ldr, void* C, long ldc, hipStream_t stream) {
+  return rt_gemm_splitk_reduce_glu(slabs, nsplit, M, N, bias, act, R, ldr, C, ldc, nullptr, stream);
 }
 
 // 64x64-tile GEMM (narrow LoRA products). out: 0 bf16, 1 fp32 store, 2 fp32 atomic add (split-K),

@@ -1,0 +1,849 @@
+// Latent attention for gfx950: per token one normed latent c [rank] and one rotated key part kr [rot]
+// shared by all heads are cached (a row of KD = rank + rot in a paged pool); per head
+//   k = [W_uk c, kr],  v = W_uv c,  score = (q_unrotated . W_uk c + q_rotated . kr) * scale,
+// softmax whose denominator also holds exp(sink_h), output times sigmoid(gate).
+//
+// Cache: pool [pages][64][KD], page table [rows][max_pages] int32 (page 0 is never given to a request:
+// rows without one point at it). A token of the batch is (row, position); its keys are 0 .. position.
+//
+// Few query tokens per request (decode, short portions) run the absorbed form: the query is moved into
+// latent space once (q_abs = [W_uk^T q_unrotated, q_rotated], KD wide), so scores and the weighted sum
+// both read the cached rows directly and all heads share them:
+//   latent_prep -> (absorb product) -> latent_decode (split over key partitions) -> latent_out
+// Longer portions expand the request's keys and values once per layer (a GEMM over the gathered rows)
+// and run a flash kernel over [unrotated | rotated] heads:
+//   latent_prep -> latent_gather -> (expand GEMM) -> latent_prefill
+// latent_any is the absorbed attention for any size and for fp32 (one workgroup per token and head).
+#include "rt_common.h"
+
+#include <algorithm>
+
+namespace rt {
+namespace la {
+
+typedef __attribute__((address_space(3))) void lds_void;
+constexpr int PAGE = 64;
+
+template <typename T> __device__ __forceinline__ float ld(const T* p);
+template <> __device__ __forceinline__ float ld<bf16_t>(const bf16_t* p) { return bf2f(*p); }
+template <> __device__ __forceinline__ float ld<float>(const float* p) { return *p; }
+template <typename T> __device__ __forceinline__ void st(T* p, float v);
+template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
+template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
+
+__device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
+  uint4 v;
+  v.x = pack2bf(a[0], a[1]);
+  v.y = pack2bf(a[2], a[3]);
+  v.z = pack2bf(b[0], b[1]);
+  v.w = pack2bf(b[2], b[3]);
+  return __builtin_bit_cast(bf16x8, v);
+}
+__device__ __forceinline__ bf16x8 cat4(const rt_s16x4& lo, const rt_s16x4& hi) {
+  typedef __attribute__((ext_vector_type(8))) short s16x8;
+  s16x8 v = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
+  return __builtin_bit_cast(bf16x8, v);
+}
+
+// ---------------------------------------------------------------------------------------------
+// prep: latent norm + rotation + cache append (layers with a latent of their own), query rotation
+// ---------------------------------------------------------------------------------------------
+struct PrepArgs {
+  void* proj; long ldp;        // [T, ldp]: q at 0 (heads of dim + rot), dkv at kv_col (rank + rot)
+  int kv_col;                  // < 0: the layer reads another layer's cache
+  const void* norm_w; float eps;
+  const float* cosT; const float* sinT; int max_pos;  // [max_pos, rdims / 2], multiplier included
+  int rdims;                   // rotated leading dimensions of the rot part (interleaved pairs)
+  const int* row; const int* pos;
+  void* pool; const int* tab; int max_pages, n_pages, n_rows;
+  void* qabs; int n_abs;       // tokens [0, n_abs): rotated query part to qabs [.., H, rank + rot]; others in place
+  int H, dim, rot, rank;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a) {
+  __shared__ float sbuf[4];
+  const int t = blockIdx.x, tid = threadIdx.x;
+  T* pr = (T*)a.proj + (long)t * a.ldp;
+  const int pos = min(max(a.pos[t], 0), a.max_pos - 1);
+  const int half = a.rdims / 2, KD = a.rank + a.rot;
+  const float* cs = a.cosT + (long)pos * half;
+  const float* sn = a.sinT + (long)pos * half;
+  if (a.kv_col >= 0) {
+    const int row = a.row[t];
+    const int pg_i = pos / PAGE;
+    const bool ok = row >= 0 && row < a.n_rows && pg_i < a.max_pages;
+    const int page = ok ? a.tab[(long)row * a.max_pages + pg_i] : -1;
+    T* src = pr + a.kv_col;
+    float s = 0.f;
+    for (int c = tid; c < a.rank; c += 256) {
+      const float v = ld(src + c);
+      s += v * v;
+    }
+    const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.rank + a.eps);
+    if (page >= 0 && page < a.n_pages) {
+      T* dst = (T*)a.pool + ((long)page * PAGE + pos % PAGE) * KD;
+      for (int c = tid; c < a.rank; c += 256) st(dst + c, ld(src + c) * rstd * ld((const T*)a.norm_w + c));
+      for (int i = tid; i < a.rot / 2; i += 256) {
+        const float u = ld(src + a.rank + 2 * i), v = ld(src + a.rank + 2 * i + 1);
+        const bool r = i < half;
+        st(dst + a.rank + 2 * i, r ? u * cs[i] - v * sn[i] : u);
+        st(dst + a.rank + 2 * i + 1, r ? v * cs[i] + u * sn[i] : v);
+      }
+    }
+  }
+  const int hp = a.rot / 2;
+  for (int e = tid; e < a.H * hp; e += 256) {
+    const int h = e / hp, i = e % hp;
+    T* q = pr + (long)h * (a.dim + a.rot) + a.dim + 2 * i;
+    const float u = ld(q), v = ld(q + 1);
+    const bool r = i < half;
+    T* d = t < a.n_abs ? (T*)a.qabs + ((long)t * a.H + h) * KD + a.rank + 2 * i : q;
+    st(d, r ? u * cs[i] - v * sn[i] : u);
+    st(d + 1, r ? v * cs[i] + u * sn[i] : v);
+  }
+}
+
+// ---------------------------------------------------------------------------------------------
+// per-head product at few rows: C[t][b][:] = A[t][b][:] W_b^T (absorb: rank x dim per head). MFMA, the
+// weights streamed straight to registers. grid (N / 64, batch, T / 16), wave = 16 columns.
+// ---------------------------------------------------------------------------------------------
+__global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict__ A, long lda, long sA,
+                                                        const bf16_t* __restrict__ W, long ldw, long sW,
+                                                        bf16_t* __restrict__ C, long ldc, long sC, int T, int N, int K) {
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
+  const int n0 = blockIdx.x * 64 + w * 16, b = blockIdx.y, t0 = blockIdx.z * 16;
+  if (n0 >= N) return;
+  const bf16_t* ap = A + (long)min(t0 + r16, T - 1) * lda + b * sA + 8 * q;
+  const bf16_t* wp = W + b * sW + (long)min(n0 + r16, N - 1) * ldw + 8 * q;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = 0; k < K; k += 32) {
+    const bool ok = k + 8 * q < K;
+    const bf16x8 wf = ok ? *(const bf16x8*)(wp + k) : bf16x8{};
+    const bf16x8 af = ok ? *(const bf16x8*)(ap + k) : bf16x8{};
+    // weight as the A operand: acc[r] = C[t0 + r16][n0 + 4 q + r]
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc, 0, 0, 0);
+  }
+  const int t = t0 + r16;
+  if (t >= T) return;
+  bf16_t* c = C + (long)t * ldc + b * sC + n0 + 4 * q;
+#pragma unroll
+  for (int r = 0; r < 4; ++r)
+    if (n0 + 4 * q + r < N) c[r] = f2bf(acc[r]);
+}
+
+// ---------------------------------------------------------------------------------------------
+// absorbed attention over the pool, split over NP key partitions
+// ---------------------------------------------------------------------------------------------
+// Workgroup = (token, group of 16 NH heads, partition), 4 waves. Per 32-key tile (one LDS image, two
+// buffers, LDS-DMA one tile ahead):
+//   scores S^T = K Q^T (key on the MFMA row, head on the lane) by waves (key half, K-dim half) for
+//   NH = 1 and (key half, head tile) for NH = 2; exchanged through LDS in accumulator layout;
+//   every wave runs the same online softmax, packs P as the next MFMA's A operand, and accumulates
+//   O += P V for its own quarter of the latent columns (V = the latent part of the same LDS image,
+//   transposed reads). Two barriers per tile.
+// A row's keys are cut in NP equal partitions (multiples of 32) from its own length, so a captured
+// launch with a fixed NP balances every length. Image rows are CPR = 8 QS + 1 16-B chunks (odd: row
+// reads conflict-free); chunks past KD come from the zero page.
+struct DecArgs {
+  const bf16_t* q;            // [T, H, KD]
+  const bf16_t* pool; const int* tab; int max_pages, n_pages, n_rows;
+  const int* row; const int* pos;
+  float* part; float* ml;     // [T, H, NP, rank], [T, H, NP, 2] (max in log2 units, sum)
+  int T, H, rank, KD, NP, HG;
+  float scale_log2;
+  const bf16_t* zpage;
+};
+
+template <int QS, int RT, int NH>
+__global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
+  constexpr int CPR = 8 * QS + 1, ROWB = CPR * 16;
+  constexpr int NI = (32 * CPR + 255) / 256;         // LDS-DMA instructions per wave and tile
+  constexpr int NIT = (32 * CPR + 63) / 64;          // of the workgroup (the last one may be half used)
+  constexpr int BUFB = NIT * 1024;
+  constexpr int QF = NH == 1 ? QS : 2 * QS;          // query fragments per wave
+  __shared__ __attribute__((aligned(16))) char smem[2 * BUFB + 4096];
+  float* sx = (float*)(smem + 2 * BUFB);             // [4 waves][64 lanes][4]
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int g = lane >> 4, r16 = lane & 15;
+  const int bid = xcd_remap(blockIdx.x, gridDim.x);
+  const int hg = bid % a.HG, part = (bid / a.HG) % a.NP, t = bid / (a.HG * a.NP);
+  const int row = min(max(a.row[t], 0), a.n_rows - 1);
+  const int len = min(a.pos[t] + 1, a.max_pages * PAGE);
+  const int per = ((len + a.NP - 1) / a.NP + 31) & ~31;
+  const int k0 = part * per, k1 = min(len, k0 + per);
+  const int h0 = hg * 16 * NH;
+  if (k0 >= k1) {  // nothing for this partition (uniform over the workgroup)
+    if (tid < 16 * NH && h0 + tid < a.H) {
+      float* m = a.ml + (((long)t * a.H + h0 + tid) * a.NP + part) * 2;
+      m[0] = -INFINITY;
+      m[1] = 0.f;
+    }
+    return;
+  }
+  const int* tab = a.tab + (long)row * a.max_pages;
+
+  // query fragments: lane holds Q[head r16][32 s + 8 g ..]
+  const int kt = w & 1, hi = w >> 1;                 // key half; K-dim half (NH = 1) or head tile (NH = 2)
+  const int qh = h0 + (NH == 2 ? hi * 16 : 0) + r16;
+  const int sbase = NH == 1 ? hi * QS : 0;
+  bf16x8 qf[QF];
+#pragma unroll
+  for (int s = 0; s < QF; ++s) {
+    const int k = 32 * (sbase + s) + 8 * g;
+    qf[s] = (qh < a.H && k < a.KD) ? *(const bf16x8*)(a.q + ((long)t * a.H + qh) * a.KD + k) : bf16x8{};
+  }
+#pragma unroll
+  for (int s = 0; s < QF; ++s) asm volatile("" : "+v"(qf[s]));
+
+  // LDS-DMA sources: instruction j of wave w covers image chunks (4 j + w) * 64 + lane
+  int src[NI];  // element offset inside the tile's first cache row, < 0: zero page
+#pragma unroll
+  for (int j = 0; j < NI; ++j) {
+    const int c = (4 * j + w) * 64 + lane;
+    const int r = c / CPR, cc = c % CPR;
+    src[j] = (r < 32 && cc * 8 < a.KD) ? r * a.KD + cc * 8 : -1;
+  }
+  auto stage = [&](int key0, int buf) {
+    int page = tab[key0 / PAGE];
+    page = min(max(page, 0), a.n_pages - 1);
+    const bf16_t* base = a.pool + ((long)page * PAGE + key0 % PAGE) * a.KD;
+#pragma unroll
+    for (int j = 0; j < NI; ++j) {
+      if (4 * j + w >= NIT) break;  // wave-uniform
+      const bf16_t* p = src[j] >= 0 ? base + src[j] : a.zpage;
+      __builtin_amdgcn_global_load_lds((const void*)p, (lds_void*)(smem + buf * BUFB + (4 * j + w) * 1024), 16, 0, 0);
+    }
+  };
+
+  f32x4 o[NH][RT];
+#pragma unroll
+  for (int n = 0; n < NH; ++n)
+#pragma unroll
+    for (int c = 0; c < RT; ++c) o[n][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m[NH], l[NH];
+#pragma unroll
+  for (int n = 0; n < NH; ++n) { m[n] = -INFINITY; l[n] = 0.f; }
+
+  stage(k0, 0);
+  int buf = 0;
+  for (int key0 = k0; key0 < k1; key0 += 32, buf ^= 1) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this tile's image (issued one tile ago)
+    asm volatile("s_barrier" ::: "memory");           // ... of every wave; the other buffer is free
+    if (key0 + 32 < k1) stage(key0 + 32, buf ^ 1);
+    const char* img = smem + buf * BUFB;
+    // ---- scores ----
+    f32x4 sp = {0.f, 0.f, 0.f, 0.f};
+    {
+      const char* kp = img + (16 * kt + r16) * ROWB + (4 * sbase + g) * 16;
+#pragma unroll
+      for (int s = 0; s < QF; ++s) {
+        const bf16x8 kf = *(const bf16x8*)(kp + s * 64);
+        sp = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], sp, 0, 0, 0);
+      }
+    }
+    *(f32x4*)(sx + (w * 64 + lane) * 4) = sp;
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    asm volatile("s_barrier" ::: "memory");
+    // ---- softmax (identical in every wave) ----
+    bf16x8 pa[NH];
+#pragma unroll
+    for (int n = 0; n < NH; ++n) {
+      f32x4 s2[2];
+#pragma unroll
+      for (int k = 0; k < 2; ++k) {
+        if constexpr (NH == 1)
+          s2[k] = *(const f32x4*)(sx + (k * 64 + lane) * 4) + *(const f32x4*)(sx + ((k + 2) * 64 + lane) * 4);
+        else
+          s2[k] = *(const f32x4*)(sx + ((k + 2 * n) * 64 + lane) * 4);
+      }
+      float mx = -INFINITY;
+#pragma unroll
+      for (int k = 0; k < 2; ++k)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int key = key0 + 16 * k + 4 * g + i;
+          s2[k][i] = key < k1 ? s2[k][i] * a.scale_log2 : -INFINITY;
+          mx = fmaxf(mx, s2[k][i]);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[n], mx);
+      const float mu = mn == -INFINITY ? 0.f : mn;
+      const float alpha = exp2f(m[n] - mu);
+      m[n] = mn;
+      float rs = 0.f;
+#pragma unroll
+      for (int k = 0; k < 2; ++k)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float p = exp2f(s2[k][i] - mu);
+          s2[k][i] = p;
+          rs += p;
+        }
+      rs += __shfl_xor(rs, 16, 64);
+      rs += __shfl_xor(rs, 32, 64);
+      l[n] = l[n] * alpha + rs;
+      pa[n] = pack_p(s2[0], s2[1]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float al = __shfl(alpha, 4 * g + i, 64);
+#pragma unroll
+        for (int c = 0; c < RT; ++c) o[n][c][i] *= al;
+      }
+    }
+    // ---- O += P V: latent columns [16 RT w, 16 RT (w + 1)) ----
+    const uint32_t va = lds_addr(img + (4 * g + ((lane >> 2) & 3)) * ROWB + w * RT * 32 + (lane & 3) * 8);
+    rt_s16x4 v[2 * RT];
+    if constexpr (RT == 8) ds_tr16_frag4<16 * ROWB, 32, 32 + 16 * ROWB>(va, va + 64, va + 128, va + 192, v);
+    else if constexpr (RT == 4) ds_tr16_frag2<16 * ROWB, 32, 32 + 16 * ROWB>(va, va + 64, v);
+    else ds_tr16_x4<16 * ROWB, 32, 32 + 16 * ROWB>(va, v[0], v[1], v[2], v[3]);
+#pragma unroll
+    for (int c = 0; c < RT; ++c) {
+      const bf16x8 vf = cat4(v[2 * c], v[2 * c + 1]);
+#pragma unroll
+      for (int n = 0; n < NH; ++n) o[n][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[n], vf, o[n][c], 0, 0, 0);
+    }
+  }
+  // o[n][c][i]: head h0 + 16 n + 4 g + i, latent column 16 (RT w + c) + r16
+#pragma unroll
+  for (int n = 0; n < NH; ++n) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int h = h0 + 16 * n + 4 * g + i;
+      if (h >= a.H) continue;
+      float* po = a.part + (((long)t * a.H + h) * a.NP + part) * a.rank;
+#pragma unroll
+      for (int c = 0; c < RT; ++c) {
+        const int col = 16 * (RT * w + c) + r16;
+        if (col < a.rank) po[col] = o[n][c][i];
+      }
+    }
+    const int h = h0 + 16 * n + r16;
+    if (w == 0 && g == 0 && h < a.H) {
+      float* pm = a.ml + (((long)t * a.H + h) * a.NP + part) * 2;
+      pm[0] = m[n];
+      pm[1] = l[n];
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------
+// merge of the partitions (+ sink), value expansion W_uv, output gate. grid (H, T / 16, VS), 4 waves
+// ---------------------------------------------------------------------------------------------
+struct OutArgs {
+  const float* part; const float* ml;
+  const float* sink;           // [H] fp32
+  const bf16_t* wuv;           // [H, vdim, rank]
+  const bf16_t* gate; long ldg; // [T, ldg], head h at h * vdim
+  bf16_t* o; long ldo;
+  int T, H, rank, vdim, NP;
+};
+
+__global__ __launch_bounds__(256) void latent_out_kernel(OutArgs a) {
+  extern __shared__ __attribute__((aligned(16))) bf16_t lat[];  // [16][LD]
+  const int h = blockIdx.x, t0 = blockIdx.y * 16;
+  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, r16 = lane & 15, q = lane >> 4;
+  const int rp = (a.rank + 31) & ~31, LD = rp + 8;
+  const float sink2 = a.sink[h] * 1.4426950408889634f;
+  // wave w merges tokens w, w + 4, ...
+  for (int r = w; r < 16; r += 4) {
+    const int t = t0 + r;
+    if (t >= a.T) {
+      for (int c = lane; c < rp; c += 64) lat[r * LD + c] = 0;
+      continue;
+    }
+    const long base = ((long)t * a.H + h) * a.NP;
+    float M = sink2;
+    for (int p = 0; p < a.NP; ++p) M = fmaxf(M, a.ml[(base + p) * 2]);
+    float L = exp2f(sink2 - M);
+    for (int p = 0; p < a.NP; ++p) {
+      const float mp = a.ml[(base + p) * 2];
+      if (mp != -INFINITY) L += a.ml[(base + p) * 2 + 1] * exp2f(mp - M);
+    }
+    const float inv = 1.f / L;
+    for (int c = 2 * lane; c < rp; c += 128) {
+      float y0 = 0.f, y1 = 0.f;
+      if (c < a.rank) {
+        for (int p = 0; p < a.NP; ++p) {
+          const float mp = a.ml[(base + p) * 2];
+          if (mp == -INFINITY) continue;
+          const float f = exp2f(mp - M);
+          const float2 v = *(const float2*)(a.part + (base + p) * a.rank + c);
+          y0 = fmaf(f, v.x, y0);
+          y1 = fmaf(f, v.y, y1);
+        }
+      }
+      *(uint32_t*)(lat + r * LD + c) = pack2bf(y0 * inv, y1 * inv);
+    }
+  }
+  __syncthreads();
+  const int nt = (a.vdim + 15) / 16;
+  for (int vt = blockIdx.z * 4 + w; vt < nt; vt += 4 * gridDim.z) {
+    const bf16_t* wp = a.wuv + ((long)h * a.vdim + min(vt * 16 + r16, a.vdim - 1)) * a.rank + 8 * q;
+    const bf16_t* lp = lat + r16 * LD + 8 * q;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+    for (int k = 0; k < rp; k += 32) {
+      const bf16x8 wf = k + 8 * q < a.rank ? *(const bf16x8*)(wp + k) : bf16x8{};
+      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, *(const bf16x8*)(lp + k), acc, 0, 0, 0);
+    }
+    const int t = t0 + r16;
+    if (t < a.T) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int v = vt * 16 + 4 * q + r;
+        if (v >= a.vdim) continue;
+        const float gx = bf2f(a.gate[(long)t * a.ldg + (long)h * a.vdim + v]);
+        a.o[(long)t * a.ldo + (long)h * a.vdim + v] = f2bf(acc[r] / (1.f + __expf(-gx)));
+      }
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------
+// segments of longer portions
+// ---------------------------------------------------------------------------------------------
+struct Seg { int row, q_off, q_len, kv_off, kv_len, pos0, pad0, pad1; };  // 8 ints
+
+// out [kv rows of all segments, KD] = the cached rows of each segment, dense
+template <typename V>
+__global__ __launch_bounds__(256) void latent_gather_kernel(const V* __restrict__ pool, const int* __restrict__ tab,
+                                                            int max_pages, int n_pages, const Seg* __restrict__ segs,
+                                                            V* __restrict__ out, int vpr) {
+  const Seg s = segs[blockIdx.y];
+  const long n = (long)s.kv_len * vpr;
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
+    const int k = (int)(i / vpr), c = (int)(i % vpr);
+    const int page = min(max(tab[(long)s.row * max_pages + min(k / PAGE, max_pages - 1)], 0), n_pages - 1);
+    out[((long)s.kv_off + k) * vpr + c] = pool[((long)page * PAGE + k % PAGE) * vpr + c];
+  }
+}
+
+// ---------------------------------------------------------------------------------------------
+// flash attention of a portion over its request's expanded keys / values
+// ---------------------------------------------------------------------------------------------
+// The structure of attn_fwd_kernel (swapped S^T = K Q^T, P straight into the next MFMA, register-
+// prefetched double-buffered K / V tiles of 64 keys): 128 query rows of one head per workgroup, 4 waves x
+// 32 rows; a K row is [W_uk c (dim) | kr (rot)] from two sources, padded to DQ columns; value width DV.
+struct PreArgs {
+  const bf16_t* q; long ldq;     // [tokens, ldq], head h at h * (dim + rot), rotated
+  const bf16_t* kv; long ldk;    // expanded [kv rows, ldk]: unrotated keys at h * dim, values at v_col + h * vdim
+  int v_col;
+  const bf16_t* kr; long ldr;    // rotated key part per kv row
+  const float* sink;
+  const bf16_t* gate; long ldg;
+  bf16_t* o; long ldo;
+  const Seg* segs; const int2* tiles; int n_tiles;   // {segment, first query row / 128}
+  int H, dim, rot, vdim;
+  float scale_log2;
+};
+
+template <int DQ>
+__device__ __forceinline__ int kq_off(int r, int c) {
+  const int sw = (DQ / 64) % 2 ? ((r >> 1) & 7) : (r & 15 & (DQ / 8 - 1));
+  return r * (DQ * 2) + ((c ^ sw) << 4);
+}
+template <int DV>
+__device__ __forceinline__ int vv_off(int r, int c) {
+  constexpr int NCH = DV / 8, RPB = 128 / DV;
+  return r * (DV * 2) + ((c ^ (((r / RPB) & (NCH / 2 - 1)) << 1)) << 4);
+}
+
+template <int DQ, int DV>
+__global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
+  constexpr int NQ = DQ / 8, NV = DV / 8, DS = DQ / 32, DT = DV / 16;
+  constexpr int KB = 64 * DQ * 2, VB = 64 * DV * 2;
+  constexpr int OROW = DV + 8;
+  constexpr int TILES = 2 * (KB + VB), OB = 128 * OROW * 2;
+  __shared__ __attribute__((aligned(16))) char smem[TILES > OB ? TILES : OB];
+  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int g = lane >> 4, r16 = lane & 15;
+  const int lin = xcd_remap(blockIdx.x, gridDim.x);
+  const int h = lin / a.n_tiles;
+  const int2 tl = a.tiles[lin % a.n_tiles];
+  const Seg sg = a.segs[tl.x];
+  const int qblk0 = tl.y * 128, q0 = qblk0 + wid * 32;
+  const int kend = min(sg.kv_len, sg.pos0 + min(qblk0 + 128, sg.q_len));
+  const int hd = a.dim + a.rot;
+
+  bf16x8 qf[2][DS];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const int qr = min(q0 + 16 * u + r16, sg.q_len - 1);
+    const bf16_t* qp = a.q + (long)(sg.q_off + qr) * a.ldq + (long)h * hd;
+#pragma unroll
+    for (int s = 0; s < DS; ++s) {
+      const int c = 32 * s + 8 * g;
+      qf[u][s] = c < hd ? *(const bf16x8*)(qp + c) : bf16x8{};
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int s = 0; s < DS; ++s) asm volatile("" : "+v"(qf[u][s]));
+
+  f32x4 o[2][DT];
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+#pragma unroll
+    for (int c = 0; c < DT; ++c) o[u][c] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m[2], l[2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) { m[u] = -INFINITY; l[u] = 0.f; }
+
+  // chunk e of the tile (K then V) by thread tid + 256 r
+  constexpr int CK = 64 * NQ / 256, CV = 64 * NV / 256;
+  u32x4 kreg[CK], vreg[CV];
+  const bf16_t* kvb = a.kv + (long)sg.kv_off * a.ldk + (long)h * a.dim;
+  const bf16_t* vb = a.kv + (long)sg.kv_off * a.ldk + a.v_col + (long)h * a.vdim;
+  const bf16_t* krb = a.kr + (long)sg.kv_off * a.ldr;
+  auto load_tile = [&](int kv0) {
+#pragma unroll
+    for (int r = 0; r < CK; ++r) {
+      const int e = tid + 256 * r, key = e / NQ, c = (e % NQ) * 8;
+      const long kk = min(kv0 + key, sg.kv_len - 1);
+      const bf16_t* p = c < a.dim ? kvb + kk * a.ldk + c : krb + kk * a.ldr + (c - a.dim);
+      kreg[r] = c < hd ? *(const u32x4*)p : u32x4{0, 0, 0, 0};
+    }
+#pragma unroll
+    for (int r = 0; r < CV; ++r) {
+      const int e = tid + 256 * r, key = e / NV, c = (e % NV) * 8;
+      const long kk = min(kv0 + key, sg.kv_len - 1);
+      vreg[r] = c < a.vdim ? *(const u32x4*)(vb + kk * a.ldk + c) : u32x4{0, 0, 0, 0};
+    }
+  };
+  auto store_tile = [&](char* kd) {
+    char* vd = kd + KB;
+#pragma unroll
+    for (int r = 0; r < CK; ++r) {
+      const int e = tid + 256 * r;
+      *(u32x4*)(kd + kq_off<DQ>(e / NQ, e % NQ)) = kreg[r];
+    }
+#pragma unroll
+    for (int r = 0; r < CV; ++r) {
+      const int e = tid + 256 * r;
+      *(u32x4*)(vd + vv_off<DV>(e / NV, e % NV)) = vreg[r];
+    }
+  };
+  load_tile(0);
+  store_tile(smem);
+  __syncthreads();
+  int cur = 0;
+  for (int kv0 = 0; kv0 < kend; kv0 += 64) {
+    const bool has_next = kv0 + 64 < kend;
+    if (has_next) load_tile(kv0 + 64);
+    char* Ks = smem + cur * (KB + VB);
+    char* Vs = Ks + KB;
+    f32x4 stt[4][2];
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int u = 0; u < 2; ++u) stt[t][u] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int t = 0; t < 4; ++t)
+#pragma unroll
+      for (int s = 0; s < DS; ++s) {
+        const bf16x8 kf = *(const bf16x8*)(Ks + kq_off<DQ>(16 * t + r16, 4 * s + g));
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+          stt[t][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[u][s], stt[t][u], 0, 0, 0);
+      }
+    const bool full = kv0 + 63 <= sg.pos0 + q0 && kv0 + 63 < kend;
+    float alpha[2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          float x = stt[t][u][i] * a.scale_log2;
+          if (!full) {
+            const int kk = kv0 + 16 * t + 4 * g + i;
+            x = kk < kend && kk <= sg.pos0 + q0 + 16 * u + r16 ? x : -INFINITY;
+          }
+          stt[t][u][i] = x;
+          mx = fmaxf(mx, x);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float mn = fmaxf(m[u], mx);
+      const float mu = mn == -INFINITY ? 0.f : mn;
+      alpha[u] = exp2f(m[u] - mu);
+      m[u] = mn;
+      float rs = 0.f;
+#pragma unroll
+      for (int t = 0; t < 4; ++t)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float p = exp2f(stt[t][u][i] - mu);
+          stt[t][u][i] = p;
+          rs += p;
+        }
+      rs += __shfl_xor(rs, 16, 64);
+      rs += __shfl_xor(rs, 32, 64);
+      l[u] = l[u] * alpha[u] + rs;
+    }
+#pragma unroll
+    for (int u = 0; u < 2; ++u)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float al = __shfl(alpha[u], 4 * g + i, 64);
+#pragma unroll
+        for (int c = 0; c < DT; ++c) o[u][c][i] *= al;
+      }
+#pragma unroll
+    for (int ks = 0; ks < 2; ++ks) {
+      bf16x8 pa[2];
+#pragma unroll
+      for (int u = 0; u < 2; ++u) pa[u] = pack_p(stt[2 * ks][u], stt[2 * ks + 1][u]);
+      const int qrow = lane >> 2 & 3, pcol = lane & 3;
+#pragma unroll
+      for (int c = 0; c < DT; ++c) {
+        const int key_a = 32 * ks + 4 * g + qrow;
+        const int col = 16 * c + 4 * pcol;
+        typedef __attribute__((ext_vector_type(4))) short s16x4;
+        typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
+        const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (lds_s16x4*)(Vs + vv_off<DV>(key_a, col >> 3) + ((col & 7) << 1)));
+        const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+            (lds_s16x4*)(Vs + vv_off<DV>(key_a + 16, col >> 3) + ((col & 7) << 1)));
+        const bf16x8 vf = cat4(lo, hi);
+#pragma unroll
+        for (int u = 0; u < 2; ++u) o[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], vf, o[u][c], 0, 0, 0);
+      }
+    }
+    if (has_next) store_tile(smem + (cur ^ 1) * (KB + VB));
+    __syncthreads();
+    cur ^= 1;
+  }
+  // the sink joins the denominator; O through LDS, gated on the way out
+  const float sink2 = a.sink[h] * 1.4426950408889634f;
+  bf16_t* Os = (bf16_t*)smem;
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    const float M = fmaxf(m[u], sink2);
+    const float f = exp2f(m[u] - M);
+    const float sc = f / (l[u] * f + exp2f(sink2 - M));
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float si = __shfl(sc, 4 * g + i, 64);
+      const int r = wid * 32 + 16 * u + 4 * g + i;
+#pragma unroll
+      for (int c = 0; c < DT; ++c) Os[r * OROW + 16 * c + r16] = f2bf(o[u][c][i] * si);
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < 128 * NV; e += 256) {
+    const int r = e / NV, c = (e % NV) * 8;
+    if (qblk0 + r < sg.q_len && c < a.vdim) {
+      const long tok = sg.q_off + qblk0 + r;
+      float v[8], x[8];
+      unpack8(*(const uint4*)(Os + r * OROW + c), v);
+      unpack8(*(const uint4*)(a.gate + tok * a.ldg + (long)h * a.vdim + c), x);
+#pragma unroll
+      for (int k = 0; k < 8; ++k) v[k] = v[k] / (1.f + __expf(-x[k]));
+      *(uint4*)(a.o + tok * a.ldo + (long)h * a.vdim + c) = pack8(v);
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------------
+// absorbed attention of any size and type: one workgroup per (token, head), 256 keys at a time
+// ---------------------------------------------------------------------------------------------
+struct LatAnyArgs {
+  const void* q; const void* pool; const int* tab; int max_pages, n_pages, n_rows;
+  const int* row; const int* pos;
+  const float* sink;
+  void* o;                     // [T, H, rank] latent outputs (softmax with the sink applied)
+  int H, rank, KD;
+  float scale;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void latent_any_kernel(LatAnyArgs a) {
+  extern __shared__ float sm[];  // q [KD], acc [rank], p [256], sbuf [4]
+  float* qs = sm;
+  float* acc = qs + a.KD;
+  float* ps = acc + a.rank;
+  float* sbuf = ps + 256;
+  const int h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x;
+  const int row = min(max(a.row[t], 0), a.n_rows - 1);
+  const int len = min(a.pos[t] + 1, a.max_pages * PAGE);
+  const int* tab = a.tab + (long)row * a.max_pages;
+  for (int c = tid; c < a.KD; c += 256) qs[c] = ld((const T*)a.q + ((long)t * a.H + h) * a.KD + c);
+  for (int c = tid; c < a.rank; c += 256) acc[c] = 0.f;
+  float m = a.sink[h], l = 1.f;  // the sink: exp(sink - m) = 1
+  __syncthreads();
+  for (int k0 = 0; k0 < len; k0 += 256) {
+    const int key = k0 + tid;
+    float s = -INFINITY;
+    if (key < len) {
+      const int page = min(max(tab[key / PAGE], 0), a.n_pages - 1);
+      const T* kp = (const T*)a.pool + ((long)page * PAGE + key % PAGE) * a.KD;
+      float d = 0.f;
+      for (int c = 0; c < a.KD; ++c) d = fmaf(qs[c], ld(kp + c), d);
+      s = d * a.scale;
+    }
+    const float mn = fmaxf(m, block_max(s, sbuf));
+    const float alpha = expf(m - mn);
+    const float p = key < len ? expf(s - mn) : 0.f;
+    ps[tid] = p;
+    l = l * alpha + block_sum(p, sbuf);
+    m = mn;
+    __syncthreads();
+    const int n = min(256, len - k0);
+    for (int c = tid; c < a.rank; c += 256) {
+      float y = acc[c] * alpha;
+      for (int k = 0; k < n; ++k) {
+        const int kk = k0 + k;
+        const int page = min(max(tab[kk / PAGE], 0), a.n_pages - 1);
+        y = fmaf(ps[k], ld((const T*)a.pool + ((long)page * PAGE + kk % PAGE) * a.KD + c), y);
+      }
+      acc[c] = y;
+    }
+    __syncthreads();
+  }
+  for (int c = tid; c < a.rank; c += 256) st((T*)a.o + ((long)t * a.H + h) * a.rank + c, acc[c] / l);
+}
+
+}  // namespace la
+}  // namespace rt
+
+using namespace rt;
+using namespace rt::la;
+
+extern "C" int rt_latent_prep(int f32, void* proj, long ldp, int kv_col, const void* norm_w, float eps,
+                              const float* cosT, const float* sinT, int max_pos, int rdims, const int* row,
+                              const int* pos, void* pool, const int* tab, int max_pages, int n_pages, int n_rows,
+                              void* qabs, int n_abs, int T, int H, int dim, int rot, int rank, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (rot % 2 || rdims % 2 || rdims > rot) return -1;
+  PrepArgs a{proj, ldp, kv_col, norm_w, eps, cosT, sinT, max_pos, rdims, row, pos, pool, tab, max_pages, n_pages,
+             n_rows, qabs, n_abs, H, dim, rot, rank};
+  if (f32) hipLaunchKernelGGL((latent_prep_kernel<float>), dim3(T), dim3(256), 0, stream, a);
+  else hipLaunchKernelGGL((latent_prep_kernel<bf16_t>), dim3(T), dim3(256), 0, stream, a);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+// bf16, K % 8 == 0, 16-B aligned rows
+extern "C" int rt_head_gemm(const void* A, long lda, long sA, const void* W, long ldw, long sW, void* C, long ldc,
+                            long sC, int T, int N, int K, int batch, hipStream_t stream) {
+  if (T <= 0 || N <= 0 || batch <= 0) return 0;
+  if (K % 8 || lda % 8 || sA % 8 || ldw % 8 || sW % 8 || batch > 65535 || (T + 15) / 16 > 65535) return -1;
+  dim3 grid((N + 63) / 64, batch, (T + 15) / 16);
+  hipLaunchKernelGGL(head_gemm_kernel, grid, dim3(256), 0, stream, (const bf16_t*)A, lda, sA, (const bf16_t*)W, ldw,
+                     sW, (bf16_t*)C, ldc, sC, T, N, K);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_latent_decode_ok(int rank, int KD) {
+  return rank % 8 == 0 && KD % 8 == 0 && rank <= 512 && KD <= 640 && (rank > 256 || KD <= 384) && (rank > 128 || KD <= 256);
+}
+
+extern "C" int rt_latent_decode(const void* q, const void* pool, const int* tab, int max_pages, int n_pages, int n_rows,
+                                const int* row, const int* pos, float* part, float* ml, int T, int H, int rank, int KD,
+                                int NP, float scale, const void* zpage, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (!rt_latent_decode_ok(rank, KD) || NP < 1 || !zpage) return -1;
+  const int NH = H > 16 ? 2 : 1;
+  const int HG = (H + 16 * NH - 1) / (16 * NH);
+  DecArgs a{(const bf16_t*)q, (const bf16_t*)pool, tab, max_pages, n_pages, n_rows, row, pos, part, ml, T, H, rank, KD,
+            NP, HG, scale * 1.4426950408889634f, (const bf16_t*)zpage};
+  dim3 grid((unsigned)((long)T * HG * NP)), block(256);
+#define LD_(QS, RT)                                                                                       \
+  do {                                                                                                    \
+    if (NH == 1) hipLaunchKernelGGL((latent_decode_kernel<QS, RT, 1>), grid, block, 0, stream, a);        \
+    else hipLaunchKernelGGL((latent_decode_kernel<QS, RT, 2>), grid, block, 0, stream, a);                \
+  } while (0)
+  if (rank <= 128) {
+    if (KD <= 192) LD_(3, 2); else LD_(4, 2);
+  } else if (rank <= 256) {
+    if (KD <= 320) LD_(5, 4); else LD_(6, 4);
+  } else {
+    if (KD <= 576) LD_(9, 8); else LD_(10, 8);
+  }
+#undef LD_
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_latent_out(const float* part, const float* ml, const float* sink, const void* wuv, const void* gate,
+                             long ldg, void* o, long ldo, int T, int H, int rank, int vdim, int NP, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (rank % 8 || rank > 2048 || (T + 15) / 16 > 65535) return -1;
+  OutArgs a{part, ml, sink, (const bf16_t*)wuv, (const bf16_t*)gate, ldg, (bf16_t*)o, ldo, T, H, rank, vdim, NP};
+  const int tt = (T + 15) / 16, nt = (vdim + 15) / 16;
+  int vs = std::max(1, std::min((nt + 3) / 4, 256 / std::max(1, H * tt)));
+  const size_t lds = (size_t)16 * (((rank + 31) & ~31) + 8) * 2;
+  hipLaunchKernelGGL(latent_out_kernel, dim3(H, tt, vs), dim3(256), lds, stream, a);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_latent_gather(int f32, const void* pool, const int* tab, int max_pages, int n_pages, const void* segs,
+                                int n_segs, int max_kv, void* out, int KD, hipStream_t stream) {
+  if (n_segs <= 0 || max_kv <= 0) return 0;
+  if (n_segs > 65535) return -1;
+  const int bytes = KD * (f32 ? 4 : 2);
+  const int vb = bytes % 16 == 0 ? 16 : 2;
+  const int vpr = bytes / vb;
+  const long n = (long)max_kv * vpr;
+  dim3 grid((unsigned)std::min<long>((n + 255) / 256, 4096), n_segs);
+  if (vb == 16)
+    hipLaunchKernelGGL((latent_gather_kernel<u32x4>), grid, dim3(256), 0, stream, (const u32x4*)pool, tab, max_pages,
+                       n_pages, (const Seg*)segs, (u32x4*)out, vpr);
+  else
+    hipLaunchKernelGGL((latent_gather_kernel<uint16_t>), grid, dim3(256), 0, stream, (const uint16_t*)pool, tab,
+                       max_pages, n_pages, (const Seg*)segs, (uint16_t*)out, vpr);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_latent_prefill_ok(int dim, int rot, int vdim) {
+  return dim % 8 == 0 && rot % 8 == 0 && vdim % 8 == 0 && dim + rot <= 256 && vdim <= 128;
+}
+
+extern "C" int rt_latent_prefill(const void* q, long ldq, const void* kv, long ldk, int v_col, const void* kr, long ldr,
+                                 const float* sink, const void* gate, long ldg, void* o, long ldo, const void* segs,
+                                 const void* tiles, int n_tiles, int H, int dim, int rot, int vdim, float scale,
+                                 hipStream_t stream) {
+  if (n_tiles <= 0) return 0;
+  if (!rt_latent_prefill_ok(dim, rot, vdim) || ldq % 8 || ldk % 8 || v_col % 8 || ldr % 8 || ldg % 8 || ldo % 8) return -1;
+  PreArgs a{(const bf16_t*)q, ldq, (const bf16_t*)kv, ldk, v_col, (const bf16_t*)kr, ldr, sink, (const bf16_t*)gate, ldg,
+            (bf16_t*)o, ldo, (const Seg*)segs, (const int2*)tiles, n_tiles, H, dim, rot, vdim,
+            scale * 1.4426950408889634f};
+  dim3 grid((unsigned)((long)n_tiles * H)), block(256);
+  const int dq = dim + rot;
+#define LP_(DQ)                                                                                         \
+  do {                                                                                                  \
+    if (vdim <= 64) hipLaunchKernelGGL((latent_prefill_kernel<DQ, 64>), grid, block, 0, stream, a);     \
+    else hipLaunchKernelGGL((latent_prefill_kernel<DQ, 128>), grid, block, 0, stream, a);               \
+  } while (0)
+  if (dq <= 64) LP_(64);
+  else if (dq <= 128) LP_(128);
+  else if (dq <= 192) LP_(192);
+  else LP_(256);
+#undef LP_
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_latent_any(int f32, const void* q, const void* pool, const int* tab, int max_pages, int n_pages,
+                             int n_rows, const int* row, const int* pos, const float* sink, void* o, int T, int H,
+                             int rank, int KD, float scale, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (T > 65535) return -1;
+  const size_t lds = (size_t)(KD + rank + 256 + 4) * 4;
+  if (lds > 65536) return -2;
+  LatAnyArgs a{q, pool, tab, max_pages, n_pages, n_rows, row, pos, sink, o, H, rank, KD, scale};
+  if (f32) hipLaunchKernelGGL((latent_any_kernel<float>), dim3(H, T), dim3(256), lds, stream, a);
+  else hipLaunchKernelGGL((latent_any_kernel<bf16_t>), dim3(H, T), dim3(256), lds, stream, a);
+  RT_LAUNCH_CHECK();
+  return 0;
+}

@@ -1,0 +1,285 @@
+// Mixture-of-experts feed-forward for gfx950: routing, the sort of (token, slot) pairs by expert, and
+// the grouped expert products at few rows per expert (many rows per expert: the GRP form of
+// gemm_big_kernel). All row counts stay on the device: every launch has a fixed grid, so a decode step
+// with these kernels can be captured in a graph.
+//
+//   moe_route    logits [T, ldl] fp32 (columns [0, E) experts, optional column E = shared gate) ->
+//                per token the `top` experts of the largest choice score softmax(z) + correction and
+//                their weights softmax(z) (not renormalised), then `nshared` slots of the shared
+//                expert (groups E .. E + nshared - 1) with weight sigmoid(shared gate);
+//   moe_sort     one workgroup per group: stable counting sort of the pairs -> group offsets, the token
+//                behind each sorted row, and the sorted row of each pair;
+//   moe_tiles    256-row tiles of the sorted rows for the grouped token-parallel GEMM;
+//   moe_rows     grouped product at few rows per group: weights streamed straight to registers as MFMA
+//                operands (each read once per 64 rows), 4 waves splitting K, reduced through LDS;
+//                PAIR: gate and up rows together with the gated linear unit in the epilogue.
+#include "rt_common.h"
+
+namespace rt {
+
+// one wave per token
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, long ldl,
+                                                        const float* __restrict__ correction, int T, int E, int top,
+                                                        int nshared, int gate_col, int* __restrict__ idx,
+                                                        float* __restrict__ wt) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (t >= T) return;
+  constexpr int MAXV = 8;  // E <= 512
+  const float* z = logits + (long)t * ldl;
+  float s[MAXV], c[MAXV];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = e < E ? z[e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
+  mx = wave_max(mx);
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    s[i] = lane + 64 * i < E ? expf(s[i] - mx) : 0.f;
+    sum += s[i];
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = s[i] / sum;
+    c[i] = e < E ? s[i] + correction[e] : -INFINITY;
+  }
+  const int slots = top + nshared;
+  for (int k = 0; k < top; ++k) {
+    // largest remaining choice score; equal scores: the lower expert. `be` always names an expert that
+    // is still free, also when scores are not comparable (NaN)
+    float bv = -INFINITY, bs = 0.f;
+    int be = 1 << 30;
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i) {
+      const int e = lane + 64 * i;
+      const bool open = e < E && c[i] != -INFINITY;
+      if (open && (be == (1 << 30) || c[i] > bv)) { bv = c[i]; bs = s[i]; be = e; }
+    }
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64), os = __shfl_xor(bs, o, 64);
+      const int oe = __shfl_xor(be, o, 64);
+      const bool take = oe != (1 << 30) && (be == (1 << 30) || ov > bv || (!(bv > ov) && oe < be));
+      if (take) { bv = ov; bs = os; be = oe; }
+    }
+    be = __builtin_amdgcn_readfirstlane(be);
+    if (be >= E) be = k;  // no open expert left (only with a choice score of -inf)
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+      if (lane + 64 * i == be) c[i] = -INFINITY;
+    if (lane == 0) {
+      idx[(long)t * slots + k] = be;
+      wt[(long)t * slots + k] = bs;
+    }
+  }
+  if (lane < nshared) {
+    idx[(long)t * slots + top + lane] = E + lane;
+    wt[(long)t * slots + top + lane] = gate_col >= 0 ? 1.f / (1.f + expf(-z[gate_col])) : 1.f;
+  }
+}
+
+// workgroup g: counts the pairs of lower groups (its offset), then places its own pairs in pair order
+__global__ __launch_bounds__(256) void moe_sort_kernel(const int* __restrict__ idx, int P, int slots, int G,
+                                                       int* __restrict__ offs, int* __restrict__ row_tok,
+                                                       int* __restrict__ pair_pos) {
+  __shared__ int cnt[4][2];
+  __shared__ int wbase[4];
+  const int g = blockIdx.x, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  int less = 0, mine = 0;
+  for (int i = tid; i < P; i += 256) {
+    const int e = idx[i];
+    less += e < g;
+    mine += e == g;
+  }
+#pragma unroll
+  for (int o = 32; o > 0; o >>= 1) {
+    less += __shfl_xor(less, o, 64);
+    mine += __shfl_xor(mine, o, 64);
+  }
+  if (lane == 0) { cnt[w][0] = less; cnt[w][1] = mine; }
+  __syncthreads();
+  const int base = cnt[0][0] + cnt[1][0] + cnt[2][0] + cnt[3][0];
+  const int total = cnt[0][1] + cnt[1][1] + cnt[2][1] + cnt[3][1];
+  if (tid == 0) {
+    offs[g] = base;
+    if (g == G - 1) offs[G] = base + total;
+  }
+  int run = base;
+  for (int i0 = 0; i0 < P; i0 += 256) {
+    const int i = i0 + tid;
+    const bool hit = i < P && idx[i] == g;
+    const unsigned long long m = __ballot(hit);
+    if (lane == 0) wbase[w] = __popcll(m);
+    __syncthreads();
+    int before = run;
+    for (int q = 0; q < w; ++q) before += wbase[q];
+    if (hit) {
+      const int pos = before + __popcll(m & ((1ull << lane) - 1));
+      row_tok[pos] = i / slots;
+      pair_pos[i] = pos;
+    }
+    run += wbase[0] + wbase[1] + wbase[2] + wbase[3];
+    __syncthreads();
+  }
+}
+
+__global__ __launch_bounds__(1024) void moe_tiles_kernel(const int* __restrict__ offs, int G, int rows, int max_tiles,
+                                                         int4* __restrict__ tiles, int* __restrict__ n_tiles) {
+  __shared__ int first[1025];
+  const int g = threadIdx.x;
+  if (g < G) first[g + 1] = (offs[g + 1] - offs[g] + rows - 1) / rows;
+  if (g == 0) first[0] = 0;
+  __syncthreads();
+  if (g == 0)
+    for (int i = 0; i < G; ++i) first[i + 1] += first[i];
+  __syncthreads();
+  if (g < G) {
+    const int b = offs[g], e = offs[g + 1];
+    for (int i = first[g]; i < first[g + 1] && i < max_tiles; ++i) {
+      const int m0 = b + (i - first[g]) * rows;
+      tiles[i] = make_int4(g, m0, min(m0 + rows, e), 0);
+    }
+  }
+  if (g == 0) *n_tiles = min(first[G], max_tiles);
+}
+
+struct MoeRowsArgs {
+  const bf16_t* A; long lda; const int* row_map;  // A row of sorted row r (null: r)
+  const bf16_t* W; long sW, ldw;                  // group g: W + g * sW; PAIR: [gate; up], N rows each
+  void* C; long ldc;
+  const int* offs;
+  int N, K;
+  GluP glu;
+};
+
+// grid (N / 16, groups). Each wave takes K / 4 of the reduction in 32-deep MFMA steps.
+template <bool PAIR, bool OUT_F32, int MT>
+__global__ __launch_bounds__(256) void moe_rows_kernel(MoeRowsArgs p) {
+  constexpr int NB = PAIR ? 2 : 1;
+  __shared__ float red[4][MT * NB][64 * 4];
+  const int g = blockIdx.y, n0 = blockIdx.x * 16;
+  const int beg = p.offs[g], end = p.offs[g + 1];
+  if (beg >= end) return;
+  const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+  const int r16 = lane & 15, q = lane >> 4;
+  const bf16_t* W = p.W + (long)g * p.sW;
+  const bf16_t* wp[NB];
+#pragma unroll
+  for (int b = 0; b < NB; ++b) wp[b] = W + (long)(b * p.N + min(n0 + r16, p.N - 1)) * p.ldw + 8 * q;
+  const int steps = (p.K + 31) / 32;
+  const int per = (steps + 3) / 4;
+  const int s0 = w * per, s1 = min(steps, s0 + per);
+  for (int m0 = beg; m0 < end; m0 += 16 * MT) {
+    const bf16_t* ap[MT];
+#pragma unroll
+    for (int i = 0; i < MT; ++i) {
+      const int r = min(m0 + 16 * i + r16, end - 1);
+      ap[i] = p.A + (long)(p.row_map ? p.row_map[r] : r) * p.lda + 8 * q;
+    }
+    f32x4 acc[MT][NB];
+#pragma unroll
+    for (int i = 0; i < MT; ++i)
+#pragma unroll
+      for (int b = 0; b < NB; ++b) acc[i][b] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int mt = min(MT, (end - m0 + 15) / 16);
+#pragma unroll 4
+    for (int s = s0; s < s1; ++s) {
+      const int k = s * 32;
+      const bool ok = k + 8 * q < p.K;  // K % 8 == 0: a lane's 8 elements are all in or all out
+      bf16x8 wf[NB];
+#pragma unroll
+      for (int b = 0; b < NB; ++b)
+        wf[b] = ok ? __builtin_bit_cast(bf16x8, load_nt16(wp[b] + k)) : bf16x8{};
+#pragma unroll
+      for (int i = 0; i < MT; ++i) {
+        if (i < mt) {
+          const bf16x8 af = ok ? *(const bf16x8*)(ap[i] + k) : bf16x8{};
+#pragma unroll
+          for (int b = 0; b < NB; ++b) acc[i][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af, wf[b], acc[i][b], 0, 0, 0);
+        }
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < MT; ++i)
+#pragma unroll
+      for (int b = 0; b < NB; ++b) *(f32x4*)&red[w][i * NB + b][lane * 4] = acc[i][b];
+    __syncthreads();
+    // acc[r]: row 4 q + r, column r16; wave w finishes tiles w, w + 4, ...
+    for (int i = w; i < mt; i += 4) {
+      f32x4 v[NB];
+#pragma unroll
+      for (int b = 0; b < NB; ++b) {
+        v[b] = *(const f32x4*)&red[0][i * NB + b][lane * 4];
+#pragma unroll
+        for (int x = 1; x < 4; ++x) v[b] += *(const f32x4*)&red[x][i * NB + b][lane * 4];
+      }
+      const int col = n0 + r16;
+      if (col < p.N) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int row = m0 + 16 * i + 4 * q + r;
+          if (row >= end) continue;
+          const float y = PAIR ? glu(v[0][r], v[NB - 1][r], p.glu) : v[0][r];
+          if constexpr (OUT_F32) ((float*)p.C)[(long)row * p.ldc + col] = y;
+          else ((bf16_t*)p.C)[(long)row * p.ldc + col] = f2bf(y);
+        }
+      }
+    }
+    __syncthreads();
+  }
+}
+
+}  // namespace rt
+
+using namespace rt;
+
+extern "C" int rt_moe_route(const float* logits, long ldl, const float* correction, int T, int E, int top, int nshared,
+                            int gate_col, int* idx, float* wt, hipStream_t stream) {
+  if (T <= 0) return 0;
+  if (E < 1 || E > 512 || top < 1 || top > E || nshared < 0 || nshared > 64) return -1;
+  hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, ldl, correction, T, E, top,
+                     nshared, gate_col, idx, wt);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+// tiles / n_tiles may be null (few rows per group: no tile list)
+extern "C" int rt_moe_sort(const int* idx, int P, int slots, int G, int* offs, int* row_tok, int* pair_pos,
+                           int tile_rows, int max_tiles, void* tiles, int* n_tiles, hipStream_t stream) {
+  if (P <= 0) return 0;
+  if (G < 1 || G > 1024) return -1;
+  hipLaunchKernelGGL(moe_sort_kernel, dim3(G), dim3(256), 0, stream, idx, P, slots, G, offs, row_tok, pair_pos);
+  if (tiles) {
+    hipLaunchKernelGGL(moe_tiles_kernel, dim3(1), dim3(1024), 0, stream, offs, G, tile_rows, max_tiles, (int4*)tiles,
+                       n_tiles);
+  }
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+// C[r] = A[row_map[r]] W_g^T (pair: gated linear unit of [gate; up] halves, N = half) for the rows of
+// every group; mean_rows: expected rows per group (picks the row tiles per pass)
+extern "C" int rt_moe_rows(const void* A, long lda, const int* row_map, const void* W, long sW, long ldw, void* C,
+                           long ldc, const int* offs, int G, int N, int K, int pair, int out_f32, int mean_rows,
+                           const float* glu_p, hipStream_t stream) {
+  if (G <= 0 || N <= 0) return 0;
+  if (K % 8 || ldw % 8 || lda % 8 || (pair && out_f32) || G > 65535) return -1;
+  MoeRowsArgs p{(const bf16_t*)A, lda, row_map, (const bf16_t*)W, sW, ldw, C, ldc, offs, N, K, GluP{}};
+  if (glu_p) { p.glu.limit = glu_p[0]; p.glu.alpha = glu_p[1]; p.glu.offset = glu_p[2]; }
+  dim3 grid((N + 15) / 16, G), block(256);
+#define MR(MTV)                                                                                          \
+  if (pair) hipLaunchKernelGGL((moe_rows_kernel<true, false, MTV>), grid, block, 0, stream, p);          \
+  else if (out_f32) hipLaunchKernelGGL((moe_rows_kernel<false, true, MTV>), grid, block, 0, stream, p);  \
+  else hipLaunchKernelGGL((moe_rows_kernel<false, false, MTV>), grid, block, 0, stream, p);
+  if (mean_rows <= 12) { MR(1) }
+  else if (mean_rows <= 28) { MR(2) }
+  else { MR(4) }
+#undef MR
+  RT_LAUNCH_CHECK();
+  return 0;
+}

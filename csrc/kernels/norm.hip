@@ -270,3 +270,188 @@ extern "C" int rt_norm_bwd(int layernorm, const void* dy, const void* h, const v
   RT_LAUNCH_CHECK();
   return 0;
 }
+
+// ---------------------------------------------------------------------------------------------
+// Branch norm: the step between two sublayers of a decoder with a norm before and after each
+// (fp32 residual stream x [T, H], everything in fp32):
+//   x += rms(y) * w_branch          (y = the sublayer's output)
+//   h  = rms(x) * w_next            (the next sublayer's input, rounded once to the activation type)
+// One workgroup per row, the row in registers: x is read and written once, y read once. The branch y is
+//   Y_NONE    absent (first norm of a pass): x = table[ids[row]] when a table is given;
+//   Y_ACT     rows of the activation type;
+//   Y_SLABS   the sum of nsplit fp32 slabs (split-K partial products; 1 slab = an fp32 tensor);
+//   Y_PAIRS   a mixture: sum over the row's K slots of pair_w[row, k] * y[pair_pos[row, k]].
+// w_next == null: no h (x only).
+// ---------------------------------------------------------------------------------------------
+namespace rt {
+
+enum BranchKind { Y_NONE = 0, Y_ACT = 1, Y_SLABS = 2, Y_PAIRS = 3, Y_PAIRS_F32 = 4 };
+
+struct BranchArgs {
+  float* x;
+  const void* y; long y_stride; int nsplit;  // Y_SLABS: slab stride in floats
+  const void* w_branch; const void* w_next; void* h;
+  const void* table; const long* ids; int vocab;
+  const float* pair_w; const int* pair_pos; int K;
+  int H;
+  float eps;
+};
+
+template <typename T> __device__ __forceinline__ float act_ld(const T* p);
+template <> __device__ __forceinline__ float act_ld<bf16_t>(const bf16_t* p) { return bf2f(*p); }
+template <> __device__ __forceinline__ float act_ld<float>(const float* p) { return *p; }
+template <typename T> __device__ __forceinline__ void act_st(T* p, float v);
+template <> __device__ __forceinline__ void act_st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
+template <> __device__ __forceinline__ void act_st<float>(float* p, float v) { *p = v; }
+
+template <typename T, int V>
+__device__ __forceinline__ void act_ldv(const T* p, float* o) {
+  if constexpr (V == 4 && sizeof(T) == 2) {
+    const uint2 v = *(const uint2*)p;
+    o[0] = __uint_as_float(v.x << 16); o[1] = __uint_as_float(v.x & 0xffff0000u);
+    o[2] = __uint_as_float(v.y << 16); o[3] = __uint_as_float(v.y & 0xffff0000u);
+  } else if constexpr (V == 4) {
+    const float4 v = *(const float4*)p;
+    o[0] = v.x; o[1] = v.y; o[2] = v.z; o[3] = v.w;
+  } else {
+#pragma unroll
+    for (int e = 0; e < V; ++e) o[e] = act_ld(p + e);
+  }
+}
+template <typename T, int V>
+__device__ __forceinline__ void act_stv(T* p, const float* o) {
+  if constexpr (V == 4 && sizeof(T) == 2) *(uint2*)p = make_uint2(pack2bf(o[0], o[1]), pack2bf(o[2], o[3]));
+  else if constexpr (V == 4) *(float4*)p = make_float4(o[0], o[1], o[2], o[3]);
+  else {
+#pragma unroll
+    for (int e = 0; e < V; ++e) act_st(p + e, o[e]);
+  }
+}
+
+// V elements per access (4, or 1 when H % 4 != 0), NV accesses per thread
+template <typename T, int KIND, int V, int NV>
+__global__ __launch_bounds__(512) void branch_norm_kernel(BranchArgs a) {
+  __shared__ float sbuf[8];
+  const long row = blockIdx.x;
+  const int nvec = a.H / V;
+  float* xr = a.x + row * a.H;
+  float x[NV][V], y[NV][V];
+  long tok = 0;
+  if (KIND == Y_NONE && a.table) {
+    tok = a.ids[row];
+    tok = tok < 0 ? 0 : (tok >= a.vocab ? a.vocab - 1 : tok);
+  }
+  float s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+#pragma unroll
+    for (int e = 0; e < V; ++e) { x[i][e] = 0.f; y[i][e] = 0.f; }
+    if (c >= nvec) continue;
+    if (KIND == Y_NONE && a.table) act_ldv<T, V>((const T*)a.table + tok * a.H + c * V, x[i]);
+    else act_ldv<float, V>(xr + c * V, x[i]);
+    if constexpr (KIND == Y_ACT) {
+      act_ldv<T, V>((const T*)a.y + row * a.H + c * V, y[i]);
+    } else if constexpr (KIND == Y_SLABS) {
+      for (int q = 0; q < a.nsplit; ++q) {
+        float t[V];
+        act_ldv<float, V>((const float*)a.y + q * a.y_stride + row * a.H + c * V, t);
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] += t[e];
+      }
+    } else if constexpr (KIND == Y_PAIRS || KIND == Y_PAIRS_F32) {
+      for (int k = 0; k < a.K; ++k) {
+        const float w = a.pair_w[row * a.K + k];
+        const long pr = a.pair_pos[row * a.K + k];
+        float t[V];
+        if constexpr (KIND == Y_PAIRS_F32) act_ldv<float, V>((const float*)a.y + pr * a.H + c * V, t);
+        else act_ldv<T, V>((const T*)a.y + pr * a.H + c * V, t);
+#pragma unroll
+        for (int e = 0; e < V; ++e) y[i][e] = fmaf(w, t[e], y[i][e]);
+      }
+    }
+#pragma unroll
+    for (int e = 0; e < V; ++e) s += y[i][e] * y[i][e];
+  }
+  if constexpr (KIND != Y_NONE) {
+    const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c >= nvec) continue;
+      float w[V];
+      act_ldv<T, V>((const T*)a.w_branch + c * V, w);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[i][e] += y[i][e] * rstd * w[e];
+    }
+  }
+  if (KIND != Y_NONE || a.table) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < nvec) act_stv<float, V>(xr + c * V, x[i]);
+    }
+  }
+  if (!a.w_next) return;
+  s = 0.f;
+#pragma unroll
+  for (int i = 0; i < NV; ++i)
+#pragma unroll
+    for (int e = 0; e < V; ++e) s += x[i][e] * x[i][e];
+  const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = threadIdx.x + i * blockDim.x;
+    if (c >= nvec) continue;
+    float w[V], o[V];
+    act_ldv<T, V>((const T*)a.w_next + c * V, w);
+#pragma unroll
+    for (int e = 0; e < V; ++e) o[e] = x[i][e] * rstd * w[e];
+    act_stv<T, V>((T*)a.h + row * a.H + c * V, o);
+  }
+}
+
+template <typename T, int KIND>
+static int launch_branch(const BranchArgs& a, int Tn, hipStream_t st) {
+  const int V = a.H % 4 == 0 ? 4 : 1;
+  const int nvec = a.H / V;
+  int threads = 64;
+  while (threads < 512 && threads * 2 < nvec) threads *= 2;
+  const int per = (nvec + threads - 1) / threads;
+#define BN_L(VV, NVV) hipLaunchKernelGGL((branch_norm_kernel<T, KIND, VV, NVV>), dim3(Tn), dim3(threads), 0, st, a)
+  if (V == 4) {
+    if (per <= 2) BN_L(4, 2);
+    else if (per <= 4) BN_L(4, 4);
+    else if (per <= 8) BN_L(4, 8);
+    else return -2;
+  } else {
+    if (per <= 8) BN_L(1, 8);
+    else if (per <= 32) BN_L(1, 32);
+    else return -2;
+  }
+#undef BN_L
+  return 0;
+}
+
+}  // namespace rt
+
+extern "C" int rt_branch_norm(int f32, int kind, float* x, const void* y, long y_stride, int nsplit,
+                              const void* w_branch, const void* w_next, void* h, const void* table, const long* ids,
+                              int vocab, const float* pair_w, const int* pair_pos, int K, int T, int H, float eps,
+                              hipStream_t stream) {
+  if (T <= 0) return 0;
+  rt::BranchArgs a{x, y, y_stride, nsplit, w_branch, w_next, h, table, ids, vocab, pair_w, pair_pos, K, H, eps};
+  int rc = -1;
+#define BK(KIND) rc = f32 ? rt::launch_branch<float, rt::KIND>(a, T, stream) : rt::launch_branch<rt::bf16_t, rt::KIND>(a, T, stream)
+  switch (kind) {
+    case rt::Y_NONE: BK(Y_NONE); break;
+    case rt::Y_ACT: BK(Y_ACT); break;
+    case rt::Y_SLABS: BK(Y_SLABS); break;
+    case rt::Y_PAIRS: BK(Y_PAIRS); break;
+    case rt::Y_PAIRS_F32: BK(Y_PAIRS_F32); break;
+  }
+#undef BK
+  if (rc) return rc;
+  RT_LAUNCH_CHECK();
+  return 0;
+}

@@ -1,7 +1,8 @@
 """Command line: ``python -m rag_tl_domainllm_optimizer_amd <command> [--config f.yaml] [--preset p]
 [--section.key=value ...]``.
 
-Commands: index | rag | sft | ppo | eval | pipeline | serve | bench | launch.
+Commands: index | rag | sft | ppo | eval | pipeline | serve | trace | bench | launch. ``trace --model DIR --dtype bfloat16 --out
+DIR --max-tokens N`` replays token ids from standard input (serve.trace).
 Multi-GPU: ``python -m rag_tl_domainllm_optimizer_amd launch --nproc 8 ppo ...`` starts one process
 per GPU through torch.distributed.run (RCCL over xGMI) as a child process.
 """
@@ -401,6 +402,17 @@ def cmd_serve(cfg, args):
     serve(cfg, host=args.host, port=args.port)
 
 
+def cmd_trace(argv):
+    from .serve.trace import run
+
+    ap = argparse.ArgumentParser(prog="trace")
+    ap.add_argument("--model", required=True, help="folder with config.json and model.safetensors")
+    ap.add_argument("--dtype", default="bfloat16", choices=["bfloat16", "float32"])
+    ap.add_argument("--out", required=True, help="folder of the <step>.f32 files")
+    ap.add_argument("--max-tokens", type=int, required=True, help="tokens of all live requests together")
+    return run(ap.parse_args(argv))
+
+
 def cmd_bench(cfg, args, rest):
     root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
     r = subprocess.run([sys.executable, os.path.join(root, "bench.py"), *rest])
@@ -422,8 +434,10 @@ def cmd_launch(args, rest):
 
 def main(argv: Optional[List[str]] = None):
     argv = list(sys.argv[1:] if argv is None else argv)
+    if argv and argv[0] == "trace":
+        return cmd_trace(argv[1:])
     ap = argparse.ArgumentParser(prog="rag_tl_domainllm_optimizer_amd")
-    ap.add_argument("command", choices=["index", "rag", "sft", "ppo", "eval", "pipeline", "serve", "bench", "launch"])
+    ap.add_argument("command", choices=["index", "rag", "sft", "ppo", "eval", "pipeline", "serve", "trace", "bench", "launch"])
     ap.add_argument("--config", default=None)
     ap.add_argument("--preset", default=None, choices=sorted(C.PRESETS))
     ap.add_argument("--query", action="append")
@@ -448,4 +462,4 @@ def main(argv: Optional[List[str]] = None):
 
 
 if __name__ == "__main__":
-    main()
+    sys.exit(main() if sys.argv[1:2] == ["trace"] else (main(), 0)[1])

@@ -1,4 +1,4 @@
-"""Model zoo: Llama-2 / Mistral / OPT decoders, BERT / MPNet sentence encoders, LoRA, value head."""
+"""Model zoo: Llama-2 / Mistral / OPT decoders, layered decoders (Vezatar), BERT / MPNet sentence encoders, LoRA, value head."""
 from __future__ import annotations
 
 import os
@@ -8,9 +8,17 @@ import torch
 from .config import PRESETS, ModelConfig, resolve_preset  # noqa: F401
 from .decoder import CausalLM, fast_random_init_, pack_enabled, packed_index  # noqa: F401
 from .encoder import SentenceEncoder  # noqa: F401
+from .layered import LayeredLM  # noqa: F401
 from .lora import LoraConfig, attach_lora, load_adapter, merge_lora, save_adapter  # noqa: F401
 from .value_head import ValueHead  # noqa: F401
 from . import io  # noqa: F401
+
+
+def model_class(cfg: ModelConfig):
+    """The module class of a configuration."""
+    if cfg.is_layered:
+        return LayeredLM
+    return CausalLM if cfg.is_decoder else SentenceEncoder
 
 
 def build_model(name_or_path: str, device="cpu", dtype=None, seed: int = 0, fast_init: bool = False):
@@ -22,7 +30,7 @@ def build_model(name_or_path: str, device="cpu", dtype=None, seed: int = 0, fast
     cfg = resolve_preset(name_or_path)
     if cfg is None:
         raise ValueError(f"unknown model {name_or_path!r}: not a local HF dir and not a preset ({sorted(PRESETS)})")
-    cls = CausalLM if cfg.is_decoder else SentenceEncoder
+    cls = model_class(cfg)
     if fast_init:
         m = cls(cfg, device=device, dtype=dtype, init=False)
         fast_random_init_(m, seed, cfg.initializer_range)

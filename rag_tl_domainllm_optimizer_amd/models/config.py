@@ -11,12 +11,114 @@ from __future__ import annotations
 import dataclasses
 import json
 from dataclasses import dataclass, field
-from typing import Optional
+from typing import List, Optional
+
+
+# ---- layered decoders: every layer lists its own mixer and feed-forward ----
+@dataclass
+class YarnSpec:
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass
+class RotarySpec:
+    base: float
+    dims: int
+    scaling: Optional[YarnSpec] = None
+
+
+@dataclass
+class LatentAttentionSpec:
+    """Mixer ``latent_attention``: keys and values of all heads from one cached latent per token."""
+    heads: int
+    dim: int                            # unrotated query / key width per head
+    rot_dim: int                        # rotated query / key width (the key part is shared by the heads)
+    vdim: int
+    kv_rank: int
+    scale: float
+    rot: RotarySpec
+    kv_from: Optional[int] = None       # read this layer's cache instead of an own one
+
+
+@dataclass
+class FeedForwardSpec:
+    """``dense``: gated unit clamped at ``limit``; ``moe``: ``top`` of ``experts`` (+ a gated shared expert)."""
+    kind: str
+    ff: int
+    limit: float = 0.0
+    experts: int = 0
+    top: int = 0
+    shared_ff: int = 0
+
+
+@dataclass
+class LayerSpec:
+    mixer: LatentAttentionSpec
+    mlp: Optional[FeedForwardSpec] = None
+
+
+def layer_spec(d: dict) -> LayerSpec:
+    """One entry of a layered config's ``layers`` list."""
+    if d["type"] != "latent_attention":
+        raise ValueError(f"unknown mixer {d['type']!r}")
+    m, r = d["mixer"], d["mixer"]["rot"]
+    sc = r.get("scaling")
+    rot = RotarySpec(float(r["base"]), int(r["dims"]),
+                     YarnSpec(*(float(sc[k]) for k in ("factor", "original", "fast", "slow"))) if sc else None)
+    mixer = LatentAttentionSpec(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], float(m["scale"]), rot,
+                                m.get("kv_from"))
+    ml = d.get("mlp")
+    if ml is None:
+        return LayerSpec(mixer)
+    if ml["kind"] == "dense":
+        return LayerSpec(mixer, FeedForwardSpec("dense", ml["ff"], limit=float(ml["limit"])))
+    if ml["kind"] != "moe":
+        raise ValueError(f"unknown feed-forward {ml['kind']!r}")
+    shared = ml.get("shared")
+    return LayerSpec(mixer, FeedForwardSpec("moe", ml["expert"]["ff"], experts=ml["router"]["experts"],
+                                            top=ml["router"]["top"], shared_ff=shared["ff"] if shared else 0))
+
+
+def layer_spec_dict(s: LayerSpec) -> dict:
+    """Inverse of :func:`layer_spec`."""
+    m = s.mixer
+    rot = {"base": m.rot.base, "dims": m.rot.dims}
+    if m.rot.scaling is not None:
+        rot["scaling"] = dataclasses.asdict(m.rot.scaling)
+    mixer = {"heads": m.heads, "dim": m.dim, "rot_dim": m.rot_dim, "vdim": m.vdim, "kv_rank": m.kv_rank,
+             "scale": m.scale, "rot": rot}
+    if m.kv_from is not None:
+        mixer["kv_from"] = m.kv_from
+    ml = None
+    if s.mlp is not None and s.mlp.kind == "dense":
+        ml = {"kind": "dense", "ff": s.mlp.ff, "limit": s.mlp.limit}
+    elif s.mlp is not None:
+        ml = {"kind": "moe", "expert": {"ff": s.mlp.ff}, "router": {"experts": s.mlp.experts, "top": s.mlp.top}}
+        if s.mlp.shared_ff:
+            ml["shared"] = {"ff": s.mlp.shared_ff}
+    return {"type": "latent_attention", "mixer": mixer, "mlp": ml}
+
+
+def _check_layers(layers: List[LayerSpec]):
+    for i, s in enumerate(layers):
+        m = s.mixer
+        if m.rot_dim % 2 or m.rot.dims % 2 or m.rot.dims > m.rot_dim:
+            raise ValueError(f"layer {i}: rotation of {m.rot.dims} of {m.rot_dim} dimensions")
+        if m.kv_from is not None:
+            src = layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+            if src is None or src.kv_from is not None or (src.kv_rank, src.rot_dim, src.rot) != (m.kv_rank, m.rot_dim, m.rot):
+                raise ValueError(f"layer {i}: kv_from {m.kv_from} must be an earlier layer with its own latent of "
+                                 "equal rank and rotation")
+        if s.mlp is not None and s.mlp.kind == "moe" and not 1 <= s.mlp.top <= s.mlp.experts:
+            raise ValueError(f"layer {i}: top {s.mlp.top} of {s.mlp.experts} experts")
 
 
 @dataclass
 class ModelConfig:
-    arch: str = "llama"                 # llama | mistral | opt | bert | mpnet
+    arch: str = "llama"                 # llama | mistral | opt | bert | mpnet | vezatar
     vocab_size: int = 32000
     hidden_size: int = 4096
     num_layers: int = 32
@@ -43,10 +145,16 @@ class ModelConfig:
     # misc
     name: str = "custom"
     initializer_range: float = 0.02
+    # layered decoders (arch "vezatar"): one spec per layer; the per-layer sizes above do not apply
+    layers: Optional[List[LayerSpec]] = None
+
+    @property
+    def is_layered(self) -> bool:
+        return self.layers is not None
 
     @property
     def is_decoder(self) -> bool:
-        return self.arch in ("llama", "mistral", "opt")
+        return self.is_layered or self.arch in ("llama", "mistral", "opt")
 
     @property
     def qkv_dim(self) -> int:
@@ -58,10 +166,30 @@ class ModelConfig:
     @classmethod
     def from_dict(cls, d):
         names = {f.name for f in dataclasses.fields(cls)}
-        return cls(**{k: v for k, v in d.items() if k in names})
+        cfg = cls(**{k: v for k, v in d.items() if k in names})
+        if cfg.layers is not None and isinstance(cfg.layers[0], dict):
+            def mixer(m):
+                r = m["rot"]
+                sc = YarnSpec(**r["scaling"]) if r["scaling"] else None
+                return LatentAttentionSpec(**{**m, "rot": RotarySpec(r["base"], r["dims"], sc)})
+            cfg.layers = [LayerSpec(mixer(x["mixer"]), FeedForwardSpec(**x["mlp"]) if x["mlp"] else None)
+                          for x in cfg.layers]
+        return cfg
 
     def num_params(self) -> int:
         H, F, V, L = self.hidden_size, self.intermediate_size, self.vocab_size, self.num_layers
+        if self.is_layered:
+            n = 2 * V * H + H
+            for s in self.layers:
+                m, f = s.mixer, s.mlp
+                n += 2 * H + m.heads * ((m.dim + m.rot_dim) * H + (m.dim + m.vdim) * m.kv_rank + 2 * m.vdim * H + 1)
+                if m.kv_from is None:
+                    n += (m.kv_rank + m.rot_dim) * H + m.kv_rank
+                if f is not None:
+                    n += 2 * H + 3 * H * f.ff * max(f.experts, 1) + 3 * H * f.shared_ff
+                    if f.kind == "moe":
+                        n += f.experts * (H + 1) + (H if f.shared_ff else 0)
+            return n
         attn = H * self.qkv_dim + self.num_heads * self.head_dim * H
         if self.arch in ("llama", "mistral"):
             mlp = 3 * H * F
@@ -72,7 +200,34 @@ class ModelConfig:
         return L * (attn + mlp) + V * H
 
 
+def layered_config(arch: str, vocab_size: int, hidden_size: int, layers: List[LayerSpec], norm_eps: float,
+                   name: str = "custom", **kw) -> ModelConfig:
+    """ModelConfig of a layered decoder. Its files name no special tokens: generation stops at the ids the
+    caller gives (the tokenizer's)."""
+    _check_layers(layers)
+    m = layers[0].mixer
+    kw = {"bos_token_id": -1, "eos_token_id": -1, "pad_token_id": 0, **kw}
+    return ModelConfig(arch=arch, vocab_size=vocab_size, hidden_size=hidden_size, num_layers=len(layers),
+                       num_heads=m.heads, num_kv_heads=1, head_dim=m.kv_rank + m.rot_dim, intermediate_size=0,
+                       max_position=1 << 20, norm_eps=norm_eps, rope_theta=m.rot.base, name=name, layers=layers, **kw)
+
+
+def _vezatar_preset(name, vocab, width, n, heads, dim, rot, vdim, rank, ff, moe, shared_ff, factor=4.0):
+    """Layers in pairs: own latent + dense feed-forward, shared latent + experts (``moe`` = (experts, top, ff))."""
+    layers = []
+    for i in range(n):
+        r = RotarySpec(10000.0, rot, YarnSpec(factor, 4096.0, 32.0, 1.0))
+        m = LatentAttentionSpec(heads, dim, rot, vdim, rank, (dim + rot) ** -0.5, r, i - 1 if i % 2 else None)
+        f = FeedForwardSpec("moe", moe[2], experts=moe[0], top=moe[1], shared_ff=shared_ff) if i % 2 and moe else \
+            FeedForwardSpec("dense", ff, limit=7.0)
+        layers.append(LayerSpec(m, f))
+    return layered_config("vezatar", vocab, width, layers, 1e-6, name, bos_token_id=1, eos_token_id=2)
+
+
 PRESETS = {
+    # a real model's layer sizes (Mistral-7B's width and head count; 64 experts, 8 used) and a test size
+    "vezatar-7b": _vezatar_preset("vezatar-7b", 32000, 4096, 32, 32, 128, 64, 128, 512, 14336, (64, 8, 1408), 2816),
+    "tiny-vezatar": _vezatar_preset("tiny-vezatar", 512, 192, 4, 6, 32, 16, 48, 64, 256, (10, 3, 64), 128),
     "mistral-7b": ModelConfig(arch="mistral", vocab_size=32000, hidden_size=4096, num_layers=32, num_heads=32,
                               num_kv_heads=8, head_dim=128, intermediate_size=14336, max_position=32768,
                               norm_eps=1e-5, rope_theta=10000.0, sliding_window=4096, name="mistral-7b"),
@@ -144,7 +299,13 @@ def resolve_preset(name: str) -> Optional[ModelConfig]:
 
 
 def config_from_hf(d: dict) -> ModelConfig:
-    """Build a ModelConfig from an HF config.json dict (llama / mistral / opt / bert / mpnet)."""
+    """Build a ModelConfig from a config.json dict: HF model types (llama / mistral / opt / bert / mpnet) or
+    a layered architecture (``"architecture": "Vezatar"``)."""
+    if "architecture" in d:
+        if d["architecture"] != "Vezatar":
+            raise ValueError(f"unsupported architecture {d['architecture']!r}")
+        return layered_config("vezatar", d["vocab"], d["width"], [layer_spec(x) for x in d["layers"]],
+                              float(d["norm"]["eps"]), d.get("_ragtl_preset", "vezatar"))
     mt = d.get("model_type", "llama")
     if mt in ("llama", "mistral"):
         H = d["hidden_size"]
@@ -182,7 +343,10 @@ def config_from_hf(d: dict) -> ModelConfig:
 
 
 def config_to_hf(cfg: ModelConfig) -> dict:
-    """HF config.json dict for save_pretrained-compatible checkpoints."""
+    """config.json dict of the checkpoints ``save_pretrained`` writes."""
+    if cfg.is_layered:
+        return {"architecture": "Vezatar", "vocab": cfg.vocab_size, "width": cfg.hidden_size,
+                "norm": {"eps": cfg.norm_eps}, "layers": [layer_spec_dict(s) for s in cfg.layers]}
     if cfg.arch in ("llama", "mistral"):
         d = {
             "architectures": ["MistralForCausalLM" if cfg.arch == "mistral" else "LlamaForCausalLM"],

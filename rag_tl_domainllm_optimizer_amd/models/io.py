@@ -87,11 +87,105 @@ def encoder_mapping(cfg: ModelConfig) -> Mapping:
     return m
 
 
+class Part:
+    """A piece of a checkpoint tensor that a native parameter holds: rows [row0, row0 + rows) of the (2-D
+    or 1-D) parameter, ``dim`` / ``start`` / the parameter side's size selecting the tensor's slice."""
+
+    __slots__ = ("name", "param", "row0", "rows", "dim", "start", "size")
+
+    def __init__(self, name, param, row0=0, rows=None, dim=None, start=0, size=None):
+        self.name, self.param, self.row0, self.rows = name, param, row0, rows
+        self.dim, self.start, self.size = dim, start, size
+
+
+def layered_mapping(cfg: ModelConfig) -> List[Part]:
+    """Tensor names of a layered decoder -> its fused parameters: [q | dkv | g] and [uk; uv] as one
+    projection each, experts stacked, the shared expert cut into parts of an expert's width behind them."""
+    m = [Part("embed", "embed"), Part("head", "lm_head"), Part("final.norm", "norm_w")]
+    for i, s in enumerate(cfg.layers):
+        L, n, x = f"l{i}", f"layers.{i}", s.mixer
+        nq, nk, ng = x.heads * (x.dim + x.rot_dim), x.kv_rank + x.rot_dim, x.heads * x.vdim
+        own = x.kv_from is None
+        m += [Part(f"{L}.norm1", f"{n}.norm1_w"), Part(f"{L}.norm1b", f"{n}.norm1b_w"),
+              Part(f"{L}.mix.q", f"{n}.mix.in_w", 0, nq), Part(f"{L}.mix.g", f"{n}.mix.in_w", nq + (nk if own else 0), ng),
+              Part(f"{L}.mix.uk", f"{n}.mix.kv_up_w", 0, x.heads * x.dim),
+              Part(f"{L}.mix.uv", f"{n}.mix.kv_up_w", x.heads * x.dim, ng),
+              Part(f"{L}.mix.sink", f"{n}.mix.sink"), Part(f"{L}.mix.o", f"{n}.mix.o_w")]
+        if own:
+            m += [Part(f"{L}.mix.dkv", f"{n}.mix.in_w", nq, nk), Part(f"{L}.mix.dkv.norm", f"{n}.mix.latent_norm_w")]
+        f = s.mlp
+        if f is None:
+            continue
+        m += [Part(f"{L}.norm2", f"{n}.norm2_w"), Part(f"{L}.norm2b", f"{n}.norm2b_w")]
+        p = f"{L}.mlp"
+        W = cfg.hidden_size
+        if f.kind == "dense":
+            m += [Part(f"{p}.gate", f"{n}.mlp.gate_up_w", 0, f.ff), Part(f"{p}.up", f"{n}.mlp.gate_up_w", f.ff, f.ff),
+                  Part(f"{p}.down", f"{n}.mlp.down_w")]
+            continue
+        m += [Part(f"{p}.router", f"{n}.mlp.router_w", 0, f.experts), Part(f"{p}.correction", f"{n}.mlp.correction")]
+        for e in range(f.experts):
+            m += [Part(f"{p}.e{e}.gate", f"{n}.mlp.gate_up_w", 2 * e * f.ff, f.ff),
+                  Part(f"{p}.e{e}.up", f"{n}.mlp.gate_up_w", (2 * e + 1) * f.ff, f.ff),
+                  Part(f"{p}.e{e}.down", f"{n}.mlp.down_w", e * W, W)]
+        if f.shared_ff:
+            m.append(Part(f"{p}.shared.sg", f"{n}.mlp.router_w", f.experts, 1))
+            for j, c0 in enumerate(range(0, f.shared_ff, f.ff)):
+                e, c = f.experts + j, min(f.ff, f.shared_ff - c0)
+                m += [Part(f"{p}.shared.gate", f"{n}.mlp.gate_up_w", 2 * e * f.ff, c, 0, c0, c),
+                      Part(f"{p}.shared.up", f"{n}.mlp.gate_up_w", (2 * e + 1) * f.ff, c, 0, c0, c),
+                      Part(f"{p}.shared.down", f"{n}.mlp.down_w", e * W, W, 1, c0, c)]
+    return m
+
+
+@torch.no_grad()
+def load_layered_state_dict(model, sd: Dict[str, torch.Tensor]):
+    """Strict load: every expected tensor present with the shape the config gives, and no other."""
+    params = dict(model.named_parameters())
+    parts = layered_mapping(model.cfg)
+    missing = sorted({p.name for p in parts} - set(sd))
+    extra = sorted(set(sd) - {p.name for p in parts})
+    if missing or extra:
+        raise KeyError(f"checkpoint tensors do not fit the config: missing {missing[:6]}, unexpected {extra[:6]}")
+    left = {}
+    for p in parts:
+        src, dst = sd[p.name], params[p.param]
+        if p.rows is not None:
+            dst = dst[p.row0:p.row0 + p.rows]
+        left[p.name] = left.get(p.name, src.numel())
+        if p.dim is not None:
+            src = src.narrow(p.dim, p.start, p.size)
+            if p.dim == 1:
+                dst = dst[:, :p.size]
+        if tuple(src.shape) != tuple(dst.shape):
+            raise ValueError(f"{p.name}: shape {tuple(sd[p.name].shape)} does not fit the config")
+        left[p.name] -= src.numel()
+        dst.copy_(src.to(dst.device, dst.dtype))
+    if any(left.values()):
+        raise ValueError(f"checkpoint tensors larger than the config: {[k for k, v in left.items() if v][:6]}")
+
+
+def layered_state_dict(model, dtype=None) -> Dict[str, torch.Tensor]:
+    params = dict(model.named_parameters())
+    pieces: Dict[str, list] = {}
+    for p in layered_mapping(model.cfg):
+        t = params[p.param].detach()
+        if p.rows is not None:
+            t = t[p.row0:p.row0 + p.rows]
+        if p.dim == 1:
+            t = t[:, :p.size]
+        pieces.setdefault(p.name, []).append((p.dim or 0, t.to("cpu")))
+    out = {k: (torch.cat([t for _, t in v], v[0][0]) if len(v) > 1 else v[0][1]) for k, v in pieces.items()}
+    return {k: (t.to(dtype) if dtype is not None else t).contiguous() for k, t in out.items()}
+
+
 def mapping_for(model) -> Mapping:
     return decoder_mapping(model.cfg) if model.cfg.is_decoder else encoder_mapping(model.cfg)
 
 
 def to_hf_state_dict(model, dtype=None) -> Dict[str, torch.Tensor]:
+    if model.cfg.is_layered:
+        return layered_state_dict(model, dtype)
     params = dict(model.named_parameters())
     out = {}
     for hf, nat, r0, rn in mapping_for(model):
@@ -105,6 +199,9 @@ def to_hf_state_dict(model, dtype=None) -> Dict[str, torch.Tensor]:
 
 @torch.no_grad()
 def load_hf_state_dict(model, sd: Dict[str, torch.Tensor], strict: bool = True, prefix_strip: str = ""):
+    if model.cfg.is_layered:
+        load_layered_state_dict(model, sd)
+        return []
     params = dict(model.named_parameters())
     missing = []
     for hf, nat, r0, rn in mapping_for(model):
@@ -193,11 +290,9 @@ def load_config(path: str) -> ModelConfig:
 
 
 def from_pretrained(path: str, device="cpu", dtype=torch.bfloat16):
-    from .decoder import CausalLM
-    from .encoder import SentenceEncoder
+    from . import model_class
 
     cfg = load_config(path)
-    cls = CausalLM if cfg.is_decoder else SentenceEncoder
-    model = cls(cfg, device=device, dtype=dtype, init=False)
+    model = model_class(cfg)(cfg, device=device, dtype=dtype, init=False)
     load_hf_state_dict(model, read_state_dict(path))
     return model

@@ -114,6 +114,86 @@ def gemm(x: torch.Tensor, w: torch.Tensor, u=None, ub=None, bias=None, act=0, ou
     return y
 
 
+@dataclass(frozen=True)
+class Glu:
+    """Gated linear unit ``g' * sigmoid(alpha g') * (u' + offset)`` with ``g' = min(g, limit)`` and
+    ``u' = clamp(u, -limit, limit)``; the default is SwiGLU, ``silu(g) * u`` without a clamp."""
+
+    limit: float = float("inf")
+    alpha: float = 1.0
+    offset: float = 0.0
+
+    def args(self) -> List[float]:
+        return [self.limit, self.alpha, self.offset]
+
+
+def project(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False, shuf=None) -> torch.Tensor:
+    """x w^T without grad, any shape and dtype: the MFMA kernels where their shape rules hold (bf16;
+    ``shuf``: tile-ordered image at M <= 16), ``gemm_any`` otherwise — also for fp32 operands, which
+    stay fp32 throughout."""
+    if not on_gpu(x):
+        return ref.gemm(x, w, out_f32=out_f32)
+    M, K = x.shape
+    N = w.shape[0]
+    if x.dtype != torch.bfloat16 or K % 8 or N % 8 or x.stride(0) % 8 or x.data_ptr() % 16 or M == 0:
+        return native().gemm_any(x, w, out_f32)
+    if M <= 64 and K % 64 == 0:
+        if shuf is not None and shuffle_decode(M) and N % 16 == 0:
+            return native().gemm(x, shuf.get(w), None, None, None, 0, out_f32, None, None, 0.0, True)
+        return gemm(x, w, out_f32=out_f32)
+    if M <= 64:
+        return native().gemm_big(x, w, ROW, ROW, None, None, None, 0, 1 if out_f32 else 0)
+    if out_f32 and N <= 512:  # narrow fp32 products (router logits): 64x64 tiles fill the chip
+        return native().gemm_small(x, w, ROW, ROW, 1, 1, None, 64)
+    return gemm(x, w, out_f32=out_f32)
+
+
+def shuffle_decode(m: int) -> bool:
+    """Decode products at ``m`` <= 16 rows stream tile-ordered weight images (RAGTL_DECODE_SHUF=0: off)."""
+    import os
+
+    return m <= 16 and os.environ.get("RAGTL_DECODE_SHUF", "1") != "0"
+
+
+def glu_project(x: torch.Tensor, w: torch.Tensor, glu: Glu, shuf=None) -> torch.Tensor:
+    """Gated linear unit of x w^T, w = [gate; up] (2F rows), without grad: in the GEMM epilogue where
+    the MFMA kernels take the shape, else a product and an elementwise pass."""
+    if not on_gpu(x):
+        return ref.glu(ref.gemm(x, w), glu.limit, glu.alpha, glu.offset)
+    M, K = x.shape
+    N = w.shape[0]
+    if x.dtype == torch.bfloat16 and x.is_contiguous() and M > 0:
+        if M <= 64 and K % 64 == 0 and N % 64 == 0:
+            sh = shuf is not None and shuffle_decode(M)
+            return native().gemm(x, shuf.get(w) if sh else w, None, None, None, ACT_SWIGLU, False, None, None, 0.0, sh,
+                                 glu.args())
+        if M > 64 and N % 256 == 0 and K % 8 == 0:
+            s, bn = splitk_plan(M, N, K, ACT_SWIGLU)
+            if s > 1:
+                slabs = torch.empty(s * M * N, dtype=torch.float32, device=x.device)
+                return native().gemm_splitk(x, w, s, slabs, None, ACT_SWIGLU, None, None, bn or 256, glu.args())
+            return native().gemm_big(x, w, ROW, ROW, None, None, None, ACT_SWIGLU, 0, 1, None, None, None, bn,
+                                     glu.args())
+    return native().glu_any(project(x, w), glu.args())
+
+
+def branch_project(x: torch.Tensor, w: torch.Tensor, shuf=None):
+    """x w^T for ``ops.branch_norm``, without grad: fp32 up to 64 rows, unreduced split-K slabs
+    (:class:`SplitK`) where the plan splits, else the activation type."""
+    if on_gpu(x) and x.dtype == torch.bfloat16:
+        M, K = x.shape
+        N = w.shape[0]
+        if M <= 64:
+            return project(x, w, True, shuf)
+        if K % 8 == 0 and N % 16 == 0:
+            s, bn = splitk_plan(M, N, K, 0)
+            if s > 1:
+                slabs = torch.empty(s * M * N, dtype=torch.float32, device=x.device)
+                native().gemm_splitk_raw(x.contiguous(), w, s, slabs, bn or 256)
+                return SplitK(slabs, s, M, N, x.dtype)
+    return project(x, w)
+
+
 ROW, KMAJ = 0, 1  # operand layouts of the token-parallel GEMM family (csrc/kernels/gemm_big.hip)
 
 
@@ -918,5 +998,22 @@ class FoldCache(dict):
                 buf = torch.empty_like(w)
                 self["w"] = buf
             torch.mul(w, norm_w.to(w.dtype)[None, :], out=buf)
+            self["key"] = key
+        return self["w"]
+
+
+class TransposeCache(dict):
+    """Per-head transpose of a weight ``w`` [H, a, b] -> [H, b, a], rebuilt in place when the source
+    changes (graph-safe address)."""
+
+    @torch.no_grad()
+    def get(self, w: torch.Tensor) -> torch.Tensor:
+        key = (w.data_ptr(), w._version)
+        if dict.get(self, "key") != key:
+            buf = dict.get(self, "w")
+            if buf is None or buf.shape != (w.shape[0], w.shape[2], w.shape[1]) or buf.device != w.device:
+                buf = torch.empty(w.shape[0], w.shape[2], w.shape[1], dtype=w.dtype, device=w.device)
+                self["w"] = buf
+            buf.copy_(w.transpose(1, 2))
             self["key"] = key
         return self["w"]

@@ -1,0 +1,60 @@
+"""Mixture-of-experts feed-forward (no grad): router, pair sort and grouped expert products.
+
+The row counts per expert stay on the device (fixed launch grids), so a decode step with experts can be
+captured in a graph. Few rows per expert stream each expert's weights once (``moe_rows``); many rows
+run the grouped form of the token-parallel MFMA GEMM; fp32 and odd sizes run ``gemm_any``."""
+from __future__ import annotations
+
+import torch
+
+from . import reference as ref
+from ._ext import native, on_gpu
+from .linear import Glu, project
+from .norm import MoePairs
+
+ROWS_PER_GROUP = 48  # expected rows per expert up to which the weight-streaming kernel is used
+
+
+def moe_route(logits: torch.Tensor, correction: torch.Tensor, top: int, nshared: int = 0, gate_col: int = -1):
+    """fp32 router logits [T, >= E] -> (groups [T, top + nshared] int32, weights fp32): the ``top`` experts of
+    the largest ``softmax + correction`` with their softmax values, then groups E .. E + nshared - 1 (the
+    shared expert's parts) with weight sigmoid(logits[:, gate_col]) (1 without a gate column)."""
+    if on_gpu(logits):
+        return native().moe_route(logits, correction, top, nshared, gate_col)
+    return ref.moe_route(logits, correction, top, nshared, gate_col)
+
+
+def moe_ff(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor, w_gu: torch.Tensor, w_down: torch.Tensor,
+           top: int, nshared: int = 0, gate_col: int = -1, glu: Glu = Glu()) -> MoePairs:
+    """Experts w_gu [G, 2F, W] / w_down [G, W, F] (G = E + nshared) applied to h [T, W]."""
+    T = h.shape[0]
+    G, F2, W = w_gu.shape
+    F = F2 // 2
+    idx, wt = moe_route(project(h, router_w, out_f32=True), correction, top, nshared, gate_col)
+    if not on_gpu(h):
+        order = torch.argsort(idx.reshape(-1), stable=True)
+        pos = torch.empty_like(order)
+        pos[order] = torch.arange(order.numel())
+        tok, grp = order // idx.shape[1], idx.reshape(-1)[order]
+        y = torch.empty(order.numel(), W, dtype=h.dtype)
+        for g in torch.unique(grp).tolist():
+            r = torch.nonzero(grp == g).flatten()
+            f = ref.glu(ref.gemm(h[tok[r]], w_gu[g]), glu.limit, glu.alpha, glu.offset)
+            y[r] = ref.gemm(f, w_down[g])
+        return MoePairs(y, wt, pos.int().view_as(idx))
+    P = idx.numel()
+    mean = (P + G - 1) // G
+    bf16 = h.dtype == torch.bfloat16 and W % 8 == 0 and F % 8 == 0
+    big = bf16 and mean > ROWS_PER_GROUP and F % 128 == 0
+    srt = native().moe_sort(idx, G, 256 if big else 0)
+    offs, tok, pos = srt[:3]
+    if big:
+        f = native().gemm_grouped(h, tok, w_gu, srt[3], srt[4], P, glu.args(), 256)
+        y = native().gemm_grouped(f, None, w_down, srt[3], srt[4], P, [], 256)
+    elif bf16:
+        f = native().moe_rows(h, tok, w_gu, offs, P, False, mean, glu.args())
+        y = native().moe_rows(f, None, w_down, offs, P, T <= 64, mean, [])
+    else:
+        f = native().glu_any(native().gemm_any(h, w_gu, offs=offs, row_map=tok), glu.args())
+        y = native().gemm_any(f, w_down, offs=offs)
+    return MoePairs(y, wt, pos.view_as(idx))

@@ -96,3 +96,51 @@ def rms_norm(x, w, eps=1e-6, residual=None):
 def layer_norm(x, w, b=None, eps=1e-5, residual=None):
     """(y, h): h = x + residual (or x), y = LayerNorm(h) * w + b."""
     return _norm(x, w, b, eps, residual, True)
+
+
+class MoePairs:
+    """Expert outputs of a mixture, one row of ``y`` [T * slots, H] per (token, slot) pair in expert
+    order; ``w`` / ``pos`` [T, slots]: each pair's weight and its row of ``y``. The weighted sum is left to
+    the consumer (:func:`branch_norm`)."""
+
+    __slots__ = ("y", "w", "pos")
+
+    def __init__(self, y, w, pos):
+        self.y, self.w, self.pos = y, w, pos
+
+    def combine(self) -> torch.Tensor:
+        return (self.y.float()[self.pos.long().reshape(-1)].view(*self.w.shape, -1) * self.w[..., None]).sum(1)
+
+
+_Y_ACT, _Y_SLABS, _Y_PAIRS, _Y_PAIRS_F32 = 1, 2, 3, 4
+
+
+def embed_norm(table, ids, w_next, eps: float):
+    """First step of a pass with an fp32 residual stream: x = table[ids] (fp32 [T, H]) and
+    h = rms(x) * w_next in the table's dtype. Returns (x, h)."""
+    if on_gpu(ids):
+        x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=ids.device)
+        h = native().branch_norm(x, 0, w_next=w_next, table=table, ids=ids.contiguous(), eps=eps)
+        return x, h
+    x = table[ids].float()
+    return x, ref.rms(x, w_next, eps).to(table.dtype)
+
+
+def branch_norm(x, y, w_branch, w_next, eps: float):
+    """Between two sublayers with a norm before and after each, on the fp32 residual ``x`` (updated in
+    place): ``x += rms(y) * w_branch``; returns ``h = rms(x) * w_next`` in the weights' dtype. ``y``: a
+    tensor, unreduced split-K slabs (``SplitK``) or a mixture's expert outputs (:class:`MoePairs`)."""
+    from .linear import SplitK
+
+    if on_gpu(x):
+        kw = dict(w_branch=w_branch, w_next=w_next, eps=eps)
+        if isinstance(y, SplitK):
+            return native().branch_norm(x, _Y_SLABS, y=y.slabs, nsplit=y.nsplit, **kw)
+        if isinstance(y, MoePairs):
+            kind = _Y_PAIRS if y.y.dtype == w_branch.dtype else _Y_PAIRS_F32
+            return native().branch_norm(x, kind, y=y.y, pair_w=y.w, pair_pos=y.pos, **kw)
+        kind = _Y_ACT if y.dtype == w_branch.dtype else _Y_SLABS
+        return native().branch_norm(x, kind, y=y.contiguous(), **kw)
+    yf = y.combine() if isinstance(y, MoePairs) else y.float()
+    x.add_(ref.rms(yf, w_branch, eps))
+    return ref.rms(x, w_next, eps).to(w_branch.dtype)

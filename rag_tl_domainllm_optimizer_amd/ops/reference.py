@@ -318,3 +318,59 @@ def ppo_advantages(old_logp, ref_logp, values, scores, resp_len, kl_coef, gamma,
         var = (((adv - mean) ** 2) * m).sum() / n
         adv = (adv - mean) * torch.rsqrt(var + eps) * m
     return adv, ret, rewards, kl.sum(-1)
+
+
+# ------------------------------------------------------- layered decoders (latent attention, experts)
+def rms(x, w, eps):
+    """RMS norm in fp32 (no rounding of the result)"""
+    xf = x.float()
+    return xf / torch.sqrt(xf.pow(2).mean(-1, keepdim=True) + eps) * w.float()
+
+
+def glu(gu, limit=math.inf, alpha=1.0, offset=0.0):
+    g, u = gu.float().chunk(2, -1)
+    g = g.clamp(max=limit)
+    return (g * torch.sigmoid(alpha * g) * (u.clamp(-limit, limit) + offset)).to(gu.dtype)
+
+
+def rotate_pairs(x, cos, sin):
+    """x [T, ..., d] with the leading 2 * cos.shape[1] columns rotated as interleaved pairs"""
+    n = cos.shape[1]
+    shape = (x.shape[0],) + (1,) * (x.dim() - 2) + (n,)
+    c, s = cos.view(shape), sin.view(shape)
+    y = x.float().clone()
+    u, v = x[..., 0:2 * n:2].float(), x[..., 1:2 * n:2].float()
+    y[..., 0:2 * n:2] = u * c - v * s
+    y[..., 1:2 * n:2] = v * c + u * s
+    return y
+
+
+def latent_attend(q, pool, tab, row, pos, sink, rank, scale, page):
+    """Absorbed latent attention: q [T, H, KD] over the pool's rows 0..pos of each token's request ->
+    [T, H, rank] fp32 (softmax denominator with the sink)."""
+    out = torch.zeros(q.shape[0], q.shape[1], rank)
+    flat = pool.reshape(-1, pool.shape[-1])
+    for r in torch.unique(row).tolist():
+        t = torch.nonzero(row == r).flatten()
+        n = int(pos[t].max()) + 1
+        k = torch.arange(n)
+        kv = flat[tab[r].long()[k // page] * page + k % page].float()
+        s = (q[t].float().reshape(-1, q.shape[-1]) @ kv.t()).view(len(t), q.shape[1], n) * scale
+        s = s.masked_fill(k[None, None, :] > pos[t].long()[:, None, None], -math.inf)
+        s = torch.cat([s, sink.view(1, -1, 1).expand(len(t), -1, 1)], -1)
+        p = torch.softmax(s, -1)[..., :-1]
+        out[t] = (p.reshape(-1, n) @ kv[:, :rank]).view(len(t), q.shape[1], rank)
+    return out
+
+
+def moe_route(logits, correction, top, nshared, gate_col):
+    E = correction.numel()
+    s = torch.softmax(logits[:, :E].float(), -1)
+    idx = (s + correction).topk(top, -1).indices
+    w = s.gather(-1, idx)
+    if nshared:
+        T = logits.shape[0]
+        gate = torch.sigmoid(logits[:, gate_col:gate_col + 1].float()) if gate_col >= 0 else torch.ones(T, 1)
+        idx = torch.cat([idx, torch.arange(E, E + nshared).expand(T, -1)], -1)
+        w = torch.cat([w, gate.expand(T, nshared)], -1)
+    return idx.int(), w.contiguous()
