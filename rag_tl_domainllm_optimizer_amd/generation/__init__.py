@@ -7,6 +7,10 @@ projections, RoPE+append, split-K decode attention, SwiGLU), final norm, LM head
 sampler (which also emits the behaviour log-prob), value head, and the bookkeeping kernel — is one
 graph replay with zero host synchronisation. Finished rows are masked on device; the host polls
 completion only every ``sync_every`` steps.
+
+Layered models (``model.ragged``) are served by the same loops over a paged cache (``paged.PagedCache``):
+their prompts run as ragged batches (``ragged.RaggedBatch``), whole or — in ``ContinuousBatcher`` — in
+portions beside the decoding rows, and their decode step is captured like the others.
 """
 from __future__ import annotations
 
@@ -19,6 +23,8 @@ import torch
 from .. import ops
 from ..models.decoder import pack_enabled, packed_index
 from ..runtime import GraphRunner
+from .paged import PAGE, PagedCache  # noqa: F401
+from .ragged import RaggedBatch, StepEngine  # noqa: F401
 
 
 @dataclass
@@ -126,7 +132,9 @@ class Generator:
     """Owns the cache and captured graph for one (model, max_batch, max_seq) configuration."""
 
     def __init__(self, model, max_batch: int, max_seq: int, device=None, use_graph: bool = True,
-                 value_head=None, sync_every: int = 16, kv_fp8: Optional[bool] = None):
+                 value_head=None, sync_every: int = 16, kv_fp8: Optional[bool] = None,
+                 cache_tokens: Optional[int] = None):
+        """``cache_tokens`` (paged models): tokens the cache pool holds, default max_batch x max_seq."""
         self.model = model
         cfg = model.cfg
         self.cfg = cfg
@@ -143,11 +151,17 @@ class Generator:
         # fp8 K/V cache (config 5): the model's setting unless given; GPU MFMA decode kernels only
         # (head_dim 128), the CPU path runs the quantise / dequantise reference
         kv_fp8 = getattr(model, "kv_fp8", False) if kv_fp8 is None else kv_fp8
-        self.cache = KVCache(cfg.num_layers, max_batch, cfg.num_kv_heads, max_seq, cfg.head_dim, self.device,
-                             model.dtype, fp8=bool(kv_fp8))
+        self.ragged = getattr(model, "ragged", False)
+        if self.ragged:
+            if kv_fp8:
+                raise ValueError(f"{cfg.arch}: no fp8 K/V cache")
+            self.cache = model.make_cache(max_batch, max_seq, cache_tokens, self.device)
+        else:
+            self.cache = KVCache(cfg.num_layers, max_batch, cfg.num_kv_heads, max_seq, cfg.head_dim, self.device,
+                                 model.dtype, fp8=bool(kv_fp8))
         dev = self.device
         B = max_batch
-        self.workspace = ops.decode_workspace(B, cfg.num_heads, cfg.num_kv_heads, cfg.head_dim, max_seq, dev) \
+        self.workspace = None if self.ragged else ops.decode_workspace(B, cfg.num_heads, cfg.num_kv_heads, cfg.head_dim, max_seq, dev) \
             if dev.type == "cuda" else None
         # device-resident decode state (static addresses for graph replay)
         self.tok_in = torch.zeros(B, dtype=torch.long, device=dev)
@@ -179,7 +193,10 @@ class Generator:
         # attn_len = kv_len + 1 and pos = kv_len - kv_start were set by the previous bookkeeping
         # (decode_update on the GPU, _update_cpu on the CPU) — no elementwise launches here
         nb = self._nb
-        cache = self.cache if nb == self.max_batch else _SubCache(self.cache, nb)
+        if self.ragged:
+            cache = self.cache.rows_view(0, nb)
+        else:
+            cache = self.cache if nb == self.max_batch else _SubCache(self.cache, nb)
         h = self.model.decode(self.tok_in[:nb], self.pos[:nb], self.kv_len[:nb], self.attn_len[:nb],
                               self.kv_start[:nb], cache, self.workspace)
         self._emit(h, params, eos_ids, pad_id)
@@ -298,7 +315,14 @@ class Generator:
         eos_list = list(eos_ids) or [cfg.eos_token_id]
         eos = torch.tensor(eos_list, dtype=torch.long, device=dev)
         # prefill on the first B rows of the cache
-        sub = _SubCache(self.cache, B)
+        if self.ragged:
+            self.cache.release_all()
+            for b, p in enumerate(prompts):
+                self.cache.reserve(b, len(p) + T)
+            self.cache.sync()
+            sub = prompts
+        else:
+            sub = _SubCache(self.cache, B)
         # generation never differentiates: run adapters on merged weights (one weight stream per
         # projection; the merged images are refreshed in place after each adapter update)
         prev_merged = self.model.set_lora_merged(self.merge_lora) if hasattr(self.model, "set_lora_merged") else None
@@ -312,11 +336,14 @@ class Generator:
         cfg, dev, MB = self.cfg, self.device, self.max_batch
         packed = None
         n_real = B * S - int(start.sum())
-        if pack_enabled() and n_real < 0.97 * B * S:
+        if self.ragged:
+            h_last = self._ragged_prefill(sub)
+        elif pack_enabled() and n_real < 0.97 * B * S:
             # varlen prefill: the projection GEMMs run on the real prompt tokens only
             packed = packed_index(start.numpy(), np.full(B, S), S, dev)
-        h_last = self.model.prefill(ids, self.kv_start[:B], sub, packed=packed) if packed is not None else \
-            self.model.prefill(ids, self.kv_start[:B], sub)
+        if not self.ragged:
+            h_last = self.model.prefill(ids, self.kv_start[:B], sub, packed=packed) if packed is not None else \
+                self.model.prefill(ids, self.kv_start[:B], sub)
         if hasattr(self.model, "refresh_decode_weights"):
             self.model.refresh_decode_weights(self._bucket(B))  # folded / tile-ordered / fp8 images of graph replays
         self._nb = self._bucket(B)
@@ -338,6 +365,12 @@ class Generator:
             ev[2].record()
             pend._recorded = True
         return pend
+
+    def _ragged_prefill(self, prompts) -> torch.Tensor:
+        """Prompts of rows 0.. as one ragged step -> the hidden state of each one's last token."""
+        batch = RaggedBatch.build([(b, p, 0) for b, p in enumerate(prompts)], self.device)
+        last = torch.tensor([int(batch.offset[b]) + len(p) - 1 for b, p in enumerate(prompts)]).to(self.device)
+        return self.model.step(batch, self.cache, last)
 
     def _ensure_graph(self, params, eos, eos_list, pad_id, T):
         """The captured decode step for (sampling parameters, output width, row bucket)."""
@@ -540,9 +573,17 @@ class ContinuousBatcher:
     power-of-two bucket of rows that covers the active ones (inactive rows in it are masked).
 
     Usage: ``admit(prompt_ids, tag)`` while ``free_rows()``; ``step(n)``; ``collect()`` returns the
-    rows that finished (a host read of the per-row flags once per call)."""
+    rows that finished (a host read of the per-row flags once per call).
 
-    def __init__(self, gen: Generator, params: SamplingParams, pad_id: int = 0, eos_ids: Sequence[int] = ()):
+    Paged models: an admitted prompt waits (first come, first served) until the pool holds its prompt and
+    new tokens, then enters in portions: while prompts are pending, a step is one ragged batch of up to
+    ``prefill_tokens`` prompt tokens beside the decoding rows' single tokens; otherwise the captured
+    decode step. Pages go back when the row is collected."""
+
+    def __init__(self, gen: Generator, params: SamplingParams, pad_id: int = 0, eos_ids: Sequence[int] = (),
+                 prefill_tokens: int = 2048):
+        self.prefill_tokens = max(1, prefill_tokens)
+        self.pending = []  # paged models: [row, prompt, tokens already in the cache (None: no pages yet)]
         self.gen, self.params, self.pad_id = gen, params, pad_id
         g = gen
         dev, MB, T = g.device, g.max_batch, params.max_new_tokens
@@ -555,6 +596,9 @@ class ContinuousBatcher:
         g.kv_start.zero_()
         g.kv_len.zero_()
         g.tok_in.fill_(pad_id)
+        if g.ragged:
+            g.cache.release_all()
+            g.cache.sync()
         if g.out_tokens is None or g.out_tokens.shape[1] != T:
             g.out_tokens = torch.full((MB, T), pad_id, dtype=torch.long, device=dev)
             g.out_logp = torch.zeros(MB, T, dtype=torch.float32, device=dev)
@@ -596,8 +640,15 @@ class ContinuousBatcher:
         for p in prompts:
             if len(p) < 1 or len(p) + self.T > g.max_seq:
                 raise ValueError(f"prompt of {len(p)} tokens + {self.T} new exceeds the cache ({g.max_seq})")
+            if g.ragged and len(p) + self.T > (g.cache.n_pages - 1) * PAGE:
+                raise ValueError(f"prompt of {len(p)} tokens + {self.T} new exceeds the cache pool")
         self.free.sort()
         rows, self.free = self.free[:len(prompts)], self.free[len(prompts):]
+        if g.ragged:
+            for b, p, tag in zip(rows, prompts, tags):
+                self.rows[b] = (tag, len(p), self.steps)
+                self.pending.append([b, list(p), None])
+            return rows
         try:
             self._admit_runs(rows, prompts, tags)
         except BaseException:
@@ -646,8 +697,61 @@ class ContinuousBatcher:
             if self.T > 1:
                 g._ensure_graph(self.params, self.eos, self.eos_list, self.pad_id, self.T)
         for _ in range(n):
-            g._replay(self.params, self.eos, self.pad_id)
-        self.steps += n
+            if not (self.pending and self._mixed_step()):
+                g._replay(self.params, self.eos, self.pad_id)
+            self.steps += 1
+
+    @torch.no_grad()
+    def _mixed_step(self) -> bool:
+        """One ragged step: the next portions of pending prompts beside every decoding row's token. False when
+        no pending prompt can get its pages yet."""
+        g = self.gen
+        budget, take = self.prefill_tokens, []
+        for e in self.pending:
+            if budget <= 0:
+                break
+            b, prompt, done = e
+            if done is None:
+                if not g.cache.can_reserve(b, len(prompt) + self.T):
+                    break
+                g.cache.reserve(b, len(prompt) + self.T)
+                e[2] = done = 0
+            n = min(budget, len(prompt) - done)
+            take.append((e, n))
+            budget -= n
+        if not take:
+            return False
+        g.cache.sync()
+        waiting = {e[0] for e in self.pending}
+        dec = [b for b in self.rows if b not in waiting]
+        # the decoding rows' tokens and positions are device state: placeholders here, filled below
+        batch = RaggedBatch.build([(b, [0], 0) for b in dec] + [(e[0], e[1][e[2]:e[2] + n], e[2]) for e, n in take],
+                                  g.device)
+        nd = len(dec)
+        if nd:
+            idx = torch.tensor(dec).to(g.device)
+            batch.ids[:nd] = g.tok_in[idx]
+            batch.pos[:nd] = g.pos[idx]
+            bound = max(self.rows[b][1] + self.T for b in dec)
+            batch.max_len = max(batch.max_len, min(bound, g.cache.max_seq))
+        want, rows = list(range(nd)), list(dec)
+        for k, (e, n) in enumerate(take):
+            e[2] += n
+            if e[2] == len(e[1]):  # the prompt is complete: its first token is sampled in this step
+                want.append(int(batch.offset[nd + k]) + n - 1)
+                rows.append(e[0])
+                b = e[0]
+                g.kv_start[b:b + 1].zero_()
+                g.kv_len[b:b + 1].fill_(len(e[1]) - 1)  # the bookkeeping advances it to the prompt length
+                g.gen_len[b:b + 1].zero_()
+                g.active[b:b + 1].fill_(1)
+        self.pending = [e for e in self.pending if e[2] is None or e[2] < len(e[1])]
+        h = g.model.step(batch, g.cache, torch.tensor(want, dtype=torch.long).to(g.device))
+        if rows:
+            full = h.new_zeros(g._bucket(max(self.rows) + 1), h.shape[1])
+            full[torch.tensor(rows).to(g.device)] = h
+            g._emit(full, self.params, self.eos, self.pad_id)
+        return True
 
     def collect(self) -> List[FinishedRow]:
         """Rows that have finished since the last call (their outputs copied to the host)."""
@@ -655,7 +759,8 @@ class ContinuousBatcher:
             return []
         g = self.gen
         act = g.active.cpu()
-        done = [b for b in self.rows if not bool(act[b])]
+        waiting = {e[0] for e in self.pending}
+        done = [b for b in self.rows if b not in waiting and not bool(act[b])]
         out = []
         if done:
             idx = torch.tensor(done, device=g.device)
@@ -666,4 +771,9 @@ class ContinuousBatcher:
                 tag, S, s0 = self.rows.pop(b)
                 out.append(FinishedRow(tag, t[:n].tolist(), lp[:n].tolist(), S, self.steps - s0))
                 self.free.append(b)
+                if g.ragged:
+                    g.cache.release(b)
+            if g.ragged:
+                g.kv_len[idx], g.pos[idx] = 0, 0
+                g.cache.sync()  # a released row's table entries are gone before its pages have a new owner
         return out

@@ -138,7 +138,7 @@ class LayeredLM(nn.Module):
         self.lm_head = nn.Parameter(torch.empty(cfg.vocab_size, cfg.hidden_size, **kw), requires_grad=False)
         self.layers = nn.ModuleList([LayeredLayer(i, s, cfg.hidden_size, cfg.norm_eps, device, dtype)
                                      for i, s in enumerate(cfg.layers)])
-        self._tables = {}
+        self._tables, self._old_tables = {}, []
         self._head_shuf = ops.ShufCache()
         if init:
             self.reset_parameters(seed)
@@ -175,15 +175,18 @@ class LayeredLM(nn.Module):
         from ..generation.paged import PagedCache
 
         dev = device or self.embed.device
+        cache = PagedCache([layer.mix.cache_width() for layer in self.layers], rows, max_seq, tokens, dev, self.dtype)
         for layer in self.layers:
-            self._rope(layer.mix.spec.rot, max_seq, dev)
-        return PagedCache([layer.mix.cache_width() for layer in self.layers], rows, max_seq, tokens, dev, self.dtype)
+            self._rope(layer.mix.spec.rot, cache.max_seq, dev)
+        return cache
 
     def _rope(self, rot, n: int, dev):
-        """cos / sin tables of at least n positions (made before any graph captures them)"""
+        """cos / sin tables of at least n positions. Made with the cache, before a graph captures them; outgrown
+        tables stay alive for the graphs that hold them."""
         key = (rot.base, rot.dims, None if rot.scaling is None else tuple(vars(rot.scaling).values()))
         t = self._tables.get(key)
         if t is None or t[0].shape[0] < n or t[0].device != torch.device(dev):
+            self._old_tables.append(t)
             t = self._tables[key] = ops.yarn_rope_tables(rot.dims, rot.base, max(n, 1), rot.scaling, dev)
         return t
 
@@ -252,6 +255,7 @@ class LayeredLM(nn.Module):
         ids = input_ids.tolist()
         for b in range(B):
             cache.reserve(b, S - start[b])
+        cache.sync()
         batch = RaggedBatch.build([(b, ids[b][start[b]:], 0) for b in range(B)], input_ids.device)
         h = self.step(batch, cache)
         out = h.new_zeros(B * S, h.shape[1])

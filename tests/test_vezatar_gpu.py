@@ -1,0 +1,435 @@
+"""Vezatar on the GPU: every kernel against fp32 torch arithmetic, and the model in fp32 and bf16 against the
+plain implementation (vezatar_oracle.py): whole prompts, portions, decoding, mixed batches with reused
+pages, far keys at every edge, greedy generation through the captured decode step and the scheduler."""
+import json
+import os
+import subprocess
+import sys
+
+import numpy as np
+import pytest
+import torch
+import vezatar_common as vc
+import vezatar_oracle as oracle
+
+from rag_tl_domainllm_optimizer_amd import ops
+from rag_tl_domainllm_optimizer_amd.generation import ContinuousBatcher, Generator, SamplingParams
+from rag_tl_domainllm_optimizer_amd.generation.paged import PAGE
+from rag_tl_domainllm_optimizer_amd.generation.ragged import StepEngine
+from rag_tl_domainllm_optimizer_amd.ops import MoePairs, SplitK, native, reference as ref
+
+pytestmark = pytest.mark.gpu
+DEV = "cuda"
+ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+F32_TOL = 2e-4   # per-position logits difference relative to their spread (fp32 rounding: up to 4e-5)
+BF16_TOL = 0.1   # bf16 activations and products: median 0.02, single positions up to 0.07
+
+
+def rel(a, b):
+    a, b = a.float().cpu(), b.float().cpu()
+    return float((a - b).norm() / b.norm().clamp_min(1e-30))
+
+
+def tokens(cfg, n, seed=0):
+    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+
+def check(got, want, dtype):
+    e = (got - want).pow(2).mean(-1).sqrt() / want.std()
+    if dtype == torch.float32:
+        assert float(e.max()) < F32_TOL, float(e.max())
+    else:  # single positions of the narrowest model, whose branch norms divide by small numbers, reach 0.22
+        assert float(e.quantile(0.9)) < BF16_TOL and float(e.max()) < 4 * BF16_TOL, (float(e.max()), float(e.median()))
+
+
+CONFIGS = {
+    "odd": vc.odd,                                                    # no MFMA kernel fits
+    "even": vc.even,                                                  # 6 heads, latent 64 + 16
+    "heads20_rank256": lambda: vc.even(20, 64, 64, 128, 256),         # two head tiles, the last half empty
+    "rank512": lambda: vc.even(16, 128, 64, 128, 512),
+    "rank136_v24": lambda: vc.even(17, 40, 8, 24, 136),               # ragged sizes on the MFMA kernels
+    "dim200": lambda: vc.even(3, 184, 24, 64, 64),
+}
+
+
+@pytest.fixture(scope="module")
+def model_of(tmp_path_factory):
+    made = {}
+
+    def get(name, dtype):
+        if (name, dtype) not in made:
+            cfg = CONFIGS[name]()
+            w = vc.weights(cfg, 1, decisive=dtype == torch.bfloat16)
+            made[name, dtype] = (cfg, w, vc.load(cfg, w, tmp_path_factory.mktemp(name), DEV, dtype))
+        return made[name, dtype]
+    return get
+
+
+# ------------------------------------------------------------------ kernels
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_gemm_any(dtype):
+    tol = 1e-6 if dtype == torch.float32 else 4e-3
+    for M, N, K in ((1, 1, 1), (3, 70, 37), (130, 65, 100)):
+        a, w = torch.randn(M, K).to(dtype), torch.randn(N, K).to(dtype)
+        want = a.float() @ w.float().T
+        assert rel(native().gemm_any(a.to(DEV), w.to(DEV)), want) < tol
+        assert rel(native().gemm_any(a.to(DEV), w.to(DEV), True), want) < 1e-6
+        a3, w3 = torch.randn(M, 3, K).to(dtype), torch.randn(3, N, K).to(dtype)
+        got = native().gemm_any(a3.to(DEV).transpose(0, 1), w3.to(DEV))
+        assert rel(got, torch.stack([a3[:, b].float() @ w3[b].float().T for b in range(3)])) < tol
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("H", [4, 130, 192, 4096])
+def test_branch_norm(dtype, H):
+    T, eps = 5, 1e-3
+    x, y = torch.randn(T, H), torch.randn(T, H).to(dtype)
+    wb, wn = torch.randn(H).to(dtype), torch.randn(H).to(dtype)
+    h_tol = 1e-6 if dtype == torch.float32 else 3e-3
+
+    def run(yy, yref):
+        xg = x.to(DEV)
+        h = ops.branch_norm(xg, yy, wb.to(DEV), wn.to(DEV), eps)
+        want = x + oracle.rms(yref, eps) * wb.float()
+        assert rel(xg, want) < 1e-6 and rel(h, oracle.rms(want, eps) * wn.float()) < h_tol
+    run(y.to(DEV), y.float())
+    slabs = torch.randn(3, T, H)
+    run(SplitK(slabs.to(DEV), 3, T, H, dtype), slabs.sum(0))
+    pos = torch.randperm(2 * T).int().view(T, 2)
+    pw = torch.rand(T, 2)
+    for pt in (dtype, torch.float32):
+        yp = torch.randn(2 * T, H).to(pt)
+        run(MoePairs(yp.to(DEV), pw.to(DEV), pos.to(DEV)), (yp.float()[pos.long()] * pw[..., None]).sum(1))
+    table, ids = torch.randn(9, H).to(dtype), torch.tensor([0, 8, 3, 3, 1])
+    xg, h = ops.embed_norm(table.to(DEV), ids.to(DEV), wn.to(DEV), eps)
+    assert torch.equal(xg.cpu(), table[ids].float()) and rel(h, oracle.rms(table[ids].float(), eps) * wn.float()) < h_tol
+
+
+@pytest.mark.parametrize("M", [1, 16, 17, 48, 64, 65, 300, 700])
+def test_gated_unit_epilogues(M):
+    for K, N in ((256, 512), (128, 192), (72, 144)):
+        x, w = torch.randn(M, K).bfloat16(), (torch.randn(N, K) * 0.15).bfloat16()
+        for glu in (ops.Glu(), ops.Glu(1.1, 1.702, 1.0)):
+            p = (x.float() @ w.float().T)
+            g, u = p.chunk(2, -1)
+            g = g.clamp(max=glu.limit)
+            want = g * torch.sigmoid(glu.alpha * g) * (u.clamp(-glu.limit, glu.limit) + glu.offset)
+            assert rel(ops.glu_project(x.to(DEV), w.to(DEV), glu, ops.ShufCache()), want) < 8e-3
+
+
+@pytest.mark.parametrize("E,top,nsh", [(5, 2, 0), (64, 8, 2), (130, 1, 1), (7, 7, 0)])
+def test_router(E, top, nsh):
+    z, c = torch.randn(37, E + 3) * 2, torch.randn(E) * 0.2
+    idx, w = native().moe_route(z.to(DEV), c.to(DEV), top, nsh, E if nsh else -1)
+    s = torch.softmax(z[:, :E], -1)
+    want = (s + c).topk(top, -1).indices
+    assert torch.equal(idx[:, :top].cpu().long(), want)
+    torch.testing.assert_close(w[:, :top].cpu(), s.gather(-1, want), rtol=1e-5, atol=1e-7)
+    for j in range(nsh):
+        assert (idx[:, top + j] == E + j).all()
+        torch.testing.assert_close(w[:, top + j].cpu(), torch.sigmoid(z[:, E]), rtol=1e-5, atol=1e-7)
+
+
+def test_router_ties_and_nan_stay_in_range():
+    E = 70
+    z = torch.zeros(3, E)
+    z[1] = float("nan")
+    z[2, 5] = float("inf")
+    idx, _ = native().moe_route(z.to(DEV), torch.zeros(E).to(DEV), 6, 0, -1)
+    idx = idx.cpu()
+    assert idx[0].tolist() == [0, 1, 2, 3, 4, 5]
+    assert int(idx.min()) >= 0 and int(idx.max()) < E and all(len(set(r)) == 6 for r in idx.tolist())
+
+
+@pytest.mark.parametrize("T,slots,G", [(1, 3, 5), (77, 4, 9), (3000, 9, 66)])
+def test_pair_sort(T, slots, G):
+    idx = torch.randint(0, G, (T, slots), generator=torch.Generator().manual_seed(T)).int()
+    idx[:, 0] = G - 1
+    offs, tok, pos, tiles, n = native().moe_sort(idx.to(DEV), G, 256)
+    order = torch.argsort(idx.reshape(-1), stable=True)
+    assert torch.equal(tok.cpu().long(), order // slots)
+    assert torch.equal(pos.cpu().long()[order], torch.arange(T * slots))
+    cnt = torch.bincount(idx.reshape(-1).long(), minlength=G)
+    assert torch.equal(offs.cpu().long(), torch.cat([torch.zeros(1, dtype=torch.long), cnt.cumsum(0)]))
+    want = [(g, a, min(a + 256, int(offs[g + 1]))) for g in range(G) for a in range(int(offs[g]), int(offs[g + 1]), 256)]
+    assert int(n) == len(want) <= tiles.shape[0] and [tuple(r[:3]) for r in tiles[:len(want)].tolist()] == want
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("T,W,F,E,top,nsh", [(1, 256, 128, 12, 4, 2), (60, 136, 40, 5, 2, 1), (300, 256, 128, 3, 2, 0),
+                                             (900, 192, 256, 6, 3, 1), (50, 44, 14, 5, 2, 2)])
+def test_expert_products(dtype, T, W, F, E, top, nsh):
+    G = E + nsh
+    h, rw = torch.randn(T, W).to(dtype), (torch.randn((E + 8) // 8 * 8 + 8, W) * 0.1).to(dtype)
+    cor = torch.randn(E) * 0.1
+    gu, dn = (torch.randn(G, 2 * F, W) * W ** -0.5).to(dtype), (torch.randn(G, W, F) * F ** -0.5).to(dtype)
+    y = ops.moe_ff(h.to(DEV), rw.to(DEV), cor.to(DEV), gu.to(DEV), dn.to(DEV), top, nsh, E if nsh else -1)
+    z = h.float() @ rw.float().T
+    s = torch.softmax(z[:, :E], -1)
+    idx = (s + cor).topk(top, -1).indices
+    want = torch.zeros(T, W)
+    for g in range(G):
+        wt = (s.gather(-1, idx) * (idx == g)).sum(-1, keepdim=True) if g < E else torch.sigmoid(z[:, E:E + 1])
+        a, b = (h.float() @ gu[g].float().T).chunk(2, -1)
+        want += wt * ((a * torch.sigmoid(a) * b) @ dn[g].float().T)
+    e = (y.combine().cpu() - want).norm(dim=-1) / want.norm(dim=-1)
+    tol = 1e-5 if dtype == torch.float32 else 1.5e-2
+    assert float(e.median()) < tol and float((e > 3 * tol).float().mean()) <= 0.02
+
+
+@pytest.mark.parametrize("H,rank,rot", [(3, 64, 16), (16, 128, 32), (17, 128, 128), (20, 200, 40), (32, 512, 64),
+                                        (40, 320, 64), (5, 512, 128)])
+@pytest.mark.parametrize("parts", [1, 3, 8])
+def test_latent_decode_and_out(H, rank, rot, parts):
+    """absorbed attention alone: page and partition borders, one key per row that stands out, sink, gate"""
+    KD, V = rank + rot, 24
+    lens = [1, 2, 31, 32, 33, 63, 64, 65, 128, 300]
+    g = torch.Generator().manual_seed(H)
+    n_pages = sum((n + 63) // 64 for n in lens) + 1
+    pool = (torch.randn(n_pages, 64, KD, generator=g)).bfloat16()
+    tab = torch.zeros(len(lens), 5, dtype=torch.int32)
+    perm = (torch.randperm(n_pages - 1, generator=g) + 1).int()
+    at = 0
+    for r, n in enumerate(lens):
+        k = (n + 63) // 64
+        tab[r, :k] = perm[at:at + k]
+        at += k
+    T = len(lens)
+    q = (torch.randn(T, H, KD, generator=g) * 0.3).bfloat16()
+    for r, n in enumerate(lens):  # the last key of the row, its first one, or the one on a page border
+        key = (n - 1, 0, min(64, n - 1))[r % 3]
+        q[r] = pool[tab[r, key // 64], key % 64] * 2
+    sink = torch.linspace(-1, 40, H)
+    gate, wuv = torch.randn(T, H * V, generator=g).bfloat16(), (torch.randn(H, V, rank, generator=g) * rank ** -0.5).bfloat16()
+    row, pos = torch.arange(T).int(), torch.tensor(lens).int() - 1
+    scale = KD ** -0.5
+    o = ref.latent_attend(q, pool, tab, row, pos, sink, rank, scale, 64)
+    want = torch.einsum("thc,hvc->thv", o, wuv.float()).reshape(T, -1) * torch.sigmoid(gate.float())
+    d = [t.to(DEV) for t in (q, pool, tab, row, pos, sink, wuv, gate)]
+    part, ml = native().latent_decode(d[0], d[1], d[2], d[3], d[4], rank, parts, scale)
+    out = torch.empty(T, H * V, dtype=torch.bfloat16, device=DEV)
+    native().latent_out(part, ml, d[5], d[6], d[7], out)
+    assert rel(out, want) < 1e-2
+    any_o = native().latent_any(d[0], d[1], d[2], d[3], d[4], d[5], rank, scale)
+    assert rel(any_o, o) < 4e-3
+
+
+@pytest.mark.parametrize("H,dim,rot,vdim", [(2, 32, 16, 48), (3, 64, 64, 128), (2, 128, 64, 128), (1, 184, 64, 64), (2, 40, 8, 8),
+                                            (2, 16, 24, 72)])
+def test_latent_prefill(H, dim, rot, vdim):
+    """portions of several requests over expanded keys and values, starts inside the context"""
+    shapes = [(0, 33), (100, 40), (0, 200), (63, 130), (5, 128)]  # (start, portion)
+    g = torch.Generator().manual_seed(dim)
+    hd = dim + rot
+    N, KV = sum(n for _, n in shapes), sum(s + n for s, n in shapes)
+    segs, tiles, qo, ko = [], [], 0, 0
+    for i, (s, n) in enumerate(shapes):
+        segs.append([0, qo, n, ko, s + n, s, 0, 0])
+        tiles += [[i, t] for t in range((n + 127) // 128)]
+        qo += n
+        ko += s + n
+    q, kr = torch.randn(N, H * hd, generator=g).bfloat16(), torch.randn(KV, rot, generator=g).bfloat16()
+    kv = torch.randn(KV, H * (dim + vdim), generator=g).bfloat16()
+    gate, sink = torch.randn(N, H * vdim, generator=g).bfloat16(), torch.linspace(-2, 8, H)
+    scale = 2.0 * hd ** -0.5
+    want = torch.zeros(N, H * vdim)
+    for (s, n), sg in zip(shapes, segs):
+        for h in range(H):
+            k = torch.cat([kv[sg[3]:sg[3] + s + n, h * dim:(h + 1) * dim], kr[sg[3]:sg[3] + s + n]], 1).float()
+            v = kv[sg[3]:sg[3] + s + n, H * dim + h * vdim:H * dim + (h + 1) * vdim].float()
+            sc = q[sg[1]:sg[1] + n, h * hd:(h + 1) * hd].float() @ k.T * scale
+            sc = sc.masked_fill(torch.arange(s + n)[None] > s + torch.arange(n)[:, None], -torch.inf)
+            p = torch.softmax(torch.cat([sc, sink[h].expand(n, 1)], 1), -1)[:, :-1]
+            want[sg[1]:sg[1] + n, h * vdim:(h + 1) * vdim] = p @ v
+    want *= torch.sigmoid(gate.float())
+    out = torch.empty(N, H * vdim, dtype=torch.bfloat16, device=DEV)
+    native().latent_prefill(q.to(DEV), kv.to(DEV), kr.to(DEV), sink.to(DEV), gate.to(DEV), out,
+                            torch.tensor(segs).int().to(DEV), torch.tensor(tiles).int().to(DEV), H, dim, rot, vdim, scale)
+    assert rel(out, want) < 1e-2
+
+
+def test_wrappers_refuse_bad_shapes():
+    n = native()
+    x = torch.randn(4, 8, device=DEV)
+    with pytest.raises(RuntimeError):
+        n.branch_norm(x, 1, y=x[:2].contiguous(), w_branch=x[0].contiguous(), eps=1e-5)
+    with pytest.raises(RuntimeError):
+        n.gemm_any(x, torch.randn(4, 9, device=DEV))
+    with pytest.raises(RuntimeError):
+        n.moe_route(x, torch.zeros(9, device=DEV), 2, 0, -1)
+    with pytest.raises(RuntimeError):
+        n.moe_route(x, torch.zeros(8, device=DEV), 9, 0, -1)
+    with pytest.raises(RuntimeError):
+        n.latent_any(torch.randn(1, 2, 12, device=DEV), torch.zeros(2, 64, 16, device=DEV),
+                     torch.zeros(1, 1, dtype=torch.int32, device=DEV), torch.zeros(1, dtype=torch.int32, device=DEV),
+                     torch.zeros(1, dtype=torch.int32, device=DEV), torch.zeros(2, device=DEV), 8, 1.0)
+
+
+# ------------------------------------------------------------------ model
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("name", list(CONFIGS))
+def test_whole_portions_and_decoding(model_of, name, dtype):
+    cfg, w, m = model_of(name, dtype)
+    t = tokens(cfg, 260, 3)
+    want = oracle.forward(cfg, w, t)
+    eng = StepEngine(m, 2, 320)
+    for sizes in ((260,), (129, 1), (2, 33, 64, 1, 100, 3)):
+        check(vc.run(eng, t, sizes), want, dtype)
+
+
+@pytest.mark.parametrize("name", ["odd", "even"])
+def test_residual_after_every_layer(model_of, name):
+    from rag_tl_domainllm_optimizer_amd.generation.ragged import RaggedBatch
+
+    cfg, w, m = model_of(name, torch.float32)
+    t = tokens(cfg, 70, 4)
+    layers, got = [], []
+    oracle.forward(cfg, w, t, layers_out=layers)
+    cache = m.make_cache(1, 128)
+    cache.reserve(0, len(t))
+    cache.sync()
+    m.step(RaggedBatch.build([(0, t, 0)], DEV), cache, layer_out=got)
+    for a, b in zip(got, layers):
+        torch.testing.assert_close(a.cpu(), b, rtol=5e-4, atol=5e-4)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("name", ["odd", "heads20_rank256"])
+def test_mixed_batches_and_reused_pages(model_of, name, dtype):
+    cfg, w, m = model_of(name, dtype)
+    rng = np.random.default_rng(1)
+    eng = StepEngine(m, 3, 8 * PAGE)
+    live, nxt, done, want, got = {}, 0, 0, {}, {}
+    while done < 8:
+        while len(live) < 3 and nxt < 8:
+            t = tokens(cfg, int(rng.integers(1, 200)), 10 + nxt)
+            if sum((len(x[1]) + PAGE - 1) // PAGE for x in live.values()) + (len(t) + PAGE - 1) // PAGE > 8:
+                break
+            want[nxt], got[nxt] = oracle.forward(cfg, w, t), []
+            live[nxt] = [eng.admit(), t, 0]
+            nxt += 1
+        part = [k for k in live if rng.random() < 0.7] or list(live)[:1]
+        ent = [(k, live[k][1][live[k][2]:live[k][2] + int(rng.choice([1, 1, 2, 40, 90]))]) for k in part]
+        lg = eng.step([(live[k][0], c, list(range(len(c)))) for k, c in ent]).cpu()
+        o = 0
+        for k, c in ent:
+            got[k].append(lg[o:o + len(c)])
+            o += len(c)
+            live[k][2] += len(c)
+            if live[k][2] == len(live[k][1]):
+                eng.release(live.pop(k)[0])
+                done += 1
+    check(torch.cat([torch.cat(got[k]) for k in want]), torch.cat([want[k] for k in want]), dtype)
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+def test_needle_at_every_edge(tmp_path, dtype):
+    cfg, w = vc.needle_model()
+    m = vc.load(cfg, w, tmp_path, DEV, dtype)
+    n = 200
+    for at in (0, 1, 31, 32, 63, 64, 127, 128, 191, 192, n - 2):
+        t = vc.needle_tokens(n, at)
+        want = oracle.forward(cfg, w, t)[-1:]
+        plain = list(t)
+        plain[at] = 7
+        assert vc.err(oracle.forward(cfg, w, plain)[-1:], want) > 3 * BF16_TOL
+        for sizes in ((n,), (n - 1, 1), (64, 40, 1)):
+            got = vc.run(StepEngine(m, 1, 256), t, sizes)[-1:]
+            assert vc.err(got, want) < (F32_TOL if dtype == torch.float32 else BF16_TOL), (at, sizes)
+
+
+@pytest.mark.parametrize("name", ["odd", "even"])
+def test_long_decoding(model_of, name):
+    """several hundred tokens one by one, across page borders, against the whole sequence at once"""
+    cfg, w, m = model_of(name, torch.float32)
+    t = tokens(cfg, 400, 6)
+    check(vc.run(StepEngine(m, 1, 448), t, (7, 1)), oracle.forward(cfg, w, t), torch.float32)
+
+
+# ------------------------------------------------------------------ generation
+@pytest.mark.parametrize("name", ["odd", "even"])
+@pytest.mark.parametrize("use_graph", [True, False])
+def test_greedy_generation(model_of, name, use_graph):
+    cfg, w, m = model_of(name, torch.float32)
+    prompts = [tokens(cfg, n, 60 + n) for n in (5, 40, 70)]
+    want = [vc.greedy(cfg, w, p, 12) for p in prompts]
+    gen = Generator(m, max_batch=4, max_seq=128, device=DEV, use_graph=use_graph)
+    p = SamplingParams(max_new_tokens=12, do_sample=False)
+    for _ in range(3):  # later calls replay the captured step on reused rows
+        out = gen.generate(prompts, p, eos_ids=[-5])
+        assert [r.tolist() for r in out.tokens] == want
+        torch.randn(64, 64, device=DEV) @ torch.randn(64, 64, device=DEV)
+        torch.cuda.synchronize()
+
+
+@pytest.mark.parametrize("name", ["even", "rank512"])
+def test_graph_replays_equal_the_eager_step(model_of, name):
+    """bf16: greedy tokens and their log-probs of the captured decode step, bitwise the eager step's"""
+    cfg, w, m = model_of(name, torch.bfloat16)
+    prompts = [tokens(cfg, n, 70 + n) for n in (9, 130, 64, 3, 77)]
+    p = SamplingParams(max_new_tokens=24, do_sample=False)
+    eager = Generator(m, max_batch=8, max_seq=192, device=DEV, use_graph=False).generate(prompts, p, eos_ids=[-5])
+    gen = Generator(m, max_batch=8, max_seq=192, device=DEV)
+    for _ in range(4):
+        out = gen.generate(prompts, p, eos_ids=[-5])
+        assert torch.equal(out.tokens, eager.tokens) and torch.equal(out.logprobs, eager.logprobs)
+
+
+def test_continuous_batching_in_portions(model_of):
+    cfg, w, m = model_of("even", torch.float32)
+    prompts = [tokens(cfg, n, 80 + n) for n in (50, 3, 170, 20, 33, 1, 90)]
+    want = [vc.greedy(cfg, w, p, 6) for p in prompts]
+    gen = Generator(m, max_batch=3, max_seq=192, device=DEV, cache_tokens=4 * PAGE)
+    for _ in range(2):
+        cb = ContinuousBatcher(gen, SamplingParams(max_new_tokens=6, do_sample=False), eos_ids=[-5], prefill_tokens=48)
+        todo, got = list(enumerate(prompts)), {}
+        for _ in range(300):
+            while todo and cb.free_rows():
+                i, pr = todo.pop(0)
+                cb.admit(pr, i)
+            cb.step(2)
+            for r in cb.collect():
+                got[r.tag] = r.tokens
+            if len(got) == len(prompts):
+                break
+        assert [got[i] for i in range(len(prompts))] == want
+        assert gen.cache.free_tokens() == 4 * PAGE
+
+
+def test_sampling_logprobs_match_rescoring(model_of):
+    cfg, w, m = model_of("even", torch.float32)
+    pr = [tokens(cfg, 20, 1), tokens(cfg, 50, 2)]
+    out = Generator(m, max_batch=2, max_seq=96, device=DEV).generate(pr, SamplingParams(max_new_tokens=8, temperature=0.8,
+                                                                                         top_k=0), eos_ids=[-5])
+    for b, p in enumerate(pr):
+        seq = p + out.tokens[b].tolist()
+        lp = torch.log_softmax(oracle.forward(cfg, w, seq) / 0.8, -1)
+        want = torch.stack([lp[len(p) - 1 + i, seq[len(p) + i]] for i in range(8)])
+        torch.testing.assert_close(out.logprobs[b].cpu(), want, rtol=1e-3, atol=1e-3)
+
+
+def test_trace_program(model_of, tmp_path):
+    """bin/trace_run as a program of its own: answers before it asks for the next step"""
+    cfg, w, m = model_of("even", torch.float32)
+    vc.load(cfg, w, tmp_path / "model")
+    t = tokens(cfg, 80, 5)
+    p = subprocess.Popen([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path / "model"), "--dtype",
+                          "float32", "--out", str(tmp_path / "out"), "--max-tokens", "128"], stdin=subprocess.PIPE,
+                         stdout=subprocess.PIPE, text=True)
+    try:
+        for i, (a, b) in enumerate(((0, 70), (70, 71), (71, 80))):
+            p.stdin.write(json.dumps({"step": i, "entries": [{"id": "x", "tokens": t[a:b], "want": [b - a - 1]}], "end": []}) + "\n")
+            p.stdin.flush()
+            line = ""
+            while not line.startswith("done"):
+                line = p.stdout.readline()
+                assert line
+            assert line.split() == ["done", str(i)]
+        p.stdin.close()
+        assert p.wait(30) == 0
+    finally:
+        p.kill()
+    want = oracle.forward(cfg, w, t)
+    for i, k in enumerate((69, 70, 79)):
+        got = torch.from_numpy(np.fromfile(tmp_path / "out" / f"{i}.f32", "<f4").copy())[None]
+        assert vc.err(got, want[k:k + 1]) < F32_TOL
