@@ -23,6 +23,8 @@ Secondary modes (not the headline; each prints its own JSON line):
   --mode sft       BASELINE config 3: RAFT-style LoRA r=16 SFT with distractor docs, tokens/s
   --mode pipeline  BASELINE config 5: RAG index -> LoRA SFT -> PPO on one policy (default
                    --model llama2-13b; --fp8 runs rollouts / reference scoring on e4m3fn weights)
+  --mode layered   prefill and decode throughput of a layered model (Vezatar) beside the closest
+                   existing decoder at equal width and depth (random weights)
 """
 from __future__ import annotations
 
@@ -88,7 +90,14 @@ def main():
     ap.add_argument("--torch-profile", default=None,
                     help="PPO mode: run one extra (untimed) step under torch.profiler after the warm-up and "
                          "write its per-op table, grouped by Python call site, to this path")
-    ap.add_argument("--mode", default="ppo", choices=["ppo", "sft", "pipeline", "serve"])
+    ap.add_argument("--mode", default="ppo", choices=["ppo", "sft", "pipeline", "serve", "layered"])
+    ap.add_argument("--layered-sizes", default="vezatar-7b/mistral-7b,vezatar-2k/mistral-2k",
+                    help="--mode layered: comma list of layered-preset/comparison-preset pairs")
+    ap.add_argument("--layered-layers", type=int, default=8, help="--mode layered: layers of either model")
+    ap.add_argument("--layered-prefill", default="8x1024,2x4096", help="--mode layered: prompts x tokens")
+    ap.add_argument("--layered-decode", default="1x1024,16x1024,64x1024,256x512",
+                    help="--mode layered: rows x context of the captured decode step")
+    ap.add_argument("--layered-only", default="", help="--mode layered: 'layered' or 'closest' runs one side (profiling)")
     ap.add_argument("--serve-concurrency", default="1,4,16",
                     help="--mode serve: closed-loop client counts (one engine, max batch = the largest)")
     ap.add_argument("--serve-requests", type=int, default=64, help="--mode serve: answers per concurrency level")
@@ -166,6 +175,9 @@ def main():
             tuning_over[k.strip()] = float(v) if "." in v else int(v)
         ops.set_tuning(**tuning_over)
         log(f"[bench] tuning overrides: {tuning_over}")
+    if args.mode == "layered":
+        run_layered(args, dev)
+        return
     if args.lora_grad_epilogue == "off":
         import importlib
 
@@ -440,6 +452,57 @@ def _timed(di, fn, steps):
     el = torch.tensor([time.perf_counter() - t0], dtype=torch.float64, device=di.device)
     parallel.all_reduce_(el, "max")
     return float(el), out, rank_spread(t_local / max(steps, 1), di.device)
+
+
+def run_layered(args, dev):
+    """Prefill and decode of a layered model and of the closest existing decoder, same width and layer
+    count, through ``Generator``: prefill = prompts to the first token, decode = replays of the captured
+    step. Medians over --steps runs after --warmup."""
+    import dataclasses
+    import statistics
+
+    from rag_tl_domainllm_optimizer_amd import models
+    from rag_tl_domainllm_optimizer_amd.generation import Generator, SamplingParams
+
+    rows = []
+    for pair in args.layered_sizes.split(","):
+        for side, name in zip(("layered", "closest"), pair.split("/")):
+            if args.layered_only and side != args.layered_only:
+                continue
+            cfg = models.resolve_preset(name)
+            n = args.layered_layers
+            cfg = dataclasses.replace(cfg, num_layers=n, layers=cfg.layers[:n] if cfg.is_layered else None)
+            m = models.model_class(cfg)(cfg, device=dev, dtype=torch.bfloat16, init=False).eval()
+            models.fast_random_init_(m, 0, 0.02)
+            if cfg.is_layered:
+                m._zero_padding()
+            shapes = [("prefill", *map(int, x.split("x"))) for x in args.layered_prefill.split(",") if x] + \
+                     [("decode", *map(int, x.split("x"))) for x in args.layered_decode.split(",") if x]
+            for phase, B, S in shapes:
+                T = 1 if phase == "prefill" else 33
+                gen = Generator(m, max_batch=B, max_seq=S + T, device=dev)
+                rng = random.Random(B * S)
+                prompts = [[rng.randrange(3, cfg.vocab_size) for _ in range(S)] for _ in range(B)]
+                p = SamplingParams(max_new_tokens=T, do_sample=False)
+                t = []
+                for i in range(args.warmup + args.steps):
+                    out = gen.generate_async(prompts, p, eos_ids=[-1]).result()
+                    if i >= args.warmup:
+                        t.append(out.timings["prefill_s"] if phase == "prefill" else out.timings["decode_s"] / (T - 1))
+                s = statistics.median(t)
+                rows.append({"model": name, "side": side, "layers": n, "phase": phase, "batch": B, "tokens": S,
+                             "ms": round(s * 1e3, 4), "us_per_layer": round(s * 1e6 / n, 1),
+                             "tokens_per_s": round((B * S if phase == "prefill" else B) / s, 1)})
+                log(rows[-1])
+                del gen
+            del m
+            torch.cuda.empty_cache()
+    dec = [r for r in rows if r["phase"] == "decode" and r["side"] == "layered"] or rows
+    best = max(dec, key=lambda r: r["tokens_per_s"])
+    print(json.dumps({"metric": "layered-model decode tokens/s (largest batch)", "value": best["tokens_per_s"],
+                      "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+                      "ms_per_step": best["ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
+                      "dtype": "bf16", "data": "synthetic", "config": {"model": best["model"], "rows": rows}}), flush=True)
 
 
 def run_serve(args, di, policy, tok, encoder, corpus, index):

@@ -25,16 +25,16 @@ int rt_gemm_grouped(const void*, long, const int*, const void*, long, long, void
                     int, int, int, const float*, const void*, int, hipStream_t);
 int rt_latent_prep(int, void*, long, int, const void*, float, const float*, const float*, int, int, const int*,
                    const int*, void*, const int*, int, int, int, void*, int, int, int, int, int, int, hipStream_t);
-int rt_head_gemm(const void*, long, long, const void*, long, long, void*, long, long, int, int, int, int, hipStream_t);
+int rt_head_gemm(const void*, long, long, const void*, long, long, void*, long, long, int, int, int, int, const void*,
+                 long, hipStream_t);
 int rt_latent_decode_ok(int, int);
 int rt_latent_decode(const void*, const void*, const int*, int, int, int, const int*, const int*, float*, float*, int,
                      int, int, int, int, float, const void*, hipStream_t);
-int rt_latent_out(const float*, const float*, const float*, const void*, const void*, long, void*, long, int, int, int,
-                  int, int, hipStream_t);
+int rt_latent_merge(const float*, const float*, const float*, void*, int, int, int, int, hipStream_t);
 int rt_latent_gather(int, const void*, const int*, int, int, const void*, int, int, void*, int, hipStream_t);
 int rt_latent_prefill_ok(int, int, int);
-int rt_latent_prefill(const void*, long, const void*, long, int, const void*, long, const float*, const void*, long,
-                      void*, long, const void*, const void*, int, int, int, int, int, float, hipStream_t);
+int rt_latent_prefill(const void*, long, const void*, long, int, int, const float*, const void*, long, void*, long,
+                      const void*, const void*, int, int, int, int, int, float, hipStream_t);
 int rt_latent_any(int, const void*, const void*, const int*, int, int, int, const int*, const int*, const float*, void*,
                   int, int, int, int, float, hipStream_t);
 }
@@ -172,15 +172,21 @@ Tensor gemm_any(const Tensor& a, const Tensor& w, bool out_f32, optional<Tensor>
   return c;
 }
 
-// out[b] = a[b] w[b]^T at few rows (bf16; strided 3-D views)
-void head_gemm(const Tensor& a, const Tensor& w, Tensor out) {
+// out[b] = a[b] w[b]^T at few rows (bf16; strided 3-D views), times sigmoid(gate [rows, batch * N])
+void head_gemm(const Tensor& a, const Tensor& w, Tensor out, const optional<Tensor>& gate) {
   TORCH_CHECK(a.is_cuda() && w.is_cuda() && a.scalar_type() == at::kBFloat16 && w.scalar_type() == at::kBFloat16 &&
                   out.scalar_type() == at::kBFloat16, "head_gemm: bf16");
   TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && out.dim() == 3 && a.size(0) == w.size(0) && out.size(0) == w.size(0) &&
                   a.size(2) == w.size(2) && out.size(1) == a.size(1) && out.size(2) == w.size(1) && a.stride(2) == 1 &&
                   w.stride(2) == 1 && out.stride(2) == 1 && al16(a) && al16(w), "head_gemm: shapes");
+  if (has(gate)) {
+    rows(*gate, "head_gemm gate");
+    TORCH_CHECK(gate->is_cuda() && gate->scalar_type() == at::kBFloat16 && gate->size(0) >= a.size(1) &&
+                    gate->size(1) == w.size(0) * w.size(1), "head_gemm: gate");
+  }
   rc_ok(rt_head_gemm(a.data_ptr(), a.stride(1), a.stride(0), w.data_ptr(), w.stride(1), w.stride(0), out.data_ptr(),
-                     out.stride(1), out.stride(0), (int)a.size(1), (int)w.size(1), (int)w.size(2), (int)w.size(0), stream()),
+                     out.stride(1), out.stride(0), (int)a.size(1), (int)w.size(1), (int)w.size(2), (int)w.size(0), ptr(gate),
+                     has(gate) ? gate->stride(0) : 0, stream()),
         "head_gemm");
 }
 
@@ -356,23 +362,19 @@ std::vector<Tensor> latent_decode(const Tensor& q, const Tensor& pool, const Ten
   return {part, ml};
 }
 
-// partitions -> sink, value expansion, gate -> out [T, H * vdim] rows
-void latent_out(const Tensor& part, const Tensor& ml, const Tensor& sink, const Tensor& wuv, const Tensor& gate, Tensor out) {
-  f32c(part, "latent_out part");
-  f32c(ml, "latent_out ml");
-  f32c(sink, "latent_out sink");
-  TORCH_CHECK(part.dim() == 4 && wuv.dim() == 3 && wuv.is_contiguous() && wuv.is_cuda() &&
-                  wuv.scalar_type() == at::kBFloat16 && gate.scalar_type() == at::kBFloat16 &&
-                  out.scalar_type() == at::kBFloat16, "latent_out: types");
-  const int64_t T = part.size(0), H = part.size(1), NP = part.size(2), rank = part.size(3), V = wuv.size(1);
-  rows(gate, "latent_out gate");
-  rows(out, "latent_out out");
-  TORCH_CHECK(wuv.size(0) == H && wuv.size(2) == rank && sink.numel() == H && ml.numel() == T * H * NP * 2 &&
-                  gate.size(0) >= T && gate.size(1) == H * V && out.size(0) >= T && out.size(1) == H * V && al16(wuv),
-              "latent_out: shapes");
-  rc_ok(rt_latent_out(part.data_ptr<float>(), ml.data_ptr<float>(), sink.data_ptr<float>(), wuv.data_ptr(), gate.data_ptr(),
-                      gate.stride(0), out.data_ptr(), out.stride(0), (int)T, (int)H, (int)rank, (int)V, (int)NP, stream()),
-        "latent_out");
+// partitions -> latent outputs [T, H, rank] (softmax with the sink)
+Tensor latent_merge(const Tensor& part, const Tensor& ml, const Tensor& sink) {
+  f32c(part, "latent_merge part");
+  f32c(ml, "latent_merge ml");
+  f32c(sink, "latent_merge sink");
+  TORCH_CHECK(part.dim() == 4, "latent_merge: part [T, H, NP, rank]");
+  const int64_t T = part.size(0), H = part.size(1), NP = part.size(2), rank = part.size(3);
+  TORCH_CHECK(sink.numel() == H && ml.numel() == T * H * NP * 2, "latent_merge: shapes");
+  Tensor o = at::empty({T, H, rank}, part.options().dtype(at::kBFloat16));
+  rc_ok(rt_latent_merge(part.data_ptr<float>(), ml.data_ptr<float>(), sink.data_ptr<float>(), o.data_ptr(), (int)T, (int)H,
+                        (int)rank, (int)NP, stream()),
+        "latent_merge");
+  return o;
 }
 
 Tensor latent_gather(const Tensor& pool, const Tensor& tab, const Tensor& segs, int64_t total, int64_t max_kv) {
@@ -386,10 +388,11 @@ Tensor latent_gather(const Tensor& pool, const Tensor& tab, const Tensor& segs, 
   return out;
 }
 
-// q / gate / out rows are the batch's tokens (segments index them); kv [rows, H (dim + vdim)], kr [rows, rot]
-void latent_prefill(const Tensor& q, const Tensor& kv, const Tensor& kr, const Tensor& sink, const Tensor& gate, Tensor out,
+// q / gate / out rows are the batch's tokens (segments index them); kv [rows, H (dim + vdim) + rot]: unrotated
+// keys, values, shared rotated key part
+void latent_prefill(const Tensor& q, const Tensor& kv, const Tensor& sink, const Tensor& gate, Tensor out,
                     const Tensor& segs, const Tensor& tiles, int64_t H, int64_t dim, int64_t rot, int64_t vdim, double scale) {
-  for (const Tensor* t : {&q, &kv, &kr, &gate}) {
+  for (const Tensor* t : {&q, &kv, &gate}) {
     rows(*t, "latent_prefill");
     TORCH_CHECK(t->is_cuda() && t->scalar_type() == at::kBFloat16 && al16(*t), "latent_prefill: bf16 rows, 16-B aligned");
   }
@@ -399,9 +402,9 @@ void latent_prefill(const Tensor& q, const Tensor& kv, const Tensor& kr, const T
   ints(tiles, "tiles");
   f32c(sink, "sink");
   TORCH_CHECK(segs.dim() == 2 && segs.size(1) == 8 && tiles.dim() == 2 && tiles.size(1) == 2, "latent_prefill: tables");
-  TORCH_CHECK(q.size(1) >= H * (dim + rot) && kv.size(1) == H * (dim + vdim) && kr.size(1) == rot && gate.size(1) == H * vdim &&
-                  out.size(1) == H * vdim && sink.numel() == H && kr.size(0) == kv.size(0), "latent_prefill: shapes");
-  rc_ok(rt_latent_prefill(q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), (int)(H * dim), kr.data_ptr(), kr.stride(0),
+  TORCH_CHECK(q.size(1) >= H * (dim + rot) && kv.size(1) == H * (dim + vdim) + rot && gate.size(1) == H * vdim &&
+                  out.size(1) == H * vdim && sink.numel() == H, "latent_prefill: shapes");
+  rc_ok(rt_latent_prefill(q.data_ptr(), q.stride(0), kv.data_ptr(), kv.stride(0), (int)(H * dim), (int)(H * (dim + vdim)),
                           sink.data_ptr<float>(), gate.data_ptr(), gate.stride(0), out.data_ptr(), out.stride(0),
                           segs.data_ptr(), tiles.data_ptr(), (int)tiles.size(0), (int)H, (int)dim, (int)rot, (int)vdim,
                           (float)scale, stream()),
@@ -434,7 +437,8 @@ void bind_layered(py::module_& m) {
         py::arg("pair_pos") = py::none(), py::arg("eps"));
   m.def("gemm_any", &gemm_any, "a w^T, any shape, bf16 / fp32, batched or grouped", py::arg("a"), py::arg("w"),
         py::arg("out_f32") = false, py::arg("out") = py::none(), py::arg("offs") = py::none(), py::arg("row_map") = py::none());
-  m.def("head_gemm", &head_gemm, "per-head a w^T at few rows");
+  m.def("head_gemm", &head_gemm, "per-head a w^T at few rows (gated)", py::arg("a"), py::arg("w"), py::arg("out"),
+        py::arg("gate") = py::none());
   m.def("glu_any", &glu_any, "gated linear unit of [gate | up] rows");
   m.def("gate_mul", &gate_mul, "a *= sigmoid(g)");
   m.def("moe_route", &moe_route, "softmax router with choice correction -> experts, weights");
@@ -445,7 +449,7 @@ void bind_layered(py::module_& m) {
   m.def("latent_decode_ok", [](int rank, int kd) { return rt_latent_decode_ok(rank, kd) != 0; });
   m.def("latent_prefill_ok", [](int dim, int rot, int vdim) { return rt_latent_prefill_ok(dim, rot, vdim) != 0; });
   m.def("latent_decode", &latent_decode, "absorbed attention partials over the paged latent cache");
-  m.def("latent_out", &latent_out, "partition merge, sink, value expansion, output gate");
+  m.def("latent_merge", &latent_merge, "partition merge with the sink");
   m.def("latent_gather", &latent_gather, "cached rows of each segment, dense");
   m.def("latent_prefill", &latent_prefill, "flash attention of prompt portions over expanded keys / values");
   m.def("latent_any", &latent_any, "absorbed attention, any size / type");

@@ -9,7 +9,8 @@
 // Few query tokens per request (decode, short portions) run the absorbed form: the query is moved into
 // latent space once (q_abs = [W_uk^T q_unrotated, q_rotated], KD wide), so scores and the weighted sum
 // both read the cached rows directly and all heads share them:
-//   latent_prep -> (absorb product) -> latent_decode (split over key partitions) -> latent_out
+//   latent_prep -> head product (absorb) -> latent_decode (split over key partitions) -> latent_merge ->
+//   head product (value expansion, gate)
 // Longer portions expand the request's keys and values once per layer (a GEMM over the gathered rows)
 // and run a flash kernel over [unrotated | rotated] heads:
 //   latent_prep -> latent_gather -> (expand GEMM) -> latent_prefill
@@ -58,6 +59,7 @@ struct PrepArgs {
   void* pool; const int* tab; int max_pages, n_pages, n_rows;
   void* qabs; int n_abs;       // tokens [0, n_abs): rotated query part to qabs [.., H, rank + rot]; others in place
   int H, dim, rot, rank;
+  int vec;                     // 16-B aligned rows and whole rotation: vector loads of the query part
 };
 
 template <typename T>
@@ -93,6 +95,25 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a) {
     }
   }
   const int hp = a.rot / 2;
+  if (sizeof(T) == 2 && a.vec) {  // 4 pairs = 16 B at a time
+    const int h4 = hp / 4;
+    for (int e = tid; e < a.H * h4; e += 256) {
+      const int h = e / h4, i = (e % h4) * 4;
+      T* q = pr + (long)h * (a.dim + a.rot) + a.dim + 2 * i;
+      float x[8], y[8];
+      unpack8(*(const uint4*)q, x);
+      const float4 c = *(const float4*)(cs + i), s = *(const float4*)(sn + i);
+      const float c4[4] = {c.x, c.y, c.z, c.w}, s4[4] = {s.x, s.y, s.z, s.w};
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        y[2 * k] = x[2 * k] * c4[k] - x[2 * k + 1] * s4[k];
+        y[2 * k + 1] = x[2 * k + 1] * c4[k] + x[2 * k] * s4[k];
+      }
+      T* d = t < a.n_abs ? (T*)a.qabs + ((long)t * a.H + h) * KD + a.rank + 2 * i : q;
+      *(uint4*)d = pack8(y);
+    }
+    return;
+  }
   for (int e = tid; e < a.H * hp; e += 256) {
     const int h = e / hp, i = e % hp;
     T* q = pr + (long)h * (a.dim + a.rot) + a.dim + 2 * i;
@@ -105,12 +126,13 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a) {
 }
 
 // ---------------------------------------------------------------------------------------------
-// per-head product at few rows: C[t][b][:] = A[t][b][:] W_b^T (absorb: rank x dim per head). MFMA, the
-// weights streamed straight to registers. grid (N / 64, batch, T / 16), wave = 16 columns.
+// per-head product at few rows: C[t][b][:] = A[t][b][:] W_b^T (absorb: rank x dim per head; value
+// expansion: vdim x rank, times sigmoid(gate[t][b N + n])). MFMA, weights streamed straight to registers. grid (N / 64, batch, T / 16), wave = 16 columns.
 // ---------------------------------------------------------------------------------------------
 __global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict__ A, long lda, long sA,
                                                         const bf16_t* __restrict__ W, long ldw, long sW,
-                                                        bf16_t* __restrict__ C, long ldc, long sC, int T, int N, int K) {
+                                                        bf16_t* __restrict__ C, long ldc, long sC, int T, int N, int K,
+                                                        const bf16_t* __restrict__ gate, long ldg) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
   const int n0 = blockIdx.x * 64 + w * 16, b = blockIdx.y, t0 = blockIdx.z * 16;
   if (n0 >= N) return;
@@ -128,9 +150,14 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict
   const int t = t0 + r16;
   if (t >= T) return;
   bf16_t* c = C + (long)t * ldc + b * sC + n0 + 4 * q;
+  const bf16_t* gp = gate + (long)t * ldg + (long)b * N + n0 + 4 * q;
 #pragma unroll
   for (int r = 0; r < 4; ++r)
-    if (n0 + 4 * q + r < N) c[r] = f2bf(acc[r]);
+    if (n0 + 4 * q + r < N) {
+      float y = acc[r];
+      if (gate) y /= 1.f + __expf(-bf2f(gp[r]));
+      c[r] = f2bf(y);
+    }
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -331,75 +358,39 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
 }
 
 // ---------------------------------------------------------------------------------------------
-// merge of the partitions (+ sink), value expansion W_uv, output gate. grid (H, T / 16, VS), 4 waves
+// merge of the partitions, with the sink in the denominator: one workgroup per (token, head)
 // ---------------------------------------------------------------------------------------------
-struct OutArgs {
-  const float* part; const float* ml;
-  const float* sink;           // [H] fp32
-  const bf16_t* wuv;           // [H, vdim, rank]
-  const bf16_t* gate; long ldg; // [T, ldg], head h at h * vdim
-  bf16_t* o; long ldo;
-  int T, H, rank, vdim, NP;
-};
-
-__global__ __launch_bounds__(256) void latent_out_kernel(OutArgs a) {
-  extern __shared__ __attribute__((aligned(16))) bf16_t lat[];  // [16][LD]
-  const int h = blockIdx.x, t0 = blockIdx.y * 16;
-  const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, r16 = lane & 15, q = lane >> 4;
-  const int rp = (a.rank + 31) & ~31, LD = rp + 8;
-  const float sink2 = a.sink[h] * 1.4426950408889634f;
-  // wave w merges tokens w, w + 4, ...
-  for (int r = w; r < 16; r += 4) {
-    const int t = t0 + r;
-    if (t >= a.T) {
-      for (int c = lane; c < rp; c += 64) lat[r * LD + c] = 0;
-      continue;
-    }
-    const long base = ((long)t * a.H + h) * a.NP;
-    float M = sink2;
-    for (int p = 0; p < a.NP; ++p) M = fmaxf(M, a.ml[(base + p) * 2]);
-    float L = exp2f(sink2 - M);
-    for (int p = 0; p < a.NP; ++p) {
-      const float mp = a.ml[(base + p) * 2];
-      if (mp != -INFINITY) L += a.ml[(base + p) * 2 + 1] * exp2f(mp - M);
-    }
-    const float inv = 1.f / L;
-    for (int c = 2 * lane; c < rp; c += 128) {
-      float y0 = 0.f, y1 = 0.f;
-      if (c < a.rank) {
-        for (int p = 0; p < a.NP; ++p) {
-          const float mp = a.ml[(base + p) * 2];
-          if (mp == -INFINITY) continue;
-          const float f = exp2f(mp - M);
-          const float2 v = *(const float2*)(a.part + (base + p) * a.rank + c);
-          y0 = fmaf(f, v.x, y0);
-          y1 = fmaf(f, v.y, y1);
-        }
-      }
-      *(uint32_t*)(lat + r * LD + c) = pack2bf(y0 * inv, y1 * inv);
-    }
-  }
-  __syncthreads();
-  const int nt = (a.vdim + 15) / 16;
-  for (int vt = blockIdx.z * 4 + w; vt < nt; vt += 4 * gridDim.z) {
-    const bf16_t* wp = a.wuv + ((long)h * a.vdim + min(vt * 16 + r16, a.vdim - 1)) * a.rank + 8 * q;
-    const bf16_t* lp = lat + r16 * LD + 8 * q;
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-    for (int k = 0; k < rp; k += 32) {
-      const bf16x8 wf = k + 8 * q < a.rank ? *(const bf16x8*)(wp + k) : bf16x8{};
-      acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, *(const bf16x8*)(lp + k), acc, 0, 0, 0);
-    }
-    const int t = t0 + r16;
-    if (t < a.T) {
+__global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ part, const float* __restrict__ ml,
+                                                           const float* __restrict__ sink, bf16_t* __restrict__ o, int H,
+                                                           int rank, int NP) {
+  const long th = blockIdx.x;
+  const int tid = threadIdx.x;
+  const float sink2 = sink[th % H] * 1.4426950408889634f;
+  const float* m = ml + th * NP * 2;
+  float M = sink2;
+  for (int p = 0; p < NP; ++p) M = fmaxf(M, m[2 * p]);
+  float L = exp2f(sink2 - M);
+  for (int p = 0; p < NP; ++p) L += m[2 * p + 1] * exp2f(m[2 * p] - M);  // an empty partition: 0 * exp2(-inf)
+  const float inv = 1.f / L;
+  for (int c = 4 * tid; c < rank; c += 512) {  // rank % 8 == 0
+    float y[4] = {0.f, 0.f, 0.f, 0.f};
+    for (int p0 = 0; p0 < NP; p0 += 4) {
+      float4 v[4];
+      float f[4];
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int v = vt * 16 + 4 * q + r;
-        if (v >= a.vdim) continue;
-        const float gx = bf2f(a.gate[(long)t * a.ldg + (long)h * a.vdim + v]);
-        a.o[(long)t * a.ldo + (long)h * a.vdim + v] = f2bf(acc[r] / (1.f + __expf(-gx)));
+      for (int j = 0; j < 4; ++j) {
+        const int p = min(p0 + j, NP - 1);
+        f[j] = p0 + j < NP ? exp2f(m[2 * p] - M) : 0.f;
+        v[j] = *(const float4*)(part + (th * NP + p) * rank + c);
       }
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (f[j] != 0.f) {  // an empty partition wrote nothing
+          y[0] = fmaf(f[j], v[j].x, y[0]); y[1] = fmaf(f[j], v[j].y, y[1]);
+          y[2] = fmaf(f[j], v[j].z, y[2]); y[3] = fmaf(f[j], v[j].w, y[3]);
+        }
     }
+    *(uint2*)(o + th * rank + c) = make_uint2(pack2bf(y[0] * inv, y[1] * inv), pack2bf(y[2] * inv, y[3] * inv));
   }
 }
 
@@ -425,14 +416,13 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const V* __restrict_
 // ---------------------------------------------------------------------------------------------
 // flash attention of a portion over its request's expanded keys / values
 // ---------------------------------------------------------------------------------------------
-// The structure of attn_fwd_kernel (swapped S^T = K Q^T, P straight into the next MFMA, register-
-// prefetched double-buffered K / V tiles of 64 keys): 128 query rows of one head per workgroup, 4 waves x
-// 32 rows; a K row is [W_uk c (dim) | kr (rot)] from two sources, padded to DQ columns; value width DV.
+// The structure of attn_fwd_kernel (swapped S^T = K Q^T, P straight into the next MFMA; here the double-
+// buffered K / V tiles of 64 keys come by LDS-DMA, one barrier per tile): 128 query rows of one head per workgroup, 4 waves x
+// 32 rows; a K row is [W_uk c (dim) | kr (rot)], padded to DQ columns; value width DV.
 struct PreArgs {
   const bf16_t* q; long ldq;     // [tokens, ldq], head h at h * (dim + rot), rotated
-  const bf16_t* kv; long ldk;    // expanded [kv rows, ldk]: unrotated keys at h * dim, values at v_col + h * vdim
-  int v_col;
-  const bf16_t* kr; long ldr;    // rotated key part per kv row
+  const bf16_t* kv; long ldk;    // expanded [kv rows, ldk]: unrotated keys at h * dim, values at v_col + h * vdim,
+  int v_col, kr_col;             // the shared rotated key part at kr_col
   const float* sink;
   const bf16_t* gate; long ldg;
   bf16_t* o; long ldo;
@@ -441,15 +431,24 @@ struct PreArgs {
   float scale_log2;
 };
 
+// LDS image of a K (V) tile: rows of DQ (DV) elements, 16-B chunk c of row r at slot c ^ swizzle(r) (an
+// involution, so the same function maps slots back to chunks). K: row reads conflict-free; V: transposed reads.
+template <int DQ>
+__device__ __forceinline__ int kq_chunk(int r, int c) {
+  return c ^ ((DQ / 64) % 2 ? ((r >> 1) & 7) : (r & 15 & (DQ / 8 - 1)));
+}
 template <int DQ>
 __device__ __forceinline__ int kq_off(int r, int c) {
-  const int sw = (DQ / 64) % 2 ? ((r >> 1) & 7) : (r & 15 & (DQ / 8 - 1));
-  return r * (DQ * 2) + ((c ^ sw) << 4);
+  return r * (DQ * 2) + (kq_chunk<DQ>(r, c) << 4);
+}
+template <int DV>
+__device__ __forceinline__ int vv_chunk(int r, int c) {
+  constexpr int NCH = DV / 8, RPB = 128 / DV;
+  return c ^ (((r / RPB) & (NCH / 2 - 1)) << 1);
 }
 template <int DV>
 __device__ __forceinline__ int vv_off(int r, int c) {
-  constexpr int NCH = DV / 8, RPB = 128 / DV;
-  return r * (DV * 2) + ((c ^ (((r / RPB) & (NCH / 2 - 1)) << 1)) << 4);
+  return r * (DV * 2) + (vv_chunk<DV>(r, c) << 4);
 }
 
 template <int DQ, int DV>
@@ -459,7 +458,8 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
   constexpr int OROW = DV + 8;
   constexpr int TILES = 2 * (KB + VB), OB = 128 * OROW * 2;
   __shared__ __attribute__((aligned(16))) char smem[TILES > OB ? TILES : OB];
-  const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int g = lane >> 4, r16 = lane & 15;
   const int lin = xcd_remap(blockIdx.x, gridDim.x);
   const int h = lin / a.n_tiles;
@@ -494,47 +494,50 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
 #pragma unroll
   for (int u = 0; u < 2; ++u) { m[u] = -INFINITY; l[u] = 0.f; }
 
-  // chunk e of the tile (K then V) by thread tid + 256 r
-  constexpr int CK = 64 * NQ / 256, CV = 64 * NV / 256;
-  u32x4 kreg[CK], vreg[CV];
-  const bf16_t* kvb = a.kv + (long)sg.kv_off * a.ldk + (long)h * a.dim;
-  const bf16_t* vb = a.kv + (long)sg.kv_off * a.ldk + a.v_col + (long)h * a.vdim;
-  const bf16_t* krb = a.kr + (long)sg.kv_off * a.ldr;
-  auto load_tile = [&](int kv0) {
+  // LDS-DMA of one tile: instruction j of this wave fills 1 KiB of the K (V) image; the lane's source chunk
+  // undoes the image's swizzle. Rows past the request's keys repeat the last one (masked); columns past the
+  // head repeat its first chunk (the query is zero there, the values are not stored).
+  constexpr int JK = KB / 4096, JV = VB / 4096;
+  const bf16_t* kvb = a.kv + (long)sg.kv_off * a.ldk;
+  auto chunk = [&](int j, bool v, int& key) -> int {  // key row and source column of the lane's chunk
+    const int e = (4 * j + wid) * 64 + lane;
+    key = v ? e / NV : e / NQ;
+    const int c = 8 * (v ? vv_chunk<DV>(key, e % NV) : kq_chunk<DQ>(key, e % NQ));
+    if (v) return a.v_col + h * a.vdim + (c < a.vdim ? c : 0);
+    return c < a.dim ? h * a.dim + c : (c < hd ? a.kr_col + c - a.dim : h * a.dim);
+  };
+  uint32_t off[JK + JV];
 #pragma unroll
-    for (int r = 0; r < CK; ++r) {
-      const int e = tid + 256 * r, key = e / NQ, c = (e % NQ) * 8;
-      const long kk = min(kv0 + key, sg.kv_len - 1);
-      const bf16_t* p = c < a.dim ? kvb + kk * a.ldk + c : krb + kk * a.ldr + (c - a.dim);
-      kreg[r] = c < hd ? *(const u32x4*)p : u32x4{0, 0, 0, 0};
-    }
+  for (int j = 0; j < JK + JV; ++j) {
+    int key;
+    const int c = chunk(j < JK ? j : j - JK, j >= JK, key);
+    off[j] = (uint32_t)key * (uint32_t)a.ldk + (uint32_t)c;
+  }
+  auto stage = [&](int kv0, int buf) {
+    char* kd = smem + buf * (KB + VB);
+    const bf16_t* base = kvb + (long)kv0 * a.ldk;
+    auto issue = [&](int j, uint32_t o) {
+      __builtin_amdgcn_global_load_lds((const void*)(base + o), (lds_void*)(kd + (j < JK ? 4 * j : KB / 1024 + 4 * (j - JK)) * 1024 +
+                                                                            wid * 1024), 16, 0, 0);
+    };
+    if (kv0 + 64 <= sg.kv_len) {
 #pragma unroll
-    for (int r = 0; r < CV; ++r) {
-      const int e = tid + 256 * r, key = e / NV, c = (e % NV) * 8;
-      const long kk = min(kv0 + key, sg.kv_len - 1);
-      vreg[r] = c < a.vdim ? *(const u32x4*)(vb + kk * a.ldk + c) : u32x4{0, 0, 0, 0};
+      for (int j = 0; j < JK + JV; ++j) issue(j, off[j]);
+    } else {  // the request's last tile
+#pragma unroll
+      for (int j = 0; j < JK + JV; ++j) {
+        int key;
+        const int c = chunk(j < JK ? j : j - JK, j >= JK, key);
+        issue(j, (uint32_t)min(key, sg.kv_len - 1 - kv0) * (uint32_t)a.ldk + (uint32_t)c);
+      }
     }
   };
-  auto store_tile = [&](char* kd) {
-    char* vd = kd + KB;
-#pragma unroll
-    for (int r = 0; r < CK; ++r) {
-      const int e = tid + 256 * r;
-      *(u32x4*)(kd + kq_off<DQ>(e / NQ, e % NQ)) = kreg[r];
-    }
-#pragma unroll
-    for (int r = 0; r < CV; ++r) {
-      const int e = tid + 256 * r;
-      *(u32x4*)(vd + vv_off<DV>(e / NV, e % NV)) = vreg[r];
-    }
-  };
-  load_tile(0);
-  store_tile(smem);
-  __syncthreads();
+  stage(0, 0);
   int cur = 0;
-  for (int kv0 = 0; kv0 < kend; kv0 += 64) {
-    const bool has_next = kv0 + 64 < kend;
-    if (has_next) load_tile(kv0 + 64);
+  for (int kv0 = 0; kv0 < kend; kv0 += 64, cur ^= 1) {
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this tile (issued one tile ago)
+    asm volatile("s_barrier" ::: "memory");           // ... of every wave; the other buffer is free
+    if (kv0 + 64 < kend) stage(kv0 + 64, cur ^ 1);
     char* Ks = smem + cur * (KB + VB);
     char* Vs = Ks + KB;
     f32x4 stt[4][2];
@@ -601,25 +604,25 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
 #pragma unroll
       for (int u = 0; u < 2; ++u) pa[u] = pack_p(stt[2 * ks][u], stt[2 * ks + 1][u]);
       const int qrow = lane >> 2 & 3, pcol = lane & 3;
+      // the 4 transposed reads of two column tiles: keys + 0 / + 16, columns + 0 / + 16. The swizzle moves a
+      // column tile by 32 B multiples that depend on the row, the same for rows 16 apart
+      const int key_a = 32 * ks + 4 * g + qrow;
 #pragma unroll
-      for (int c = 0; c < DT; ++c) {
-        const int key_a = 32 * ks + 4 * g + qrow;
-        const int col = 16 * c + 4 * pcol;
-        typedef __attribute__((ext_vector_type(4))) short s16x4;
-        typedef __attribute__((address_space(3))) s16x4 lds_s16x4;
-        const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-            (lds_s16x4*)(Vs + vv_off<DV>(key_a, col >> 3) + ((col & 7) << 1)));
-        const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-            (lds_s16x4*)(Vs + vv_off<DV>(key_a + 16, col >> 3) + ((col & 7) << 1)));
-        const bf16x8 vf = cat4(lo, hi);
+      for (int c = 0; c < DT; c += 2) {
+        const uint32_t a0 = lds_addr(Vs + vv_off<DV>(key_a, 2 * c + (pcol >> 1)) + ((pcol & 1) << 3));
+        const uint32_t a1 = lds_addr(Vs + vv_off<DV>(key_a, 2 * c + 2 + (pcol >> 1)) + ((pcol & 1) << 3));
+        rt_s16x4 l0, h0, l1, h1;
+        ds_tr16_2x2<16 * DV * 2>(a0, a1, l0, h0, l1, h1);
+        const bf16x8 v0 = cat4(l0, h0), v1 = cat4(l1, h1);
 #pragma unroll
-        for (int u = 0; u < 2; ++u) o[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], vf, o[u][c], 0, 0, 0);
+        for (int u = 0; u < 2; ++u) {
+          o[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], v0, o[u][c], 0, 0, 0);
+          o[u][c + 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], v1, o[u][c + 1], 0, 0, 0);
+        }
       }
     }
-    if (has_next) store_tile(smem + (cur ^ 1) * (KB + VB));
-    __syncthreads();
-    cur ^= 1;
   }
+  __syncthreads();  // the last tile's images become the O staging area
   // the sink joins the denominator; O through LDS, gated on the way out
   const float sink2 = a.sink[h] * 1.4426950408889634f;
   bf16_t* Os = (bf16_t*)smem;
@@ -723,7 +726,8 @@ extern "C" int rt_latent_prep(int f32, void* proj, long ldp, int kv_col, const v
   if (T <= 0) return 0;
   if (rot % 2 || rdims % 2 || rdims > rot) return -1;
   PrepArgs a{proj, ldp, kv_col, norm_w, eps, cosT, sinT, max_pos, rdims, row, pos, pool, tab, max_pages, n_pages,
-             n_rows, qabs, n_abs, H, dim, rot, rank};
+             n_rows, qabs, n_abs, H, dim, rot, rank, 0};
+  a.vec = rdims == rot && rot % 8 == 0 && dim % 8 == 0 && rank % 8 == 0 && ldp % 8 == 0 && (uintptr_t)proj % 16 == 0;
   if (f32) hipLaunchKernelGGL((latent_prep_kernel<float>), dim3(T), dim3(256), 0, stream, a);
   else hipLaunchKernelGGL((latent_prep_kernel<bf16_t>), dim3(T), dim3(256), 0, stream, a);
   RT_LAUNCH_CHECK();
@@ -732,12 +736,13 @@ extern "C" int rt_latent_prep(int f32, void* proj, long ldp, int kv_col, const v
 
 // bf16, K % 8 == 0, 16-B aligned rows
 extern "C" int rt_head_gemm(const void* A, long lda, long sA, const void* W, long ldw, long sW, void* C, long ldc,
-                            long sC, int T, int N, int K, int batch, hipStream_t stream) {
+                            long sC, int T, int N, int K, int batch, const void* gate, long ldg,
+                            hipStream_t stream) {
   if (T <= 0 || N <= 0 || batch <= 0) return 0;
   if (K % 8 || lda % 8 || sA % 8 || ldw % 8 || sW % 8 || batch > 65535 || (T + 15) / 16 > 65535) return -1;
   dim3 grid((N + 63) / 64, batch, (T + 15) / 16);
   hipLaunchKernelGGL(head_gemm_kernel, grid, dim3(256), 0, stream, (const bf16_t*)A, lda, sA, (const bf16_t*)W, ldw,
-                     sW, (bf16_t*)C, ldc, sC, T, N, K);
+                     sW, (bf16_t*)C, ldc, sC, T, N, K, (const bf16_t*)gate, ldg);
   RT_LAUNCH_CHECK();
   return 0;
 }
@@ -773,15 +778,12 @@ extern "C" int rt_latent_decode(const void* q, const void* pool, const int* tab,
   return 0;
 }
 
-extern "C" int rt_latent_out(const float* part, const float* ml, const float* sink, const void* wuv, const void* gate,
-                             long ldg, void* o, long ldo, int T, int H, int rank, int vdim, int NP, hipStream_t stream) {
+extern "C" int rt_latent_merge(const float* part, const float* ml, const float* sink, void* o, int T, int H, int rank,
+                               int NP, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (rank % 8 || rank > 2048 || (T + 15) / 16 > 65535) return -1;
-  OutArgs a{part, ml, sink, (const bf16_t*)wuv, (const bf16_t*)gate, ldg, (bf16_t*)o, ldo, T, H, rank, vdim, NP};
-  const int tt = (T + 15) / 16, nt = (vdim + 15) / 16;
-  int vs = std::max(1, std::min((nt + 3) / 4, 256 / std::max(1, H * tt)));
-  const size_t lds = (size_t)16 * (((rank + 31) & ~31) + 8) * 2;
-  hipLaunchKernelGGL(latent_out_kernel, dim3(H, tt, vs), dim3(256), lds, stream, a);
+  if (rank % 8 || NP < 1) return -1;
+  hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((long)T * H)), dim3(128), 0, stream, part, ml, sink, (bf16_t*)o,
+                     H, rank, NP);
   RT_LAUNCH_CHECK();
   return 0;
 }
@@ -809,13 +811,13 @@ extern "C" int rt_latent_prefill_ok(int dim, int rot, int vdim) {
   return dim % 8 == 0 && rot % 8 == 0 && vdim % 8 == 0 && dim + rot <= 256 && vdim <= 128;
 }
 
-extern "C" int rt_latent_prefill(const void* q, long ldq, const void* kv, long ldk, int v_col, const void* kr, long ldr,
+extern "C" int rt_latent_prefill(const void* q, long ldq, const void* kv, long ldk, int v_col, int kr_col,
                                  const float* sink, const void* gate, long ldg, void* o, long ldo, const void* segs,
                                  const void* tiles, int n_tiles, int H, int dim, int rot, int vdim, float scale,
                                  hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (!rt_latent_prefill_ok(dim, rot, vdim) || ldq % 8 || ldk % 8 || v_col % 8 || ldr % 8 || ldg % 8 || ldo % 8) return -1;
-  PreArgs a{(const bf16_t*)q, ldq, (const bf16_t*)kv, ldk, v_col, (const bf16_t*)kr, ldr, sink, (const bf16_t*)gate, ldg,
+  if (!rt_latent_prefill_ok(dim, rot, vdim) || ldq % 8 || ldk % 8 || v_col % 8 || kr_col % 8 || ldg % 8 || ldo % 8) return -1;
+  PreArgs a{(const bf16_t*)q, ldq, (const bf16_t*)kv, ldk, v_col, kr_col, sink, (const bf16_t*)gate, ldg,
             (bf16_t*)o, ldo, (const Seg*)segs, (const int2*)tiles, n_tiles, H, dim, rot, vdim,
             scale * 1.4426950408889634f};
   dim3 grid((unsigned)((long)n_tiles * H)), block(256);

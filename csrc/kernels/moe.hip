@@ -49,33 +49,33 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
     c[i] = e < E ? s[i] + correction[e] : -INFINITY;
   }
   const int slots = top + nshared;
+  // order-preserving integer keys: (score, lower expert first); 0 = taken or out of range. Every float,
+  // also a NaN, has a place in this order, so a chosen expert is always a free one
+  unsigned key[MAXV];
+#pragma unroll
+  for (int i = 0; i < MAXV; ++i) {
+    const unsigned u = __float_as_uint(c[i]);
+    key[i] = lane + 64 * i < E ? max(u & 0x80000000u ? ~u : u | 0x80000000u, 1u) : 0u;
+  }
   for (int k = 0; k < top; ++k) {
-    // largest remaining choice score; equal scores: the lower expert. `be` always names an expert that
-    // is still free, also when scores are not comparable (NaN)
-    float bv = -INFINITY, bs = 0.f;
-    int be = 1 << 30;
-#pragma unroll
-    for (int i = 0; i < MAXV; ++i) {
-      const int e = lane + 64 * i;
-      const bool open = e < E && c[i] != -INFINITY;
-      if (open && (be == (1 << 30) || c[i] > bv)) { bv = c[i]; bs = s[i]; be = e; }
-    }
-#pragma unroll
-    for (int o = 32; o > 0; o >>= 1) {
-      const float ov = __shfl_xor(bv, o, 64), os = __shfl_xor(bs, o, 64);
-      const int oe = __shfl_xor(be, o, 64);
-      const bool take = oe != (1 << 30) && (be == (1 << 30) || ov > bv || (!(bv > ov) && oe < be));
-      if (take) { bv = ov; bs = os; be = oe; }
-    }
-    be = __builtin_amdgcn_readfirstlane(be);
-    if (be >= E) be = k;  // no open expert left (only with a choice score of -inf)
+    unsigned bk = 0, bi = 0;
 #pragma unroll
     for (int i = 0; i < MAXV; ++i)
-      if (lane + 64 * i == be) c[i] = -INFINITY;
-    if (lane == 0) {
-      idx[(long)t * slots + k] = be;
-      wt[(long)t * slots + k] = bs;
+      if (64 * i < E && key[i] > bk) { bk = key[i]; bi = i; }
+    unsigned long long best = ((unsigned long long)bk << 32) | (0xffffffffu - (lane + 64 * bi));
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const unsigned long long other = __shfl_xor(best, o, 64);
+      best = other > best ? other : best;
     }
+    const int e = (int)(0xffffffffu - (unsigned)best);
+#pragma unroll
+    for (int i = 0; i < MAXV; ++i)
+      if (lane + 64 * i == e) {  // the owner lane records its choice
+        key[i] = 0;
+        idx[(long)t * slots + k] = e;
+        wt[(long)t * slots + k] = s[i];
+      }
   }
   if (lane < nshared) {
     idx[(long)t * slots + top + lane] = E + lane;
@@ -83,18 +83,32 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
   }
 }
 
-// workgroup g: counts the pairs of lower groups (its offset), then places its own pairs in pair order
-__global__ __launch_bounds__(256) void moe_sort_kernel(const int* __restrict__ idx, int P, int slots, int G,
-                                                       int* __restrict__ offs, int* __restrict__ row_tok,
-                                                       int* __restrict__ pair_pos) {
-  __shared__ int cnt[4][2];
-  __shared__ int wbase[4];
+// workgroup g: counts the pairs of lower groups (its offset), then places its own pairs in pair order.
+// Four consecutive pairs per thread and pass.
+__global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ idx, int P, int slots, int G,
+                                                        int* __restrict__ offs, int* __restrict__ row_tok,
+                                                        int* __restrict__ pair_pos) {
+  __shared__ int cnt[16][2];
+  __shared__ int wsum[2][16];
   const int g = blockIdx.x, tid = threadIdx.x, lane = tid & 63, w = tid >> 6;
+  auto load4 = [&](int i0, int (&e)[4]) {
+    if (i0 + 3 < P) {
+      const int4 v = *(const int4*)(idx + i0);
+      e[0] = v.x; e[1] = v.y; e[2] = v.z; e[3] = v.w;
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) e[j] = i0 + j < P ? idx[i0 + j] : 0x7fffffff;
+    }
+  };
   int less = 0, mine = 0;
-  for (int i = tid; i < P; i += 256) {
-    const int e = idx[i];
-    less += e < g;
-    mine += e == g;
+  for (int i0 = tid * 4; i0 < P; i0 += 4096) {
+    int e[4];
+    load4(i0, e);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      less += e[j] < g;
+      mine += e[j] == g;
+    }
   }
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) {
@@ -103,28 +117,43 @@ __global__ __launch_bounds__(256) void moe_sort_kernel(const int* __restrict__ i
   }
   if (lane == 0) { cnt[w][0] = less; cnt[w][1] = mine; }
   __syncthreads();
-  const int base = cnt[0][0] + cnt[1][0] + cnt[2][0] + cnt[3][0];
-  const int total = cnt[0][1] + cnt[1][1] + cnt[2][1] + cnt[3][1];
+  int base = 0, total = 0;
+#pragma unroll
+  for (int q = 0; q < 16; ++q) { base += cnt[q][0]; total += cnt[q][1]; }
   if (tid == 0) {
     offs[g] = base;
     if (g == G - 1) offs[G] = base + total;
   }
-  int run = base;
-  for (int i0 = 0; i0 < P; i0 += 256) {
-    const int i = i0 + tid;
-    const bool hit = i < P && idx[i] == g;
-    const unsigned long long m = __ballot(hit);
-    if (lane == 0) wbase[w] = __popcll(m);
-    __syncthreads();
-    int before = run;
-    for (int q = 0; q < w; ++q) before += wbase[q];
-    if (hit) {
-      const int pos = before + __popcll(m & ((1ull << lane) - 1));
-      row_tok[pos] = i / slots;
-      pair_pos[i] = pos;
+  if (total == 0) return;
+  int run = base, ph = 0;
+  for (int b0 = 0; b0 < P; b0 += 4096, ph ^= 1) {
+    const int i0 = b0 + tid * 4;
+    int e[4] = {-1, -1, -1, -1}, c = 0;
+    if (i0 < P) load4(i0, e);
+#pragma unroll
+    for (int j = 0; j < 4; ++j) c += e[j] == g;
+    int inc = c;  // inclusive scan over the wave
+#pragma unroll
+    for (int o = 1; o < 64; o <<= 1) {
+      const int v = __shfl_up(inc, o, 64);
+      if (lane >= o) inc += v;
     }
-    run += wbase[0] + wbase[1] + wbase[2] + wbase[3];
+    if (lane == 63) wsum[ph][w] = inc;
     __syncthreads();
+    int pos = run + inc - c, all = 0;
+#pragma unroll
+    for (int q = 0; q < 16; ++q) {
+      const int v = wsum[ph][q];
+      if (q < w) pos += v;
+      all += v;
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      if (e[j] == g) {
+        row_tok[pos] = (i0 + j) / slots;
+        pair_pos[i0 + j] = pos++;
+      }
+    run += all;
   }
 }
 
@@ -157,10 +186,13 @@ struct MoeRowsArgs {
   GluP glu;
 };
 
-// grid (N / 16, groups). Each wave takes K / 4 of the reduction in 32-deep MFMA steps.
+// grid (N / 16, groups). Each wave takes K / 4 of the reduction in 32-deep MFMA steps, U steps of operands
+// in registers and the next U in flight (non-temporal weight loads: with the compiler's own schedule this
+// streamed 2.7 TB/s, with the explicit double buffer 4.6).
 template <bool PAIR, bool OUT_F32, int MT>
 __global__ __launch_bounds__(256) void moe_rows_kernel(MoeRowsArgs p) {
   constexpr int NB = PAIR ? 2 : 1;
+  constexpr int U = MT == 4 ? 2 : 4;
   __shared__ float red[4][MT * NB][64 * 4];
   const int g = blockIdx.y, n0 = blockIdx.x * 16;
   const int beg = p.offs[g], end = p.offs[g + 1];
@@ -172,8 +204,8 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(MoeRowsArgs p) {
 #pragma unroll
   for (int b = 0; b < NB; ++b) wp[b] = W + (long)(b * p.N + min(n0 + r16, p.N - 1)) * p.ldw + 8 * q;
   const int steps = (p.K + 31) / 32;
-  const int per = (steps + 3) / 4;
-  const int s0 = w * per, s1 = min(steps, s0 + per);
+  const int groups = (steps + U - 1) / U, per = (groups + 3) / 4;
+  const int s0 = w * per, s1 = min(groups, s0 + per);
   for (int m0 = beg; m0 < end; m0 += 16 * MT) {
     const bf16_t* ap[MT];
 #pragma unroll
@@ -187,21 +219,34 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(MoeRowsArgs p) {
 #pragma unroll
       for (int b = 0; b < NB; ++b) acc[i][b] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int mt = min(MT, (end - m0 + 15) / 16);
-#pragma unroll 4
-    for (int s = s0; s < s1; ++s) {
-      const int k = s * 32;
-      const bool ok = k + 8 * q < p.K;  // K % 8 == 0: a lane's 8 elements are all in or all out
-      bf16x8 wf[NB];
+    bf16x8 wf[2][NB][U], af[2][MT][U];
+    auto load = [&](int s, int d) {
 #pragma unroll
-      for (int b = 0; b < NB; ++b)
-        wf[b] = ok ? __builtin_bit_cast(bf16x8, load_nt16(wp[b] + k)) : bf16x8{};
+      for (int u = 0; u < U; ++u) {
+        const int k = (s * U + u) * 32;
+        const bool ok = k + 8 * q < p.K;  // K % 8 == 0: a lane's 8 elements are all in or all out
 #pragma unroll
-      for (int i = 0; i < MT; ++i) {
-        if (i < mt) {
-          const bf16x8 af = ok ? *(const bf16x8*)(ap[i] + k) : bf16x8{};
+        for (int b = 0; b < NB; ++b) wf[d][b][u] = ok ? __builtin_bit_cast(bf16x8, load_nt16(wp[b] + k)) : bf16x8{};
 #pragma unroll
-          for (int b = 0; b < NB; ++b) acc[i][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af, wf[b], acc[i][b], 0, 0, 0);
-        }
+        for (int i = 0; i < MT; ++i) af[d][i][u] = ok ? *(const bf16x8*)(ap[i] + k) : bf16x8{};
+      }
+    };
+    auto mul = [&](int d) {
+#pragma unroll
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int i = 0; i < MT; ++i)
+#pragma unroll
+          for (int b = 0; b < NB; ++b)
+            acc[i][b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[d][i][u], wf[d][b][u], acc[i][b], 0, 0, 0);
+    };
+    if (s0 < s1) load(s0, 0);
+    for (int s = s0; s < s1; s += 2) {
+      if (s + 1 < s1) load(s + 1, 1);
+      mul(0);
+      if (s + 1 < s1) {
+        if (s + 2 < s1) load(s + 2, 0);
+        mul(1);
       }
     }
 #pragma unroll
@@ -253,7 +298,7 @@ extern "C" int rt_moe_sort(const int* idx, int P, int slots, int G, int* offs, i
                            int tile_rows, int max_tiles, void* tiles, int* n_tiles, hipStream_t stream) {
   if (P <= 0) return 0;
   if (G < 1 || G > 1024) return -1;
-  hipLaunchKernelGGL(moe_sort_kernel, dim3(G), dim3(256), 0, stream, idx, P, slots, G, offs, row_tok, pair_pos);
+  hipLaunchKernelGGL(moe_sort_kernel, dim3(G), dim3(1024), 0, stream, idx, P, slots, G, offs, row_tok, pair_pos);
   if (tiles) {
     hipLaunchKernelGGL(moe_tiles_kernel, dim3(1), dim3(1024), 0, stream, offs, G, tile_rows, max_tiles, (int4*)tiles,
                        n_tiles);

@@ -360,14 +360,26 @@ __global__ __launch_bounds__(512) void branch_norm_kernel(BranchArgs a) {
         for (int e = 0; e < V; ++e) y[i][e] += t[e];
       }
     } else if constexpr (KIND == Y_PAIRS || KIND == Y_PAIRS_F32) {
-      for (int k = 0; k < a.K; ++k) {
-        const float w = a.pair_w[row * a.K + k];
-        const long pr = a.pair_pos[row * a.K + k];
-        float t[V];
-        if constexpr (KIND == Y_PAIRS_F32) act_ldv<float, V>((const float*)a.y + pr * a.H + c * V, t);
-        else act_ldv<T, V>((const T*)a.y + pr * a.H + c * V, t);
+      for (int k0 = 0; k0 < a.K; k0 += 4) {  // four pairs' rows in flight
+        float w[4], t[4][V];
+        long pr[4];
 #pragma unroll
-        for (int e = 0; e < V; ++e) y[i][e] = fmaf(w, t[e], y[i][e]);
+        for (int j = 0; j < 4; ++j) {
+          const long o = row * a.K + min(k0 + j, a.K - 1);
+          w[j] = k0 + j < a.K ? a.pair_w[o] : 0.f;
+          pr[j] = a.pair_pos[o];
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          if constexpr (KIND == Y_PAIRS_F32) act_ldv<float, V>((const float*)a.y + pr[j] * a.H + c * V, t[j]);
+          else act_ldv<T, V>((const T*)a.y + pr[j] * a.H + c * V, t[j]);
+        }
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (k0 + j < a.K) {
+#pragma unroll
+            for (int e = 0; e < V; ++e) y[i][e] = fmaf(w[j], t[j][e], y[i][e]);
+          }
       }
     }
 #pragma unroll

@@ -34,5 +34,7 @@ def build_model(name_or_path: str, device="cpu", dtype=None, seed: int = 0, fast
     if fast_init:
         m = cls(cfg, device=device, dtype=dtype, init=False)
         fast_random_init_(m, seed, cfg.initializer_range)
+        if cfg.is_layered:
+            m._zero_padding()
         return m
     return cls(cfg, device=device, dtype=dtype, init=True, seed=seed)

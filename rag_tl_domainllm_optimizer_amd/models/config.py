@@ -225,8 +225,13 @@ def _vezatar_preset(name, vocab, width, n, heads, dim, rot, vdim, rank, ff, moe,
 
 
 PRESETS = {
-    # a real model's layer sizes (Mistral-7B's width and head count; 64 experts, 8 used) and a test size
+    # real models' layer sizes (Mistral-7B's width and head count, and half of both; 64 experts), a comparison
+    # decoder of the half width, and a test size
     "vezatar-7b": _vezatar_preset("vezatar-7b", 32000, 4096, 32, 32, 128, 64, 128, 512, 14336, (64, 8, 1408), 2816),
+    "vezatar-2k": _vezatar_preset("vezatar-2k", 32000, 2048, 24, 16, 128, 64, 128, 512, 7168, (64, 6, 896), 1792),
+    "mistral-2k": ModelConfig(arch="mistral", vocab_size=32000, hidden_size=2048, num_layers=24, num_heads=16,
+                              num_kv_heads=4, head_dim=128, intermediate_size=7168, max_position=32768,
+                              norm_eps=1e-5, rope_theta=10000.0, sliding_window=4096, name="mistral-2k"),
     "tiny-vezatar": _vezatar_preset("tiny-vezatar", 512, 192, 4, 6, 32, 16, 48, 64, 256, (10, 3, 64), 128),
     "mistral-7b": ModelConfig(arch="mistral", vocab_size=32000, hidden_size=4096, num_layers=32, num_heads=32,
                               num_kv_heads=8, head_dim=128, intermediate_size=14336, max_position=32768,

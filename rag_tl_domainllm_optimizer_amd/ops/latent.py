@@ -93,7 +93,8 @@ def latent_attention(proj: torch.Tensor, d: LatentDims, kv_up: torch.Tensor, sin
         if fast:
             nat.head_gemm(qn, uk_t.get(uk), dst)
             part, ml = nat.latent_decode(qabs, pool, tab, row, pos, C, _np_parts(n_abs, H, batch.max_len), d.scale)
-            nat.latent_out(part, ml, sink, uv, gate[:n_abs], out[:n_abs])
+            o = nat.latent_merge(part, ml, sink)
+            nat.head_gemm(o.transpose(0, 1), uv, out[:n_abs].view(n_abs, H, V).transpose(0, 1), gate[:n_abs])
         else:
             nat.gemm_any(qn, uk_t.get(uk), False, dst)
             o = nat.latent_any(qabs, pool, tab, row, pos, sink, C, d.scale)
@@ -103,9 +104,11 @@ def latent_attention(proj: torch.Tensor, d: LatentDims, kv_up: torch.Tensor, sin
         rows = dense.get(dense_key)
         if rows is None:
             rows = dense[dense_key] = nat.latent_gather(pool, tab, batch.segs, batch.kv_total, batch.max_kv)
-        kv = project(rows[:, :C], kv_up)
-        nat.latent_prefill(proj[:, :d.q_cols], kv, rows[:, C:], sink, gate, out, batch.segs, batch.tiles, H, D, R, V,
-                           d.scale)
+        n_up = H * (D + V)
+        kv = torch.empty(rows.shape[0], n_up + R, dtype=proj.dtype, device=proj.device)
+        project(rows[:, :C], kv_up, out=kv[:, :n_up])
+        kv[:, n_up:] = rows[:, C:]
+        nat.latent_prefill(proj[:, :d.q_cols], kv, sink, gate, out, batch.segs, batch.tiles, H, D, R, V, d.scale)
     return out
 
 

@@ -127,25 +127,26 @@ class Glu:
         return [self.limit, self.alpha, self.offset]
 
 
-def project(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False, shuf=None) -> torch.Tensor:
+def project(x: torch.Tensor, w: torch.Tensor, out_f32: bool = False, shuf=None, out=None) -> torch.Tensor:
     """x w^T without grad, any shape and dtype: the MFMA kernels where their shape rules hold (bf16;
     ``shuf``: tile-ordered image at M <= 16), ``gemm_any`` otherwise — also for fp32 operands, which
-    stay fp32 throughout."""
+    stay fp32 throughout. ``out``: rows to write (may be strided)."""
     if not on_gpu(x):
-        return ref.gemm(x, w, out_f32=out_f32)
+        y = ref.gemm(x, w, out_f32=out_f32)
+        return y if out is None else out.copy_(y)
     M, K = x.shape
     N = w.shape[0]
     if x.dtype != torch.bfloat16 or K % 8 or N % 8 or x.stride(0) % 8 or x.data_ptr() % 16 or M == 0:
-        return native().gemm_any(x, w, out_f32)
+        return native().gemm_any(x, w, out_f32, out)
     if M <= 64 and K % 64 == 0:
         if shuf is not None and shuffle_decode(M) and N % 16 == 0:
-            return native().gemm(x, shuf.get(w), None, None, None, 0, out_f32, None, None, 0.0, True)
-        return gemm(x, w, out_f32=out_f32)
+            return native().gemm(x, shuf.get(w), None, None, None, 0, out_f32, out, None, 0.0, True)
+        return gemm(x, w, out_f32=out_f32, out=out)
     if M <= 64:
-        return native().gemm_big(x, w, ROW, ROW, None, None, None, 0, 1 if out_f32 else 0)
+        return native().gemm_big(x, w, ROW, ROW, None, None, None, 0, 1 if out_f32 else 0, 1, out)
     if out_f32 and N <= 512:  # narrow fp32 products (router logits): 64x64 tiles fill the chip
-        return native().gemm_small(x, w, ROW, ROW, 1, 1, None, 64)
-    return gemm(x, w, out_f32=out_f32)
+        return native().gemm_small(x, w, ROW, ROW, 1, 1, out, 64)
+    return gemm(x, w, out_f32=out_f32, out=out)
 
 
 def shuffle_decode(m: int) -> bool:

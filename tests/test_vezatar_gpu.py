@@ -180,7 +180,7 @@ def test_expert_products(dtype, T, W, F, E, top, nsh):
 @pytest.mark.parametrize("H,rank,rot", [(3, 64, 16), (16, 128, 32), (17, 128, 128), (20, 200, 40), (32, 512, 64),
                                         (40, 320, 64), (5, 512, 128)])
 @pytest.mark.parametrize("parts", [1, 3, 8])
-def test_latent_decode_and_out(H, rank, rot, parts):
+def test_latent_decode_merge_and_expansion(H, rank, rot, parts):
     """absorbed attention alone: page and partition borders, one key per row that stands out, sink, gate"""
     KD, V = rank + rot, 24
     lens = [1, 2, 31, 32, 33, 63, 64, 65, 128, 300]
@@ -208,7 +208,7 @@ def test_latent_decode_and_out(H, rank, rot, parts):
     d = [t.to(DEV) for t in (q, pool, tab, row, pos, sink, wuv, gate)]
     part, ml = native().latent_decode(d[0], d[1], d[2], d[3], d[4], rank, parts, scale)
     out = torch.empty(T, H * V, dtype=torch.bfloat16, device=DEV)
-    native().latent_out(part, ml, d[5], d[6], d[7], out)
+    native().head_gemm(native().latent_merge(part, ml, d[5]).transpose(0, 1), d[6], out.view(T, H, V).transpose(0, 1), d[7])
     assert rel(out, want) < 1e-2
     any_o = native().latent_any(d[0], d[1], d[2], d[3], d[4], d[5], rank, scale)
     assert rel(any_o, o) < 4e-3
@@ -243,7 +243,7 @@ def test_latent_prefill(H, dim, rot, vdim):
             want[sg[1]:sg[1] + n, h * vdim:(h + 1) * vdim] = p @ v
     want *= torch.sigmoid(gate.float())
     out = torch.empty(N, H * vdim, dtype=torch.bfloat16, device=DEV)
-    native().latent_prefill(q.to(DEV), kv.to(DEV), kr.to(DEV), sink.to(DEV), gate.to(DEV), out,
+    native().latent_prefill(q.to(DEV), torch.cat([kv, kr], 1).to(DEV), sink.to(DEV), gate.to(DEV), out,
                             torch.tensor(segs).int().to(DEV), torch.tensor(tiles).int().to(DEV), H, dim, rot, vdim, scale)
     assert rel(out, want) < 1e-2
 
