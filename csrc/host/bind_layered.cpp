@@ -20,7 +20,7 @@ int rt_gate_mul(int, void*, const void*, long, long, int, hipStream_t);
 int rt_moe_route(const float*, long, const float*, int, int, int, int, int, int*, float*, hipStream_t);
 int rt_moe_sort(const int*, int, int, int, int*, int*, int*, int, int, void*, int*, hipStream_t);
 int rt_moe_rows(const void*, long, const int*, const void*, long, long, void*, long, const int*, int, int, int, int, int,
-                int, const float*, hipStream_t);
+                int, int, const float*, hipStream_t);
 int rt_gemm_grouped(const void*, long, const int*, const void*, long, long, void*, long, const void*, const int*, int,
                     int, int, int, const float*, const void*, int, hipStream_t);
 int rt_latent_prep(int, void*, long, int, const void*, float, const float*, const float*, int, int, const int*,
@@ -29,7 +29,7 @@ int rt_head_gemm(const void*, long, long, const void*, long, long, void*, long, 
                  long, hipStream_t);
 int rt_latent_decode_ok(int, int);
 int rt_latent_decode(const void*, const void*, const int*, int, int, int, const int*, const int*, float*, float*, int,
-                     int, int, int, int, float, const void*, hipStream_t);
+                     int, int, int, int, float, hipStream_t);
 int rt_latent_merge(const float*, const float*, const float*, void*, int, int, int, int, hipStream_t);
 int rt_latent_gather(int, const void*, const int*, int, int, const void*, int, int, void*, int, hipStream_t);
 int rt_latent_prefill_ok(int, int, int);
@@ -246,7 +246,7 @@ std::vector<Tensor> moe_sort(const Tensor& idx, int64_t G, int64_t tile_rows) {
 
 // rows of a sorted by group times w [G, N or 2N, K] (glu given: [gate; up] with the gated unit)
 Tensor moe_rows(const Tensor& a, const optional<Tensor>& row_map, const Tensor& w, const Tensor& offs, int64_t n_rows,
-                bool out_f32, int64_t mean_rows, const std::vector<double>& glu) {
+                bool out_f32, int64_t mean_rows, bool ring, const std::vector<double>& glu) {
   TORCH_CHECK(a.is_cuda() && a.scalar_type() == at::kBFloat16 && w.scalar_type() == at::kBFloat16 && w.is_cuda(), "moe_rows: bf16");
   rows(a, "moe_rows");
   ints(offs, "moe_rows offs");
@@ -264,7 +264,7 @@ Tensor moe_rows(const Tensor& a, const optional<Tensor>& row_map, const Tensor& 
   float g[3];
   if (pair) for (int i = 0; i < 3; ++i) g[i] = Glu(glu).v[i];
   rc_ok(rt_moe_rows(a.data_ptr(), a.stride(0), (const int*)ptr(row_map), w.data_ptr(), w.stride(0), w.stride(1), c.data_ptr(),
-                    N, offs.data_ptr<int>(), (int)G, (int)N, (int)K, pair, out_f32, (int)mean_rows, pair ? g : nullptr, stream()),
+                    N, offs.data_ptr<int>(), (int)G, (int)N, (int)K, pair, out_f32, (int)mean_rows, ring, pair ? g : nullptr, stream()),
         "moe_rows");
   return c;
 }
@@ -357,7 +357,7 @@ std::vector<Tensor> latent_decode(const Tensor& q, const Tensor& pool, const Ten
   Tensor ml = at::empty({T, H, NP, 2}, q.options().dtype(at::kFloat));
   rc_ok(rt_latent_decode(q.data_ptr(), pool.data_ptr(), tab.data_ptr<int>(), pl.max_pages(), pl.pages(), pl.rows(),
                          row.data_ptr<int>(), pos.data_ptr<int>(), part.data_ptr<float>(), ml.data_ptr<float>(), (int)T,
-                         (int)H, (int)rank, pl.kd(), (int)NP, (float)scale, zero_page(q).data_ptr(), stream()),
+                         (int)H, (int)rank, pl.kd(), (int)NP, (float)scale, stream()),
         "latent_decode");
   return {part, ml};
 }

@@ -32,6 +32,9 @@ template <typename T> __device__ __forceinline__ void st(T* p, float v);
 template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
 
+// v_exp_f32: arguments here are <= 0 (or -inf -> 0), where the library function's range handling does nothing
+__device__ __forceinline__ float fexp2(float x) { return __builtin_amdgcn_exp2f(x); }
+
 __device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
   uint4 v;
   v.x = pack2bf(a[0], a[1]);
@@ -138,13 +141,24 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict
   if (n0 >= N) return;
   const bf16_t* ap = A + (long)min(t0 + r16, T - 1) * lda + b * sA + 8 * q;
   const bf16_t* wp = W + b * sW + (long)min(n0 + r16, N - 1) * ldw + 8 * q;
+  // weight as the A operand: acc[r] = C[t0 + r16][n0 + 4 q + r]
   f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  int k = 0;
+  for (; k + 256 <= K; k += 256) {  // eight steps' operands in flight
+    bf16x8 wf[8], af[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      wf[u] = *(const bf16x8*)(wp + k + 32 * u);
+      af[u] = *(const bf16x8*)(ap + k + 32 * u);
+    }
+#pragma unroll
+    for (int u = 0; u < 8; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], af[u], acc, 0, 0, 0);
+  }
 #pragma unroll 4
-  for (int k = 0; k < K; k += 32) {
+  for (; k < K; k += 32) {
     const bool ok = k + 8 * q < K;
     const bf16x8 wf = ok ? *(const bf16x8*)(wp + k) : bf16x8{};
     const bf16x8 af = ok ? *(const bf16x8*)(ap + k) : bf16x8{};
-    // weight as the A operand: acc[r] = C[t0 + r16][n0 + 4 q + r]
     acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc, 0, 0, 0);
   }
   const int t = t0 + r16;
@@ -167,12 +181,12 @@ __global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict
 // buffers, LDS-DMA one tile ahead):
 //   scores S^T = K Q^T (key on the MFMA row, head on the lane) by waves (key half, K-dim half) for
 //   NH = 1 and (key half, head tile) for NH = 2; exchanged through LDS in accumulator layout;
-//   every wave runs the same online softmax, packs P as the next MFMA's A operand, and accumulates
-//   O += P V for its own quarter of the latent columns (V = the latent part of the same LDS image,
-//   transposed reads). Two barriers per tile.
+//   every wave runs the same online softmax, packs P as the next MFMA's B operand, and accumulates
+//   O^T += V^T P^T (head on the lane again) for its own quarter of the latent columns (V = the latent part of the same LDS image,
+//   transposed reads). Two tiles' images are in flight or in use; three barriers per tile.
 // A row's keys are cut in NP equal partitions (multiples of 32) from its own length, so a captured
 // launch with a fixed NP balances every length. Image rows are CPR = 8 QS + 1 16-B chunks (odd: row
-// reads conflict-free); chunks past KD come from the zero page.
+// reads conflict-free); chunks past KD repeat the row's last one.
 struct DecArgs {
   const bf16_t* q;            // [T, H, KD]
   const bf16_t* pool; const int* tab; int max_pages, n_pages, n_rows;
@@ -180,7 +194,6 @@ struct DecArgs {
   float* part; float* ml;     // [T, H, NP, rank], [T, H, NP, 2] (max in log2 units, sum)
   int T, H, rank, KD, NP, HG;
   float scale_log2;
-  const bf16_t* zpage;
 };
 
 template <int QS, int RT, int NH>
@@ -197,11 +210,19 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
   const int g = lane >> 4, r16 = lane & 15;
   const int bid = xcd_remap(blockIdx.x, gridDim.x);
   const int hg = bid % a.HG, part = (bid / a.HG) % a.NP, t = bid / (a.HG * a.NP);
+  const int h0 = hg * 16 * NH;
+  // query fragments: lane holds Q[head r16][32 s + 8 g ..]
+  const int kt = w & 1, hi = w >> 1;                 // key half; K-dim half (NH = 1) or head tile (NH = 2)
+  const int qh = h0 + (NH == 2 ? hi * 16 : 0) + r16;
+  const int sbase = NH == 1 ? hi * QS : 0;
+  bf16x8 qf[QF];
+  const bf16_t* qp = a.q + ((long)t * a.H + min(qh, a.H - 1)) * a.KD;  // heads past the last repeat it (not stored)
+#pragma unroll
+  for (int s = 0; s < QF; ++s) qf[s] = *(const bf16x8*)(qp + min(32 * (sbase + s) + 8 * g, a.KD - 8));
   const int row = min(max(a.row[t], 0), a.n_rows - 1);
   const int len = min(a.pos[t] + 1, a.max_pages * PAGE);
   const int per = ((len + a.NP - 1) / a.NP + 31) & ~31;
   const int k0 = part * per, k1 = min(len, k0 + per);
-  const int h0 = hg * 16 * NH;
   if (k0 >= k1) {  // nothing for this partition (uniform over the workgroup)
     if (tid < 16 * NH && h0 + tid < a.H) {
       float* m = a.ml + (((long)t * a.H + h0 + tid) * a.NP + part) * 2;
@@ -212,36 +233,21 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
   }
   const int* tab = a.tab + (long)row * a.max_pages;
 
-  // query fragments: lane holds Q[head r16][32 s + 8 g ..]
-  const int kt = w & 1, hi = w >> 1;                 // key half; K-dim half (NH = 1) or head tile (NH = 2)
-  const int qh = h0 + (NH == 2 ? hi * 16 : 0) + r16;
-  const int sbase = NH == 1 ? hi * QS : 0;
-  bf16x8 qf[QF];
-#pragma unroll
-  for (int s = 0; s < QF; ++s) {
-    const int k = 32 * (sbase + s) + 8 * g;
-    qf[s] = (qh < a.H && k < a.KD) ? *(const bf16x8*)(a.q + ((long)t * a.H + qh) * a.KD + k) : bf16x8{};
-  }
-#pragma unroll
-  for (int s = 0; s < QF; ++s) asm volatile("" : "+v"(qf[s]));
-
   // LDS-DMA sources: instruction j of wave w covers image chunks (4 j + w) * 64 + lane
-  int src[NI];  // element offset inside the tile's first cache row, < 0: zero page
+  uint32_t src[NI];  // element offset from the tile's first cache row
 #pragma unroll
   for (int j = 0; j < NI; ++j) {
     const int c = (4 * j + w) * 64 + lane;
-    const int r = c / CPR, cc = c % CPR;
-    src[j] = (r < 32 && cc * 8 < a.KD) ? r * a.KD + cc * 8 : -1;
+    src[j] = (uint32_t)(min(c / CPR, 31) * a.KD + min(c % CPR * 8, a.KD - 8));
   }
-  auto stage = [&](int key0, int buf) {
-    int page = tab[key0 / PAGE];
-    page = min(max(page, 0), a.n_pages - 1);
+  auto page_of = [&](int key0) { return min(max(tab[key0 / PAGE], 0), a.n_pages - 1); };
+  auto stage = [&](int key0, int page, int buf) {
     const bf16_t* base = a.pool + ((long)page * PAGE + key0 % PAGE) * a.KD;
 #pragma unroll
     for (int j = 0; j < NI; ++j) {
-      if (4 * j + w >= NIT) break;  // wave-uniform
-      const bf16_t* p = src[j] >= 0 ? base + src[j] : a.zpage;
-      __builtin_amdgcn_global_load_lds((const void*)p, (lds_void*)(smem + buf * BUFB + (4 * j + w) * 1024), 16, 0, 0);
+      if (4 * j + w < NIT)  // wave-uniform
+        __builtin_amdgcn_global_load_lds((const void*)(base + src[j]), (lds_void*)(smem + buf * BUFB + (4 * j + w) * 1024),
+                                         16, 0, 0);
     }
   };
 
@@ -254,24 +260,37 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
 #pragma unroll
   for (int n = 0; n < NH; ++n) { m[n] = -INFINITY; l[n] = 0.f; }
 
-  stage(k0, 0);
+  const bool more = w < NIT % 4;  // this wave issues NIT / 4 + 1 instructions per tile, else NIT / 4
+  stage(k0, page_of(k0), 0);
+  if (k0 + 32 < k1) stage(k0 + 32, page_of(k0 + 32), 1);
+  if (a.KD < 64 * QS) {  // columns past KD: zero in the query, anything finite in the image
+#pragma unroll
+    for (int s = 0; s < QF; ++s)
+      if (32 * (sbase + s) + 8 * g >= a.KD) qf[s] = bf16x8{};
+  }
+#pragma unroll
+  for (int s = 0; s < QF; ++s) asm volatile("" : "+v"(qf[s]));
   int buf = 0;
   for (int key0 = k0; key0 < k1; key0 += 32, buf ^= 1) {
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // this tile's image (issued one tile ago)
-    asm volatile("s_barrier" ::: "memory");           // ... of every wave; the other buffer is free
-    if (key0 + 32 < k1) stage(key0 + 32, buf ^ 1);
+    const bool n1 = key0 + 32 < k1, n2 = key0 + 64 < k1;
+    const int page2 = n2 ? page_of(key0 + 64) : 0;
+    // this tile's image; the next tile's instructions stay in flight
+    if (!n1) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    else if (more) asm volatile("s_waitcnt vmcnt(%0)" :: "n"(NIT / 4 + 1) : "memory");
+    else asm volatile("s_waitcnt vmcnt(%0)" :: "n"(NIT / 4) : "memory");
+    asm volatile("s_barrier" ::: "memory");           // ... of every wave
     const char* img = smem + buf * BUFB;
     // ---- scores ----
-    f32x4 sp = {0.f, 0.f, 0.f, 0.f};
+    f32x4 sp[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};  // two independent MFMA chains
     {
       const char* kp = img + (16 * kt + r16) * ROWB + (4 * sbase + g) * 16;
 #pragma unroll
       for (int s = 0; s < QF; ++s) {
         const bf16x8 kf = *(const bf16x8*)(kp + s * 64);
-        sp = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], sp, 0, 0, 0);
+        sp[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[s], sp[s & 1], 0, 0, 0);
       }
     }
-    *(f32x4*)(sx + (w * 64 + lane) * 4) = sp;
+    *(f32x4*)(sx + (w * 64 + lane) * 4) = sp[0] + sp[1];
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     asm volatile("s_barrier" ::: "memory");
     // ---- softmax (identical in every wave) ----
@@ -286,27 +305,27 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
         else
           s2[k] = *(const f32x4*)(sx + ((k + 2 * n) * 64 + lane) * 4);
       }
-      float mx = -INFINITY;
+      if (key0 + 32 > k1) {  // the row's last tile
 #pragma unroll
-      for (int k = 0; k < 2; ++k)
+        for (int k = 0; k < 2; ++k)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int key = key0 + 16 * k + 4 * g + i;
-          s2[k][i] = key < k1 ? s2[k][i] * a.scale_log2 : -INFINITY;
-          mx = fmaxf(mx, s2[k][i]);
-        }
+          for (int i = 0; i < 4; ++i)
+            if (key0 + 16 * k + 4 * g + i >= k1) s2[k][i] = -INFINITY;
+      }
+      float mx = fmaxf(fmaxf(fmaxf(s2[0][0], s2[0][1]), fmaxf(s2[0][2], s2[0][3])),
+                       fmaxf(fmaxf(s2[1][0], s2[1][1]), fmaxf(s2[1][2], s2[1][3])));
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m[n], mx);
-      const float mu = mn == -INFINITY ? 0.f : mn;
-      const float alpha = exp2f(m[n] - mu);
+      // every tile holds a key of the row, so mn is finite; scale > 0 (launcher)
+      const float mn = fmaxf(m[n], mx * a.scale_log2);
+      const float alpha = fexp2(m[n] - mn);
       m[n] = mn;
       float rs = 0.f;
 #pragma unroll
       for (int k = 0; k < 2; ++k)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float p = exp2f(s2[k][i] - mu);
+          const float p = fexp2(fmaf(s2[k][i], a.scale_log2, -mn));
           s2[k][i] = p;
           rs += p;
         }
@@ -314,11 +333,10 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
       rs += __shfl_xor(rs, 32, 64);
       l[n] = l[n] * alpha + rs;
       pa[n] = pack_p(s2[0], s2[1]);
+      // O^T: the head is the lane's column, as in the scores (most tiles bring no new maximum)
+      if (__any(alpha != 1.f)) {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float al = __shfl(alpha, 4 * g + i, 64);
-#pragma unroll
-        for (int c = 0; c < RT; ++c) o[n][c][i] *= al;
+        for (int c = 0; c < RT; ++c) o[n][c] *= alpha;
       }
     }
     // ---- O += P V: latent columns [16 RT w, 16 RT (w + 1)) ----
@@ -331,64 +349,67 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
     for (int c = 0; c < RT; ++c) {
       const bf16x8 vf = cat4(v[2 * c], v[2 * c + 1]);
 #pragma unroll
-      for (int n = 0; n < NH; ++n) o[n][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[n], vf, o[n][c], 0, 0, 0);
+      for (int n = 0; n < NH; ++n) o[n][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pa[n], o[n][c], 0, 0, 0);
+    }
+    if (n2) {  // every wave is done with this image: the tile after the next one takes its place
+      asm volatile("s_barrier" ::: "memory");
+      stage(key0 + 64, page2, buf);
     }
   }
-  // o[n][c][i]: head h0 + 16 n + 4 g + i, latent column 16 (RT w + c) + r16
+  // o[n][c][i]: head h0 + 16 n + r16, latent column 16 (RT w + c) + 4 g + i
 #pragma unroll
   for (int n = 0; n < NH; ++n) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int h = h0 + 16 * n + 4 * g + i;
-      if (h >= a.H) continue;
-      float* po = a.part + (((long)t * a.H + h) * a.NP + part) * a.rank;
-#pragma unroll
-      for (int c = 0; c < RT; ++c) {
-        const int col = 16 * (RT * w + c) + r16;
-        if (col < a.rank) po[col] = o[n][c][i];
-      }
-    }
     const int h = h0 + 16 * n + r16;
-    if (w == 0 && g == 0 && h < a.H) {
-      float* pm = a.ml + (((long)t * a.H + h) * a.NP + part) * 2;
-      pm[0] = m[n];
-      pm[1] = l[n];
-    }
+    if (h >= a.H) continue;
+    const long th = ((long)t * a.H + h) * a.NP + part;
+    float* po = a.part + th * a.rank + 16 * RT * w + 4 * g;
+#pragma unroll
+    for (int c = 0; c < RT; ++c)
+      if (16 * (RT * w + c) + 4 * g < a.rank) *(f32x4*)(po + 16 * c) = o[n][c];  // rank % 8 == 0
+    if (w == 0 && g == 0) *(float2*)(a.ml + th * 2) = make_float2(m[n], l[n]);
   }
 }
 
 // ---------------------------------------------------------------------------------------------
 // merge of the partitions, with the sink in the denominator: one workgroup per (token, head)
 // ---------------------------------------------------------------------------------------------
+constexpr int MERGE_MAX = 1024;  // partitions
+
 __global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ part, const float* __restrict__ ml,
                                                            const float* __restrict__ sink, bf16_t* __restrict__ o, int H,
                                                            int rank, int NP) {
+  __shared__ float fac[MERGE_MAX];
+  __shared__ float sbuf[2];
   const long th = blockIdx.x;
   const int tid = threadIdx.x;
   const float sink2 = sink[th % H] * 1.4426950408889634f;
   const float* m = ml + th * NP * 2;
-  float M = sink2;
-  for (int p = 0; p < NP; ++p) M = fmaxf(M, m[2 * p]);
-  float L = exp2f(sink2 - M);
-  for (int p = 0; p < NP; ++p) L += m[2 * p + 1] * exp2f(m[2 * p] - M);  // an empty partition: 0 * exp2(-inf)
-  const float inv = 1.f / L;
+  float mx = -INFINITY;
+  for (int p = tid; p < NP; p += 128) {
+    fac[p] = m[2 * p];
+    mx = fmaxf(mx, fac[p]);
+  }
+  const float M = fmaxf(block_max(mx, sbuf), sink2);
+  float L = 0.f;
+  for (int p = tid; p < NP; p += 128) {
+    fac[p] = exp2f(fac[p] - M);  // 0 for an empty partition
+    L += m[2 * p + 1] * fac[p];
+  }
+  const float inv = 1.f / (block_sum(L, sbuf) + exp2f(sink2 - M));
   for (int c = 4 * tid; c < rank; c += 512) {  // rank % 8 == 0
     float y[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int p0 = 0; p0 < NP; p0 += 4) {
-      float4 v[4];
-      float f[4];
+    for (int p0 = 0; p0 < NP; p0 += 8) {  // eight partitions' rows in flight
+      float4 v[8];
 #pragma unroll
-      for (int j = 0; j < 4; ++j) {
-        const int p = min(p0 + j, NP - 1);
-        f[j] = p0 + j < NP ? exp2f(m[2 * p] - M) : 0.f;
-        v[j] = *(const float4*)(part + (th * NP + p) * rank + c);
-      }
+      for (int j = 0; j < 8; ++j) v[j] = *(const float4*)(part + (th * NP + min(p0 + j, NP - 1)) * rank + c);
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (f[j] != 0.f) {  // an empty partition wrote nothing
-          y[0] = fmaf(f[j], v[j].x, y[0]); y[1] = fmaf(f[j], v[j].y, y[1]);
-          y[2] = fmaf(f[j], v[j].z, y[2]); y[3] = fmaf(f[j], v[j].w, y[3]);
+      for (int j = 0; j < 8; ++j) {
+        const float f = p0 + j < NP ? fac[p0 + j] : 0.f;
+        if (f != 0.f) {  // an empty partition wrote nothing
+          y[0] = fmaf(f, v[j].x, y[0]); y[1] = fmaf(f, v[j].y, y[1]);
+          y[2] = fmaf(f, v[j].z, y[2]); y[3] = fmaf(f, v[j].w, y[3]);
         }
+      }
     }
     *(uint2*)(o + th * rank + c) = make_uint2(pack2bf(y[0] * inv, y[1] * inv), pack2bf(y[2] * inv, y[3] * inv));
   }
@@ -416,7 +437,7 @@ __global__ __launch_bounds__(256) void latent_gather_kernel(const V* __restrict_
 // ---------------------------------------------------------------------------------------------
 // flash attention of a portion over its request's expanded keys / values
 // ---------------------------------------------------------------------------------------------
-// The structure of attn_fwd_kernel (swapped S^T = K Q^T, P straight into the next MFMA; here the double-
+// The structure of attn_fwd_kernel (swapped S^T = K Q^T, P straight into the next MFMA, here O^T = V^T P^T; the double-
 // buffered K / V tiles of 64 keys come by LDS-DMA, one barrier per tile): 128 query rows of one head per workgroup, 4 waves x
 // 32 rows; a K row is [W_uk c (dim) | kr (rot)], padded to DQ columns; value width DV.
 struct PreArgs {
@@ -554,35 +575,35 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
         for (int u = 0; u < 2; ++u)
           stt[t][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[u][s], stt[t][u], 0, 0, 0);
       }
-    const bool full = kv0 + 63 <= sg.pos0 + q0 && kv0 + 63 < kend;
+    if (!(kv0 + 63 <= sg.pos0 + q0 && kv0 + 63 < kend)) {  // the diagonal or the last tile
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+          for (int i = 0; i < 4; ++i) {
+            const int kk = kv0 + 16 * t + 4 * g + i;
+            if (!(kk < kend && kk <= sg.pos0 + q0 + 16 * u + r16)) stt[t][u][i] = -INFINITY;
+          }
+    }
     float alpha[2];
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       float mx = -INFINITY;
 #pragma unroll
       for (int t = 0; t < 4; ++t)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          float x = stt[t][u][i] * a.scale_log2;
-          if (!full) {
-            const int kk = kv0 + 16 * t + 4 * g + i;
-            x = kk < kend && kk <= sg.pos0 + q0 + 16 * u + r16 ? x : -INFINITY;
-          }
-          stt[t][u][i] = x;
-          mx = fmaxf(mx, x);
-        }
+        mx = fmaxf(mx, fmaxf(fmaxf(stt[t][u][0], stt[t][u][1]), fmaxf(stt[t][u][2], stt[t][u][3])));
       mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
       mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float mn = fmaxf(m[u], mx);
-      const float mu = mn == -INFINITY ? 0.f : mn;
-      alpha[u] = exp2f(m[u] - mu);
+      const float mn = fmaxf(m[u], mx * a.scale_log2);  // scale > 0 (launcher); key 0 keeps it finite
+      alpha[u] = fexp2(m[u] - mn);
       m[u] = mn;
       float rs = 0.f;
 #pragma unroll
       for (int t = 0; t < 4; ++t)
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-          const float p = exp2f(stt[t][u][i] - mu);
+          const float p = fexp2(fmaf(stt[t][u][i], a.scale_log2, -mn));
           stt[t][u][i] = p;
           rs += p;
         }
@@ -590,14 +611,13 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
       rs += __shfl_xor(rs, 32, 64);
       l[u] = l[u] * alpha[u] + rs;
     }
+    // O^T: the query is the lane's column, as in the scores (most tiles bring no new maximum)
+    if (__any(alpha[0] != 1.f || alpha[1] != 1.f)) {
 #pragma unroll
-    for (int u = 0; u < 2; ++u)
+      for (int u = 0; u < 2; ++u)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const float al = __shfl(alpha[u], 4 * g + i, 64);
-#pragma unroll
-        for (int c = 0; c < DT; ++c) o[u][c][i] *= al;
-      }
+        for (int c = 0; c < DT; ++c) o[u][c] *= alpha[u];
+    }
 #pragma unroll
     for (int ks = 0; ks < 2; ++ks) {
       bf16x8 pa[2];
@@ -616,8 +636,8 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
         const bf16x8 v0 = cat4(l0, h0), v1 = cat4(l1, h1);
 #pragma unroll
         for (int u = 0; u < 2; ++u) {
-          o[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], v0, o[u][c], 0, 0, 0);
-          o[u][c + 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pa[u], v1, o[u][c + 1], 0, 0, 0);
+          o[u][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v0, pa[u], o[u][c], 0, 0, 0);
+          o[u][c + 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v1, pa[u], o[u][c + 1], 0, 0, 0);
         }
       }
     }
@@ -631,13 +651,11 @@ __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
     const float M = fmaxf(m[u], sink2);
     const float f = exp2f(m[u] - M);
     const float sc = f / (l[u] * f + exp2f(sink2 - M));
+    const int r = wid * 32 + 16 * u + r16;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const float si = __shfl(sc, 4 * g + i, 64);
-      const int r = wid * 32 + 16 * u + 4 * g + i;
-#pragma unroll
-      for (int c = 0; c < DT; ++c) Os[r * OROW + 16 * c + r16] = f2bf(o[u][c][i] * si);
-    }
+    for (int c = 0; c < DT; ++c)
+      *(uint2*)(Os + r * OROW + 16 * c + 4 * g) =
+          make_uint2(pack2bf(o[u][c][0] * sc, o[u][c][1] * sc), pack2bf(o[u][c][2] * sc, o[u][c][3] * sc));
   }
   __syncthreads();
   for (int e = tid; e < 128 * NV; e += 256) {
@@ -753,13 +771,13 @@ extern "C" int rt_latent_decode_ok(int rank, int KD) {
 
 extern "C" int rt_latent_decode(const void* q, const void* pool, const int* tab, int max_pages, int n_pages, int n_rows,
                                 const int* row, const int* pos, float* part, float* ml, int T, int H, int rank, int KD,
-                                int NP, float scale, const void* zpage, hipStream_t stream) {
+                                int NP, float scale, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (!rt_latent_decode_ok(rank, KD) || NP < 1 || !zpage) return -1;
+  if (!rt_latent_decode_ok(rank, KD) || NP < 1 || !(scale > 0)) return -1;
   const int NH = H > 16 ? 2 : 1;
   const int HG = (H + 16 * NH - 1) / (16 * NH);
   DecArgs a{(const bf16_t*)q, (const bf16_t*)pool, tab, max_pages, n_pages, n_rows, row, pos, part, ml, T, H, rank, KD,
-            NP, HG, scale * 1.4426950408889634f, (const bf16_t*)zpage};
+            NP, HG, scale * 1.4426950408889634f};
   dim3 grid((unsigned)((long)T * HG * NP)), block(256);
 #define LD_(QS, RT)                                                                                       \
   do {                                                                                                    \
@@ -781,7 +799,7 @@ extern "C" int rt_latent_decode(const void* q, const void* pool, const int* tab,
 extern "C" int rt_latent_merge(const float* part, const float* ml, const float* sink, void* o, int T, int H, int rank,
                                int NP, hipStream_t stream) {
   if (T <= 0) return 0;
-  if (rank % 8 || NP < 1) return -1;
+  if (rank % 8 || NP < 1 || NP > MERGE_MAX) return -1;
   hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((long)T * H)), dim3(128), 0, stream, part, ml, sink, (bf16_t*)o,
                      H, rank, NP);
   RT_LAUNCH_CHECK();
@@ -816,7 +834,7 @@ extern "C" int rt_latent_prefill(const void* q, long ldq, const void* kv, long l
                                  const void* tiles, int n_tiles, int H, int dim, int rot, int vdim, float scale,
                                  hipStream_t stream) {
   if (n_tiles <= 0) return 0;
-  if (!rt_latent_prefill_ok(dim, rot, vdim) || ldq % 8 || ldk % 8 || v_col % 8 || kr_col % 8 || ldg % 8 || ldo % 8) return -1;
+  if (!(scale > 0) || !rt_latent_prefill_ok(dim, rot, vdim) || ldq % 8 || ldk % 8 || v_col % 8 || kr_col % 8 || ldg % 8 || ldo % 8) return -1;
   PreArgs a{(const bf16_t*)q, ldq, (const bf16_t*)kv, ldk, v_col, kr_col, sink, (const bf16_t*)gate, ldg,
             (bf16_t*)o, ldo, (const Seg*)segs, (const int2*)tiles, n_tiles, H, dim, rot, vdim,
             scale * 1.4426950408889634f};

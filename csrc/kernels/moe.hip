@@ -279,6 +279,109 @@ __global__ __launch_bounds__(256) void moe_rows_kernel(MoeRowsArgs p) {
   }
 }
 
+// Grouped product at up to 64 rows per group and pass, weights and rows through an LDS-DMA ring (the
+// structure of gemm_m64_kernel): workgroup = 64 weight rows (PAIR: 32 gate + 32 up) of one group, 64-deep
+// K-steps of X[64] and W[64] rows in a 4-slot ring, three steps in flight. Wave w owns rows [16 w, 16 w + 16)
+// and skips their X loads and products when the group has none there. K % 64 == 0, N % 64 == 0 (PAIR: 32).
+constexpr int RING_SLOTS = 4, RING_SLOT = 2 * 64 * 128;
+__device__ __forceinline__ int ring_swz(int row) { return (row >> 1) & 7; }
+
+template <bool PAIR, bool OUT_F32>
+__global__ __launch_bounds__(256, 2) void moe_ring_kernel(MoeRowsArgs p) {
+  typedef __attribute__((address_space(3))) void lds_void;
+  __shared__ __attribute__((aligned(16))) char smem[RING_SLOTS * RING_SLOT];  // the only __shared__ object
+  const int g = blockIdx.y, cg = blockIdx.x;
+  const int beg = p.offs[g], end = p.offs[g + 1];
+  if (beg >= end) return;
+  const int tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int frow = lane & 15, fq = lane >> 4;
+  const int nk = p.K / 64;
+  const bf16_t* W = p.W + (long)g * p.sW;
+  const bf16_t* wp[2];
+  int lr[2], ck[2];
+#pragma unroll
+  for (int j = 0; j < 2; ++j) {
+    lr[j] = (wid * 2 + j) * 8 + (lane >> 3);
+    ck[j] = ((lane & 7) ^ ring_swz(lr[j])) * 8;
+    const int wr = PAIR ? (lr[j] < 32 ? cg * 32 + lr[j] : p.N + cg * 32 + lr[j] - 32) : cg * 64 + lr[j];
+    wp[j] = W + (long)wr * p.ldw + ck[j];
+  }
+  for (int m0 = beg; m0 < end; m0 += 64) {
+    const bool mine = m0 + 16 * wid < end;  // wave-uniform
+    const bf16_t* xp[2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      const int r = min(m0 + lr[j], end - 1);
+      xp[j] = p.A + (long)(p.row_map ? p.row_map[r] : r) * p.lda + ck[j];
+    }
+    auto stage = [&](int t) {
+      char* slot = smem + (t % RING_SLOTS) * RING_SLOT;
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+        __builtin_amdgcn_global_load_lds((const void*)(wp[j] + t * 64), (lds_void*)(slot + 8192 + (wid * 2 + j) * 1024), 16, 0, 0);
+      if (mine) {
+#pragma unroll
+        for (int j = 0; j < 2; ++j)
+          __builtin_amdgcn_global_load_lds((const void*)(xp[j] + t * 64), (lds_void*)(slot + (wid * 2 + j) * 1024), 16, 0, 0);
+      }
+    };
+    f32x4 acc[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    // row pointers loaded above are in registers before the counted waits start
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < RING_SLOTS - 1; ++i)
+      if (i < nk) stage(i);
+    for (int i = 0; i < nk; ++i) {
+      const int ahead = min(RING_SLOTS - 2, nk - 1 - i);  // later steps stay in flight
+      if (mine) {
+        if (ahead >= 2) asm volatile("s_waitcnt vmcnt(8)" ::: "memory");
+        else if (ahead == 1) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      } else {
+        if (ahead >= 2) asm volatile("s_waitcnt vmcnt(4)" ::: "memory");
+        else if (ahead == 1) asm volatile("s_waitcnt vmcnt(2)" ::: "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+      }
+      asm volatile("s_barrier" ::: "memory");
+      // the slot read in the previous step is free: every wave is past it
+      if (i + RING_SLOTS - 1 < nk) stage(i + RING_SLOTS - 1);
+      if (!mine) continue;
+      const char* slot = smem + (i % RING_SLOTS) * RING_SLOT;
+      const int ar = wid * 16 + frow;
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk) {
+        const int c = kk * 4 + fq;
+        const bf16x8 a = *(const bf16x8*)(slot + ar * 128 + ((c ^ ring_swz(ar)) << 4));
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int br = j * 16 + frow;
+          const bf16x8 b = *(const bf16x8*)(slot + 8192 + br * 128 + ((c ^ ring_swz(br)) << 4));
+          acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, acc[j], 0, 0, 0);
+        }
+      }
+    }
+    // lane holds C[16 wid + 4 fq + r][16 j + frow]
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = m0 + 16 * wid + 4 * fq + r;
+      if (row >= end) continue;
+#pragma unroll
+      for (int j = 0; j < (PAIR ? 2 : 4); ++j) {
+        const int col = (PAIR ? cg * 32 : cg * 64) + 16 * j + frow;
+        const float y = PAIR ? glu(acc[j][r], acc[j + (PAIR ? 2 : 0)][r], p.glu) : acc[j][r];
+        if constexpr (OUT_F32) ((float*)p.C)[(long)row * p.ldc + col] = y;
+        else ((bf16_t*)p.C)[(long)row * p.ldc + col] = f2bf(y);
+      }
+    }
+    // every wave has read its last slots before the next pass stages over them
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    asm volatile("s_barrier" ::: "memory");
+  }
+}
+
 }  // namespace rt
 
 using namespace rt;
@@ -308,15 +411,25 @@ extern "C" int rt_moe_sort(const int* idx, int P, int slots, int G, int* offs, i
 }
 
 // C[r] = A[row_map[r]] W_g^T (pair: gated linear unit of [gate; up] halves, N = half) for the rows of
-// every group; mean_rows: expected rows per group (picks the row tiles per pass)
+// every group; mean_rows: expected rows per group (picks the row tiles per pass); ring: the LDS-DMA form
 extern "C" int rt_moe_rows(const void* A, long lda, const int* row_map, const void* W, long sW, long ldw, void* C,
                            long ldc, const int* offs, int G, int N, int K, int pair, int out_f32, int mean_rows,
-                           const float* glu_p, hipStream_t stream) {
+                           int ring, const float* glu_p, hipStream_t stream) {
   if (G <= 0 || N <= 0) return 0;
   if (K % 8 || ldw % 8 || lda % 8 || (pair && out_f32) || G > 65535) return -1;
   MoeRowsArgs p{(const bf16_t*)A, lda, row_map, (const bf16_t*)W, sW, ldw, C, ldc, offs, N, K, GluP{}};
   if (glu_p) { p.glu.limit = glu_p[0]; p.glu.alpha = glu_p[1]; p.glu.offset = glu_p[2]; }
-  dim3 grid((N + 15) / 16, G), block(256);
+  dim3 block(256);
+  if (ring) {
+    if (K % 64 || N % (pair ? 32 : 64)) return -3;
+    dim3 rg(N / (pair ? 32 : 64), G);
+    if (pair) hipLaunchKernelGGL((moe_ring_kernel<true, false>), rg, block, 0, stream, p);
+    else if (out_f32) hipLaunchKernelGGL((moe_ring_kernel<false, true>), rg, block, 0, stream, p);
+    else hipLaunchKernelGGL((moe_ring_kernel<false, false>), rg, block, 0, stream, p);
+    RT_LAUNCH_CHECK();
+    return 0;
+  }
+  dim3 grid((N + 15) / 16, G);
 #define MR(MTV)                                                                                          \
   if (pair) hipLaunchKernelGGL((moe_rows_kernel<true, false, MTV>), grid, block, 0, stream, p);          \
   else if (out_f32) hipLaunchKernelGGL((moe_rows_kernel<false, true, MTV>), grid, block, 0, stream, p);  \

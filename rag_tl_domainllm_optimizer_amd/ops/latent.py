@@ -57,7 +57,7 @@ def _np_parts(T: int, heads: int, max_len: int) -> int:
     """Key partitions of the split decode attention: enough workgroups for the chip (two per CU), at least
     64 keys each."""
     groups = T * ((heads + 31) // 32 if heads > 16 else 1)
-    return max(1, min((512 + groups - 1) // groups, (max_len + 63) // 64))
+    return max(1, min((512 + groups - 1) // groups, (max_len + 63) // 64, 512))
 
 
 def latent_attention(proj: torch.Tensor, d: LatentDims, kv_up: torch.Tensor, sink: torch.Tensor, cos, sin, batch, pool,
@@ -78,7 +78,7 @@ def latent_attention(proj: torch.Tensor, d: LatentDims, kv_up: torch.Tensor, sin
     if not on_gpu(proj):
         return _latent_attention_cpu(proj, d, uk, uv, sink, cos, sin, row, pos, pool, tab, kv_col, norm_w, eps, gate)
     nat = native()
-    bf16 = proj.dtype == torch.bfloat16
+    bf16 = proj.dtype == torch.bfloat16 and d.scale > 0
     fast = bf16 and D % 8 == 0 and R % 8 == 0 and proj.stride(0) % 8 == 0 and nat.latent_decode_ok(C, d.kd)
     expand = bf16 and C % 8 == 0 and batch.segs is not None and proj.stride(0) % 8 == 0 \
         and nat.latent_prefill_ok(D, R, V)

@@ -12,7 +12,9 @@ from ._ext import native, on_gpu
 from .linear import Glu, project
 from .norm import MoePairs
 
-ROWS_PER_GROUP = 48  # expected rows per expert up to which the weight-streaming kernel is used
+# expected rows per expert from which the next form is faster (64 experts of 4096 x 1408 on one MI355X):
+RING_ROWS = 5              # LDS-DMA ring instead of register streaming
+TILE_ROWS_IN, TILE_ROWS_OUT = 33, 57  # 256-row MFMA tiles instead of the ring (gate / up, down)
 
 
 def moe_route(logits: torch.Tensor, correction: torch.Tensor, top: int, nshared: int = 0, gate_col: int = -1):
@@ -45,15 +47,19 @@ def moe_ff(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor, w_
     P = idx.numel()
     mean = (P + G - 1) // G
     bf16 = h.dtype == torch.bfloat16 and W % 8 == 0 and F % 8 == 0
-    big = bf16 and mean > ROWS_PER_GROUP and F % 128 == 0
-    srt = native().moe_sort(idx, G, 256 if big else 0)
+    tiles = bf16 and mean >= TILE_ROWS_IN and F % 128 == 0
+    srt = native().moe_sort(idx, G, 256 if tiles else 0)
     offs, tok, pos = srt[:3]
-    if big:
-        f = native().gemm_grouped(h, tok, w_gu, srt[3], srt[4], P, glu.args(), 256)
-        y = native().gemm_grouped(f, None, w_down, srt[3], srt[4], P, [], 256)
-    elif bf16:
-        f = native().moe_rows(h, tok, w_gu, offs, P, False, mean, glu.args())
-        y = native().moe_rows(f, None, w_down, offs, P, T <= 64, mean, [])
+    if bf16:
+        ring = mean >= RING_ROWS
+        if tiles:
+            f = native().gemm_grouped(h, tok, w_gu, srt[3], srt[4], P, glu.args(), 256)
+        else:
+            f = native().moe_rows(h, tok, w_gu, offs, P, False, mean, ring and W % 64 == 0 and F % 32 == 0, glu.args())
+        if tiles and mean >= TILE_ROWS_OUT:
+            y = native().gemm_grouped(f, None, w_down, srt[3], srt[4], P, [], 256)
+        else:
+            y = native().moe_rows(f, None, w_down, offs, P, T <= 64, mean, ring and W % 64 == 0 and F % 64 == 0, [])
     else:
         f = native().glu_any(native().gemm_any(h, w_gu, offs=offs, row_map=tok), glu.args())
         y = native().gemm_any(f, w_down, offs=offs)

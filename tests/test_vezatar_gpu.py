@@ -157,7 +157,8 @@ def test_pair_sort(T, slots, G):
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("T,W,F,E,top,nsh", [(1, 256, 128, 12, 4, 2), (60, 136, 40, 5, 2, 1), (300, 256, 128, 3, 2, 0),
-                                             (900, 192, 256, 6, 3, 1), (50, 44, 14, 5, 2, 2)])
+                                             (900, 192, 256, 6, 3, 1), (50, 44, 14, 5, 2, 2), (70, 256, 64, 4, 3, 1),
+                                             (150, 128, 96, 9, 2, 1)])
 def test_expert_products(dtype, T, W, F, E, top, nsh):
     G = E + nsh
     h, rw = torch.randn(T, W).to(dtype), (torch.randn((E + 8) // 8 * 8 + 8, W) * 0.1).to(dtype)
