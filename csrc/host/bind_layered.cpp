@@ -17,7 +17,7 @@ int rt_gemm_any(int, int, const void*, long, long, const void*, long, long, void
                 const int*, const int*, hipStream_t);
 int rt_glu_any(int, const void*, long, void*, long, int, const float*, hipStream_t);
 int rt_gate_mul(int, void*, const void*, long, long, int, hipStream_t);
-int rt_moe_route(const float*, long, const float*, int, int, int, int, int, int*, float*, hipStream_t);
+int rt_moe_route(const float*, long, int, long, const float*, int, int, int, int, int, int*, float*, hipStream_t);
 int rt_moe_sort(const int*, int, int, int, int*, int*, int*, int, int, void*, int*, hipStream_t);
 int rt_moe_rows(const void*, long, const int*, const void*, long, long, void*, long, const int*, int, int, int, int, int,
                 int, int, const float*, hipStream_t);
@@ -208,17 +208,19 @@ void gate_mul(Tensor a, const Tensor& g) {
   rc_ok(rt_gate_mul(is_f32(a), a.data_ptr(), g.data_ptr(), g.stride(0), a.size(0), (int)a.size(1), stream()), "gate_mul");
 }
 
-// -> (idx [T, top + nshared] int32, weights [T, top + nshared] fp32)
-std::vector<Tensor> moe_route(const Tensor& logits, const Tensor& correction, int64_t top, int64_t nshared, int64_t gate_col) {
+// logits [T, >= E] fp32, or [nslab * T, ..] split-K slabs -> (idx [T, top + nshared] int32, weights fp32)
+std::vector<Tensor> moe_route(const Tensor& logits, const Tensor& correction, int64_t top, int64_t nshared, int64_t gate_col,
+                              int64_t nslab) {
   TORCH_CHECK(logits.is_cuda() && is_f32(logits), "moe_route: fp32 logits");
   rows(logits, "moe_route");
   f32c(correction, "moe_route correction");
-  const int64_t T = logits.size(0), E = correction.numel();
+  TORCH_CHECK(nslab >= 1 && logits.size(0) % nslab == 0, "moe_route: slabs");
+  const int64_t T = logits.size(0) / nslab, E = correction.numel();
   TORCH_CHECK(logits.size(1) >= E && gate_col < logits.size(1), "moe_route: columns");
   Tensor idx = at::empty({T, top + nshared}, logits.options().dtype(at::kInt));
   Tensor wt = at::empty({T, top + nshared}, logits.options());
-  rc_ok(rt_moe_route(logits.data_ptr<float>(), logits.stride(0), correction.data_ptr<float>(), (int)T, (int)E, (int)top,
-                     (int)nshared, (int)gate_col, idx.data_ptr<int>(), wt.data_ptr<float>(), stream()),
+  rc_ok(rt_moe_route(logits.data_ptr<float>(), logits.stride(0), (int)nslab, T * logits.stride(0), correction.data_ptr<float>(),
+                     (int)T, (int)E, (int)top, (int)nshared, (int)gate_col, idx.data_ptr<int>(), wt.data_ptr<float>(), stream()),
         "moe_route");
   return {idx, wt};
 }
@@ -441,7 +443,8 @@ void bind_layered(py::module_& m) {
         py::arg("gate") = py::none());
   m.def("glu_any", &glu_any, "gated linear unit of [gate | up] rows");
   m.def("gate_mul", &gate_mul, "a *= sigmoid(g)");
-  m.def("moe_route", &moe_route, "softmax router with choice correction -> experts, weights");
+  m.def("moe_route", &moe_route, "softmax router with choice correction -> experts, weights", py::arg("logits"),
+        py::arg("correction"), py::arg("top"), py::arg("nshared"), py::arg("gate_col"), py::arg("nslab") = 1);
   m.def("moe_sort", &moe_sort, "stable sort of (token, slot) pairs by expert");
   m.def("moe_rows", &moe_rows, "grouped product at few rows per group");
   m.def("gemm_grouped", &gemm_grouped, "grouped product over 256-row tiles");

@@ -130,48 +130,77 @@ __global__ __launch_bounds__(256) void latent_prep_kernel(PrepArgs a) {
 
 // ---------------------------------------------------------------------------------------------
 // per-head product at few rows: C[t][b][:] = A[t][b][:] W_b^T (absorb: rank x dim per head; value
-// expansion: vdim x rank, times sigmoid(gate[t][b N + n])). MFMA, weights streamed straight to registers. grid (N / 64, batch, T / 16), wave = 16 columns.
+// expansion: vdim x rank, times sigmoid(gate[t][b N + n])). MFMA, weights streamed straight to registers. grid (N / 64, batch, T / (16 MT)), wave = 16 columns x 16 MT rows.
 // ---------------------------------------------------------------------------------------------
+template <int MT>
 __global__ __launch_bounds__(256) void head_gemm_kernel(const bf16_t* __restrict__ A, long lda, long sA,
                                                         const bf16_t* __restrict__ W, long ldw, long sW,
                                                         bf16_t* __restrict__ C, long ldc, long sC, int T, int N, int K,
-                                                        const bf16_t* __restrict__ gate, long ldg) {
+                                                        const bf16_t* __restrict__ gate, long ldg, int vec) {
   const int lane = threadIdx.x & 63, w = threadIdx.x >> 6, r16 = lane & 15, q = lane >> 4;
-  const int n0 = blockIdx.x * 64 + w * 16, b = blockIdx.y, t0 = blockIdx.z * 16;
-  if (n0 >= N) return;
-  const bf16_t* ap = A + (long)min(t0 + r16, T - 1) * lda + b * sA + 8 * q;
-  const bf16_t* wp = W + b * sW + (long)min(n0 + r16, N - 1) * ldw + 8 * q;
-  // weight as the A operand: acc[r] = C[t0 + r16][n0 + 4 q + r]
-  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
-  int k = 0;
-  for (; k + 256 <= K; k += 256) {  // eight steps' operands in flight
-    bf16x8 wf[8], af[8];
+  const int n0 = blockIdx.x * 64 + w * 16, b = blockIdx.y, t0 = blockIdx.z * 16 * MT;
+  __shared__ __attribute__((aligned(16))) bf16_t tile[16 * MT][72];  // 64 columns, padded rows
+  const bf16_t* ap[MT];
 #pragma unroll
-    for (int u = 0; u < 8; ++u) {
+  for (int i = 0; i < MT; ++i) ap[i] = A + (long)min(t0 + 16 * i + r16, T - 1) * lda + b * sA + 8 * q;
+  const bf16_t* wp = W + b * sW + (long)min(n0 + r16, N - 1) * ldw + 8 * q;
+  // weight as the A operand: acc[i][r] = C[t0 + 16 i + r16][n0 + 4 q + r]
+  f32x4 acc[MT];
+#pragma unroll
+  for (int i = 0; i < MT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  constexpr int U = MT == 1 ? 8 : 4;  // steps' operands in flight
+  int k = 0;
+  for (; k + 32 * U <= K; k += 32 * U) {
+    bf16x8 wf[U], af[MT][U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
       wf[u] = *(const bf16x8*)(wp + k + 32 * u);
-      af[u] = *(const bf16x8*)(ap + k + 32 * u);
+#pragma unroll
+      for (int i = 0; i < MT; ++i) af[i][u] = *(const bf16x8*)(ap[i] + k + 32 * u);
     }
 #pragma unroll
-    for (int u = 0; u < 8; ++u) acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], af[u], acc, 0, 0, 0);
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int i = 0; i < MT; ++i) acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[u], af[i][u], acc[i], 0, 0, 0);
   }
-#pragma unroll 4
   for (; k < K; k += 32) {
     const bool ok = k + 8 * q < K;
     const bf16x8 wf = ok ? *(const bf16x8*)(wp + k) : bf16x8{};
-    const bf16x8 af = ok ? *(const bf16x8*)(ap + k) : bf16x8{};
-    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc, 0, 0, 0);
-  }
-  const int t = t0 + r16;
-  if (t >= T) return;
-  bf16_t* c = C + (long)t * ldc + b * sC + n0 + 4 * q;
-  const bf16_t* gp = gate + (long)t * ldg + (long)b * N + n0 + 4 * q;
 #pragma unroll
-  for (int r = 0; r < 4; ++r)
-    if (n0 + 4 * q + r < N) {
-      float y = acc[r];
-      if (gate) y /= 1.f + __expf(-bf2f(gp[r]));
-      c[r] = f2bf(y);
+    for (int i = 0; i < MT; ++i) {
+      const bf16x8 af = ok ? *(const bf16x8*)(ap[i] + k) : bf16x8{};
+      acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, af, acc[i], 0, 0, 0);
     }
+  }
+  // through LDS: whole 128-B row pieces out, the gate read the same way
+#pragma unroll
+  for (int i = 0; i < MT; ++i)
+    *(uint2*)&tile[16 * i + r16][16 * w + 4 * q] = make_uint2(pack2bf(acc[i][0], acc[i][1]), pack2bf(acc[i][2], acc[i][3]));
+  __syncthreads();
+  const int c0 = blockIdx.x * 64;
+  for (int e = threadIdx.x; e < 16 * MT * 8; e += 256) {
+    const int r = e >> 3, c = (e & 7) * 8, t = t0 + r;
+    if (t >= T || c0 + c >= N) continue;
+    bf16_t* o = C + (long)t * ldc + b * sC + c0 + c;
+    const bf16_t* gp = gate + (long)t * ldg + (long)b * N + c0 + c;
+    if (vec) {
+      uint4 v = *(const uint4*)&tile[r][c];
+      if (gate) {
+        float y[8], x[8];
+        unpack8(v, y);
+        unpack8(*(const uint4*)gp, x);
+#pragma unroll
+        for (int k = 0; k < 8; ++k) y[k] /= 1.f + __expf(-x[k]);
+        v = pack8(y);
+      }
+      *(uint4*)o = v;
+    } else {
+      for (int k = 0; k < 8 && c0 + c + k < N; ++k) {
+        const float y = bf2f(tile[r][c + k]);
+        o[k] = f2bf(gate ? y / (1.f + __expf(-bf2f(gp[k]))) : y);
+      }
+    }
+  }
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -758,9 +787,15 @@ extern "C" int rt_head_gemm(const void* A, long lda, long sA, const void* W, lon
                             hipStream_t stream) {
   if (T <= 0 || N <= 0 || batch <= 0) return 0;
   if (K % 8 || lda % 8 || sA % 8 || ldw % 8 || sW % 8 || batch > 65535 || (T + 15) / 16 > 65535) return -1;
-  dim3 grid((N + 63) / 64, batch, (T + 15) / 16);
-  hipLaunchKernelGGL(head_gemm_kernel, grid, dim3(256), 0, stream, (const bf16_t*)A, lda, sA, (const bf16_t*)W, ldw,
-                     sW, (bf16_t*)C, ldc, sC, T, N, K, (const bf16_t*)gate, ldg);
+  const int mt = T > 128 ? 4 : 1;
+  // 16-B output pieces (and gate reads)
+  const int vec = N % 8 == 0 && ldc % 8 == 0 && sC % 8 == 0 && (uintptr_t)C % 16 == 0 &&
+                  (!gate || (ldg % 8 == 0 && (uintptr_t)gate % 16 == 0));
+  dim3 grid((N + 63) / 64, batch, (T + 16 * mt - 1) / (16 * mt));
+#define HG_(M) hipLaunchKernelGGL(head_gemm_kernel<M>, grid, dim3(256), 0, stream, (const bf16_t*)A, lda, sA, (const bf16_t*)W, \
+                                  ldw, sW, (bf16_t*)C, ldc, sC, T, N, K, (const bf16_t*)gate, ldg, vec)
+  if (mt == 4) HG_(4); else HG_(1);
+#undef HG_
   RT_LAUNCH_CHECK();
   return 0;
 }

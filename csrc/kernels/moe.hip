@@ -3,7 +3,7 @@
 // gemm_big_kernel). All row counts stay on the device: every launch has a fixed grid, so a decode step
 // with these kernels can be captured in a graph.
 //
-//   moe_route    logits [T, ldl] fp32 (columns [0, E) experts, optional column E = shared gate) ->
+//   moe_route    logits [T, ldl] fp32, or nslab split-K slabs of them (columns [0, E) experts, optional column E = shared gate) ->
 //                per token the `top` experts of the largest choice score softmax(z) + correction and
 //                their weights softmax(z) (not renormalised), then `nshared` slots of the shared
 //                expert (groups E .. E + nshared - 1) with weight sigmoid(shared gate);
@@ -18,8 +18,8 @@
 namespace rt {
 
 // one wave per token
-__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, long ldl,
-                                                        const float* __restrict__ correction, int T, int E, int top,
+__global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict__ logits, long ldl, int nslab,
+                                                        long sstride, const float* __restrict__ correction, int T, int E, int top,
                                                         int nshared, int gate_col, int* __restrict__ idx,
                                                         float* __restrict__ wt) {
   const int t = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
@@ -31,7 +31,11 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
 #pragma unroll
   for (int i = 0; i < MAXV; ++i) {
     const int e = lane + 64 * i;
-    s[i] = e < E ? z[e] : -INFINITY;
+    s[i] = -INFINITY;
+    if (e < E) {
+      s[i] = z[e];
+      for (int q = 1; q < nslab; ++q) s[i] += z[q * sstride + e];
+    }
     mx = fmaxf(mx, s[i]);
   }
   mx = wave_max(mx);
@@ -79,7 +83,10 @@ __global__ __launch_bounds__(256) void moe_route_kernel(const float* __restrict_
   }
   if (lane < nshared) {
     idx[(long)t * slots + top + lane] = E + lane;
-    wt[(long)t * slots + top + lane] = gate_col >= 0 ? 1.f / (1.f + expf(-z[gate_col])) : 1.f;
+    float zg = 0.f;
+    if (gate_col >= 0)
+      for (int q = 0; q < nslab; ++q) zg += z[q * sstride + gate_col];
+    wt[(long)t * slots + top + lane] = gate_col >= 0 ? 1.f / (1.f + expf(-zg)) : 1.f;
   }
 }
 
@@ -386,11 +393,11 @@ __global__ __launch_bounds__(256, 2) void moe_ring_kernel(MoeRowsArgs p) {
 
 using namespace rt;
 
-extern "C" int rt_moe_route(const float* logits, long ldl, const float* correction, int T, int E, int top, int nshared,
+extern "C" int rt_moe_route(const float* logits, long ldl, int nslab, long sstride, const float* correction, int T, int E, int top, int nshared,
                             int gate_col, int* idx, float* wt, hipStream_t stream) {
   if (T <= 0) return 0;
   if (E < 1 || E > 512 || top < 1 || top > E || nshared < 0 || nshared > 64) return -1;
-  hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, ldl, correction, T, E, top,
+  hipLaunchKernelGGL(moe_route_kernel, dim3((T + 3) / 4), dim3(256), 0, stream, logits, ldl, nslab, sstride, correction, T, E, top,
                      nshared, gate_col, idx, wt);
   RT_LAUNCH_CHECK();
   return 0;

@@ -243,6 +243,9 @@ class LayeredLM(nn.Module):
         if "key" in self._head_shuf:
             self._head_shuf.get(self.lm_head)
 
+    def add_lora(self, *a, **kw):
+        raise NotImplementedError(f"{self.cfg.arch}: layered models are inference-only (no adapters, no backward)")
+
     @torch.no_grad()
     def forward(self, input_ids: torch.Tensor, kv_start: Optional[torch.Tensor] = None) -> torch.Tensor:
         """input_ids [B, S] (left-padded; kv_start[b] = first real token) -> final hidden [B * S, width] (zeros

@@ -9,7 +9,7 @@ import torch
 
 from . import reference as ref
 from ._ext import native, on_gpu
-from .linear import Glu, project
+from .linear import ROW, Glu, project
 from .norm import MoePairs
 
 # expected rows per expert from which the next form is faster (64 experts of 4096 x 1408 on one MI355X):
@@ -17,13 +17,26 @@ RING_ROWS = 5              # LDS-DMA ring instead of register streaming
 TILE_ROWS_IN, TILE_ROWS_OUT = 33, 57  # 256-row MFMA tiles instead of the ring (gate / up, down)
 
 
-def moe_route(logits: torch.Tensor, correction: torch.Tensor, top: int, nshared: int = 0, gate_col: int = -1):
-    """fp32 router logits [T, >= E] -> (groups [T, top + nshared] int32, weights fp32): the ``top`` experts of
-    the largest ``softmax + correction`` with their softmax values, then groups E .. E + nshared - 1 (the
+def moe_route(logits: torch.Tensor, correction: torch.Tensor, top: int, nshared: int = 0, gate_col: int = -1,
+              nslab: int = 1):
+    """fp32 router logits [T, >= E] (or ``nslab`` slabs of them, stacked) -> (groups [T, top + nshared] int32,
+    weights fp32): the ``top`` experts of the largest ``softmax + correction`` with their softmax values, then groups E .. E + nshared - 1 (the
     shared expert's parts) with weight sigmoid(logits[:, gate_col]) (1 without a gate column)."""
     if on_gpu(logits):
-        return native().moe_route(logits, correction, top, nshared, gate_col)
+        return native().moe_route(logits, correction, top, nshared, gate_col, nslab)
     return ref.moe_route(logits, correction, top, nshared, gate_col)
+
+
+def router_logits(h: torch.Tensor, router_w: torch.Tensor):
+    """(fp32 logits h W^T, slabs): above 64 rows the narrow product is split over K into slabs that fill the
+    chip, summed by the routing kernel."""
+    T, K = h.shape
+    N = router_w.shape[0]
+    if on_gpu(h) and h.dtype == torch.bfloat16 and T > 64 and K % 64 == 0 and N % 8 == 0:
+        ns = max(1, min(K // 256, 1024 // max(1, ((T + 63) // 64) * ((N + 63) // 64)), 16))
+        if ns > 1:
+            return native().gemm_small(h, router_w, ROW, ROW, 3, ns, None, 64), ns
+    return project(h, router_w, out_f32=True), 1
 
 
 def moe_ff(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor, w_gu: torch.Tensor, w_down: torch.Tensor,
@@ -32,7 +45,8 @@ def moe_ff(h: torch.Tensor, router_w: torch.Tensor, correction: torch.Tensor, w_
     T = h.shape[0]
     G, F2, W = w_gu.shape
     F = F2 // 2
-    idx, wt = moe_route(project(h, router_w, out_f32=True), correction, top, nshared, gate_col)
+    z, nslab = router_logits(h, router_w)
+    idx, wt = moe_route(z, correction, top, nshared, gate_col, nslab)
     if not on_gpu(h):
         order = torch.argsort(idx.reshape(-1), stable=True)
         pos = torch.empty_like(order)

@@ -314,6 +314,34 @@ def test_cli_rag_answers_with_a_layered_policy(capsys):
     assert "answer" in json.loads(line)
 
 
+def test_serving_engines_with_a_layered_policy():
+    """the RAG pipeline's answers, one by one, equal those of the continuous engine under load"""
+    from rag_tl_domainllm_optimizer_amd.rag import RagPipeline
+    from rag_tl_domainllm_optimizer_amd.retrieval import Encoder, FlatIndex
+    from rag_tl_domainllm_optimizer_amd.serve import ContinuousEngine
+    from rag_tl_domainllm_optimizer_amd.tokenizer import Tokenizer
+
+    pol = models.LayeredLM(models.resolve_preset("tiny-vezatar"), dtype=torch.float32, seed=1)
+    enc_m = models.build_model("tiny-bert", device="cpu", dtype=torch.float32, seed=2).eval()
+    tok = Tokenizer.synthetic(pol.cfg.vocab_size, pol.cfg.arch)
+    enc = Encoder(enc_m, Tokenizer.synthetic(enc_m.cfg.vocab_size, enc_m.cfg.arch), max_length=32)
+    words = tok.words()
+    docs = [" ".join(words[(7 * i + j) % len(words)] for j in range(12)) for i in range(30)]
+    index = FlatIndex(enc.dim, "ip", "cpu")
+    index.add(enc.encode(docs))
+    pipe = RagPipeline(enc, index, docs, pol, tok, top_k=2, sampling=SamplingParams(max_new_tokens=4, do_sample=False),
+                       max_prompt_tokens=96, max_batch=2, use_graph=False)
+    qs = [f"{words[i]} {words[i + 3]}" for i in range(5)]
+    direct = [pipe.answer([q])[0].answer for q in qs]
+    with ContinuousEngine(pipe, chunk=2) as eng:
+        assert [a.answer for a in eng.answer_many(qs, timeout=60)] == direct
+
+
+def test_layered_models_refuse_adapters():
+    with pytest.raises(NotImplementedError):
+        models.build_model("tiny-vezatar:random").add_lora(8)
+
+
 def test_wrong_config_values_are_read_not_assumed(odd):
     """every constant of config.json reaches the result: changing any of them changes the logits"""
     cfg, w, _ = odd
