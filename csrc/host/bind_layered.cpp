@@ -11,11 +11,12 @@
 #include <vector>
 
 extern "C" {
-int rt_branch_norm(int, int, float*, const void*, long, int, const void*, const void*, void*, const void*, const long*,
-                   int, const float*, const int*, int, int, int, float, hipStream_t);
+int rt_branch_norm(int, int, float*, const void*, long, int, const void*, const void*, const void*, float, void*,
+                   const void*, const long*, int, const float*, const int*, int, int, int, float, hipStream_t);
 int rt_gemm_any(int, int, const void*, long, long, const void*, long, long, void*, long, long, int, int, int, int,
                 const int*, const int*, hipStream_t);
 int rt_glu_any(int, const void*, long, void*, long, int, const float*, hipStream_t);
+int rt_act_any(int, const float*, void*, long, int, hipStream_t);
 int rt_gate_mul(int, void*, const void*, long, long, int, hipStream_t);
 int rt_moe_route(const float*, long, int, long, const float*, int, int, int, int, int, int*, float*, hipStream_t);
 int rt_moe_sort(const int*, int, int, int, int*, int*, int*, int, int, void*, int*, hipStream_t);
@@ -30,11 +31,31 @@ int rt_head_gemm(const void*, long, long, const void*, long, long, void*, long, 
 int rt_latent_decode_ok(int, int);
 int rt_latent_decode(const void*, const void*, const int*, int, int, int, const int*, const int*, float*, float*, int,
                      int, int, int, int, float, hipStream_t);
-int rt_latent_merge(const float*, const float*, const float*, void*, int, int, int, int, hipStream_t);
+int rt_partition_merge(const float*, const float*, const float*, void*, long, int, int, int, int, float, hipStream_t);
 int rt_latent_gather(int, const void*, const int*, int, int, const void*, int, int, void*, int, hipStream_t);
 int rt_latent_prefill_ok(int, int, int);
 int rt_latent_prefill(const void*, long, const void*, long, int, int, const float*, const void*, long, void*, long,
                       const void*, const void*, int, int, int, int, int, float, hipStream_t);
+int rt_window_prep(int, void*, long, int, int, int, const void*, const void*, float, const float*, const float*, int, int,
+                   const int*, const int*, void*, const int*, int, int, int, int, int, int, int, int, hipStream_t);
+int rt_window_decode_ok(int, int, int, int);
+int rt_window_decode(const void*, long, const void*, const int*, int, int, int, const int*, const int*, float*, float*, int,
+                     int, int, int, int, int, int, int, float, float, hipStream_t);
+int rt_window_prefill_ok(int, int);
+int rt_window_prefill(const void*, long, const void*, const int*, int, int, int, void*, long, const void*, const void*, int,
+                      int, int, int, int, int, int, float, float, float, hipStream_t);
+int rt_window_any(int, const void*, long, const void*, const int*, int, int, int, const int*, const int*, void*, long, int,
+                  int, int, int, int, int, int, float, float, float, hipStream_t);
+struct RtDelta {  // mirrors csrc/kernels/delta_rule.hip
+  const void* x; long ldx; const void* b; long ldb; const void* a; long lda; const void* z; long ldz;
+  const void* conv; const float* A_log; const float* dt; const void* norm_w; float eps;
+  const int* row; const int* pos; float* S; void* ring; int n_rows; void* out; long ldo; float out_scale;
+  int H, K, D, V, taps, channel, silu;
+};
+int rt_delta_step(int, const RtDelta*, int, hipStream_t);
+long rt_delta_ws(int);
+int rt_delta_runs(int, const RtDelta*, const void*, const void*, const int*, int, int, int, int, float*, void*, float*,
+                  hipStream_t);
 int rt_latent_any(int, const void*, const void*, const int*, int, int, int, const int*, const int*, const float*, void*,
                   int, int, int, int, float, hipStream_t);
 }
@@ -86,17 +107,20 @@ const Tensor& zero_page(const Tensor& like) {
 }
 
 // x [T, H] fp32 in place; kind 0 none / embedding, 1 rows of the activation type, 2 fp32 slabs
-// [nsplit, T, H], 3 pairs (activation type), 4 pairs (fp32). Returns h (or None without w_next).
+// [nsplit, T, H], 3 pairs (activation type), 4 pairs (fp32). Returns h (plain: x rounded, without w_next) or
+// None.
 py::object branch_norm(Tensor x, int64_t kind, const optional<Tensor>& y, int64_t nsplit, const optional<Tensor>& w_branch,
                        const optional<Tensor>& w_next, const optional<Tensor>& table, const optional<Tensor>& ids,
-                       const optional<Tensor>& pair_w, const optional<Tensor>& pair_pos, double eps) {
+                       const optional<Tensor>& pair_w, const optional<Tensor>& pair_pos, double eps,
+                       const optional<Tensor>& scale, double next_mul, bool plain) {
   f32c(x, "branch_norm x");
   TORCH_CHECK(x.dim() == 2, "branch_norm: x [T, H]");
   const int64_t T = x.size(0), H = x.size(1);
-  TORCH_CHECK(kind >= 0 && kind <= 4 && (kind == 0) == !has(w_branch), "branch_norm: kind / w_branch");
+  TORCH_CHECK(kind >= 0 && kind <= 4 && (kind == 0 || has(w_branch)) && (kind != 0 || !has(w_branch) || has(table)) &&
+                  !(plain && has(w_next)), "branch_norm: kind / w_branch");
   const Tensor& like = has(w_branch) ? *w_branch : (has(w_next) ? *w_next : *table);
   act_type(like, "branch_norm weights");
-  for (const auto* w : {&w_branch, &w_next})
+  for (const auto* w : {&w_branch, &w_next, &scale})
     if (has(*w)) TORCH_CHECK((*w)->numel() == H && (*w)->is_contiguous() && (*w)->scalar_type() == like.scalar_type(), "branch_norm: weights");
   int64_t K = 0, vocab = 0;
   if (kind == 0) {
@@ -126,12 +150,13 @@ py::object branch_norm(Tensor x, int64_t kind, const optional<Tensor>& y, int64_
     }
   }
   Tensor h;
-  if (has(w_next)) h = at::empty({T, H}, like.options());
-  rc_ok(rt_branch_norm(is_f32(like), (int)kind, x.data_ptr<float>(), ptr(y), T * H, (int)nsplit, ptr(w_branch), ptr(w_next),
-                       has(w_next) ? h.data_ptr() : nullptr, ptr(table), (const long*)ptr(ids), (int)vocab,
-                       (const float*)ptr(pair_w), (const int*)ptr(pair_pos), (int)K, (int)T, (int)H, (float)eps, stream()),
+  const bool want = has(w_next) || plain;
+  if (want) h = at::empty({T, H}, like.options());
+  rc_ok(rt_branch_norm(is_f32(like), (int)kind, x.data_ptr<float>(), ptr(y), T * H, (int)nsplit, ptr(w_branch), ptr(scale),
+                       ptr(w_next), (float)next_mul, want ? h.data_ptr() : nullptr, ptr(table), (const long*)ptr(ids),
+                       (int)vocab, (const float*)ptr(pair_w), (const int*)ptr(pair_pos), (int)K, (int)T, (int)H, (float)eps, stream()),
         "branch_norm");
-  return has(w_next) ? py::cast(h) : py::none();
+  return want ? py::cast(h) : py::none();
 }
 
 // out = a w^T. 2-D operands; 3-D: batched (strided views with unit last stride); offs: grouped (w 3-D,
@@ -197,6 +222,14 @@ Tensor glu_any(const Tensor& gu, const std::vector<double>& glu) {
   Tensor y = at::empty({gu.size(0), gu.size(1) / 2}, gu.options());
   rc_ok(rt_glu_any(is_f32(gu), gu.data_ptr(), gu.stride(0), y.data_ptr(), gu.size(0), (int)(gu.size(1) / 2), Glu(glu).v, stream()),
         "glu_any");
+  return y;
+}
+
+// activation of an fp32 product: act 8 = max(x, 0)^2
+Tensor act_any(const Tensor& x, int64_t act, bool out_f32) {
+  f32c(x, "act_any");
+  Tensor y = at::empty(x.sizes(), x.options().dtype(out_f32 ? at::kFloat : at::kBFloat16));
+  rc_ok(rt_act_any(out_f32, x.data_ptr<float>(), y.data_ptr(), x.numel(), (int)act, stream()), "act_any");
   return y;
 }
 
@@ -373,8 +406,8 @@ Tensor latent_merge(const Tensor& part, const Tensor& ml, const Tensor& sink) {
   const int64_t T = part.size(0), H = part.size(1), NP = part.size(2), rank = part.size(3);
   TORCH_CHECK(sink.numel() == H && ml.numel() == T * H * NP * 2, "latent_merge: shapes");
   Tensor o = at::empty({T, H, rank}, part.options().dtype(at::kBFloat16));
-  rc_ok(rt_latent_merge(part.data_ptr<float>(), ml.data_ptr<float>(), sink.data_ptr<float>(), o.data_ptr(), (int)T, (int)H,
-                        (int)rank, (int)NP, stream()),
+  rc_ok(rt_partition_merge(part.data_ptr<float>(), ml.data_ptr<float>(), sink.data_ptr<float>(), o.data_ptr(), H * rank, (int)T,
+                           (int)H, (int)rank, (int)NP, 1.f, stream()),
         "latent_merge");
   return o;
 }
@@ -430,18 +463,176 @@ Tensor latent_any(const Tensor& q, const Tensor& pool, const Tensor& tab, const 
   return o;
 }
 
+// ---- grouped-query attention over a paged window ----
+// pool [pages, 64, G (D + V)] (inside a page: [G][64][D + V])
+struct Win {
+  int H, G, D, V, size, keep;
+  float scale, cap;
+  // {heads, key heads, key width, value width, window (0: none), kept first tokens}, {scale, softcap (0: none)}
+  Win(const std::vector<int64_t>& d, const std::vector<double>& f, const Pool& pl) {
+    TORCH_CHECK(d.size() == 6 && f.size() == 2, "window attention: dims {6}, {2}");
+    H = (int)d[0]; G = (int)d[1]; D = (int)d[2]; V = (int)d[3]; size = (int)d[4]; keep = (int)d[5];
+    scale = (float)f[0]; cap = (float)f[1];
+    TORCH_CHECK(H > 0 && G > 0 && H % G == 0 && D > 0 && V > 0 && size >= 0 && keep >= 0 && pl.kd() == G * (D + V) &&
+                    pl.rows() > 0 && pl.max_pages() > 0, "window attention: sizes");
+  }
+};
+
+// proj [N, ..] = q | k | v from column col: q normed and rotated in place, k and v to the cache
+void window_prep(Tensor proj, int64_t col, const optional<Tensor>& q_norm, const optional<Tensor>& k_norm, double eps,
+                 const Tensor& cosT, const Tensor& sinT, const Tensor& row, const Tensor& pos, Tensor pool, const Tensor& tab,
+                 const std::vector<int64_t>& dims, const std::vector<double>& fs) {
+  Pool pl(pool, tab);
+  const Win w(dims, fs, pl);
+  rows(proj, "window_prep proj");
+  same(pool, proj, "window_prep");
+  const int64_t T = proj.size(0), nq = (int64_t)w.H * w.D, nk = (int64_t)w.G * w.D;
+  tok_index(row, pos, T);
+  f32c(cosT, "cos");
+  f32c(sinT, "sin");
+  TORCH_CHECK(cosT.dim() == 2 && cosT.sizes() == sinT.sizes() && cosT.size(0) >= 1 && 2 * cosT.size(1) <= w.D && col >= 0 &&
+                  col + nq + nk + (int64_t)w.G * w.V <= proj.size(1), "window_prep: shapes");
+  if (has(q_norm)) {
+    same(pool, *q_norm, "window_prep q norm");
+    TORCH_CHECK(q_norm->is_contiguous() && q_norm->numel() == nq, "window_prep: q norm");
+  }
+  if (has(k_norm)) {
+    same(pool, *k_norm, "window_prep k norm");
+    TORCH_CHECK(k_norm->is_contiguous() && k_norm->numel() == nk, "window_prep: k norm");
+  }
+  rc_ok(rt_window_prep(is_f32(pool), proj.data_ptr(), proj.stride(0), (int)col, (int)(col + nq), (int)(col + nq + nk), ptr(q_norm),
+                       ptr(k_norm), (float)eps, cosT.data_ptr<float>(), sinT.data_ptr<float>(), (int)cosT.size(0),
+                       (int)cosT.size(1), row.data_ptr<int>(), pos.data_ptr<int>(), pool.data_ptr(), tab.data_ptr<int>(),
+                       pl.max_pages(), pl.pages(), pl.rows(), (int)T, w.H, w.G, w.D, w.V, stream()),
+        "window_prep");
+}
+
+// tokens [0, T) of q [.., H D] and out [.., H V] (strided rows), keys and values from the cache
+void window_decode(const Tensor& q, const Tensor& pool, const Tensor& tab, const Tensor& row, const Tensor& pos, Tensor out,
+                   int64_t NP, double out_scale, const std::vector<int64_t>& dims, const std::vector<double>& fs) {
+  Pool pl(pool, tab);
+  const Win w(dims, fs, pl);
+  rows(q, "window_decode q");
+  rows(out, "window_decode out");
+  const int64_t T = q.size(0);
+  tok_index(row, pos, T);
+  TORCH_CHECK(pool.scalar_type() == at::kBFloat16 && q.scalar_type() == at::kBFloat16 && out.scalar_type() == at::kBFloat16 &&
+                  q.is_cuda() && out.is_cuda() && q.size(1) == (int64_t)w.H * w.D && out.size(0) == T &&
+                  out.size(1) == (int64_t)w.H * w.V && NP >= 1 && NP <= 1024 && al16(q), "window_decode: shapes");
+  Tensor part = at::empty({T, w.H, NP, w.V}, q.options().dtype(at::kFloat));
+  Tensor ml = at::empty({T, w.H, NP, 2}, q.options().dtype(at::kFloat));
+  rc_ok(rt_window_decode(q.data_ptr(), q.stride(0), pool.data_ptr(), tab.data_ptr<int>(), pl.max_pages(), pl.pages(), pl.rows(),
+                         row.data_ptr<int>(), pos.data_ptr<int>(), part.data_ptr<float>(), ml.data_ptr<float>(), (int)T, w.H, w.G,
+                         w.D, w.V, (int)NP, w.size, w.keep, w.scale, w.cap, stream()),
+        "window_decode");
+  rc_ok(rt_partition_merge(part.data_ptr<float>(), ml.data_ptr<float>(), nullptr, out.data_ptr(), out.stride(0), (int)T, w.H, w.V,
+                           (int)NP, (float)out_scale, stream()),
+        "partition_merge");
+}
+
+void window_prefill(const Tensor& q, const Tensor& pool, const Tensor& tab, Tensor out, const Tensor& segs, const Tensor& tiles,
+                    double out_scale, const std::vector<int64_t>& dims, const std::vector<double>& fs) {
+  Pool pl(pool, tab);
+  const Win w(dims, fs, pl);
+  rows(q, "window_prefill q");
+  rows(out, "window_prefill out");
+  ints(segs, "segs");
+  ints(tiles, "tiles");
+  TORCH_CHECK(pool.scalar_type() == at::kBFloat16 && q.scalar_type() == at::kBFloat16 && out.scalar_type() == at::kBFloat16 &&
+                  q.is_cuda() && out.is_cuda() && q.size(1) == (int64_t)w.H * w.D && out.size(0) == q.size(0) &&
+                  out.size(1) == (int64_t)w.H * w.V && al16(q) && segs.dim() == 2 && segs.size(1) == 8 && tiles.dim() == 2 &&
+                  tiles.size(1) == 2, "window_prefill: shapes");
+  rc_ok(rt_window_prefill(q.data_ptr(), q.stride(0), pool.data_ptr(), tab.data_ptr<int>(), pl.max_pages(), pl.pages(), pl.rows(),
+                          out.data_ptr(), out.stride(0), segs.data_ptr(), tiles.data_ptr(), (int)tiles.size(0), w.H, w.G, w.D,
+                          w.V, w.size, w.keep, w.scale, w.cap, (float)out_scale, stream()),
+        "window_prefill");
+}
+
+void window_any(const Tensor& q, const Tensor& pool, const Tensor& tab, const Tensor& row, const Tensor& pos, Tensor out,
+                double out_scale, const std::vector<int64_t>& dims, const std::vector<double>& fs) {
+  Pool pl(pool, tab);
+  const Win w(dims, fs, pl);
+  rows(q, "window_any q");
+  rows(out, "window_any out");
+  same(pool, q, "window_any");
+  same(pool, out, "window_any");
+  tok_index(row, pos, q.size(0));
+  TORCH_CHECK(q.size(1) == (int64_t)w.H * w.D && out.size(0) == q.size(0) && out.size(1) == (int64_t)w.H * w.V, "window_any: shapes");
+  rc_ok(rt_window_any(is_f32(pool), q.data_ptr(), q.stride(0), pool.data_ptr(), tab.data_ptr<int>(), pl.max_pages(), pl.pages(),
+                      pl.rows(), row.data_ptr<int>(), pos.data_ptr<int>(), out.data_ptr(), out.stride(0), (int)q.size(0), w.H,
+                      w.G, w.D, w.V, w.size, w.keep, w.scale, w.cap, (float)out_scale, stream()),
+        "window_any");
+}
+
+// ---- gated delta rule ----
+// x [N, C] (q | k | v projections), b [N, H], a [N, H or H D], z [N, H V], out [N, H V]: strided rows of one
+// type; S [rows, H, D, V] fp32, ring [rows, taps, C]. Tokens [0, n_single): one per request; the rest by runs
+// [R, 4] {row, first token, tokens, position}, chunks [.., 2] {run, chunk}, first_chunk [R].
+void delta_rule(const Tensor& x, const Tensor& b, const Tensor& a, const Tensor& z, const Tensor& conv, const Tensor& A_log,
+                const Tensor& dt, const Tensor& norm_w, double eps, const Tensor& row, const Tensor& pos, Tensor S, Tensor ring,
+                Tensor out, double out_scale, int64_t K, bool silu, int64_t n_single, const optional<Tensor>& runs,
+                const optional<Tensor>& chunks, const optional<Tensor>& first_chunk) {
+  act_type(x, "delta_rule x");
+  for (const Tensor* t : {&x, &b, &a, &z, (const Tensor*)&out}) {
+    rows(*t, "delta_rule rows");
+    same(x, *t, "delta_rule");
+    TORCH_CHECK(t->size(0) == x.size(0), "delta_rule: one row per token");
+  }
+  f32c(S, "delta_rule state");
+  f32c(A_log, "delta_rule A_log");
+  f32c(dt, "delta_rule dt");
+  same(x, ring, "delta_rule ring");
+  same(x, conv, "delta_rule conv");
+  same(x, norm_w, "delta_rule norm");
+  const int64_t N = x.size(0);
+  TORCH_CHECK(S.dim() == 4 && S.size(0) >= 1, "delta_rule: S [rows, H, D, V]");
+  const int64_t H = S.size(1), D = S.size(2), V = S.size(3), C = x.size(1);
+  TORCH_CHECK(K >= 1 && H % K == 0 && C == 2 * K * D + H * V && conv.dim() == 2 && conv.size(0) == C && conv.is_contiguous() &&
+                  conv.size(1) >= 1, "delta_rule: channels");
+  const int64_t taps = conv.size(1);
+  const bool channel = dt.numel() == H * D && a.size(1) == H * D && !(D == 1);
+  TORCH_CHECK(A_log.numel() == H && (channel || (dt.numel() == H && a.size(1) == H)) && b.size(1) == H && z.size(1) == H * V &&
+                  out.size(1) == H * V && norm_w.numel() == V && norm_w.is_contiguous(), "delta_rule: shapes");
+  TORCH_CHECK(ring.dim() == 3 && ring.size(0) == S.size(0) && ring.size(1) == taps && ring.size(2) == C && ring.is_contiguous(),
+              "delta_rule: ring [rows, taps, C]");
+  tok_index(row, pos, N);
+  TORCH_CHECK(n_single >= 0 && n_single <= N && (n_single == N || has(runs)), "delta_rule: runs");
+  RtDelta d{x.data_ptr(), x.stride(0), b.data_ptr(), b.stride(0), a.data_ptr(), a.stride(0), z.data_ptr(), z.stride(0),
+            conv.data_ptr(), A_log.data_ptr<float>(), dt.data_ptr<float>(), norm_w.data_ptr(), (float)eps, row.data_ptr<int>(),
+            pos.data_ptr<int>(), S.data_ptr<float>(), ring.data_ptr(), (int)S.size(0), out.data_ptr(), out.stride(0),
+            (float)out_scale, (int)H, (int)K, (int)D, (int)V, (int)taps, channel, silu};
+  rc_ok(rt_delta_step(is_f32(x), &d, (int)n_single, stream()), "delta_step");
+  if (n_single == N) return;
+  ints(*runs, "delta_rule runs");
+  TORCH_CHECK(has(chunks) && has(first_chunk), "delta_rule: chunks");
+  ints(*chunks, "delta_rule chunks");
+  ints(*first_chunk, "delta_rule first_chunk");
+  TORCH_CHECK(runs->dim() == 2 && runs->size(1) == 4 && chunks->dim() == 2 && chunks->size(1) == 2 && first_chunk->numel() == runs->size(0) &&
+                  al16(*runs) && reinterpret_cast<uintptr_t>(chunks->data_ptr()) % 8 == 0, "delta_rule: tables");
+  const long per = rt_delta_ws((int)D);
+  TORCH_CHECK(per > 0, "delta_rule: key width ", D, " above 256");
+  Tensor ws = at::empty({chunks->size(0) * H * per}, x.options().dtype(at::kFloat));
+  Tensor v = at::empty({N, H * V}, x.options()), o = at::empty({N, H * V}, x.options().dtype(at::kFloat));
+  rc_ok(rt_delta_runs(is_f32(x), &d, runs->data_ptr(), chunks->data_ptr(), first_chunk->data_ptr<int>(), (int)runs->size(0),
+                      (int)chunks->size(0), (int)n_single, (int)(N - n_single), ws.data_ptr<float>(), v.data_ptr(),
+                      o.data_ptr<float>(), stream()),
+        "delta_runs");
+}
+
 }  // namespace
 
 void bind_layered(py::module_& m) {
   m.def("branch_norm", &branch_norm, "x += rms(y) w_branch; h = rms(x) w_next (fp32 residual)", py::arg("x"), py::arg("kind"),
         py::arg("y") = py::none(), py::arg("nsplit") = 1, py::arg("w_branch") = py::none(), py::arg("w_next") = py::none(),
         py::arg("table") = py::none(), py::arg("ids") = py::none(), py::arg("pair_w") = py::none(),
-        py::arg("pair_pos") = py::none(), py::arg("eps"));
+        py::arg("pair_pos") = py::none(), py::arg("eps"), py::arg("scale") = py::none(), py::arg("next_mul") = 1.0,
+        py::arg("plain") = false);
   m.def("gemm_any", &gemm_any, "a w^T, any shape, bf16 / fp32, batched or grouped", py::arg("a"), py::arg("w"),
         py::arg("out_f32") = false, py::arg("out") = py::none(), py::arg("offs") = py::none(), py::arg("row_map") = py::none());
   m.def("head_gemm", &head_gemm, "per-head a w^T at few rows (gated)", py::arg("a"), py::arg("w"), py::arg("out"),
         py::arg("gate") = py::none());
   m.def("glu_any", &glu_any, "gated linear unit of [gate | up] rows");
+  m.def("act_any", &act_any, "activation of an fp32 product");
   m.def("gate_mul", &gate_mul, "a *= sigmoid(g)");
   m.def("moe_route", &moe_route, "softmax router with choice correction -> experts, weights", py::arg("logits"),
         py::arg("correction"), py::arg("top"), py::arg("nshared"), py::arg("gate_col"), py::arg("nslab") = 1);
@@ -455,5 +646,12 @@ void bind_layered(py::module_& m) {
   m.def("latent_merge", &latent_merge, "partition merge with the sink");
   m.def("latent_gather", &latent_gather, "cached rows of each segment, dense");
   m.def("latent_prefill", &latent_prefill, "flash attention of prompt portions over expanded keys / values");
+  m.def("window_prep", &window_prep, "q / k norm, rotation in halves, cache append");
+  m.def("window_decode_ok", [](int H, int G, int D, int V) { return rt_window_decode_ok(H, G, D, V) != 0; });
+  m.def("window_prefill_ok", [](int D, int V) { return rt_window_prefill_ok(D, V) != 0; });
+  m.def("window_decode", &window_decode, "windowed attention, few tokens per request");
+  m.def("window_prefill", &window_prefill, "windowed flash attention of prompt portions from the pages");
+  m.def("window_any", &window_any, "windowed attention, any size / type");
+  m.def("delta_rule", &delta_rule, "gated delta rule over a ragged batch");
   m.def("latent_any", &latent_any, "absorbed attention, any size / type");
 }

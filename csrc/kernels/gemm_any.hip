@@ -5,7 +5,7 @@
 // (K % 64 at few rows, K % 8, N % 8). 64x64 tile per workgroup, 4x4 outputs per thread, K-steps of 16
 // through LDS as fp32 with the next step's loads in flight during the products.
 //
-// Also here: the elementwise steps of that path (gated linear unit, output gate).
+// Also here: the elementwise steps of that path (gated linear unit, squared relu, output gate).
 #include "rt_common.h"
 
 namespace rt {
@@ -107,6 +107,19 @@ __global__ __launch_bounds__(256) void glu_any_kernel(const T* __restrict__ gu, 
   any_st(y + i, g / (1.f + expf(-(gp.alpha * g))) * (u + gp.offset));
 }
 
+// y = max(x, 0)^2 of an fp32 product (act 8), or a rounding copy (act 0)
+template <typename T>
+__global__ __launch_bounds__(256) void act_any_kernel(const float* __restrict__ x, T* __restrict__ y, long n, int act) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n) return;
+  float v = x[i];
+  if (act == 8) {
+    v = fmaxf(v, 0.f);
+    v *= v;
+  }
+  any_st(y + i, v);
+}
+
 // a [T, N] *= sigmoid(g [T, N]) (output gate of an attention layer)
 template <typename T>
 __global__ __launch_bounds__(256) void gate_mul_kernel(T* __restrict__ a, const T* __restrict__ g, long ldg, long n,
@@ -149,6 +162,16 @@ extern "C" int rt_glu_any(int f32, const void* gu, long ldg, void* y, long T, in
   dim3 grid((unsigned)((n + 255) / 256)), block(256);
   if (f32) hipLaunchKernelGGL((glu_any_kernel<float>), grid, block, 0, stream, (const float*)gu, ldg, (float*)y, n, F, gp);
   else hipLaunchKernelGGL((glu_any_kernel<bf16_t>), grid, block, 0, stream, (const bf16_t*)gu, ldg, (bf16_t*)y, n, F, gp);
+  RT_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int rt_act_any(int f32, const float* x, void* y, long n, int act, hipStream_t stream) {
+  if (n <= 0) return 0;
+  if (act != 0 && act != 8) return -1;
+  dim3 grid((unsigned)((n + 255) / 256)), block(256);
+  if (f32) hipLaunchKernelGGL((act_any_kernel<float>), grid, block, 0, stream, x, (float*)y, n, act);
+  else hipLaunchKernelGGL((act_any_kernel<bf16_t>), grid, block, 0, stream, x, (bf16_t*)y, n, act);
   RT_LAUNCH_CHECK();
   return 0;
 }

@@ -27,7 +27,8 @@ enum Act { ACT_NONE = 0, ACT_RELU = 1, ACT_GELU = 2, ACT_GELU_TANH = 3, ACT_SILU
            // skinny kernels only: B = fused [gate; up] weight (2F rows), C[M, F] = silu(X gate^T) * (X up^T).
            // Column group g reads gate rows [32g, 32g+32) and up rows [F+32g, F+32g+32), so the pair of
            // every output lands in one lane (SwiGLU fused into the gate/up GEMM of a decode step)
-           ACT_SWIGLU = 5 };
+           ACT_SWIGLU = 5,
+           ACT_RELU2 = 8 };  // max(x, 0)^2
 
 __device__ __forceinline__ float apply_act(float x, int act) {
   switch (act) {
@@ -38,6 +39,7 @@ __device__ __forceinline__ float apply_act(float x, int act) {
       return 0.5f * x * (1.f + tanhf(k0 * (x + k1 * x * x * x)));
     }
     case ACT_SILU: return x / (1.f + __expf(-x));
+    case ACT_RELU2: { const float r = fmaxf(x, 0.f); return r * r; }
     default: return x;
   }
 }

@@ -62,7 +62,8 @@ enum Out { O_BF16 = 0, O_F32 = 1, O_F32_ATOMIC = 2, O_F32_SLAB = 3 };
 // rotate by the angle table row rope_pos[row] (cos / sin [positions, rope_d / 2] fp32). A head never
 // straddles a tile (rope_d divides 128), so both halves are in the LDS-staged tile. Arithmetic of
 // rope_qkv_kernel (sign +1) on the bf16-rounded GEMM output: bitwise the GEMM + rope pair.
-enum Epi { E_NONE = 0, E_RELU = 1, E_GELU = 2, E_GELU_TANH = 3, E_SILU = 4, E_SWIGLU = 5, E_DSWIGLU = 6, E_ROPE = 7 };
+enum Epi { E_NONE = 0, E_RELU = 1, E_GELU = 2, E_GELU_TANH = 3, E_SILU = 4, E_SWIGLU = 5, E_DSWIGLU = 6, E_ROPE = 7,
+           E_RELU2 = 8 };  // max(x, 0)^2
 
 struct Args {
   const bf16_t* A; long lda;
@@ -110,6 +111,7 @@ __device__ __forceinline__ float act_fn(float x, int act) {
       return 0.5f * x * (1.f + tanhf(k0 * (x + k1 * x * x * x)));
     }
     case E_SILU: return x / (1.f + __expf(-x));
+    case E_RELU2: { const float r = fmaxf(x, 0.f); return r * r; }
     default: return x;
   }
 }
@@ -871,6 +873,7 @@ static int launch_gemm_big(const Args& p, int layout_a, int layout_b, int act, i
       case 0: GB_LAUNCH(ROW, ROW, O_BF16, E_NONE, 128); break;
       case E_SWIGLU: GB_LAUNCH(ROW, ROW, O_BF16, E_SWIGLU, 128); break;
       case E_ROPE: GB_LAUNCH(ROW, ROW, O_BF16, E_ROPE, 128); break;
+      case E_RELU2: GB_LAUNCH(ROW, ROW, O_BF16, E_RELU2, 128); break;
       case 10: GB_LAUNCH(ROW, ROW, O_F32, E_NONE, 128); break;
       case 30: GB_LAUNCH(ROW, ROW, O_F32_SLAB, E_NONE, 128); break;
       case 100: GB_LAUNCH(ROW, KMAJ, O_BF16, E_NONE, 128); break;
@@ -886,6 +889,7 @@ static int launch_gemm_big(const Args& p, int layout_a, int layout_b, int act, i
       case E_SILU: GB_LAUNCH(ROW, ROW, O_BF16, E_SILU, 256); break;
       case E_SWIGLU: GB_LAUNCH(ROW, ROW, O_BF16, E_SWIGLU, 256); break;
       case E_ROPE: GB_LAUNCH(ROW, ROW, O_BF16, E_ROPE, 256); break;
+      case E_RELU2: GB_LAUNCH(ROW, ROW, O_BF16, E_RELU2, 256); break;
       default: return -4;
     }
   } else if (key == 10 && act == E_DSWIGLU) {
@@ -912,7 +916,7 @@ static int launch_gemm_big(const Args& p, int layout_a, int layout_b, int act, i
 
 static bool bn128_supported(int layout_a, int layout_b, int act, int out) {
   const int key = layout_a * 100 + layout_b * 10 + out;
-  return (key == 0 && (act == E_NONE || act == E_SWIGLU || act == E_ROPE)) ||
+  return (key == 0 && (act == E_NONE || act == E_SWIGLU || act == E_ROPE || act == E_RELU2)) ||
          (act == E_NONE && (key == 1 || key == 3 || key == 10)) || (key == 10 && act == E_DSWIGLU);
 }
 

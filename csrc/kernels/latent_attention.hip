@@ -15,39 +15,14 @@
 // and run a flash kernel over [unrotated | rotated] heads:
 //   latent_prep -> latent_gather -> (expand GEMM) -> latent_prefill
 // latent_any is the absorbed attention for any size and for fp32 (one workgroup per token and head).
-#include "rt_common.h"
+#include "rt_paged.h"
 
 #include <algorithm>
 
 namespace rt {
 namespace la {
 
-typedef __attribute__((address_space(3))) void lds_void;
-constexpr int PAGE = 64;
-
-template <typename T> __device__ __forceinline__ float ld(const T* p);
-template <> __device__ __forceinline__ float ld<bf16_t>(const bf16_t* p) { return bf2f(*p); }
-template <> __device__ __forceinline__ float ld<float>(const float* p) { return *p; }
-template <typename T> __device__ __forceinline__ void st(T* p, float v);
-template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
-template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
-
-// v_exp_f32: arguments here are <= 0 (or -inf -> 0), where the library function's range handling does nothing
-__device__ __forceinline__ float fexp2(float x) { return __builtin_amdgcn_exp2f(x); }
-
-__device__ __forceinline__ bf16x8 pack_p(const f32x4& a, const f32x4& b) {
-  uint4 v;
-  v.x = pack2bf(a[0], a[1]);
-  v.y = pack2bf(a[2], a[3]);
-  v.z = pack2bf(b[0], b[1]);
-  v.w = pack2bf(b[2], b[3]);
-  return __builtin_bit_cast(bf16x8, v);
-}
-__device__ __forceinline__ bf16x8 cat4(const rt_s16x4& lo, const rt_s16x4& hi) {
-  typedef __attribute__((ext_vector_type(8))) short s16x8;
-  s16x8 v = {lo[0], lo[1], lo[2], lo[3], hi[0], hi[1], hi[2], hi[3]};
-  return __builtin_bit_cast(bf16x8, v);
-}
+using namespace paged;
 
 // ---------------------------------------------------------------------------------------------
 // prep: latent norm + rotation + cache append (layers with a latent of their own), query rotation
@@ -400,55 +375,8 @@ __global__ __launch_bounds__(256, 2) void latent_decode_kernel(DecArgs a) {
 }
 
 // ---------------------------------------------------------------------------------------------
-// merge of the partitions, with the sink in the denominator: one workgroup per (token, head)
-// ---------------------------------------------------------------------------------------------
-constexpr int MERGE_MAX = 1024;  // partitions
-
-__global__ __launch_bounds__(128) void latent_merge_kernel(const float* __restrict__ part, const float* __restrict__ ml,
-                                                           const float* __restrict__ sink, bf16_t* __restrict__ o, int H,
-                                                           int rank, int NP) {
-  __shared__ float fac[MERGE_MAX];
-  __shared__ float sbuf[2];
-  const long th = blockIdx.x;
-  const int tid = threadIdx.x;
-  const float sink2 = sink[th % H] * 1.4426950408889634f;
-  const float* m = ml + th * NP * 2;
-  float mx = -INFINITY;
-  for (int p = tid; p < NP; p += 128) {
-    fac[p] = m[2 * p];
-    mx = fmaxf(mx, fac[p]);
-  }
-  const float M = fmaxf(block_max(mx, sbuf), sink2);
-  float L = 0.f;
-  for (int p = tid; p < NP; p += 128) {
-    fac[p] = exp2f(fac[p] - M);  // 0 for an empty partition
-    L += m[2 * p + 1] * fac[p];
-  }
-  const float inv = 1.f / (block_sum(L, sbuf) + exp2f(sink2 - M));
-  for (int c = 4 * tid; c < rank; c += 512) {  // rank % 8 == 0
-    float y[4] = {0.f, 0.f, 0.f, 0.f};
-    for (int p0 = 0; p0 < NP; p0 += 8) {  // eight partitions' rows in flight
-      float4 v[8];
-#pragma unroll
-      for (int j = 0; j < 8; ++j) v[j] = *(const float4*)(part + (th * NP + min(p0 + j, NP - 1)) * rank + c);
-#pragma unroll
-      for (int j = 0; j < 8; ++j) {
-        const float f = p0 + j < NP ? fac[p0 + j] : 0.f;
-        if (f != 0.f) {  // an empty partition wrote nothing
-          y[0] = fmaf(f, v[j].x, y[0]); y[1] = fmaf(f, v[j].y, y[1]);
-          y[2] = fmaf(f, v[j].z, y[2]); y[3] = fmaf(f, v[j].w, y[3]);
-        }
-      }
-    }
-    *(uint2*)(o + th * rank + c) = make_uint2(pack2bf(y[0] * inv, y[1] * inv), pack2bf(y[2] * inv, y[3] * inv));
-  }
-}
-
-// ---------------------------------------------------------------------------------------------
 // segments of longer portions
 // ---------------------------------------------------------------------------------------------
-struct Seg { int row, q_off, q_len, kv_off, kv_len, pos0, pad0, pad1; };  // 8 ints
-
 // out [kv rows of all segments, KD] = the cached rows of each segment, dense
 template <typename V>
 __global__ __launch_bounds__(256) void latent_gather_kernel(const V* __restrict__ pool, const int* __restrict__ tab,
@@ -480,26 +408,6 @@ struct PreArgs {
   int H, dim, rot, vdim;
   float scale_log2;
 };
-
-// LDS image of a K (V) tile: rows of DQ (DV) elements, 16-B chunk c of row r at slot c ^ swizzle(r) (an
-// involution, so the same function maps slots back to chunks). K: row reads conflict-free; V: transposed reads.
-template <int DQ>
-__device__ __forceinline__ int kq_chunk(int r, int c) {
-  return c ^ ((DQ / 64) % 2 ? ((r >> 1) & 7) : (r & 15 & (DQ / 8 - 1)));
-}
-template <int DQ>
-__device__ __forceinline__ int kq_off(int r, int c) {
-  return r * (DQ * 2) + (kq_chunk<DQ>(r, c) << 4);
-}
-template <int DV>
-__device__ __forceinline__ int vv_chunk(int r, int c) {
-  constexpr int NCH = DV / 8, RPB = 128 / DV;
-  return c ^ (((r / RPB) & (NCH / 2 - 1)) << 1);
-}
-template <int DV>
-__device__ __forceinline__ int vv_off(int r, int c) {
-  return r * (DV * 2) + (vv_chunk<DV>(r, c) << 4);
-}
 
 template <int DQ, int DV>
 __global__ __launch_bounds__(256, 2) void latent_prefill_kernel(PreArgs a) {
@@ -827,16 +735,6 @@ extern "C" int rt_latent_decode(const void* q, const void* pool, const int* tab,
     if (KD <= 576) LD_(9, 8); else LD_(10, 8);
   }
 #undef LD_
-  RT_LAUNCH_CHECK();
-  return 0;
-}
-
-extern "C" int rt_latent_merge(const float* part, const float* ml, const float* sink, void* o, int T, int H, int rank,
-                               int NP, hipStream_t stream) {
-  if (T <= 0) return 0;
-  if (rank % 8 || NP < 1 || NP > MERGE_MAX) return -1;
-  hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((long)T * H)), dim3(128), 0, stream, part, ml, sink, (bf16_t*)o,
-                     H, rank, NP);
   RT_LAUNCH_CHECK();
   return 0;
 }

@@ -272,16 +272,18 @@ extern "C" int rt_norm_bwd(int layernorm, const void* dy, const void* h, const v
 }
 
 // ---------------------------------------------------------------------------------------------
-// Branch norm: the step between two sublayers of a decoder with a norm before and after each
+// Branch norm: the step between two sublayers of a decoder with a norm after each, and maybe one before
 // (fp32 residual stream x [T, H], everything in fp32):
-//   x += rms(y) * w_branch          (y = the sublayer's output)
-//   h  = rms(x) * w_next            (the next sublayer's input, rounded once to the activation type)
+//   x += rms(y) * w_branch [* scale]     (y = the sublayer's output)
+//   h  = rms(x) * w_next * next_mul      (the next sublayer's input, rounded once to the activation type)
+//   h  = x                               (w_next == null: sublayers that read the stream itself)
 // One workgroup per row, the row in registers: x is read and written once, y read once. The branch y is
-//   Y_NONE    absent (first norm of a pass): x = table[ids[row]] when a table is given;
+//   Y_NONE    absent (first norm of a pass): x = table[ids[row]] when a table is given, normed and weighted
+//             with w_branch if there is one;
 //   Y_ACT     rows of the activation type;
 //   Y_SLABS   the sum of nsplit fp32 slabs (split-K partial products; 1 slab = an fp32 tensor);
 //   Y_PAIRS   a mixture: sum over the row's K slots of pair_w[row, k] * y[pair_pos[row, k]].
-// w_next == null: no h (x only).
+// h == null: x only.
 // ---------------------------------------------------------------------------------------------
 namespace rt {
 
@@ -290,7 +292,7 @@ enum BranchKind { Y_NONE = 0, Y_ACT = 1, Y_SLABS = 2, Y_PAIRS = 3, Y_PAIRS_F32 =
 struct BranchArgs {
   float* x;
   const void* y; long y_stride; int nsplit;  // Y_SLABS: slab stride in floats
-  const void* w_branch; const void* w_next; void* h;
+  const void* w_branch; const void* scale; const void* w_next; float next_mul; void* h;
   const void* table; const long* ids; int vocab;
   const float* pair_w; const int* pair_pos; int K;
   int H;
@@ -383,7 +385,19 @@ __global__ __launch_bounds__(512) void branch_norm_kernel(BranchArgs a) {
       }
     }
 #pragma unroll
-    for (int e = 0; e < V; ++e) s += y[i][e] * y[i][e];
+    for (int e = 0; e < V; ++e) s += KIND == Y_NONE ? x[i][e] * x[i][e] : y[i][e] * y[i][e];
+  }
+  if (KIND == Y_NONE && a.table && a.w_branch) {
+    const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c >= nvec) continue;
+      float w[V];
+      act_ldv<T, V>((const T*)a.w_branch + c * V, w);
+#pragma unroll
+      for (int e = 0; e < V; ++e) x[i][e] *= rstd * w[e];
+    }
   }
   if constexpr (KIND != Y_NONE) {
     const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
@@ -393,6 +407,12 @@ __global__ __launch_bounds__(512) void branch_norm_kernel(BranchArgs a) {
       if (c >= nvec) continue;
       float w[V];
       act_ldv<T, V>((const T*)a.w_branch + c * V, w);
+      if (a.scale) {
+        float f[V];
+        act_ldv<T, V>((const T*)a.scale + c * V, f);
+#pragma unroll
+        for (int e = 0; e < V; ++e) w[e] *= f[e];
+      }
 #pragma unroll
       for (int e = 0; e < V; ++e) x[i][e] += y[i][e] * rstd * w[e];
     }
@@ -404,13 +424,21 @@ __global__ __launch_bounds__(512) void branch_norm_kernel(BranchArgs a) {
       if (c < nvec) act_stv<float, V>(xr + c * V, x[i]);
     }
   }
-  if (!a.w_next) return;
+  if (!a.h) return;
+  if (!a.w_next) {
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = threadIdx.x + i * blockDim.x;
+      if (c < nvec) act_stv<T, V>((T*)a.h + row * a.H + c * V, x[i]);
+    }
+    return;
+  }
   s = 0.f;
 #pragma unroll
   for (int i = 0; i < NV; ++i)
 #pragma unroll
     for (int e = 0; e < V; ++e) s += x[i][e] * x[i][e];
-  const float rstd = 1.f / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
+  const float rstd = a.next_mul / sqrtf(block_sum(s, sbuf) / a.H + a.eps);
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
     const int c = threadIdx.x + i * blockDim.x;
@@ -448,11 +476,11 @@ static int launch_branch(const BranchArgs& a, int Tn, hipStream_t st) {
 }  // namespace rt
 
 extern "C" int rt_branch_norm(int f32, int kind, float* x, const void* y, long y_stride, int nsplit,
-                              const void* w_branch, const void* w_next, void* h, const void* table, const long* ids,
-                              int vocab, const float* pair_w, const int* pair_pos, int K, int T, int H, float eps,
+                              const void* w_branch, const void* scale, const void* w_next, float next_mul, void* h,
+                              const void* table, const long* ids, int vocab, const float* pair_w, const int* pair_pos, int K, int T, int H, float eps,
                               hipStream_t stream) {
   if (T <= 0) return 0;
-  rt::BranchArgs a{x, y, y_stride, nsplit, w_branch, w_next, h, table, ids, vocab, pair_w, pair_pos, K, H, eps};
+  rt::BranchArgs a{x, y, y_stride, nsplit, w_branch, scale, w_next, next_mul, h, table, ids, vocab, pair_w, pair_pos, K, H, eps};
   int rc = -1;
 #define BK(KIND) rc = f32 ? rt::launch_branch<float, rt::KIND>(a, T, stream) : rt::launch_branch<rt::bf16_t, rt::KIND>(a, T, stream)
   switch (kind) {

@@ -14,6 +14,7 @@ portions beside the decoding rows, and their decode step is captured like the ot
 """
 from __future__ import annotations
 
+import contextlib
 from dataclasses import dataclass, field
 from typing import List, Optional, Sequence
 
@@ -377,8 +378,10 @@ class Generator:
         key = (T, params.inv_temp, params.top_k, params.top_p, params.greedy, params.seed, tuple(eos_list), pad_id,
                self._nb)
         if self.use_graph and self.runner.needs(key):
-            # the EOS tensor is created per call: the runner keeps the captured one alive
-            self.runner.capture(lambda: self._step(params, eos, pad_id), key, keep=(eos,), restore=self._state())
+            # the EOS tensor is created per call: the runner keeps the captured one alive. Recurrent states
+            # must not advance in the warm-up: its rows are parked
+            with self.cache.parked() if self.ragged else contextlib.nullcontext():
+                self.runner.capture(lambda: self._step(params, eos, pad_id), key, keep=(eos,), restore=self._state())
 
     def _replay(self, params, eos, pad_id):
         if self.use_graph:

@@ -1,11 +1,13 @@
 """Paged cache: per layer a pool of pages of 64 tokens, and one page table row per request.
 
 The pool is sized for the tokens that live requests hold at any time (each rounded up to whole pages), not
-for rows x longest sequence. Page 0 belongs to nobody: table entries without a page point at it, so a
+for rows x longest sequence. Layers with recurrent state have one slot per row beside it: tensors
+[rows, ...] that belong to the row's request and count as zero at its position 0. Page 0 belongs to nobody: table entries without a page point at it, so a
 decode graph's idle rows write there. Pools start as zeros and only ever hold finite values, so masked
 keys of a reused page are harmless. Allocation is host bookkeeping; ``sync`` uploads the table."""
 from __future__ import annotations
 
+import contextlib
 from typing import List, Optional
 
 import numpy as np
@@ -16,15 +18,18 @@ PAGE = 64
 
 class PagedCache:
     def __init__(self, widths: List[int], rows: int, max_seq: int, tokens: Optional[int] = None, device="cpu",
-                 dtype=torch.bfloat16):
+                 dtype=torch.bfloat16, states=None):
         """``widths``: cached elements per token of every layer (0: no cache of its own); ``tokens``: capacity
-        of the pool (default rows x max_seq)."""
+        of the pool (default rows x max_seq); ``states``: per layer the (shape, dtype) of its state tensors'
+        slots."""
         self.rows = rows
         self.max_pages = max(1, (max_seq + PAGE - 1) // PAGE)
         self.max_seq = self.max_pages * PAGE
         cap = rows * self.max_pages if tokens is None else (tokens + PAGE - 1) // PAGE
         self.n_pages = cap + 1
         self._pools = [torch.zeros(self.n_pages, PAGE, w, device=device, dtype=dtype) if w else None for w in widths]
+        self._states = [tuple(torch.zeros(rows, *shape, device=device, dtype=dt) for shape, dt in s)
+                        for s in (states or [()] * len(widths))]
         self._host = np.zeros((rows, self.max_pages), dtype=np.int32)
         self.table = torch.zeros(rows, self.max_pages, dtype=torch.int32, device=device)
         self.row_ids = torch.arange(rows, dtype=torch.int32, device=device)
@@ -35,9 +40,24 @@ class PagedCache:
     def pool(self, layer: int) -> torch.Tensor:
         return self._pools[layer]
 
+    def state(self, layer: int):
+        """the layer's state tensors, [rows, ...] each"""
+        return self._states[layer]
+
     @property
     def nbytes(self) -> int:
-        return sum(p.numel() * p.element_size() for p in self._pools if p is not None)
+        held = [p for p in self._pools if p is not None] + [t for s in self._states for t in s]
+        return sum(p.numel() * p.element_size() for p in held)
+
+    @contextlib.contextmanager
+    def parked(self):
+        """No row takes part: a decode step of ``rows_view`` that runs inside (a graph's warm-up) neither
+        appends to the pools nor advances a state."""
+        self.row_ids.fill_(-1)
+        try:
+            yield
+        finally:
+            self.row_ids.copy_(torch.arange(self.rows, dtype=torch.int32))
 
     def free_tokens(self) -> int:
         return len(self.free) * PAGE
@@ -86,4 +106,4 @@ class PagedRows:
     def __init__(self, cache: PagedCache, row0: int, n: int):
         self.table, self.max_seq = cache.table, cache.max_seq
         self.row_ids = cache.row_ids[row0:row0 + n]
-        self.pool = cache.pool
+        self.pool, self.state = cache.pool, cache.state

@@ -1,7 +1,8 @@
 """Ragged batches: portions of prompts beside single decoded tokens, one step of the model for all of them.
 
-``RaggedBatch`` is the device form of a step: token ids, cache rows and positions (entries with short
-portions first), plus the segment and query-tile tables of the longer ones. ``StepEngine`` is the step
+``RaggedBatch`` is the device form of a step: token ids, cache rows and positions (single tokens first, then
+short portions, then longer ones), the segment and query-tile tables of the longer ones for attention, and the
+runs and chunks of everything above one token for recurrent layers. ``StepEngine`` is the step
 function over a paged cache with explicit tokens: requests are admitted into rows, advanced by any
 portions, and released; sampling loops (``Generator``, ``ContinuousBatcher``) drive the same model step."""
 from __future__ import annotations
@@ -13,30 +14,37 @@ import torch
 
 SHORT_TOKENS = 32   # portions up to this many tokens attend in the absorbed form, token by token
 QUERY_TILE = 128    # query rows per workgroup of the portions' attention kernel
+CHUNK = 16          # tokens per chunk of a recurrent layer's portions (csrc/kernels/delta_rule.hip)
 
 
 class RaggedBatch:
-    __slots__ = ("ids", "row", "pos", "n_short", "segs", "tiles", "kv_total", "max_kv", "max_len", "offset")
+    __slots__ = ("ids", "row", "pos", "n_single", "n_short", "segs", "tiles", "kv_total", "max_kv", "max_len", "offset",
+                 "runs", "chunks", "first_chunk")
 
-    def __init__(self, ids, row, pos, n_short, max_len, segs=None, tiles=None, kv_total=0, max_kv=0, offset=()):
-        self.ids, self.row, self.pos, self.n_short = ids, row, pos, n_short
+    def __init__(self, ids, row, pos, n_single, n_short, max_len, segs=None, tiles=None, kv_total=0, max_kv=0, offset=(),
+                 runs=None, chunks=None, first_chunk=None):
+        self.ids, self.row, self.pos = ids, row, pos
+        self.n_single, self.n_short = n_single, n_short  # tokens of one-token entries, and with the short portions'
         self.segs, self.tiles, self.kv_total, self.max_kv = segs, tiles, kv_total, max_kv
         self.max_len = max_len      # keys of the longest short token's request (bound)
         self.offset = offset        # first token of every entry, in the order given
+        # entries of two and more tokens: {row, first token, tokens, position} each, {run, chunk of the run} each,
+        # every run's first chunk
+        self.runs, self.chunks, self.first_chunk = runs, chunks, first_chunk
 
     @classmethod
     def single(cls, tokens, rows, pos, max_len: int) -> "RaggedBatch":
         """One token per row, everything on the device already (decode)."""
-        return cls(tokens, rows, pos, tokens.shape[0], max_len)
+        return cls(tokens, rows, pos, tokens.shape[0], tokens.shape[0], max_len)
 
     @classmethod
     def build(cls, entries: Sequence[Tuple[int, Sequence[int], int]], device) -> "RaggedBatch":
         """``entries``: (cache row, tokens, position of the first)."""
         lens = np.array([len(t) for _, t, _ in entries], dtype=np.int64)
-        order = np.argsort(lens > SHORT_TOKENS, kind="stable")
+        order = np.argsort((lens > 1).astype(np.int64) + (lens > SHORT_TOKENS), kind="stable")
         offset = np.zeros(len(entries), dtype=np.int64)
-        n, kv, max_len, n_short = 0, 0, 1, 0
-        segs, tiles, parts_i, parts_r, parts_p = [], [], [], [], []
+        n, kv, max_len, n_single, n_short = 0, 0, 1, 0, 0
+        segs, tiles, runs, parts_i, parts_r, parts_p = [], [], [], [], [], []
         max_kv = 0
         for e in order:
             row, toks, start = entries[e]
@@ -45,6 +53,10 @@ class RaggedBatch:
             parts_i.append(np.asarray(toks, dtype=np.int32))
             parts_r.append(np.full(L, row, dtype=np.int32))
             parts_p.append(np.arange(start, start + L, dtype=np.int32))
+            if L > 1:
+                runs.append((row, n, L, start))
+            else:
+                n_single += 1
             if L <= SHORT_TOKENS:
                 n_short += L
             else:
@@ -55,15 +67,19 @@ class RaggedBatch:
             max_len = max(max_len, start + L)
             n += L
         tiles = [t[1:] for t in sorted(tiles, key=lambda t: -t[0])]  # heaviest first
-        pad = -3 * n % 4
-        flat = np.concatenate(parts_i + parts_r + parts_p + [np.zeros(pad, np.int32),
-                                                             np.asarray(segs, np.int32).reshape(-1),
-                                                             np.asarray(tiles, np.int32).reshape(-1)])
+        per = np.array([(r[2] + CHUNK - 1) // CHUNK for r in runs], dtype=np.int64)
+        first = np.concatenate([np.zeros(1, np.int64), np.cumsum(per)])
+        chunks = np.stack([np.repeat(np.arange(len(runs)), per), np.arange(int(first[-1])) - np.repeat(first[:-1], per)], 1)
+        tables = [np.asarray(segs, np.int32).reshape(-1, 8), np.asarray(runs, np.int32).reshape(-1, 4),
+                  np.asarray(tiles, np.int32).reshape(-1, 2), chunks.astype(np.int32), first[:-1].astype(np.int32)]
+        flat = np.concatenate(parts_i + parts_r + parts_p + [np.zeros(-3 * n % 4, np.int32)] + [t.reshape(-1) for t in tables])
         buf = torch.from_numpy(flat).to(device)
-        at = 3 * n + pad
-        st = buf[at:at + 8 * len(segs)].view(-1, 8) if segs else None
-        tt = buf[at + 8 * len(segs):].view(-1, 2) if segs else None
-        return cls(buf[:n].long(), buf[n:2 * n], buf[2 * n:3 * n], n_short, max_len, st, tt, kv, max_kv, offset)
+        at, dev = 3 * n + -3 * n % 4, []
+        for t in tables:
+            dev.append(buf[at:at + t.size].view(t.shape) if t.size else None)
+            at += t.size
+        st, rt, tt, ct, ft = dev
+        return cls(buf[:n].long(), buf[n:2 * n], buf[2 * n:3 * n], n_single, n_short, max_len, st, tt, kv, max_kv, offset, rt, ct, ft)
 
 
 class StepEngine:

@@ -1,4 +1,4 @@
-"""Model zoo: Llama-2 / Mistral / OPT decoders, layered decoders (Vezatar), BERT / MPNet sentence encoders, LoRA, value head."""
+"""Model zoo: Llama-2 / Mistral / OPT decoders, layered decoders (Vezatar, Pafolorn), BERT / MPNet sentence encoders, LoRA, value head."""
 from __future__ import annotations
 
 import os

@@ -13,7 +13,8 @@ from typing import Callable, Dict, List, Tuple
 
 import torch
 
-from .config import ModelConfig, config_from_hf, config_to_hf
+from .config import (LatentAttentionSpec, ModelConfig, ParallelSpec, WindowAttentionSpec, config_from_hf, config_to_hf,
+                     with_ranks)
 
 # (hf_name, native_param_name, row_start, row_count) ; row_count None = whole tensor
 Mapping = List[Tuple[str, str, int, int]]
@@ -88,37 +89,88 @@ def encoder_mapping(cfg: ModelConfig) -> Mapping:
 
 
 class Part:
-    """A piece of a checkpoint tensor that a native parameter holds: rows [row0, row0 + rows) of the (2-D
-    or 1-D) parameter, ``dim`` / ``start`` / the parameter side's size selecting the tensor's slice."""
+    """A piece of a checkpoint tensor that a native parameter holds: rows [row0, row0 + rows) and columns
+    [col0, col0 + cols) of the (2-D or 1-D) parameter; ``dim`` / ``start`` / ``size`` select the tensor's
+    slice."""
 
-    __slots__ = ("name", "param", "row0", "rows", "dim", "start", "size")
+    __slots__ = ("name", "param", "row0", "rows", "dim", "start", "size", "col0", "cols")
 
-    def __init__(self, name, param, row0=0, rows=None, dim=None, start=0, size=None):
+    def __init__(self, name, param, row0=0, rows=None, dim=None, start=0, size=None, col0=0, cols=None):
         self.name, self.param, self.row0, self.rows = name, param, row0, rows
         self.dim, self.start, self.size = dim, start, size
+        self.col0, self.cols = col0, size if dim == 1 and cols is None else cols
+
+    def of(self, t: torch.Tensor) -> torch.Tensor:
+        """The part's place in the native parameter ``t``."""
+        if self.rows is not None:
+            t = t[self.row0:self.row0 + self.rows]
+        return t if self.cols is None else t[:, self.col0:self.col0 + self.cols]
+
+
+def _latent_parts(L: str, n: str, x: LatentAttentionSpec) -> List[Part]:
+    nq, nk, ng = x.heads * (x.dim + x.rot_dim), x.kv_rank + x.rot_dim, x.heads * x.vdim
+    own = x.kv_from is None
+    m = [Part(f"{L}.q", f"{n}.in_w", 0, nq), Part(f"{L}.g", f"{n}.in_w", nq + (nk if own else 0), ng),
+         Part(f"{L}.uk", f"{n}.kv_up_w", 0, x.heads * x.dim), Part(f"{L}.uv", f"{n}.kv_up_w", x.heads * x.dim, ng),
+         Part(f"{L}.sink", f"{n}.sink"), Part(f"{L}.o", f"{n}.o_w")]
+    if own:
+        m += [Part(f"{L}.dkv", f"{n}.in_w", nq, nk), Part(f"{L}.dkv.norm", f"{n}.latent_norm_w")]
+    return m
+
+
+def _branch_parts(L: str, n: str, spec) -> List[Part]:
+    """One mixer, or two side by side: input projections stacked, output projections side by side."""
+    from .layered import in_layout, out_layout
+
+    m = []
+    pair = isinstance(spec, ParallelSpec)
+    rows, _ = in_layout(spec)
+    cols, _ = out_layout(spec)
+    for side, x in ((("left", spec.left), ("right", spec.right)) if pair else (("mix", spec),)):
+        t = f"{L}.{side}" if pair else L
+        m += [Part(f"{t}.{k}", f"{n}.in_w", r0, rn) for k, (r0, rn) in rows[side].items()]
+        m.append(Part(f"{t}.o", f"{n}.o_w", col0=cols[side][0], cols=cols[side][1]))
+        q = f"{n}.{side}"
+        if isinstance(x, WindowAttentionSpec):
+            m += [Part(f"{t}.q.norm", f"{q}.q_norm_w"), Part(f"{t}.k.norm", f"{q}.k_norm_w")]
+            continue
+        c0 = 0
+        for k, c in (("q", x.kv_heads * x.dim), ("k", x.kv_heads * x.dim), ("v", x.heads * x.vdim)):
+            m.append(Part(f"{t}.{k}.conv", f"{q}.conv_w", c0, c))
+            c0 += c
+        m += [Part(f"{t}.A_log", f"{q}.A_log"), Part(f"{t}.dt_bias", f"{q}.dt_bias"), Part(f"{t}.norm", f"{q}.out_norm_w")]
+        if x.channel:
+            m += [Part(f"{t}.a2", f"{q}.a2_w", cols=x.a_rank), Part(f"{t}.g2", f"{q}.g2_w", cols=x.g_rank)]
+    return m
 
 
 def layered_mapping(cfg: ModelConfig) -> List[Part]:
-    """Tensor names of a layered decoder -> its fused parameters: [q | dkv | g] and [uk; uv] as one
-    projection each, experts stacked, the shared expert cut into parts of an expert's width behind them."""
-    m = [Part("embed", "embed"), Part("head", "lm_head"), Part("final.norm", "norm_w")]
+    """Tensor names of a layered decoder -> its fused parameters: the projections of a mixer's input as one
+    matrix, [uk; uv] and the taps of q, k and v as one each, experts stacked, the shared expert cut into
+    parts of an expert's width behind them."""
+    m = [Part("embed", "embed"), Part("final.norm", "norm_w")]
+    if not cfg.tie_embeddings:
+        m.append(Part("head", "lm_head"))
+    if cfg.embed_norm:
+        m.append(Part("embed.norm", "embed_norm_w"))
     for i, s in enumerate(cfg.layers):
-        L, n, x = f"l{i}", f"layers.{i}", s.mixer
-        nq, nk, ng = x.heads * (x.dim + x.rot_dim), x.kv_rank + x.rot_dim, x.heads * x.vdim
-        own = x.kv_from is None
-        m += [Part(f"{L}.norm1", f"{n}.norm1_w"), Part(f"{L}.norm1b", f"{n}.norm1b_w"),
-              Part(f"{L}.mix.q", f"{n}.mix.in_w", 0, nq), Part(f"{L}.mix.g", f"{n}.mix.in_w", nq + (nk if own else 0), ng),
-              Part(f"{L}.mix.uk", f"{n}.mix.kv_up_w", 0, x.heads * x.dim),
-              Part(f"{L}.mix.uv", f"{n}.mix.kv_up_w", x.heads * x.dim, ng),
-              Part(f"{L}.mix.sink", f"{n}.mix.sink"), Part(f"{L}.mix.o", f"{n}.mix.o_w")]
-        if own:
-            m += [Part(f"{L}.mix.dkv", f"{n}.mix.in_w", nq, nk), Part(f"{L}.mix.dkv.norm", f"{n}.mix.latent_norm_w")]
+        L, n = f"l{i}", f"layers.{i}"
+        latent = isinstance(s.mixer, LatentAttentionSpec)
+        m += (_latent_parts if latent else _branch_parts)(f"{L}.mix", f"{n}.mix", s.mixer)
         f = s.mlp
+        for j in "12" if f is not None else "1":
+            m.append(Part(f"{L}.norm{j}", f"{n}.norm{j}_w"))
+            if cfg.norms == "both":
+                m.append(Part(f"{L}.norm{j}b", f"{n}.norm{j}b_w"))
+            if cfg.layer_scale:
+                m.append(Part(f"{L}.ls{j}", f"{n}.ls{j}"))
         if f is None:
             continue
-        m += [Part(f"{L}.norm2", f"{n}.norm2_w"), Part(f"{L}.norm2b", f"{n}.norm2b_w")]
         p = f"{L}.mlp"
         W = cfg.hidden_size
+        if f.kind == "relu2":
+            m += [Part(f"{p}.up", f"{n}.mlp.up_w"), Part(f"{p}.down", f"{n}.mlp.down_w")]
+            continue
         if f.kind == "dense":
             m += [Part(f"{p}.gate", f"{n}.mlp.gate_up_w", 0, f.ff), Part(f"{p}.up", f"{n}.mlp.gate_up_w", f.ff, f.ff),
                   Part(f"{p}.down", f"{n}.mlp.down_w")]
@@ -149,14 +201,10 @@ def load_layered_state_dict(model, sd: Dict[str, torch.Tensor]):
         raise KeyError(f"checkpoint tensors do not fit the config: missing {missing[:6]}, unexpected {extra[:6]}")
     left = {}
     for p in parts:
-        src, dst = sd[p.name], params[p.param]
-        if p.rows is not None:
-            dst = dst[p.row0:p.row0 + p.rows]
+        src, dst = sd[p.name], p.of(params[p.param])
         left[p.name] = left.get(p.name, src.numel())
         if p.dim is not None:
             src = src.narrow(p.dim, p.start, p.size)
-            if p.dim == 1:
-                dst = dst[:, :p.size]
         if tuple(src.shape) != tuple(dst.shape):
             raise ValueError(f"{p.name}: shape {tuple(sd[p.name].shape)} does not fit the config")
         left[p.name] -= src.numel()
@@ -169,11 +217,7 @@ def layered_state_dict(model, dtype=None) -> Dict[str, torch.Tensor]:
     params = dict(model.named_parameters())
     pieces: Dict[str, list] = {}
     for p in layered_mapping(model.cfg):
-        t = params[p.param].detach()
-        if p.rows is not None:
-            t = t[p.row0:p.row0 + p.rows]
-        if p.dim == 1:
-            t = t[:, :p.size]
+        t = p.of(params[p.param].detach())
         pieces.setdefault(p.name, []).append((p.dim or 0, t.to("cpu")))
     out = {k: (torch.cat([t for _, t in v], v[0][0]) if len(v) > 1 else v[0][1]) for k, v in pieces.items()}
     return {k: (t.to(dtype) if dtype is not None else t).contiguous() for k, t in out.items()}
@@ -293,6 +337,9 @@ def from_pretrained(path: str, device="cpu", dtype=torch.bfloat16):
     from . import model_class
 
     cfg = load_config(path)
+    sd = read_state_dict(path)
+    if cfg.is_layered:
+        with_ranks(cfg, {k: tuple(t.shape) for k, t in sd.items()})
     model = model_class(cfg)(cfg, device=device, dtype=dtype, init=False)
-    load_hf_state_dict(model, read_state_dict(path))
+    load_hf_state_dict(model, sd)
     return model

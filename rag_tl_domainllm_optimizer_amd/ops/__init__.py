@@ -5,9 +5,11 @@ from .linear import (  # noqa: F401
     ACT_DSWIGLU, ACT_IDS, ACT_SWIGLU, KMAJ, ROW, FoldCache, LoRAGroup, ShufCache, SplitK, gemm, gemm_big, gemm_decode, gemm_nn, gemm_tn, linear,
     swiglu_mlp, gemm_rope, linear_rope, rope_fusable,
     refresh_lora_batched,
-    linear_deferred, batch_invariant, Glu, project, glu_project, branch_project, TransposeCache)
+    linear_deferred, batch_invariant, Glu, project, glu_project, act_project, branch_project, TransposeCache, ACT_RELU2)
 from .norm import MoePairs, branch_norm, embed_norm, layer_norm, rms_norm  # noqa: F401
 from .moe import moe_ff, moe_route  # noqa: F401
+from .window import WindowDims, window_attention  # noqa: F401
+from .delta import delta_rule  # noqa: F401
 from .latent import LatentDims, latent_attention, yarn_rope_tables  # noqa: F401
 from .attention import (  # noqa: F401
     attention, decode_attention, decode_step_attention, decode_workspace, flash_attention_packed, gather_rows, packed_inverse, scatter_rows,

@@ -29,8 +29,9 @@ import torch
 from . import reference as ref
 from ._ext import native, on_gpu
 
-ACT_IDS = {None: 0, "none": 0, "relu": 1, "gelu": 2, "gelu_tanh": 3, "gelu_new": 3, "silu": 4, "swiglu": 5}
+ACT_IDS = {None: 0, "none": 0, "relu": 1, "gelu": 2, "gelu_tanh": 3, "gelu_new": 3, "silu": 4, "swiglu": 5, "relu2": 8}
 ACT_SWIGLU = 5  # w = [gate; up] (2F rows) -> silu(x gate^T) * (x up^T), [.., F]
+ACT_RELU2 = 8  # max(x, 0)^2
 ACT_DSWIGLU = 6  # gemm_big NN epilogue: d[gate | up] from dF and the [gate | up] pre-activation
 
 
@@ -42,7 +43,7 @@ def splitk_plan(M: int, N: int, K: int, act: int = 0):
     the last partial wave on 256x128 tiles)."""
     if M > 512:
         return 1, 0
-    bn = 128 if act in (0, ACT_SWIGLU) else 256
+    bn = 128 if act in (0, ACT_SWIGLU, ACT_RELU2) else 256
     tiles = ((M + 255) // 256) * (N // bn if act == ACT_SWIGLU else (N + bn - 1) // bn)
     if tiles >= 128:
         return 1, bn
@@ -176,6 +177,22 @@ def glu_project(x: torch.Tensor, w: torch.Tensor, glu: Glu, shuf=None) -> torch.
             return native().gemm_big(x, w, ROW, ROW, None, None, None, ACT_SWIGLU, 0, 1, None, None, None, bn,
                                      glu.args())
     return native().glu_any(project(x, w), glu.args())
+
+
+def act_project(x: torch.Tensor, w: torch.Tensor, act: int, shuf=None) -> torch.Tensor:
+    """act(x w^T) without grad: in the GEMM epilogue where the MFMA kernels take the shape, else on an fp32
+    product."""
+    if not on_gpu(x):
+        return ref.gemm(x, w, act=act)
+    M, K = x.shape
+    N = w.shape[0]
+    if x.dtype == torch.bfloat16 and M > 0 and K % 8 == 0 and N % 8 == 0 and x.stride(0) % 8 == 0 and x.data_ptr() % 16 == 0:
+        if M <= 64 and K % 64 == 0:
+            sh = shuf is not None and shuffle_decode(M) and N % 16 == 0
+            return native().gemm(x, shuf.get(w) if sh else w, None, None, None, act, False, None, None, 0.0, sh)
+        if M > 64:
+            return gemm(x, w, act=act)
+    return native().act_any(project(x, w, True), act, x.dtype == torch.float32)
 
 
 def branch_project(x: torch.Tensor, w: torch.Tensor, shuf=None):

@@ -115,25 +115,30 @@ class MoePairs:
 _Y_ACT, _Y_SLABS, _Y_PAIRS, _Y_PAIRS_F32 = 1, 2, 3, 4
 
 
-def embed_norm(table, ids, w_next, eps: float):
-    """First step of a pass with an fp32 residual stream: x = table[ids] (fp32 [T, H]) and
-    h = rms(x) * w_next in the table's dtype. Returns (x, h)."""
+def embed_norm(table, ids, w_next, eps: float, w_embed=None):
+    """First step of a pass with an fp32 residual stream: x = table[ids] (fp32 [T, H]; normed and weighted with
+    ``w_embed`` if given) and h = rms(x) * w_next in the table's dtype (``w_next`` None: h = x, rounded).
+    Returns (x, h)."""
     if on_gpu(ids):
         x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=ids.device)
-        h = native().branch_norm(x, 0, w_next=w_next, table=table, ids=ids.contiguous(), eps=eps)
+        h = native().branch_norm(x, 0, w_branch=w_embed, w_next=w_next, table=table, ids=ids.contiguous(), eps=eps,
+                                 plain=w_next is None)
         return x, h
     x = table[ids].float()
-    return x, ref.rms(x, w_next, eps).to(table.dtype)
+    if w_embed is not None:
+        x = ref.rms(x, w_embed, eps)
+    return x, (x if w_next is None else ref.rms(x, w_next, eps)).to(table.dtype, copy=True)
 
 
-def branch_norm(x, y, w_branch, w_next, eps: float):
-    """Between two sublayers with a norm before and after each, on the fp32 residual ``x`` (updated in
-    place): ``x += rms(y) * w_branch``; returns ``h = rms(x) * w_next`` in the weights' dtype. ``y``: a
-    tensor, unreduced split-K slabs (``SplitK``) or a mixture's expert outputs (:class:`MoePairs`)."""
+def branch_norm(x, y, w_branch, w_next, eps: float, scale=None, next_mul: float = 1.0):
+    """Between two sublayers with a norm after each, on the fp32 residual ``x`` (updated in place):
+    ``x += rms(y) * w_branch [* scale]``; returns ``h = rms(x) * w_next * next_mul`` in the weights' dtype, or
+    x itself rounded (``w_next`` None: sublayers without a norm ahead). ``y``: a tensor, unreduced split-K
+    slabs (``SplitK``) or a mixture's expert outputs (:class:`MoePairs`)."""
     from .linear import SplitK
 
     if on_gpu(x):
-        kw = dict(w_branch=w_branch, w_next=w_next, eps=eps)
+        kw = dict(w_branch=w_branch, w_next=w_next, eps=eps, scale=scale, next_mul=next_mul, plain=w_next is None)
         if isinstance(y, SplitK):
             return native().branch_norm(x, _Y_SLABS, y=y.slabs, nsplit=y.nsplit, **kw)
         if isinstance(y, MoePairs):
@@ -141,6 +146,7 @@ def branch_norm(x, y, w_branch, w_next, eps: float):
             return native().branch_norm(x, kind, y=y.y, pair_w=y.w, pair_pos=y.pos, **kw)
         kind = _Y_ACT if y.dtype == w_branch.dtype else _Y_SLABS
         return native().branch_norm(x, kind, y=y.contiguous(), **kw)
-    yf = y.combine() if isinstance(y, MoePairs) else y.float()
-    x.add_(ref.rms(yf, w_branch, eps))
-    return ref.rms(x, w_next, eps).to(w_branch.dtype)
+    yf = ref.rms(y.combine() if isinstance(y, MoePairs) else y.float(), w_branch, eps)
+    x.add_(yf if scale is None else yf * scale.float())
+    h = x if w_next is None else ref.rms(x, w_next, eps) * next_mul
+    return h.to(w_branch.dtype, copy=True)

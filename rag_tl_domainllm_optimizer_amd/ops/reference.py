@@ -12,6 +12,7 @@ import torch
 import torch.nn.functional as F
 
 ACT_NONE, ACT_RELU, ACT_GELU, ACT_GELU_TANH, ACT_SILU = 0, 1, 2, 3, 4
+ACT_RELU2 = 8
 
 
 def apply_act(y: torch.Tensor, act: int) -> torch.Tensor:
@@ -23,6 +24,8 @@ def apply_act(y: torch.Tensor, act: int) -> torch.Tensor:
         return F.gelu(y, approximate="tanh")
     if act == ACT_SILU:
         return F.silu(y)
+    if act == ACT_RELU2:
+        return F.relu(y).square()
     return y
 
 
@@ -343,6 +346,14 @@ def rotate_pairs(x, cos, sin):
     y[..., 0:2 * n:2] = u * c - v * s
     y[..., 1:2 * n:2] = v * c + u * s
     return y
+
+
+def rotate_halves(x, cos, sin):
+    """x [T, heads, d] with column i < cos.shape[1] turned together with column i + cos.shape[1]"""
+    n = cos.shape[1]
+    c, s = cos[:, None], sin[:, None]
+    u, v = x[..., :n].float(), x[..., n:2 * n].float()
+    return torch.cat([u * c - v * s, v * c + u * s, x[..., 2 * n:].float()], -1)
 
 
 def latent_attend(q, pool, tab, row, pos, sink, rank, scale, page):

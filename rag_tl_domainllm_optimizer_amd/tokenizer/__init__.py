@@ -22,12 +22,12 @@ FAMILY_SPECIALS = {
              "mask": ("[MASK]", 103)},
     "mpnet": {"bos": ("<s>", 0), "pad": ("<pad>", 1), "eos": ("</s>", 2), "unk": ("<unk>", 3)},
 }
-_TEMPLATE = {"llama": "bos", "mistral": "bos", "vezatar": "bos", "opt": "bos", "bert": "cls_sep", "mpnet": "cls_sep"}
+_TEMPLATE = {"llama": "bos", "mistral": "bos", "vezatar": "bos", "pafolorn": "bos", "opt": "bos", "bert": "cls_sep", "mpnet": "cls_sep"}
 PUNCT = list(".,;:?!'\"()-")
 
 
 def family_of(arch: str) -> str:
-    return {"mistral": "llama", "llama": "llama", "vezatar": "llama"}.get(arch, arch)
+    return {"mistral": "llama", "llama": "llama", "vezatar": "llama", "pafolorn": "llama"}.get(arch, arch)
 
 
 def synthetic_words(n: int, seed: int = 1234) -> List[str]:
