@@ -1,0 +1,388 @@
+"""Pafolorn on the CPU path (fp32): reading and writing its files, every mechanism against the plain
+implementation in pafolorn_oracle.py, cache and state slots, ragged batches, scheduler, generation, trace replay."""
+import copy
+import io
+import json
+
+import numpy as np
+import pafolorn_common as pc
+import pafolorn_oracle as oracle
+import pytest
+import torch
+
+from rag_tl_domainllm_optimizer_amd import models, ops
+from rag_tl_domainllm_optimizer_amd.generation import ContinuousBatcher, Generator, SamplingParams
+from rag_tl_domainllm_optimizer_amd.generation.paged import PAGE, PagedCache
+from rag_tl_domainllm_optimizer_amd.generation.ragged import CHUNK, SHORT_TOKENS, RaggedBatch, StepEngine
+from rag_tl_domainllm_optimizer_amd.models import io as mio
+from rag_tl_domainllm_optimizer_amd.models.config import ModelConfig, config_from_hf, config_to_hf, with_ranks
+
+TOL = 2e-4  # fp32 rounding reaches 3e-5 on these models
+
+
+def tokens(cfg, n, seed=0):
+    return torch.randint(0, cfg["vocab"], (n,), generator=torch.Generator().manual_seed(seed)).tolist()
+
+
+def build(cfg, w):
+    c = with_ranks(config_from_hf(cfg), {k: tuple(v.shape) for k, v in w.items()})
+    m = models.LayeredLM(c, dtype=torch.float32, init=False)
+    mio.load_layered_state_dict(m, w)
+    return m
+
+
+@pytest.fixture(scope="module")
+def odd(tmp_path_factory):
+    cfg = pc.odd()
+    w = pc.weights(cfg, 1)
+    return cfg, w, pc.load(cfg, w, tmp_path_factory.mktemp("odd"))
+
+
+# ------------------------------------------------------------------ files and registry
+def test_config_round_trip():
+    for cfg in (pc.odd(), pc.even()):
+        c = config_from_hf(cfg)
+        assert c.is_layered and c.is_decoder and models.model_class(c) is models.LayeredLM
+        assert config_to_hf(c) == json.loads(json.dumps(cfg))
+        assert ModelConfig.from_dict(json.loads(json.dumps(c.to_dict()))) == c
+    m = models.LayeredLM(models.resolve_preset("tiny-pafolorn"), dtype=torch.float32)
+    n = sum(p.numel() for k, p in m.named_parameters() if not k.endswith(("in_w", "o_w", "a2_w", "g2_w")))
+    for layer in m.layers:  # parameters as the files count them: without the padding between the blocks
+        x = layer.mix
+        n += sum(r for s in x.rows.values() for _, r in s.values()) * m.cfg.hidden_size
+        n += sum(c for _, c in x.cols.values()) * m.cfg.hidden_size
+        for b, _, _ in x.branches():
+            if hasattr(b, "a2_w"):
+                n += b.a2_w.shape[0] * b.spec.a_rank + b.g2_w.shape[0] * b.spec.g_rank
+    assert n == m.cfg.num_params()
+
+
+def test_config_refuses_bad_values():
+    def left(l):
+        return l[0]["mixer"]["left"]
+    for edit in (lambda l: left(l).update(kv_heads=4), lambda l: left(l)["rot"].update(dims=12),
+                 lambda l: left(l)["rot"].update(dims=5), lambda l: left(l)["mask"].update(size=-1),
+                 lambda l: l[1]["mixer"].update(kv_heads=3), lambda l: l[1]["mixer"].update(conv=0),
+                 lambda l: l[0].update(type="other"), lambda l: l[0]["mlp"].update(kind="other")):
+        cfg = pc.odd()
+        edit(cfg["layers"])
+        with pytest.raises(ValueError):
+            config_from_hf(cfg)
+
+
+def test_load_is_strict(tmp_path, odd):
+    cfg, w, _ = odd
+    for edit in (lambda d: d.pop("l0.mix.right.k.conv"), lambda d: d.pop("l1.mix.a1"), lambda d: d.update(extra=torch.zeros(2)),
+                 lambda d: d.update({"l1.mix.a2": d["l1.mix.a2"][:-1].clone()}),
+                 lambda d: d.update({"l3.norm2": d["l3.norm1"].clone()})):
+        d = dict(w)
+        edit(d)
+        with pytest.raises((KeyError, ValueError)):
+            pc.load(cfg, d, tmp_path / "x")
+
+
+def test_save_pretrained_round_trip(tmp_path, odd):
+    cfg, w, m = odd
+    mio.save_pretrained(m, str(tmp_path / "s"))
+    sd = mio.read_state_dict(str(tmp_path / "s"))
+    assert set(sd) == set(w)
+    for k in w:
+        assert torch.equal(sd[k].view_as(w[k]), w[k]), k
+    m2 = models.build_model(str(tmp_path / "s"), dtype=torch.float32)
+    assert config_to_hf(m2.cfg) == config_to_hf(m.cfg)
+    for a, b in zip(m.parameters(), m2.parameters()):
+        assert torch.equal(a, b)
+
+
+def test_random_init_keeps_padding_zero():
+    m = models.LayeredLM(models.resolve_preset("tiny-pafolorn"), dtype=torch.float32, seed=3)
+    for layer in m.layers:
+        before = [p.clone() for p in layer.mix.parameters()]
+        layer.mix.zero_padding()
+        assert all(torch.equal(a, b) for a, b in zip(before, layer.mix.parameters()))
+    t = tokens({"vocab": 512}, 30, 1)
+    sd = mio.layered_state_dict(m)
+    assert pc.err(pc.run(StepEngine(m, 1, 64), t, (11, 1)), oracle.forward(config_to_hf(m.cfg), sd, t)) < TOL
+
+
+# ------------------------------------------------------------------ single mechanisms
+@pytest.mark.parametrize("size,keep,rot", [(5, 0, 4), (5, 3, 8), (70, 66, 2), (1, 1, 8), (64, 64, 6), (500, 0, 8)])
+def test_window_attention(size, keep, rot):
+    mx = pc.attn(6, 3, 8, 5, size, keep, rot=rot, softcap=2.0)
+    T, W = 150, 20
+    g = torch.Generator().manual_seed(size)
+    w = {"p." + k: torch.randn(n, W, generator=g) for k, n in (("q", 48), ("k", 24), ("v", 15))}
+    w["p.q.norm"], w["p.k.norm"] = torch.rand(48, generator=g) + 0.5, torch.rand(24, generator=g) + 0.5
+    h = torch.randn(T, W, generator=g)
+    want = oracle.window_attention(w, "p.", mx, h, 0.01)
+    spec = models.config._window_spec(mx)
+    d = ops.WindowDims(6, 3, 8, 5, spec.scale, spec.softcap, spec.window, spec.keep_first)
+    cache = PagedCache([d.cache_width], 2, T, dtype=torch.float32)
+    cos, sin = ops.yarn_rope_tables(spec.rot.dims, spec.rot.base, cache.max_seq)
+    cache.reserve(1, T)
+    cache.sync()
+    proj = torch.cat([torch.zeros(T, 3), h @ torch.cat([w["p.q"], w["p.k"], w["p.v"]]).T, torch.zeros(T, 2)], 1)
+    got, at = torch.zeros(T, 34), 0
+    for n in (1, 63, 2, 40, 44):
+        b = RaggedBatch.build([(1, [0] * n, at)], "cpu")
+        ops.window_attention(proj[at:at + n], 3, d, w["p.q.norm"], w["p.k.norm"], 0.01, cos, sin, b, cache.pool(0),
+                             cache.table, got[at:at + n, 2:32], 0.25)
+        at += n
+    torch.testing.assert_close(got[:, 2:32], 0.25 * want, rtol=1e-4, atol=1e-5)
+    assert got[:, :2].abs().max() == 0 and got[:, 32:].abs().max() == 0
+
+
+@pytest.mark.parametrize("ch", [True, False])
+@pytest.mark.parametrize("H,K,D,V,taps", [(4, 2, 6, 5, 4), (3, 3, 1, 7, 1), (2, 1, 16, 8, 2), (1, 1, 5, 1, 7)])
+def test_delta_rule(ch, H, K, D, V, taps):
+    """projections in, gated read-outs out; portions and a slot that held another request's state"""
+    mx, W, T = pc.delta(H, K, D, V, taps), 14, 60
+    cfg = pc.config(8, W, [pc.channel(mx) if ch else pc.parallel(pc.attn(1, 1, 2, 2, 3, 0), mx, 1, 1)])
+    w = {k: v.float() for k, v in pc.weights(cfg, H + D).items()}
+    p = "l0.mix." if ch else "l0.mix.right."
+    h = torch.randn(T, W, generator=torch.Generator().manual_seed(T))
+    want = oracle.delta_mixer(w, p, mx, h, 0.02, ch)
+    a = (h @ w[p + "a1"].T) @ w[p + "a2"].T if ch else h @ w[p + "a"].T
+    z = (h @ w[p + "g1"].T) @ w[p + "g2"].T if ch else h @ w[p + "g"].T
+    x, b = h @ torch.cat([w[p + k] for k in "qkv"]).T, h @ w[p + "b"].T
+    conv = torch.cat([w[p + k + ".conv"] for k in "qkv"])
+    state, ring = torch.randn(2, H, D, V) * 9, torch.randn(2, taps, x.shape[1]) * 9
+    got, at = torch.zeros(T, H * V), 0
+    for n in (1, 1, 2, 17, 1, 16, 22):
+        s = slice(at, at + n)
+        ops.delta_rule(x[s], b[s], a[s], z[s], conv, w[p + "A_log"], w[p + "dt_bias"], w[p + "norm"], 0.02,
+                       RaggedBatch.build([(1, [0] * n, at)], "cpu"), state, ring, got[s], 1.5, K, not ch)
+        at += n
+    torch.testing.assert_close(got, 1.5 * want, rtol=1e-4, atol=1e-5)
+
+
+def test_output_norm_with_scale_and_squared_relu():
+    x, y, w, ls, wn = (torch.randn(5, 12) if i < 2 else torch.randn(12) for i in range(5))
+    want = x + oracle.rms(y, 0.1) * w * ls
+    xs = x.clone()
+    h = ops.branch_norm(xs, y, w, None, 0.1, ls)
+    torch.testing.assert_close(xs, want)
+    assert torch.equal(h, xs) and h.data_ptr() != xs.data_ptr()
+    h = ops.branch_norm(x.clone(), y, w, wn, 0.1, ls, 0.3)
+    torch.testing.assert_close(h, oracle.rms(want, 0.1) * wn * 0.3)
+    e, ids = torch.randn(9, 12), torch.tensor([3, 3, 8])
+    xe, he = ops.embed_norm(e, ids, None, 0.1, w)
+    torch.testing.assert_close(xe, oracle.rms(e[ids], 0.1) * w)
+    assert torch.equal(xe, he) and he.data_ptr() != xe.data_ptr()
+    up, down = torch.randn(7, 12), torch.randn(12, 7)
+    got = ops.branch_project(ops.act_project(x, up, ops.ACT_RELU2), down)
+    torch.testing.assert_close(got, oracle.dense_ff({"up": up, "down": down}, "", x), rtol=1e-4, atol=1e-4)
+
+
+# ------------------------------------------------------------------ the step
+def test_layers_and_logits_against_oracle(odd):
+    cfg, w, m = odd
+    t = tokens(cfg, 90)
+    layers = []
+    want = oracle.forward(cfg, w, t, layers_out=layers)
+    cache = m.make_cache(1, 128)
+    cache.reserve(0, len(t))
+    cache.sync()
+    got = []
+    h = m.step(RaggedBatch.build([(0, t, 0)], "cpu"), cache, layer_out=got)
+    for a, b in zip(got, layers):
+        torch.testing.assert_close(a, b, rtol=1e-4, atol=1e-4)
+    assert pc.err(m.logits(h), want) < TOL
+    assert pc.err(m.logits(m(torch.tensor([t]))), want) < TOL
+
+
+def test_every_mechanism_shows_in_the_logits(odd):
+    """each planted mistake moves the oracle's logits far beyond the tolerance of these tests"""
+    cfg, w, _ = odd
+    t = tokens(cfg, 70)
+    want = oracle.forward(cfg, w, t)
+    for fault in ("interleaved", "window_off_by_one", "no_kept", "kept_off_by_one", "head_norm", "no_qk_norm", "no_rotation",
+                  "no_softcap", "taps_reversed", "no_conv", "read_before_write", "state_lost", "head_modulo", "no_unit",
+                  "no_decay", "no_gate", "no_scales", "relu_only", "no_embed_norm", "no_layer_scale", "no_logit_scale"):
+        n = 6 if fault == "no_unit" else len(t)  # without unit keys the state soon overflows
+        assert pc.err(oracle.forward(cfg, w, t[:n], fault=(fault,)), want[:n]) > 30 * TOL, fault
+
+
+@pytest.mark.parametrize("sizes", [(1,), (2,), (3, 5), (33, 2, 64), (CHUNK, CHUNK + 1, 1), (SHORT_TOKENS, SHORT_TOKENS + 1),
+                                   (63, 1, 1, 64, 65)])
+def test_portions(odd, sizes):
+    cfg, w, m = odd
+    t = tokens(cfg, 150, 2)
+    assert pc.err(pc.run(StepEngine(m, 1, 192), t, sizes), oracle.forward(cfg, w, t)) < TOL
+
+
+def test_mixed_batches_and_reused_slots(odd):
+    """unequal requests in one batch, left out of steps, released, their pages and slots used again in another
+    order: every logit as if alone"""
+    cfg, w, m = odd
+    rng = np.random.default_rng(0)
+    eng = StepEngine(m, 3, 5 * PAGE)
+    live, done, nxt, want = {}, 0, 0, {}
+    while done < 7:
+        while len(live) < 3 and nxt < 7:
+            t = tokens(cfg, int(rng.integers(1, 100)), 10 + nxt)
+            if sum((len(x[1]) + PAGE - 1) // PAGE for x in live.values()) + (len(t) + PAGE - 1) // PAGE > 5:
+                break
+            want[nxt] = oracle.forward(cfg, w, t)
+            live[nxt] = [eng.admit(), t, 0]
+            nxt += 1
+        part = [k for k in live if rng.random() < 0.7] or list(live)[:1]
+        ent = [(k, live[k][1][live[k][2]:live[k][2] + int(rng.choice([1, 1, 2, 30, 50]))]) for k in part]
+        lg = eng.step([(live[k][0], c, list(range(len(c)))) for k, c in ent])
+        o = 0
+        for k, c in ent:
+            assert pc.err(lg[o:o + len(c)], want[k][live[k][2]:live[k][2] + len(c)]) < TOL, k
+            o += len(c)
+            live[k][2] += len(c)
+            if live[k][2] == len(live[k][1]):
+                eng.release(live.pop(k)[0])
+                done += 1
+
+
+@pytest.mark.parametrize("size,keep", [(70, 5), (64, 64), (128, 0), (33, 66)])
+def test_needle_at_every_edge(size, keep):
+    """one key among hundreds, just inside and just outside the window and the kept tokens, at page borders"""
+    cfg, w = pc.needle_model(size, keep)
+    m = build(cfg, w)
+    n = 200
+    for at in sorted({0, keep - 1, keep, keep + 1, 63, 64, 65, n - size - 1, n - size, n - size + 1, n - 2}):
+        if not 0 <= at < n - 1:
+            continue
+        asks = [a for a in (at + 1, at + size - 1, at + size, n - 1) if at < a < n]
+        t = pc.needle_tokens(n, at, asks)
+        want = oracle.forward(cfg, w, t)
+        plain = list(t)
+        plain[at] = 7
+        moved = oracle.forward(cfg, w, plain)
+        for a in asks:
+            seen = a - at < size or at < keep
+            e = pc.err(moved[a:a + 1], want[a:a + 1])
+            assert e > 0.2 if seen else e < 1e-6, (at, a)
+        for sizes in ((n,), (n - 1, 1), (64, 40, 1), (7, 2)):
+            assert pc.err(pc.run(StepEngine(m, 1, 256), t, sizes), want) < TOL, (at, sizes)
+
+
+@pytest.mark.parametrize("ch", [True, False])
+def test_far_memory(ch):
+    """a write that only the carried state remembers, read hundreds of tokens later"""
+    cfg, w = pc.memory_model(ch)
+    m = build(cfg, w)
+    n = 300
+    t = pc.needle_tokens(n, 3, [n - 1])
+    want = oracle.forward(cfg, w, t)
+    assert pc.err(oracle.forward(cfg, w, t, fault=("state_lost",))[-1:], want[-1:]) > 0.2
+    eng = StepEngine(m, 1, 320)
+    for sizes in ((n,), (n - 1, 1), (64, 40, 1), (2,)):
+        assert pc.err(pc.run(eng, t, sizes), want) < TOL, sizes
+
+
+def test_first_tokens_and_single_token(odd):
+    cfg, w, m = odd
+    for n in (1, 2, 3):
+        t = tokens(cfg, n, 40 + n)
+        assert pc.err(pc.run(StepEngine(m, 1, 64), t, (n,)), oracle.forward(cfg, w, t)) < TOL
+
+
+# ------------------------------------------------------------------ cache and slots
+def test_state_slots():
+    c = PagedCache([8, 0], rows=3, max_seq=100, states=[[], [((2, 3), torch.float32), ((4,), torch.bfloat16)]])
+    assert c.pool(1) is None and c.state(0) == () and [tuple(t.shape) for t in c.state(1)] == [(3, 2, 3), (3, 4)]
+    assert c.nbytes == c.pool(0).numel() * 2 + 18 * 4 + 12 * 2
+    with c.parked():
+        assert c.row_ids.tolist() == [-1] * 3 and c.rows_view(1, 2).row_ids.tolist() == [-1] * 2
+    assert c.row_ids.tolist() == [0, 1, 2]
+
+
+def test_batch_tables_of_recurrent_runs():
+    b = RaggedBatch.build([(2, [1] * 40, 5), (0, [1], 9), (1, [1, 1], 0), (3, [1] * 16, 16)], "cpu")
+    assert b.n_single == 1 and b.offset.tolist() == [19, 0, 1, 3]
+    assert b.runs.tolist() == [[1, 1, 2, 0], [3, 3, 16, 16], [2, 19, 40, 5]]
+    assert b.chunks.tolist() == [[0, 0], [1, 0], [2, 0], [2, 1], [2, 2]] and b.first_chunk.tolist() == [0, 1, 2]
+    b = RaggedBatch.build([(0, [1], 9), (1, [4], 3)], "cpu")
+    assert b.n_single == 2 and b.runs is None and b.chunks is None
+
+
+# ------------------------------------------------------------------ generation, scheduler, trace, CLI
+def test_greedy_generation(odd):
+    cfg, w, m = odd
+    prompts = [tokens(cfg, n, 60 + n) for n in (5, 40, 1, 70)]
+    want = [pc.greedy(cfg, w, p, 6) for p in prompts]
+    gen = Generator(m, max_batch=4, max_seq=96, device="cpu")
+    p = SamplingParams(max_new_tokens=6, do_sample=False)
+    for _ in range(2):  # the second call reuses rows, slots and pages
+        out = gen.generate(prompts, p, eos_ids=[-5])
+        assert [r.tolist() for r in out.tokens] == want
+
+
+def test_continuous_batching_in_portions(odd):
+    """more requests than rows, a pool too small for all of them, prompts entering 16 tokens at a time: a waiting
+    or half-read prompt's state must not advance with the decoding rows"""
+    cfg, w, m = odd
+    prompts = [tokens(cfg, n, 80 + n) for n in (50, 3, 70, 20, 33, 1)]
+    want = [pc.greedy(cfg, w, p, 5) for p in prompts]
+    gen = Generator(m, max_batch=3, max_seq=128, device="cpu", cache_tokens=3 * PAGE)
+    cb = ContinuousBatcher(gen, SamplingParams(max_new_tokens=5, do_sample=False), eos_ids=[-5], prefill_tokens=16)
+    todo, got = list(enumerate(prompts)), {}
+    for _ in range(200):
+        while todo and cb.free_rows():
+            i, pr = todo.pop(0)
+            cb.admit(pr, i)
+        cb.step(1)
+        for r in cb.collect():
+            got[r.tag] = r.tokens
+        if len(got) == len(prompts):
+            break
+    assert [got[i] for i in range(len(prompts))] == want
+    assert gen.cache.free_tokens() == 3 * PAGE
+
+
+def test_trace_replay(tmp_path, odd):
+    from rag_tl_domainllm_optimizer_amd.serve.trace import replay
+
+    cfg, w, m = odd
+    a, b = tokens(cfg, 40, 1), tokens(cfg, 9, 2)
+    steps = [{"step": 0, "entries": [{"id": "a", "tokens": a[:39], "want": [0, 38]}], "end": []},
+             {"step": 1, "entries": [{"id": "b", "tokens": b[:2], "want": []}], "end": []},
+             {"step": 5, "entries": [{"id": "b", "tokens": b[2:], "want": [6, 0]}, {"id": "a", "tokens": a[39:], "want": [0]}],
+              "end": ["a", "b"]}]
+    said = []
+    assert replay(m, io.StringIO("\n".join(json.dumps(s) for s in steps)), str(tmp_path), 128, said.append) == 3
+    assert said == ["done 0", "done 1", "done 5"]
+    wa, wb = oracle.forward(cfg, w, a), oracle.forward(cfg, w, b)
+    for name, rows in (("0.f32", [wa[0], wa[38]]), ("5.f32", [wb[8], wb[2], wa[39]])):
+        got = torch.from_numpy(np.fromfile(tmp_path / name, "<f4").reshape(-1, cfg["vocab"]).copy())
+        assert pc.err(got, torch.stack(rows)) < TOL
+
+
+def test_cli_rag_answers_with_this_policy(capsys):
+    from rag_tl_domainllm_optimizer_amd import cli
+
+    cli.main(["rag", "--model.policy=tiny-pafolorn:random", "--model.encoder=tiny-bert:random", "--ppo.max_new_tokens=4",
+              "--ppo.max_prompt_tokens=64", "--data.synthetic_docs=24", "--retrieval.index=flat", "--query", "what is it"])
+    line = [x for x in capsys.readouterr().out.splitlines() if x.startswith("{")][-1]
+    assert "answer" in json.loads(line)
+
+
+def test_config_values_are_read_not_assumed(odd):
+    """every constant of config.json reaches the result: changing any of them changes the logits"""
+    cfg, w, _ = odd
+    t = tokens(cfg, 60, 9)
+    base = pc.run(StepEngine(build(cfg, w), 1, 64), t, (60,))
+
+    def left(c, **kw):
+        for x in c["layers"]:
+            if x["type"] == "parallel":
+                for k, v in kw.items():
+                    d = x["mixer"]["left"]
+                    d = d["rot"] if k in ("base", "dims") else d["mask"] if k in ("size", "keep_first") else d
+                    d[k] = v
+    edits = [lambda c: c["norm"].update(eps=0.5), lambda c: c.update(logit_scale=2.0),
+             lambda c: c["layers"][0]["mixer"].update(left_scale=0.1), lambda c: c["layers"][4]["mixer"].update(right_scale=-1.0)]
+    edits += [lambda c, kw=kw: left(c, **kw) for kw in (dict(scale=1.1), dict(softcap=0.7), dict(base=9.0), dict(dims=4),
+                                                        dict(size=17), dict(keep_first=12))]
+    for e in edits:
+        c = copy.deepcopy(cfg)
+        e(c)
+        got = pc.run(StepEngine(build(c, w), 1, 64), t, (60,))
+        assert pc.err(got, oracle.forward(c, w, t)) < TOL
+        assert pc.err(got, base) > 10 * TOL
