@@ -10,8 +10,8 @@
 // that is used again needs no clearing. Rows < 0 (parked) read zeros and write nothing.
 //
 //   delta_step    one token per request: everything in one kernel, the state read and written once
-//   portions:     delta_prep (chunks of 16 tokens, all in parallel) -> delta_scan (chunks in order, fp32 MFMA)
-//                 -> delta_out (norm, gate), delta_commit (ring)
+//   portions:     delta_prep (chunks of 16 tokens, all in parallel) -> delta_scan (chunks in order, fp32 MFMA;
+//                 value columns in parallel) -> delta_out (norm, gate), delta_commit (ring)
 //
 // Chunk form (tokens 1..16 of a chunk, G_i = summed log decays, S0 = state ahead of it):
 //   A_ij = beta_i sum_d k_id k_jd e^(G_id - G_jd)  (j < i),  P_ij = sum_d q_id k_jd e^(G_id - G_jd)  (j <= i)
@@ -201,7 +201,8 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
 // portions
 // ---------------------------------------------------------------------------------------------
 // runs: {row, first token, tokens, position of the first}; chunks: {run, chunk of the run}, a run's chunks
-// consecutive. Workspace per (chunk, head): KT, QT, KE [CH][DP], EG [DP], T, P [CH][CH] floats.
+// consecutive. Workspace per (chunk, head): k e^G, q e^G [CH][DP], k e^(G_16 - G) transposed [DP][CH], e^G_16 [DP],
+// T, P [CH][CH] floats.
 struct Work {
   const int4* runs; const int2* chunks;
   float* ws;
@@ -212,13 +213,74 @@ template <int DP> struct Lay {
   static constexpr int KT = 0, QT = CH * DP, KE = 2 * CH * DP, EG = 3 * CH * DP, T = EG + DP, P = T + CH * CH, N = P + CH * CH;
 };
 
-template <typename T, int DP>
+// N consecutive elements: 8 bf16 or 4 floats (16 bytes, aligned), or 1
+template <typename T, int N>
+__device__ __forceinline__ void ldn(const T* p, float* o) {
+  if constexpr (N == 8) unpack8(*(const uint4*)p, o);
+  else if constexpr (N == 4) *(f32x4*)o = *(const f32x4*)p;
+  else o[0] = ld(p);
+}
+template <typename T, int N>
+__device__ __forceinline__ void stn(T* p, const float* o) {
+  if constexpr (N == 8) *(uint4*)p = pack8(o);
+  else if constexpr (N == 4) *(f32x4*)p = *(const f32x4*)o;
+  else st(p, o[0]);
+}
+
+// N floats, aligned to 16 bytes from four on
+template <int N>
+__device__ __forceinline__ void ldf(const float* p, float* o) {
+  if constexpr (N % 4 == 0) {
+#pragma unroll
+    for (int k = 0; k < N; k += 4) *(f32x4*)(o + k) = *(const f32x4*)(p + k);
+  } else {
+    o[0] = p[0];
+  }
+}
+template <int N>
+__device__ __forceinline__ void stf(float* p, const float* o) { ldf<N>(o, p); }
+
+// convolution and silu of channels c .. c + N - 1 at positions p .. p + 3, zeros from position p + n on
+template <typename T, int N>
+__device__ __forceinline__ void conv4(const Conv<T>& cv, int p, int n, int c, float (&y)[4][N]) {
+  const int taps = cv.a.taps;
+  const T* w = (const T*)cv.a.conv + (long)c * taps;
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int e = 0; e < N; ++e) y[i][e] = 0.f;
+  for (int j = 0; j < taps; ++j) {
+    float wj[N];
+#pragma unroll
+    for (int e = 0; e < N; ++e) wj[e] = ld(w + e * taps + j);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int q = p + i - (taps - 1 - j);
+      const T* src = q >= cv.start ? cv.x + (long)(q - cv.start) * cv.a.ldx : cv.ring + (long)(max(q, 0) % taps) * cv.C;
+      if (i < n && (q >= cv.start || (cv.ring && q >= 0))) {
+        __attribute__((aligned(16))) float v[N];
+        ldn<T, N>(src + c, v);
+#pragma unroll
+        for (int e = 0; e < N; ++e) y[i][e] = fmaf(wj[e], v[e], y[i][e]);
+      }
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int e = 0; e < N; ++e) y[i][e] *= sigmoid(y[i][e]);
+}
+
+// workgroup = (head, chunk); CHN: a decay per key channel, else per head. N: elements per access
+template <typename T, int DP, bool CHN, int N>
 __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
   constexpr int LD = DP + 4, R = DP / 16;
   using L = Lay<DP>;
-  __shared__ __attribute__((aligned(16))) float kx[CH][LD], qx[CH][LD], G[CH][LD];
-  __shared__ float As[CH][CH + 1], Ps[CH][CH + 1], beta[CH], dot[CH];
-  const int h = blockIdx.x, ci = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+  __shared__ __attribute__((aligned(16))) float kx[CH][LD], qx[CH][LD], G[CHN ? CH : 1][LD];
+  __shared__ float As[CH][CH + 1], Ps[CH][CH + 1], beta[CH], dot[CH], Gs[CH];
+  __shared__ f32x4 red[CHN ? 1 : 3][2][64];
+  const int h = blockIdx.x, ci = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
+  const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int2 ck = w.chunks[ci];
   const int4 run = w.runs[ck.x];
   const int n = min(CH, run.z - ck.y * CH), p0 = run.w + ck.y * CH, t0 = run.y + ck.y * CH;
@@ -227,64 +289,108 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
   const Conv<T> conv{a, (const T*)a.x + (long)run.y * a.ldx,
                      carry ? (const T*)a.ring + (long)run.x * a.taps * C : nullptr, run.w, C};
   const float A = expf(a.A_log[h]);
-  if (tid < CH) beta[tid] = tid < n ? sigmoid(ld((const T*)a.b + (long)(t0 + tid) * a.ldb + h)) : 0.f;
-  for (int e = tid; e < CH * DP; e += 256) {
-    const int i = e / DP, d = e % DP;
-    float k = 0.f, q = 0.f, g = 0.f;
-    if (i < n && d < D) {
-      q = conv(p0 + i, kh * D + d);
-      k = conv(p0 + i, KD + kh * D + d);
-      g = a.channel ? -A * softplus(ld((const T*)a.a + (long)(t0 + i) * a.lda + (long)h * D + d) + a.dt[(long)h * D + d])
-                    : -A * softplus(ld((const T*)a.a + (long)(t0 + i) * a.lda + h) + a.dt[h]);
-    }
-    kx[i][d] = k;
-    qx[i][d] = q;
-    G[i][d] = g;
-  }
-  for (int e = tid; e < n * V; e += 256) {
-    const int i = e / V, c = e % V;
-    st((T*)w.v + (long)(t0 + i) * a.H * V + (long)h * V + c, conv(p0 + i, 2 * KD + h * V + c));
-  }
-  __syncthreads();
-  for (int i = wid; i < CH; i += 4) {  // unit vectors
-    float kk = 0.f, qq = 0.f, qk = 0.f;
-    for (int d = lane; d < D; d += 64) {
-      kk += kx[i][d] * kx[i][d];
-      qq += qx[i][d] * qx[i][d];
-      qk += qx[i][d] * kx[i][d];
-    }
-    const float ik = 1.f / sqrtf(wave_sum(kk) + 1e-6f), iq = 1.f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)D);
-    qk = wave_sum(qk);
-    for (int d = lane; d < D; d += 64) {
-      kx[i][d] *= ik;
-      qx[i][d] *= iq;
-    }
-    if (lane == 0) dot[i] = qk * ik * iq;
-  }
-  for (int d = tid; d < DP; d += 256) {
-    float s = 0.f;
+  if (tid < CH) {
+    const T* bp = (const T*)a.b + (long)(t0 + tid) * a.ldb + h;
+    beta[tid] = tid < n ? sigmoid(ld(bp)) : 0.f;
+    if constexpr (!CHN) {  // summed log decays
+      float g = tid < n ? -A * softplus(ld((const T*)a.a + (long)(t0 + tid) * a.lda + h) + a.dt[h]) : 0.f;
 #pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      s += G[i][d];
-      G[i][d] = s;
+      for (int o = 1; o < CH; o *= 2) {
+        const float up = __shfl_up(g, o, CH);
+        if (tid >= o) g += up;
+      }
+      Gs[tid] = g;
+    }
+  }
+  const int gd = D / N, gv = V / N, ng = 2 * gd + gv;
+  for (int e = tid; e < 4 * ng; e += 256) {  // four tokens of N channels
+    const int i0 = e / ng * 4, gr = e % ng;
+    const int c = gr < gd ? kh * D + gr * N : (gr < 2 * gd ? KD + kh * D + (gr - gd) * N : 2 * KD + h * V + (gr - 2 * gd) * N);
+    __attribute__((aligned(16))) float y[4][N];
+    conv4<T, N>(conv, p0 + i0, n - i0, c, y);
+    if (gr >= 2 * gd) {
+      T* v = (T*)w.v + (long)(t0 + i0) * a.H * V + (c - 2 * KD);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (i0 + i < n) stn<T, N>(v + (long)i * a.H * V, y[i]);
+    } else {
+      float* x = gr < gd ? &qx[i0][gr * N] : &kx[i0][(gr - gd) * N];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) stf<N>(x + i * LD, y[i]);
+    }
+  }
+  if (D < DP)
+    for (int e = tid; e < CH * (DP - D); e += 256) {
+      const int i = e / (DP - D), d = D + e % (DP - D);
+      kx[i][d] = 0.f;
+      qx[i][d] = 0.f;
+      if constexpr (CHN) G[i][d] = 0.f;
+    }
+  if constexpr (CHN) {
+    for (int e = tid; e < CH * gd; e += 256) {
+      const int i = e / gd, d = e % gd * N;
+      __attribute__((aligned(16))) float v[N];
+#pragma unroll
+      for (int k = 0; k < N; ++k) v[k] = 0.f;
+      if (i < n) {
+        ldn<T, N>((const T*)a.a + (long)(t0 + i) * a.lda + (long)h * D + d, v);
+#pragma unroll
+        for (int k = 0; k < N; ++k) v[k] = -A * softplus(v[k] + a.dt[(long)h * D + d + k]);
+      }
+      stf<N>(&G[i][d], v);
     }
   }
   __syncthreads();
-  {  // A and P: wave = level of the split, half size s
-    const int m = lane & 15, g = lane >> 4, s = 8 >> wid;
-    const int piv = (m & ~(2 * s - 1)) + s - 1;
-    f32x4 ka = {0.f, 0.f, 0.f, 0.f}, pa = {0.f, 0.f, 0.f, 0.f};
+  {  // unit vectors: 16 threads per token
+    const int i = tid >> 4;
+    float kk = 0.f, qq = 0.f, qk = 0.f;
+    for (int d = 4 * (tid & 15); d < DP; d += 64) {
+      const f32x4 k4 = *(const f32x4*)&kx[i][d], q4 = *(const f32x4*)&qx[i][d];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        kk = fmaf(k4[j], k4[j], kk);
+        qq = fmaf(q4[j], q4[j], qq);
+        qk = fmaf(q4[j], k4[j], qk);
+      }
+    }
+#pragma unroll
+    for (int o = 8; o > 0; o >>= 1) {
+      kk += __shfl_xor(kk, o, 64);
+      qq += __shfl_xor(qq, o, 64);
+      qk += __shfl_xor(qk, o, 64);
+    }
+    const float ik = 1.f / sqrtf(kk + 1e-6f), iq = 1.f / sqrtf(qq + 1e-6f) / sqrtf((float)D);
+    for (int d = 4 * (tid & 15); d < DP; d += 64) {
+      *(f32x4*)&kx[i][d] *= ik;
+      *(f32x4*)&qx[i][d] *= iq;
+    }
+    if ((tid & 15) == 0) dot[i] = qk * ik * iq;
+  }
+  if constexpr (CHN) {
+    for (int d = tid; d < DP; d += 256) {
+      float s = 0.f;
+#pragma unroll
+      for (int i = 0; i < CH; ++i) {
+        s += G[i][d];
+        G[i][d] = s;
+      }
+    }
+  }
+  __syncthreads();
+  float* ws = w.ws + ((long)ci * a.H + h) * L::N;
+  const int m = lane & 15, g = lane >> 4;
+  f32x4 ka = {0.f, 0.f, 0.f, 0.f}, pa = {0.f, 0.f, 0.f, 0.f};
+  if constexpr (CHN) {  // A and P: wave = level of the split, half size s
+    const int s = 8 >> wid, piv = (m & ~(2 * s - 1)) + s - 1;
 #pragma unroll 2
     for (int r = 0; r < R; ++r) {
       const int d = 16 * r + 4 * g;
-      const float4 k4 = *(const float4*)&kx[m][d], q4 = *(const float4*)&qx[m][d];
-      const float4 g4 = *(const float4*)&G[m][d], v4 = *(const float4*)&G[piv][d];
-      const float kk[4] = {k4.x, k4.y, k4.z, k4.w}, qq[4] = {q4.x, q4.y, q4.z, q4.w};
-      const float dd[4] = {g4.x - v4.x, g4.y - v4.y, g4.z - v4.z, g4.w - v4.w};
+      const f32x4 k4 = *(const f32x4*)&kx[m][d], q4 = *(const f32x4*)&qx[m][d];
+      const f32x4 g4 = *(const f32x4*)&G[m][d], v4 = *(const f32x4*)&G[piv][d];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const float e = expf(-fabsf(dd[i]));
-        const float x = kk[i] * e, y = qq[i] * e;
+        const float e = expf(-fabsf(g4[i] - v4[i]));
+        const float x = k4[i] * e, y = q4[i] * e;
         ka = __builtin_amdgcn_mfma_f32_16x16x4f32(x, x, ka, 0, 0, 0);
         pa = __builtin_amdgcn_mfma_f32_16x16x4f32(y, x, pa, 0, 0, 0);
       }
@@ -297,166 +403,223 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
         Ps[r][m] = pa[i];
       }
     }
-  }
-  __syncthreads();
-  float* ws = w.ws + ((long)ci * a.H + h) * L::N;
-  if (tid < CH) {  // column tid of T, by forward substitution
-    float x[CH];
+  } else {  // one product each, the key width cut over the waves
+    for (int r = wid; r < R; r += 4) {
+      const int d = 16 * r + 4 * g;
+      const f32x4 k4 = *(const f32x4*)&kx[m][d], q4 = *(const f32x4*)&qx[m][d];
 #pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      float y = i == tid ? beta[i] : 0.f;
+      for (int i = 0; i < 4; ++i) {
+        ka = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[i], k4[i], ka, 0, 0, 0);
+        pa = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[i], k4[i], pa, 0, 0, 0);
+      }
+    }
+    if (wid) {
+      red[wid - 1][0][lane] = ka;
+      red[wid - 1][1][lane] = pa;
+    }
+    __syncthreads();
+    if (wid == 0) {
 #pragma unroll
-      for (int j = 0; j < i; ++j) y = fmaf(-As[i][j], x[j], y);
-      x[i] = y;
-      ws[L::T + i * CH + tid] = y;
+      for (int j = 0; j < 3; ++j) {
+        ka += red[j][0][lane];
+        pa += red[j][1][lane];
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int r = 4 * g + i;
+        const float e = expf(fminf(Gs[r] - Gs[m], 0.f));
+        As[r][m] = r > m ? beta[r] * ka[i] * e : 0.f;
+        Ps[r][m] = pa[i] * e;
+      }
+      asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");  // read below by other lanes of this wave
     }
   }
-  if (tid >= 64 && tid < 64 + CH) {  // column of P
-    const int c = tid - 64;
+  // Scaled operands: the waves that do not solve for T. Everything they read is in place since the last barrier.
+  if constexpr (CHN) __syncthreads();
+  if (wid == 0) {
+    if (tid < CH) {  // column tid of T, by forward substitution (this wave's own LDS writes, or behind the barrier)
+      float x[CH];
 #pragma unroll
-    for (int i = 0; i < CH; ++i) ws[L::P + i * CH + c] = i > c ? Ps[i][c] : (i == c ? dot[i] : 0.f);
+      for (int i = 0; i < CH; ++i) {
+        float y = i == tid ? beta[i] : 0.f;
+#pragma unroll
+        for (int j = 0; j < i; ++j) y = fmaf(-As[i][j], x[j], y);
+        x[i] = y;
+        ws[L::T + i * CH + tid] = y;
+      }
+    } else if (tid < 2 * CH) {  // column of P
+      const int c = tid - CH;
+#pragma unroll
+      for (int i = 0; i < CH; ++i) ws[L::P + i * CH + c] = i > c ? Ps[i][c] : (i == c ? dot[i] : 0.f);
+    }
+    return;
   }
-  for (int e = tid; e < CH * DP / 4; e += 256) {
+  const int tw = tid - 64;  // 192 threads
+  auto gl = [&](int i, int d) { return CHN ? G[i][d] : Gs[i]; };
+  for (int e = tw; e < CH * DP / 4; e += 192) {
     const int i = e / (DP / 4), d = e % (DP / 4) * 4;
-    const float4 k4 = *(const float4*)&kx[i][d], q4 = *(const float4*)&qx[i][d];
-    const float4 g4 = *(const float4*)&G[i][d], l4 = *(const float4*)&G[CH - 1][d];
-    const float ex = expf(g4.x), ey = expf(g4.y), ez = expf(g4.z), ew = expf(g4.w);
-    *(float4*)(ws + L::KT + i * DP + d) = make_float4(k4.x * ex, k4.y * ey, k4.z * ez, k4.w * ew);
-    *(float4*)(ws + L::QT + i * DP + d) = make_float4(q4.x * ex, q4.y * ey, q4.z * ez, q4.w * ew);
-    *(float4*)(ws + L::KE + i * DP + d) = make_float4(k4.x * expf(l4.x - g4.x), k4.y * expf(l4.y - g4.y),
-                                                      k4.z * expf(l4.z - g4.z), k4.w * expf(l4.w - g4.w));
+    const f32x4 k4 = *(const f32x4*)&kx[i][d], q4 = *(const f32x4*)&qx[i][d];
+    f32x4 ex;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) ex[j] = (CHN || j == 0) ? expf(gl(i, d + j)) : ex[0];
+    *(f32x4*)(ws + L::KT + i * DP + d) = k4 * ex;
+    *(f32x4*)(ws + L::QT + i * DP + d) = q4 * ex;
   }
-  for (int d = tid; d < DP; d += 256) ws[L::EG + d] = expf(G[CH - 1][d]);
+  for (int e = tw; e < DP * 4; e += 192) {
+    const int d = e >> 2, i = (e & 3) * 4;
+    f32x4 y;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) y[j] = kx[i + j][d] * expf(gl(CH - 1, d) - gl(i + j, d));
+    *(f32x4*)(ws + L::KE + d * CH + i) = y;
+  }
+  for (int d = tw; d < DP; d += 192) ws[L::EG + d] = expf(gl(CH - 1, d));
 }
 
-// Workgroup = (run, head, 64 value columns), wave = 16 columns: the state's columns as DP / 16 MFMA
-// accumulators (row 16 r + 4 g + i, column lane % 16), which are at once the B operands of the products with
-// S0 (k index of step (r, i): row 16 r + 4 g + i for lane group g). The chunk's operands are shared through
-// LDS, two buffers, the next chunk's loads in flight during the products.
+// Workgroup = (run, head, 16 value columns); NW waves hold RW 16-row tiles of the state's columns each, as MFMA
+// accumulators (row 16 r + 4 g + i, column lane % 16), which are at once the B operands of the products with S0
+// (k index of step (r, i): row 16 r + 4 g + i for lane group g). The waves' shares of those products meet in LDS,
+// one barrier per chunk; every wave solves for U by itself. Operands go straight to registers, two chunks ahead.
+template <int RW> struct ScanOps { f32x4 k[RW], q[RW], e[RW], g[RW], t, p; float v[4]; };
+
 template <typename T, int DP>
-__global__ __launch_bounds__(256) void delta_scan_kernel(Args a, Work w, const int* first_chunk) {
-  constexpr int LD = DP + 4, R = DP / 16;
+__global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 : 256) void delta_scan_kernel(Args a, Work w, const int* first_chunk) {
+  constexpr int R = DP / 16, NW = R < 4 ? R : 4, RW = R / NW;
   using L = Lay<DP>;
-  constexpr int N4 = L::N / 4, NLD = (N4 + 255) / 256;
-  // LDS image of a chunk: KT, QT, KE rows padded to LD, then EG, T, P
-  constexpr int IK = 0, IQ = CH * LD, IE = 2 * CH * LD, IG = 3 * CH * LD, IT = IG + DP, IP = IT + CH * CH, IN = IP + CH * CH;
-  __shared__ __attribute__((aligned(16))) float sm[2][IN];
+  __shared__ f32x4 part[2][NW][2][64];
   const int tid = threadIdx.x, lane = tid & 63, m = lane & 15, g = lane >> 4;
   const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
-  const int VB = (a.V + 63) / 64;
-  const int vb = blockIdx.x % VB, h = blockIdx.x / VB % a.H, ri = blockIdx.x / (VB * a.H);
+  const int VB = (a.V + 15) / 16, lin = xcd_remap(blockIdx.x, gridDim.x);
+  const int vb = lin % VB, h = lin / VB % a.H, ri = lin / (VB * a.H);
   const int4 run = w.runs[ri];
   const int nc = (run.z + CH - 1) / CH, c0 = first_chunk[ri];
-  const int col = vb * 64 + wid * 16 + m;
-  const bool ok = col < a.V;
-  const bool live = run.x >= 0 && run.x < a.n_rows;
+  const int col = vb * 16 + m, d0 = 16 * RW * wid;
+  const bool ok = col < a.V, live = run.x >= 0 && run.x < a.n_rows;
   float* Sp = a.S + ((long)max(run.x, 0) * a.H + h) * a.D * a.V + (ok ? col : 0);
-  f32x4 S[R];
-#pragma unroll
-  for (int r = 0; r < R; ++r)
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int d = 16 * r + 4 * g + i;
-      S[r][i] = live && run.w > 0 && ok && d < a.D ? Sp[(long)d * a.V] : 0.f;
-    }
-  float4 pre[NLD];
-  auto load = [&](int c) {
-    const float4* src = (const float4*)(w.ws + ((long)(c0 + c) * a.H + h) * L::N);
-#pragma unroll
-    for (int j = 0; j < NLD; ++j) pre[j] = src[min(tid + 256 * j, N4 - 1)];
-  };
-  auto place = [&](int b) {
-#pragma unroll
-    for (int j = 0; j < NLD; ++j) {
-      const int e = (tid + 256 * j) * 4;
-      if (e >= L::N) continue;
-      const int at = e < L::EG ? e / DP * LD + e % DP : IG + e - L::EG;
-      *(float4*)&sm[b][at] = pre[j];
-    }
-  };
   const long ldv = (long)a.H * a.V;
   const T* vp = (const T*)w.v + (long)run.y * ldv + (long)h * a.V + (ok ? col : 0);
   float* op = w.o + (long)run.y * ldv + (long)h * a.V + (ok ? col : 0);
-  float vn[4];
-  auto load_v = [&](int c) {
+  const float* wp = w.ws + ((long)c0 * a.H + h) * L::N;
+  auto load_kq = [&](ScanOps<RW>& s, int c) {
+    const float* p = wp + (long)min(c, nc - 1) * a.H * L::N + m * DP + d0 + 4 * g;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = c * CH + 4 * g + i;
-      vn[i] = ok && t < run.z ? ld(vp + (long)t * ldv) : 0.f;
+    for (int r = 0; r < RW; ++r) {
+      s.k[r] = *(const f32x4*)(p + L::KT + 16 * r);
+      s.q[r] = *(const f32x4*)(p + L::QT + 16 * r);
     }
   };
-  load(0);
-  load_v(0);
-  for (int c = 0; c < nc; ++c) {
-    const float* s = sm[c & 1];
-    place(c & 1);
-    float v[4];
+  auto load_rest = [&](ScanOps<RW>& s, int c) {
+    c = min(c, nc - 1);
+    const float* p = wp + (long)c * a.H * L::N;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) v[i] = vn[i];
-    __syncthreads();  // this image is whole; the other one is written only after the next barrier's arrivals
-    if (c + 1 < nc) {
-      load(c + 1);
-      load_v(c + 1);
+    for (int i = 0; i < 4; ++i) s.v[i] = ld(vp + (long)min(c * CH + 4 * g + i, run.z - 1) * ldv);  // past the run: beta is 0
+    s.t = *(const f32x4*)(p + L::T + m * CH + 4 * g);
+#pragma unroll
+    for (int r = 0; r < RW; ++r) {
+      s.e[r] = *(const f32x4*)(p + L::KE + (d0 + 16 * r + m) * CH + 4 * g);
+      s.g[r] = *(const f32x4*)(p + L::EG + d0 + 16 * r + 4 * g);
     }
+    s.p = *(const f32x4*)(p + L::P + m * CH + 4 * g);
+  };
+  f32x4 S[RW];
+  auto chunk = [&](ScanOps<RW>& s, int c) {
     f32x4 x[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}}, o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
 #pragma unroll
-    for (int r = 0; r < R; ++r) {
-      const f32x4 k4 = *(const f32x4*)(s + IK + m * LD + 16 * r + 4 * g), q4 = *(const f32x4*)(s + IQ + m * LD + 16 * r + 4 * g);
+    for (int r = 0; r < RW; ++r)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) x[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(s.k[r][i], S[r][i], x[i & 1], 0, 0, 0);
+#pragma unroll
+    for (int r = 0; r < RW; ++r)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(s.q[r][i], S[r][i], o[i & 1], 0, 0, 0);
+    load_kq(s, c + 2);
+    const int b = c & 1;
+    part[b][wid][0][lane] = x[0] + x[1];
+    part[b][wid][1][lane] = o[0] + o[1];
+    // the shares are whole; this buffer is written again only behind the next chunk's barrier. Global loads stay in flight
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    asm volatile("s_barrier" ::: "memory");
+    f32x4 wv = {s.v[0], s.v[1], s.v[2], s.v[3]}, u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < NW; ++j) wv -= part[b][j][0][lane];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(s.t[i], wv[i], u, 0, 0, 0);
+#pragma unroll
+    for (int r = 0; r < RW; ++r) S[r] *= s.g[r];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int r = 0; r < RW; ++r) S[r] = __builtin_amdgcn_mfma_f32_16x16x4f32(s.e[r][i], u[i], S[r], 0, 0, 0);
+    if (wid == (c & (NW - 1))) {  // one wave finishes the read-outs
+      f32x4 oo = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < NW; ++j) oo += part[b][j][1][lane];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(s.p[i], u[i], oo, 0, 0, 0);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        x[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(k4[i], S[r][i], x[i & 1], 0, 0, 0);
-        o[i & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(q4[i], S[r][i], o[i & 1], 0, 0, 0);
+        const int t = c * CH + 4 * g + i;
+        if (ok && t < run.z) op[(long)t * ldv] = oo[i];
       }
     }
-    f32x4 wv, u = {0.f, 0.f, 0.f, 0.f};
+    load_rest(s, c + 2);
+  };
+  ScanOps<RW> s0, s1;
+  load_kq(s0, 0);
+  load_rest(s0, 0);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) wv[i] = v[i] - (x[0][i] + x[1][i]);
-    const f32x4 t4 = *(const f32x4*)(s + IT + m * CH + 4 * g), p4 = *(const f32x4*)(s + IP + m * CH + 4 * g);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(t4[i], wv[i], u, 0, 0, 0);
-    f32x4 oo = o[0] + o[1];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(p4[i], u[i], oo, 0, 0, 0);
-#pragma unroll
-    for (int r = 0; r < R; ++r) {
-      f32x4 d = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int i = 0; i < 4; ++i)
-        d = __builtin_amdgcn_mfma_f32_16x16x4f32(s[IE + (4 * g + i) * LD + 16 * r + m], u[i], d, 0, 0, 0);
-      const f32x4 eg = *(const f32x4*)(s + IG + 16 * r + 4 * g);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) S[r][i] = fmaf(S[r][i], eg[i], d[i]);
-    }
+  for (int r = 0; r < RW; ++r)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int t = c * CH + 4 * g + i;
-      if (ok && t < run.z) op[(long)t * ldv] = oo[i];
+      const int d = d0 + 16 * r + 4 * g + i;
+      S[r][i] = live && run.w > 0 && ok && d < a.D ? Sp[(long)d * a.V] : 0.f;
     }
+  load_kq(s1, 1);
+  load_rest(s1, 1);
+  for (int c = 0; c < nc; c += 2) {
+    chunk(s0, c);
+    if (c + 1 < nc) chunk(s1, c + 1);
   }
   if (live && ok) {
 #pragma unroll
-    for (int r = 0; r < R; ++r)
+    for (int r = 0; r < RW; ++r)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int d = 16 * r + 4 * g + i;
+        const int d = d0 + 16 * r + 4 * g + i;
         if (d < a.D) Sp[(long)d * a.V] = S[r][i];
       }
   }
 }
 
-// read-outs -> normed, weighted, gated rows: wave = one (token, head)
-template <typename T>
-__global__ __launch_bounds__(256) void delta_out_kernel(Args a, const float* __restrict__ o, int t0) {
-  const int lane = threadIdx.x & 63, h = blockIdx.x * 4 + (threadIdx.x >> 6);
-  const long t = t0 + (long)blockIdx.y;
-  if (h >= a.H) return;
+// read-outs -> normed, weighted, gated rows: LPR lanes (a power of two) per (token, head), N columns each at a time
+template <typename T, int N>
+__global__ __launch_bounds__(256) void delta_out_kernel(Args a, const float* __restrict__ o, long row0, long rows, int LPR) {
+  const int lane = threadIdx.x & 63, l = lane & (LPR - 1);
+  const long th = row0 + ((long)blockIdx.x * 256 + threadIdx.x) / LPR;  // token * H + head
+  const bool in = th < row0 + rows;
+  const long t = (in ? th : row0) / a.H;
+  const int h = (int)((in ? th : row0) % a.H);
   const float* op = o + (t * a.H + h) * a.V;
   float s = 0.f;
-  for (int c = lane; c < a.V; c += 64) s += op[c] * op[c];
-  const float r = a.out_scale / sqrtf(wave_sum(s) / a.V + a.eps);
-  for (int c = lane; c < a.V; c += 64)
-    st((T*)a.out + t * a.ldo + (long)h * a.V + c,
-       op[c] * r * ld((const T*)a.norm_w + c) * gate_of(ld((const T*)a.z + t * a.ldz + (long)h * a.V + c), a.silu));
+  for (int c = l * N; c < a.V; c += LPR * N) {
+    __attribute__((aligned(16))) float ov[N];
+    ldf<N>(op + c, ov);
+#pragma unroll
+    for (int e = 0; e < N; ++e) s = fmaf(ov[e], ov[e], s);
+  }
+  for (int x = LPR >> 1; x > 0; x >>= 1) s += __shfl_xor(s, x, 64);
+  const float r = a.out_scale / sqrtf(s / a.V + a.eps);
+  if (!in) return;
+  const T* z = (const T*)a.z + t * a.ldz + (long)h * a.V;
+  T* out = (T*)a.out + t * a.ldo + (long)h * a.V;
+  for (int c = l * N; c < a.V; c += LPR * N) {
+    __attribute__((aligned(16))) float ov[N], zv[N], wv[N], y[N];
+    ldf<N>(op + c, ov);
+    ldn<T, N>(z + c, zv);
+    ldn<T, N>((const T*)a.norm_w + c, wv);
+#pragma unroll
+    for (int e = 0; e < N; ++e) y[e] = ov[e] * r * wv[e] * gate_of(zv[e], a.silu);
+    stn<T, N>(out + c, y);
+  }
 }
 
 // the last projections of every run into its row's ring (behind delta_prep, which reads the old ones)
@@ -515,20 +678,32 @@ static int step(const Args& a, int n, hipStream_t st_) {
 template <typename T, int DP>
 static int runs_(const Args& a, const Work& w, const int* first_chunk, int n_runs, int n_chunks, int t0, int n_tokens,
                  hipStream_t st_) {
+  constexpr int N = 16 / sizeof(T);
+  auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
+  const bool vec = a.D % N == 0 && a.V % N == 0 && a.ldx % N == 0 && al(a.x) && al(a.ring) && al(w.v) &&
+                   (!a.channel || (a.lda % N == 0 && al(a.a)));
+  const bool vec_out = a.V % N == 0 && a.ldz % N == 0 && a.ldo % N == 0 && al(a.z) && al(a.out) && al(a.norm_w) && al(w.o);
   for (int c0 = 0; c0 < n_chunks; c0 += 65535) {
     Work q = w;
     q.chunks = w.chunks + c0;
     q.ws = w.ws + (long)c0 * a.H * Lay<DP>::N;
-    hipLaunchKernelGGL((delta_prep_kernel<T, DP>), dim3(a.H, std::min(n_chunks - c0, 65535)), dim3(256), 0, st_, a, q);
+    const dim3 grid(a.H, std::min(n_chunks - c0, 65535));
+    if (a.channel && vec) hipLaunchKernelGGL((delta_prep_kernel<T, DP, true, N>), grid, dim3(256), 0, st_, a, q);
+    else if (a.channel) hipLaunchKernelGGL((delta_prep_kernel<T, DP, true, 1>), grid, dim3(256), 0, st_, a, q);
+    else if (vec) hipLaunchKernelGGL((delta_prep_kernel<T, DP, false, N>), grid, dim3(256), 0, st_, a, q);
+    else hipLaunchKernelGGL((delta_prep_kernel<T, DP, false, 1>), grid, dim3(256), 0, st_, a, q);
     RT_LAUNCH_CHECK();
   }
-  hipLaunchKernelGGL((delta_scan_kernel<T, DP>), dim3((unsigned)((long)n_runs * a.H * ((a.V + 63) / 64))), dim3(256), 0, st_, a,
-                     w, first_chunk);
+  hipLaunchKernelGGL((delta_scan_kernel<T, DP>), dim3((unsigned)((long)n_runs * a.H * ((a.V + 15) / 16))),
+                     dim3(std::min(DP * 4, 256)), 0, st_, a, w, first_chunk);
   RT_LAUNCH_CHECK();
-  for (int c = 0; c < n_tokens; c += 65535) {
-    hipLaunchKernelGGL((delta_out_kernel<T>), dim3((a.H + 3) / 4, std::min(n_tokens - c, 65535)), dim3(256), 0, st_, a, w.o, t0 + c);
-    RT_LAUNCH_CHECK();
-  }
+  int lpr = 1;
+  while (lpr < 64 && lpr * (vec_out ? N : 1) < a.V) lpr *= 2;
+  const long rows = (long)n_tokens * a.H, row0 = (long)t0 * a.H;
+  const dim3 grid((unsigned)((rows * lpr + 255) / 256));
+  if (vec_out) hipLaunchKernelGGL((delta_out_kernel<T, N>), grid, dim3(256), 0, st_, a, w.o, row0, rows, lpr);
+  else hipLaunchKernelGGL((delta_out_kernel<T, 1>), grid, dim3(256), 0, st_, a, w.o, row0, rows, lpr);
+  RT_LAUNCH_CHECK();
   const int C = 2 * a.K * a.D + a.H * a.V;
   hipLaunchKernelGGL((delta_commit_kernel<T>), dim3((C + 255) / 256, n_runs), dim3(256), 0, st_, a, w.runs);
   RT_LAUNCH_CHECK();
