@@ -612,7 +612,7 @@ void delta_rule(const Tensor& x, const Tensor& b, const Tensor& a, const Tensor&
   const long per = rt_delta_ws((int)D);
   TORCH_CHECK(per > 0, "delta_rule: key width ", D, " above 256");
   Tensor ws = at::empty({chunks->size(0) * H * per}, x.options().dtype(at::kFloat));
-  Tensor v = at::empty({N, H * V}, x.options()), o = at::empty({N, H * V}, x.options().dtype(at::kFloat));
+  Tensor v = at::empty({N, (H * V + 1) / 2 * 2}, x.options()), o = at::empty({N, H * V}, x.options().dtype(at::kFloat));
   rc_ok(rt_delta_runs(is_f32(x), &d, runs->data_ptr(), chunks->data_ptr(), first_chunk->data_ptr<int>(), (int)runs->size(0),
                       (int)chunks->size(0), (int)n_single, (int)(N - n_single), ws.data_ptr<float>(), v.data_ptr(),
                       o.data_ptr<float>(), stream()),

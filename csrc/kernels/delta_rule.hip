@@ -35,7 +35,7 @@ template <typename T> __device__ __forceinline__ void st(T* p, float v);
 template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
 
-__device__ __forceinline__ float sigmoid(float x) { return 1.f / (1.f + expf(-x)); }
+__device__ __forceinline__ float sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + expf(-x)); }
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float gate_of(float z, bool silu) { return (silu ? z : 1.f) * sigmoid(z); }
 
@@ -205,8 +205,10 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
 // T, P [CH][CH] floats.
 struct Work {
   const int4* runs; const int2* chunks;
-  float* ws;
-  void* v;      // [N, H * V] convolved values, rows of the batch's tokens
+  float* ws;    // a head's chunks side by side
+  int n_chunks, chunk0;
+  long ldv;
+  void* v;      // [N, ldv] convolved values, rows of the batch's tokens; ldv = H * V, even
   float* o;     // [N, H * V] read-outs
 };
 template <int DP> struct Lay {
@@ -240,26 +242,44 @@ __device__ __forceinline__ void ldf(const float* p, float* o) {
 template <int N>
 __device__ __forceinline__ void stf(float* p, const float* o) { ldf<N>(o, p); }
 
-// convolution and silu of channels c .. c + N - 1 at positions p .. p + 3, zeros from position p + n on
-template <typename T, int N>
+// convolution and silu of channels c .. c + N - 1 at positions p .. p + 3, zeros from position p + n on. TAPS: their
+// number (every load issued ahead), 0: any
+template <typename T, int N, int TAPS>
 __device__ __forceinline__ void conv4(const Conv<T>& cv, int p, int n, int c, float (&y)[4][N]) {
-  const int taps = cv.a.taps;
+  const int taps = TAPS ? TAPS : cv.a.taps;
   const T* w = (const T*)cv.a.conv + (long)c * taps;
+  // a row that counts as zero stays unread
+  auto row = [&](int q, float (&v)[N]) {
+    const T* src = q >= cv.start ? cv.x + (long)(q - cv.start) * cv.a.ldx : cv.ring + (long)(max(q, 0) % taps) * cv.C;
+#pragma unroll
+    for (int e = 0; e < N; ++e) v[e] = 0.f;
+    if (q < p + n && (q >= cv.start || (cv.ring && q >= 0))) ldn<T, N>(src + c, v);
+  };
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int e = 0; e < N; ++e) y[i][e] = 0.f;
-  for (int j = 0; j < taps; ++j) {
-    float wj[N];
+  if constexpr (TAPS > 0) {
+    __attribute__((aligned(16))) float v[TAPS + 3][N], f[TAPS][N];  // f: the weights as they lie, [channel][tap]
 #pragma unroll
-    for (int e = 0; e < N; ++e) wj[e] = ld(w + e * taps + j);
+    for (int j = 0; j < TAPS + 3; ++j) row(p - (TAPS - 1) + j, v[j]);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int q = p + i - (taps - 1 - j);
-      const T* src = q >= cv.start ? cv.x + (long)(q - cv.start) * cv.a.ldx : cv.ring + (long)(max(q, 0) % taps) * cv.C;
-      if (i < n && (q >= cv.start || (cv.ring && q >= 0))) {
+    for (int j = 0; j < TAPS; ++j) ldn<T, N>(w + j * N, f[j]);
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < N; ++e) y[i][e] = fmaf((&f[0][0])[e * TAPS + j], v[i + j][e], y[i][e]);
+  } else {
+    for (int j = 0; j < taps; ++j) {
+      float wj[N];
+#pragma unroll
+      for (int e = 0; e < N; ++e) wj[e] = ld(w + e * taps + j);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
         __attribute__((aligned(16))) float v[N];
-        ldn<T, N>(src + c, v);
+        row(p + i - (taps - 1 - j), v);
 #pragma unroll
         for (int e = 0; e < N; ++e) y[i][e] = fmaf(wj[e], v[e], y[i][e]);
       }
@@ -268,11 +288,11 @@ __device__ __forceinline__ void conv4(const Conv<T>& cv, int p, int n, int c, fl
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
-    for (int e = 0; e < N; ++e) y[i][e] *= sigmoid(y[i][e]);
+    for (int e = 0; e < N; ++e) y[i][e] = i < n ? y[i][e] * sigmoid(y[i][e]) : 0.f;
 }
 
 // workgroup = (head, chunk); CHN: a decay per key channel, else per head. N: elements per access
-template <typename T, int DP, bool CHN, int N>
+template <typename T, int DP, bool CHN, int N, int TAPS>
 __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
   constexpr int LD = DP + 4, R = DP / 16;
   using L = Lay<DP>;
@@ -307,12 +327,12 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
     const int i0 = e / ng * 4, gr = e % ng;
     const int c = gr < gd ? kh * D + gr * N : (gr < 2 * gd ? KD + kh * D + (gr - gd) * N : 2 * KD + h * V + (gr - 2 * gd) * N);
     __attribute__((aligned(16))) float y[4][N];
-    conv4<T, N>(conv, p0 + i0, n - i0, c, y);
+    conv4<T, N, TAPS>(conv, p0 + i0, n - i0, c, y);
     if (gr >= 2 * gd) {
-      T* v = (T*)w.v + (long)(t0 + i0) * a.H * V + (c - 2 * KD);
+      T* v = (T*)w.v + (long)(t0 + i0) * w.ldv + (c - 2 * KD);
 #pragma unroll
       for (int i = 0; i < 4; ++i)
-        if (i0 + i < n) stn<T, N>(v + (long)i * a.H * V, y[i]);
+        if (i0 + i < n) stn<T, N>(v + i * w.ldv, y[i]);
     } else {
       float* x = gr < gd ? &qx[i0][gr * N] : &kx[i0][(gr - gd) * N];
 #pragma unroll
@@ -377,7 +397,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
     }
   }
   __syncthreads();
-  float* ws = w.ws + ((long)ci * a.H + h) * L::N;
+  float* ws = w.ws + ((long)h * w.n_chunks + w.chunk0 + ci) * L::N;
   const int m = lane & 15, g = lane >> 4;
   f32x4 ka = {0.f, 0.f, 0.f, 0.f}, pa = {0.f, 0.f, 0.f, 0.f};
   if constexpr (CHN) {  // A and P: wave = level of the split, half size s
@@ -478,11 +498,20 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
 // Workgroup = (run, head, 16 value columns); NW waves hold RW 16-row tiles of the state's columns each, as MFMA
 // accumulators (row 16 r + 4 g + i, column lane % 16), which are at once the B operands of the products with S0
 // (k index of step (r, i): row 16 r + 4 g + i for lane group g). The waves' shares of those products meet in LDS,
-// one barrier per chunk; every wave solves for U by itself. Operands go straight to registers, two chunks ahead.
-template <int RW> struct ScanOps { f32x4 k[RW], q[RW], e[RW], g[RW], t, p; float v[4]; };
+// one barrier per chunk; every wave solves for U by itself, and one more finishes the read-outs off the chain from
+// chunk to chunk. Operands go straight to registers, two chunks ahead.
+// Values stay the 32-bit words they were loaded as until they are used (anything done at the load waits for it); a
+// lane's bf16 value is the word's upper half if `odd`
+template <typename T> __device__ __forceinline__ float of_word(uint32_t r, bool odd) {
+  return __uint_as_float(sizeof(T) == 4 || odd ? (sizeof(T) == 4 ? r : r & 0xffff0000u) : r << 16);
+}
+template <int RW> struct ScanOps { f32x4 k[RW], q[RW], e[RW], g[RW], t; uint32_t v[4]; };
+// uniform base, the lane's byte offset
+template <typename V> __device__ __forceinline__ V at(const void* base, uint32_t off) { return *(const V*)((const char*)base + off); }
+struct ReadOps { f32x4 t, p; uint32_t v[4]; };
 
 template <typename T, int DP>
-__global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 : 256) void delta_scan_kernel(Args a, Work w, const int* first_chunk) {
+__global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 + 64 : 320, DP > 128 ? 2 : 4) void delta_scan_kernel(Args a, Work w, const int* first_chunk) {
   constexpr int R = DP / 16, NW = R < 4 ? R : 4, RW = R / NW;
   using L = Lay<DP>;
   __shared__ f32x4 part[2][NW][2][64];
@@ -495,31 +524,85 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 : 256) void delta_scan_kernel(
   const int col = vb * 16 + m, d0 = 16 * RW * wid;
   const bool ok = col < a.V, live = run.x >= 0 && run.x < a.n_rows;
   float* Sp = a.S + ((long)max(run.x, 0) * a.H + h) * a.D * a.V + (ok ? col : 0);
-  const long ldv = (long)a.H * a.V;
-  const T* vp = (const T*)w.v + (long)run.y * ldv + (long)h * a.V + (ok ? col : 0);
-  float* op = w.o + (long)run.y * ldv + (long)h * a.V + (ok ? col : 0);
-  const float* wp = w.ws + ((long)c0 * a.H + h) * L::N;
+  const long ldo = (long)a.H * a.V, vc = (long)h * a.V + (ok ? col : 0);
+  constexpr int PER = 4 / sizeof(T);  // values per word
+  const uint32_t* vp = (const uint32_t*)w.v + (long)run.y * w.ldv / PER;
+  const uint32_t ldw = (uint32_t)(w.ldv / PER), vw = (uint32_t)(vc / PER);
+  const bool odd = vc & 1;
+  float* op = w.o + (long)run.y * ldo;
+  const float* wp = w.ws + ((long)h * w.n_chunks + c0) * L::N;
+  const uint32_t o_kq = 4 * (m * DP + d0 + 4 * g), o_e = 4 * (L::KE + (d0 + m) * CH + 4 * g), o_g = 4 * (L::EG + d0 + 4 * g),
+                 o_t = 4 * (L::T + m * CH + 4 * g);
   auto load_kq = [&](ScanOps<RW>& s, int c) {
-    const float* p = wp + (long)min(c, nc - 1) * a.H * L::N + m * DP + d0 + 4 * g;
+    const float* p = wp + (long)min(c, nc - 1) * L::N;
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
-      s.k[r] = *(const f32x4*)(p + L::KT + 16 * r);
-      s.q[r] = *(const f32x4*)(p + L::QT + 16 * r);
+      s.k[r] = at<f32x4>(p + L::KT + 16 * r, o_kq);
+      s.q[r] = at<f32x4>(p + L::QT + 16 * r, o_kq);
     }
+  };
+  auto load_tv = [&](auto& s, int c) {  // c < nc
+    const uint32_t* p = vp + (long)c * CH * ldw;
+    const int last = run.z - 1 - c * CH;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)  // past the run: beta is 0
+      s.v[i] = at<uint32_t>(p, 4 * (__umul24((uint32_t)min(4 * g + i, last), ldw) + vw));
+    s.t = at<f32x4>(wp + (long)c * L::N, o_t);
   };
   auto load_rest = [&](ScanOps<RW>& s, int c) {
     c = min(c, nc - 1);
-    const float* p = wp + (long)c * a.H * L::N;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) s.v[i] = ld(vp + (long)min(c * CH + 4 * g + i, run.z - 1) * ldv);  // past the run: beta is 0
-    s.t = *(const f32x4*)(p + L::T + m * CH + 4 * g);
+    load_tv(s, c);
+    const float* p = wp + (long)c * L::N;
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
-      s.e[r] = *(const f32x4*)(p + L::KE + (d0 + 16 * r + m) * CH + 4 * g);
-      s.g[r] = *(const f32x4*)(p + L::EG + d0 + 16 * r + 4 * g);
+      s.e[r] = at<f32x4>(p + 16 * r * CH, o_e);
+      s.g[r] = at<f32x4>(p + 16 * r, o_g);
     }
-    s.p = *(const f32x4*)(p + L::P + m * CH + 4 * g);
   };
+  // U from the shares of k e^G S0 in buffer b
+  auto solve = [&](auto& s, int b) {
+#pragma unroll
+    for (int i = 0; i < 4; ++i) asm volatile("" : "+v"(s.v[i]));  // nothing of this chunk is used ahead of its barrier
+    f32x4 wv = {of_word<T>(s.v[0], odd), of_word<T>(s.v[1], odd), of_word<T>(s.v[2], odd), of_word<T>(s.v[3], odd)}, u = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int j = 0; j < NW; ++j) wv -= part[b][j][0][lane];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(s.t[i], wv[i], u, 0, 0, 0);
+    return u;
+  };
+  if (wid == NW) {  // read-outs
+    ReadOps r0, r1;
+    auto load = [&](ReadOps& s, int c) {
+      c = min(c, nc - 1);
+      load_tv(s, c);
+      s.p = at<f32x4>(wp + (long)c * L::N + (L::P - L::T), o_t);
+    };
+    auto read = [&](ReadOps& s, int c) {
+      const int b = c & 1;
+      asm volatile("s_barrier" ::: "memory");
+      const f32x4 u = solve(s, b);
+      f32x4 oo = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int j = 0; j < NW; ++j) oo += part[b][j][1][lane];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(s.p[i], u[i], oo, 0, 0, 0);
+      float* oc = op + (long)c * CH * ldo;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (ok && 4 * g + i < run.z - c * CH) *(float*)((char*)oc + 4 * (__umul24((uint32_t)(4 * g + i), (uint32_t)ldo) + (uint32_t)vc)) = oo[i];
+      load(s, c + 2);
+    };
+    load(r0, 0);
+    load(r1, 1);
+    __builtin_amdgcn_s_waitcnt(0x0f70);
+    int c = 0;
+    for (; c + 1 < nc; c += 2) {
+      read(r0, c);
+      read(r1, c + 1);
+    }
+    if (c < nc) read(r0, c);
+    return;
+  }
   f32x4 S[RW];
   auto chunk = [&](ScanOps<RW>& s, int c) {
     f32x4 x[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}}, o[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
@@ -538,29 +621,16 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 : 256) void delta_scan_kernel(
     // the shares are whole; this buffer is written again only behind the next chunk's barrier. Global loads stay in flight
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     asm volatile("s_barrier" ::: "memory");
-    f32x4 wv = {s.v[0], s.v[1], s.v[2], s.v[3]}, u = {0.f, 0.f, 0.f, 0.f};
+    const f32x4 u = solve(s, b);
 #pragma unroll
-    for (int j = 0; j < NW; ++j) wv -= part[b][j][0][lane];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u = __builtin_amdgcn_mfma_f32_16x16x4f32(s.t[i], wv[i], u, 0, 0, 0);
-#pragma unroll
-    for (int r = 0; r < RW; ++r) S[r] *= s.g[r];
+    for (int r = 0; r < RW; ++r) {
+      asm volatile("" : "+v"(s.g[r]));
+      S[r] *= s.g[r];
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int r = 0; r < RW; ++r) S[r] = __builtin_amdgcn_mfma_f32_16x16x4f32(s.e[r][i], u[i], S[r], 0, 0, 0);
-    if (wid == (c & (NW - 1))) {  // one wave finishes the read-outs
-      f32x4 oo = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int j = 0; j < NW; ++j) oo += part[b][j][1][lane];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) oo = __builtin_amdgcn_mfma_f32_16x16x4f32(s.p[i], u[i], oo, 0, 0, 0);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = c * CH + 4 * g + i;
-        if (ok && t < run.z) op[(long)t * ldv] = oo[i];
-      }
-    }
     load_rest(s, c + 2);
   };
   ScanOps<RW> s0, s1;
@@ -575,10 +645,13 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 : 256) void delta_scan_kernel(
     }
   load_kq(s1, 1);
   load_rest(s1, 1);
-  for (int c = 0; c < nc; c += 2) {
+  __builtin_amdgcn_s_waitcnt(0x0f70);  // vmcnt(0): the waits in the loop then count from the loop's own order of loads
+  int c = 0;
+  for (; c + 1 < nc; c += 2) {
     chunk(s0, c);
-    if (c + 1 < nc) chunk(s1, c + 1);
+    chunk(s1, c + 1);
   }
+  if (c < nc) chunk(s0, c);
   if (live && ok) {
 #pragma unroll
     for (int r = 0; r < RW; ++r)
@@ -680,22 +753,27 @@ static int runs_(const Args& a, const Work& w, const int* first_chunk, int n_run
                  hipStream_t st_) {
   constexpr int N = 16 / sizeof(T);
   auto al = [](const void* p) { return (uintptr_t)p % 16 == 0; };
-  const bool vec = a.D % N == 0 && a.V % N == 0 && a.ldx % N == 0 && al(a.x) && al(a.ring) && al(w.v) &&
+  const bool vec = a.D % N == 0 && a.V % N == 0 && a.ldx % N == 0 && al(a.x) && al(a.ring) && al(a.conv) && al(w.v) &&
                    (!a.channel || (a.lda % N == 0 && al(a.a)));
   const bool vec_out = a.V % N == 0 && a.ldz % N == 0 && a.ldo % N == 0 && al(a.z) && al(a.out) && al(a.norm_w) && al(w.o);
   for (int c0 = 0; c0 < n_chunks; c0 += 65535) {
     Work q = w;
     q.chunks = w.chunks + c0;
-    q.ws = w.ws + (long)c0 * a.H * Lay<DP>::N;
+    q.chunk0 = c0;
     const dim3 grid(a.H, std::min(n_chunks - c0, 65535));
-    if (a.channel && vec) hipLaunchKernelGGL((delta_prep_kernel<T, DP, true, N>), grid, dim3(256), 0, st_, a, q);
-    else if (a.channel) hipLaunchKernelGGL((delta_prep_kernel<T, DP, true, 1>), grid, dim3(256), 0, st_, a, q);
-    else if (vec) hipLaunchKernelGGL((delta_prep_kernel<T, DP, false, N>), grid, dim3(256), 0, st_, a, q);
-    else hipLaunchKernelGGL((delta_prep_kernel<T, DP, false, 1>), grid, dim3(256), 0, st_, a, q);
+#define DR_PREP(CHN)                                                                                                          \
+  do {                                                                                                                        \
+    if (!vec) hipLaunchKernelGGL((delta_prep_kernel<T, DP, CHN, 1, 0>), grid, dim3(256), 0, st_, a, q);                       \
+    else if (a.taps == 4) hipLaunchKernelGGL((delta_prep_kernel<T, DP, CHN, N, 4>), grid, dim3(256), 0, st_, a, q);           \
+    else hipLaunchKernelGGL((delta_prep_kernel<T, DP, CHN, N, 0>), grid, dim3(256), 0, st_, a, q);                            \
+  } while (0)
+    if (a.channel) DR_PREP(true);
+    else DR_PREP(false);
+#undef DR_PREP
     RT_LAUNCH_CHECK();
   }
   hipLaunchKernelGGL((delta_scan_kernel<T, DP>), dim3((unsigned)((long)n_runs * a.H * ((a.V + 15) / 16))),
-                     dim3(std::min(DP * 4, 256)), 0, st_, a, w, first_chunk);
+                     dim3(std::min(DP * 4, 256) + 64), 0, st_, a, w, first_chunk);
   RT_LAUNCH_CHECK();
   int lpr = 1;
   while (lpr < 64 && lpr * (vec_out ? N : 1) < a.V) lpr *= 2;
@@ -750,7 +828,7 @@ extern "C" int rt_delta_runs(int f32, const RtDelta* d, const void* runs, const 
   if (n_runs <= 0) return 0;
   if (n_runs > 65535) return -1;
   const Args a = make_args(*d);
-  const Work w{(const int4*)runs, (const int2*)chunks, ws, v, o};
+  const Work w{(const int4*)runs, (const int2*)chunks, ws, n_chunks, 0, ((long)a.H * a.V + 1) / 2 * 2, v, o};
 #define DR_(DP)                                                                                       \
   return f32 ? runs_<float, DP>(a, w, first_chunk, n_runs, n_chunks, t0, n_tokens, stream)            \
              : runs_<bf16_t, DP>(a, w, first_chunk, n_runs, n_chunks, t0, n_tokens, stream)
