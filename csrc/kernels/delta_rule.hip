@@ -202,7 +202,8 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
 // ---------------------------------------------------------------------------------------------
 // runs: {row, first token, tokens, position of the first}; chunks: {run, chunk of the run}, a run's chunks
 // consecutive. Workspace per (chunk, head): k e^G, q e^G [CH][DP], k e^(G_16 - G) transposed [DP][CH], e^G_16 [DP],
-// T, P [CH][CH] floats.
+// T, P [CH][CH] floats, the matrices as the MFMA's first operand: row m, column 16 r + 4 g + i of a [CH][..] one (of
+// rows 16 r + m, column 4 g + i of the transposed one) is element (r * 64 + 16 g + m) * 4 + i, so a wave loads 1 KB runs.
 struct Work {
   const int4* runs; const int2* chunks;
   float* ws;    // a head's chunks side by side
@@ -212,6 +213,7 @@ struct Work {
   float* o;     // [N, H * V] read-outs
 };
 template <int DP> struct Lay {
+  static __device__ __forceinline__ int sq(int row, int col) { return (16 * (col >> 2) + row) * 4 + (col & 3); }  // T, P
   static constexpr int KT = 0, QT = CH * DP, KE = 2 * CH * DP, EG = 3 * CH * DP, T = EG + DP, P = T + CH * CH, N = P + CH * CH;
 };
 
@@ -465,32 +467,32 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(Args a, Work w) {
 #pragma unroll
         for (int j = 0; j < i; ++j) y = fmaf(-As[i][j], x[j], y);
         x[i] = y;
-        ws[L::T + i * CH + tid] = y;
+        ws[L::T + L::sq(i, tid)] = y;
       }
     } else if (tid < 2 * CH) {  // column of P
       const int c = tid - CH;
 #pragma unroll
-      for (int i = 0; i < CH; ++i) ws[L::P + i * CH + c] = i > c ? Ps[i][c] : (i == c ? dot[i] : 0.f);
+      for (int i = 0; i < CH; ++i) ws[L::P + L::sq(i, c)] = i > c ? Ps[i][c] : (i == c ? dot[i] : 0.f);
     }
     return;
   }
   const int tw = tid - 64;  // 192 threads
   auto gl = [&](int i, int d) { return CHN ? G[i][d] : Gs[i]; };
   for (int e = tw; e < CH * DP / 4; e += 192) {
-    const int i = e / (DP / 4), d = e % (DP / 4) * 4;
-    const f32x4 k4 = *(const f32x4*)&kx[i][d], q4 = *(const f32x4*)&qx[i][d];
+    const int em = e & 15, d = 16 * (e >> 6) + 4 * (e >> 4 & 3);  // token em, channels d .. d + 3
+    const f32x4 k4 = *(const f32x4*)&kx[em][d], q4 = *(const f32x4*)&qx[em][d];
     f32x4 ex;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) ex[j] = (CHN || j == 0) ? expf(gl(i, d + j)) : ex[0];
-    *(f32x4*)(ws + L::KT + i * DP + d) = k4 * ex;
-    *(f32x4*)(ws + L::QT + i * DP + d) = q4 * ex;
+    for (int j = 0; j < 4; ++j) ex[j] = (CHN || j == 0) ? expf(gl(em, d + j)) : ex[0];
+    *(f32x4*)(ws + L::KT + 4 * e) = k4 * ex;
+    *(f32x4*)(ws + L::QT + 4 * e) = q4 * ex;
   }
-  for (int e = tw; e < DP * 4; e += 192) {
-    const int d = e >> 2, i = (e & 3) * 4;
+  for (int e = tw; e < CH * DP / 4; e += 192) {
+    const int d = 16 * (e >> 6) + (e & 15), i = 4 * (e >> 4 & 3);  // channel d, tokens i .. i + 3
     f32x4 y;
 #pragma unroll
     for (int j = 0; j < 4; ++j) y[j] = kx[i + j][d] * expf(gl(CH - 1, d) - gl(i + j, d));
-    *(f32x4*)(ws + L::KE + d * CH + i) = y;
+    *(f32x4*)(ws + L::KE + 4 * e) = y;
   }
   for (int d = tw; d < DP; d += 192) ws[L::EG + d] = expf(gl(CH - 1, d));
 }
@@ -531,14 +533,13 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 + 64 : 320, DP > 128 ? 2 : 4) 
   const bool odd = vc & 1;
   float* op = w.o + (long)run.y * ldo;
   const float* wp = w.ws + ((long)h * w.n_chunks + c0) * L::N;
-  const uint32_t o_kq = 4 * (m * DP + d0 + 4 * g), o_e = 4 * (L::KE + (d0 + m) * CH + 4 * g), o_g = 4 * (L::EG + d0 + 4 * g),
-                 o_t = 4 * (L::T + m * CH + 4 * g);
+  const uint32_t o_m = 16 * lane, o_s = 16 * (RW * wid * 64 + lane), o_g = 4 * (d0 + 4 * g);  // the wave's row tiles
   auto load_kq = [&](ScanOps<RW>& s, int c) {
     const float* p = wp + (long)min(c, nc - 1) * L::N;
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
-      s.k[r] = at<f32x4>(p + L::KT + 16 * r, o_kq);
-      s.q[r] = at<f32x4>(p + L::QT + 16 * r, o_kq);
+      s.k[r] = at<f32x4>(p + L::KT + 256 * r, o_s);
+      s.q[r] = at<f32x4>(p + L::QT + 256 * r, o_s);
     }
   };
   auto load_tv = [&](auto& s, int c) {  // c < nc
@@ -547,7 +548,7 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 + 64 : 320, DP > 128 ? 2 : 4) 
 #pragma unroll
     for (int i = 0; i < 4; ++i)  // past the run: beta is 0
       s.v[i] = at<uint32_t>(p, 4 * (__umul24((uint32_t)min(4 * g + i, last), ldw) + vw));
-    s.t = at<f32x4>(wp + (long)c * L::N, o_t);
+    s.t = at<f32x4>(wp + (long)c * L::N + L::T, o_m);
   };
   auto load_rest = [&](ScanOps<RW>& s, int c) {
     c = min(c, nc - 1);
@@ -555,8 +556,8 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 + 64 : 320, DP > 128 ? 2 : 4) 
     const float* p = wp + (long)c * L::N;
 #pragma unroll
     for (int r = 0; r < RW; ++r) {
-      s.e[r] = at<f32x4>(p + 16 * r * CH, o_e);
-      s.g[r] = at<f32x4>(p + 16 * r, o_g);
+      s.e[r] = at<f32x4>(p + L::KE + 256 * r, o_s);
+      s.g[r] = at<f32x4>(p + L::EG + 16 * r, o_g);
     }
   };
   // U from the shares of k e^G S0 in buffer b
@@ -575,7 +576,7 @@ __global__ __launch_bounds__(DP / 16 < 4 ? DP * 4 + 64 : 320, DP > 128 ? 2 : 4) 
     auto load = [&](ReadOps& s, int c) {
       c = min(c, nc - 1);
       load_tv(s, c);
-      s.p = at<f32x4>(wp + (long)c * L::N + (L::P - L::T), o_t);
+      s.p = at<f32x4>(wp + (long)c * L::N + L::P, o_m);
     };
     auto read = [&](ReadOps& s, int c) {
       const int b = c & 1;
