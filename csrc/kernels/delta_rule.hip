@@ -35,6 +35,19 @@ template <typename T> __device__ __forceinline__ void st(T* p, float v);
 template <> __device__ __forceinline__ void st<bf16_t>(bf16_t* p, float v) { *p = f2bf(v); }
 template <> __device__ __forceinline__ void st<float>(float* p, float v) { *p = v; }
 
+// N floats, aligned to 16 bytes from four on
+template <int N>
+__device__ __forceinline__ void ldf(const float* p, float* o) {
+  if constexpr (N % 4 == 0) {
+#pragma unroll
+    for (int k = 0; k < N; k += 4) *(f32x4*)(o + k) = *(const f32x4*)(p + k);
+  } else {
+    o[0] = p[0];
+  }
+}
+template <int N>
+__device__ __forceinline__ void stf(float* p, const float* o) { ldf<N>(o, p); }
+
 __device__ __forceinline__ float sigmoid(float x) { return __builtin_amdgcn_rcpf(1.f + expf(-x)); }
 __device__ __forceinline__ float softplus(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float gate_of(float z, bool silu) { return (silu ? z : 1.f) * sigmoid(z); }
@@ -73,58 +86,109 @@ struct Conv {
 };
 
 // ---------------------------------------------------------------------------------------------
-// one token per request. Thread = VEC value columns x NR key rows of the state, held in registers; the
-// projections' part (convolutions, unit norms, decays) runs while the state is on its way.
+// one token per request. Thread = VEC value columns x NR key rows of the state, held in registers. The small inputs are
+// on their way first (as the words they lie in memory as: a conversion would wait for them), then the state; the
+// projections' part (convolutions, unit norms, decays) runs meanwhile.
 // ---------------------------------------------------------------------------------------------
+template <typename T> __device__ __forceinline__ uint32_t word(const T* p);
+template <> __device__ __forceinline__ uint32_t word<bf16_t>(const bf16_t* p) { return *p; }
+template <> __device__ __forceinline__ uint32_t word<float>(const float* p) { return __float_as_uint(*p); }
+template <typename T> __device__ __forceinline__ float value(uint32_t w) { return __uint_as_float(sizeof(T) == 2 ? w << 16 : w); }
+
 template <typename T, int VEC, int NR, int BLOCK>
 __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
-  extern __shared__ float sm[];  // k, q (unit, decayed later), g [D]; v, o [V]; sums [2][RG][V]; red [2 * BLOCK / 64]
+  extern __shared__ __attribute__((aligned(16))) float sm[];  // sums [2][RG][V]; k, q, g [D]; v, o [V]
+  constexpr int PRE = 2, TAP = 4;  // channels per thread and their last taps that are loaded ahead
   const int h = blockIdx.x, t = blockIdx.y, tid = threadIdx.x, lane = tid & 63;
-  const int D = a.D, V = a.V, kh = h / (a.H / a.K);
+  const int D = a.D, V = a.V, taps = a.taps, kh = h / (a.H / a.K);
   const int ncol = (V + VEC - 1) / VEC, RG = BLOCK / ncol;
-  float* ks = sm;
+  float* sum = sm;
+  float* ks = sum + 2 * RG * V;
   float* qs = ks + D;
   float* gs = qs + D;
   float* vs = gs + D;
   float* os = vs + V;
-  float* sum = os + V;
-  const int row = a.row[t], pos = max(a.pos[t], 0);
-  const bool live = row >= 0 && row < a.n_rows, carry = live && pos > 0;
+  const int row_ = a.row[t], pos = max(a.pos[t], 0);
+  const bool live = row_ >= 0 && row_ < a.n_rows, carry = live && pos > 0;
+  const int row = live ? row_ : 0;
   const int cg = tid % ncol, rg = tid / ncol;
   const bool mine = rg < RG;
-  float* Sp = a.S + (((long)max(row, 0) * a.H + h) * D) * V + cg * VEC;
+  const int KD = a.K * D, C = 2 * KD + a.H * V, nch = 2 * D + V, slot = pos % taps;
+  const T* xt = (const T*)a.x + (long)t * a.ldx;
+  const T* conv = (const T*)a.conv;
+  T* ring = (T*)a.ring + (long)row * taps * C;
+  auto chan = [&](int i) { return i < D ? kh * D + i : (i < 2 * D ? KD + kh * D + i - D : 2 * KD + h * V + i - 2 * D); };
+  auto past = [&](int c, int back) {  // the channel's input `back` < taps tokens ago (a finite or stale word: see seen)
+    int s = slot - back;
+    if (s < 0) s += taps;
+    return word(back ? ring + (long)s * C + c : xt + c);
+  };
+  auto seen = [&](int back) { return back < taps && (back == 0 || (carry && pos >= back)); };
+  uint32_t xw[PRE][TAP], ww[PRE][TAP];
+#pragma unroll
+  for (int k = 0; k < PRE; ++k) {
+    const int c = chan(min(tid + k * BLOCK, nch - 1));
+#pragma unroll
+    for (int j = 0; j < TAP; ++j) {
+      const int back = min(j, taps - 1);
+      xw[k][j] = past(c, back);
+      ww[k][j] = word(conv + (long)c * taps + taps - 1 - back);
+    }
+  }
+  const T* ap = (const T*)a.a + (long)t * a.lda + (a.channel ? (long)h * D + min(tid, D - 1) : h);
+  const uint32_t aw = word(ap), bw = word((const T*)a.b + (long)t * a.ldb + h);
+  const float dt = a.dt[a.channel ? (long)h * D + min(tid, D - 1) : h], A_log = a.A_log[h];
+  const T* zp = (const T*)a.z + (long)t * a.ldz + (long)h * V;
+  const uint32_t zw = word(zp + min(tid, V - 1)), nw = word((const T*)a.norm_w + min(tid, V - 1));
+  asm volatile("" ::: "memory");
+  float* Sp = a.S + (((long)row * a.H + h) * D) * V + (mine ? cg * VEC : 0);
   float s[NR][VEC];
 #pragma unroll
-  for (int j = 0; j < NR; ++j) {
-    const int d = rg + j * RG;
+  for (int j = 0; j < NR; ++j)
 #pragma unroll
     for (int e = 0; e < VEC; ++e) s[j][e] = 0.f;
-    if (carry && mine && d < D) {
+  if (carry) {  // threads and rows past the edge repeat the last row; they take no part below
+#pragma unroll
+    for (int j = 0; j < NR; ++j) {
+      const float* p = Sp + (long)min(rg + j * RG, D - 1) * V;
       if constexpr (VEC == 4) {
-        const float4 v = *(const float4*)(Sp + (long)d * V);
+        const float4 v = *(const float4*)p;
         s[j][0] = v.x; s[j][1] = v.y; s[j][2] = v.z; s[j][3] = v.w;
       } else {
-        s[j][0] = Sp[(long)d * V];
+        s[j][0] = *p;
       }
     }
   }
-  const int KD = a.K * D, C = 2 * KD + a.H * V;
-  const T* xt = (const T*)a.x + (long)t * a.ldx;
-  T* ring = (T*)a.ring + (long)max(row, 0) * a.taps * C;
-  const Conv<T> conv{a, xt, carry ? ring : nullptr, pos, C};
-  for (int i = tid; i < 2 * D + V; i += BLOCK) {
-    const int c = i < D ? kh * D + i : (i < 2 * D ? KD + kh * D + i - D : 2 * KD + h * V + i - 2 * D);
-    const float y = conv(pos, c);
+  auto put = [&](int i, int c, float y) {
+    y *= sigmoid(y);
     (i < D ? qs[i] : (i < 2 * D ? ks[i - D] : vs[i - 2 * D])) = y;
     // the slot of this position is read by nobody at this position; heads that share a key head share the write
-    if (live && (i >= 2 * D || h % (a.H / a.K) == 0)) ring[(long)(pos % a.taps) * C + c] = xt[c];
+    if (live && (i >= 2 * D || h % (a.H / a.K) == 0)) ring[(long)slot * C + c] = xt[c];
+  };
+  auto older = [&](int c, int j0) {  // taps from j0 tokens ago on
+    float y = 0.f;
+    for (int j = taps - 1; j >= j0; --j)
+      if (seen(j)) y = fmaf(ld(conv + (long)c * taps + taps - 1 - j), value<T>(past(c, j)), y);
+    return y;
+  };
+#pragma unroll
+  for (int k = 0; k < PRE; ++k) {
+    const int i = tid + k * BLOCK;
+    if (i >= nch) continue;
+    const int c = chan(i);
+    float y = older(c, TAP);
+#pragma unroll
+    for (int j = TAP - 1; j >= 0; --j) y = seen(j) ? fmaf(value<T>(ww[k][j]), value<T>(xw[k][j]), y) : y;
+    put(i, c, y);
   }
-  const float A = expf(a.A_log[h]);
+  for (int i = tid + PRE * BLOCK; i < nch; i += BLOCK) put(i, chan(i), older(chan(i), 0));
+  const float A = expf(A_log);
   if (a.channel) {
-    for (int d = tid; d < D; d += BLOCK)
+    if (tid < D) gs[tid] = expf(-A * softplus(value<T>(aw) + dt));
+    for (int d = tid + BLOCK; d < D; d += BLOCK)
       gs[d] = expf(-A * softplus(ld((const T*)a.a + (long)t * a.lda + (long)h * D + d) + a.dt[(long)h * D + d]));
   } else {
-    const float g = expf(-A * softplus(ld((const T*)a.a + (long)t * a.lda + h) + a.dt[h]));
+    const float g = expf(-A * softplus(value<T>(aw) + dt));
     for (int d = tid; d < D; d += BLOCK) gs[d] = g;
   }
   __syncthreads();
@@ -136,8 +200,8 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
   }
   const float iq = 1.f / sqrtf(wave_sum(qq) + 1e-6f) / sqrtf((float)D), ik = 1.f / sqrtf(wave_sum(kk) + 1e-6f);
   qk = wave_sum(qk) * iq * ik;
-  const float beta = sigmoid(ld((const T*)a.b + (long)t * a.ldb + h));
-  float pk[VEC], pq[VEC];
+  const float beta = sigmoid(value<T>(bw));
+  __attribute__((aligned(16))) float pk[VEC], pq[VEC];
 #pragma unroll
   for (int e = 0; e < VEC; ++e) { pk[e] = 0.f; pq[e] = 0.f; }
 #pragma unroll
@@ -154,25 +218,30 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
     }
   }
   if (mine) {
-#pragma unroll
-    for (int e = 0; e < VEC; ++e) {
-      sum[rg * V + cg * VEC + e] = pk[e];
-      sum[(RG + rg) * V + cg * VEC + e] = pq[e];
-    }
+    stf<VEC>(sum + rg * V + cg * VEC, pk);
+    stf<VEC>(sum + (RG + rg) * V + cg * VEC, pq);
   }
   __syncthreads();
   float u[VEC];
   if (mine) {
+    __attribute__((aligned(16))) float sk[VEC], sq[VEC], x[VEC];
+#pragma unroll
+    for (int e = 0; e < VEC; ++e) { sk[e] = 0.f; sq[e] = 0.f; }
+#pragma unroll 4
+    for (int r = 0; r < RG; ++r) {
+      ldf<VEC>(sum + r * V + cg * VEC, x);
+#pragma unroll
+      for (int e = 0; e < VEC; ++e) sk[e] += x[e];
+      if (rg == 0) {
+        ldf<VEC>(sum + (RG + r) * V + cg * VEC, x);
+#pragma unroll
+        for (int e = 0; e < VEC; ++e) sq[e] += x[e];
+      }
+    }
 #pragma unroll
     for (int e = 0; e < VEC; ++e) {
-      const int c = cg * VEC + e;
-      float sk = 0.f, sq = 0.f;
-      for (int r = 0; r < RG; ++r) {
-        sk += sum[r * V + c];
-        sq += sum[(RG + r) * V + c];
-      }
-      u[e] = beta * (vs[c] - sk);
-      if (rg == 0) os[c] = fmaf(qk, u[e], sq);  // S^T q behind the write
+      u[e] = beta * (vs[cg * VEC + e] - sk[e]);
+      if (rg == 0) os[cg * VEC + e] = fmaf(qk, u[e], sq[e]);  // S^T q behind the write
     }
     if (live) {
 #pragma unroll
@@ -192,9 +261,9 @@ __global__ __launch_bounds__(BLOCK) void delta_step_kernel(Args a) {
   float oo = 0.f;
   for (int c = lane; c < V; c += 64) oo += os[c] * os[c];
   const float r = a.out_scale / sqrtf(wave_sum(oo) / V + a.eps);
-  for (int c = tid; c < V; c += BLOCK)
-    st((T*)a.out + (long)t * a.ldo + (long)h * V + c,
-       os[c] * r * ld((const T*)a.norm_w + c) * gate_of(ld((const T*)a.z + (long)t * a.ldz + (long)h * V + c), a.silu));
+  T* out = (T*)a.out + (long)t * a.ldo + (long)h * V;
+  if (tid < V) st(out + tid, os[tid] * r * value<T>(nw) * gate_of(value<T>(zw), a.silu));
+  for (int c = tid + BLOCK; c < V; c += BLOCK) st(out + c, os[c] * r * ld((const T*)a.norm_w + c) * gate_of(ld(zp + c), a.silu));
 }
 
 // ---------------------------------------------------------------------------------------------
@@ -230,19 +299,6 @@ __device__ __forceinline__ void stn(T* p, const float* o) {
   else if constexpr (N == 4) *(f32x4*)p = *(const f32x4*)o;
   else st(p, o[0]);
 }
-
-// N floats, aligned to 16 bytes from four on
-template <int N>
-__device__ __forceinline__ void ldf(const float* p, float* o) {
-  if constexpr (N % 4 == 0) {
-#pragma unroll
-    for (int k = 0; k < N; k += 4) *(f32x4*)(o + k) = *(const f32x4*)(p + k);
-  } else {
-    o[0] = p[0];
-  }
-}
-template <int N>
-__device__ __forceinline__ void stf(float* p, const float* o) { ldf<N>(o, p); }
 
 // convolution and silu of channels c .. c + N - 1 at positions p .. p + 3, zeros from position p + n on. TAPS: their
 // number (every load issued ahead), 0: any

@@ -49,7 +49,7 @@ __device__ __forceinline__ void stn(T* p, const float* o) {
 // N consecutive elements per access: 8 (bf16, D, V and half multiples of 8, aligned rows) or 1
 template <typename T, int N>
 __global__ __launch_bounds__(256) void window_prep_kernel(PrepArgs a) {
-  __shared__ float sbuf[4];
+  __shared__ float sbuf[8];
   const int t = blockIdx.x, tid = threadIdx.x;
   T* pr = (T*)a.proj + (long)t * a.ldp;
   const int p_raw = a.pos[t], pos = min(max(p_raw, 0), a.max_pos - 1);
@@ -62,14 +62,14 @@ __global__ __launch_bounds__(256) void window_prep_kernel(PrepArgs a) {
   T* dst = (T*)a.pool + ((long)max(page, 0) * a.G * PAGE + pos % PAGE) * (a.D + a.V);  // + head * PAGE * (D + V)
   const long hs = (long)PAGE * (a.D + a.V);
 
-  auto rstd_of = [&](const T* x, int n) {
+  auto squares = [&](const T* x, int n) {
     float s = 0.f, v[N];
     for (int e = tid * N; e < n; e += 256 * N) {
       ldn<T, N>(x + e, v);
 #pragma unroll
       for (int k = 0; k < N; ++k) s += v[k] * v[k];
     }
-    return 1.f / sqrtf(block_sum(s, sbuf) / n + a.eps);
+    return s;
   };
   // one thread normalises and turns both halves of its pairs, so rows may be written in place
   auto turn = [&](T* x, const T* w, int heads, float rstd, bool to_cache) {
@@ -105,8 +105,19 @@ __global__ __launch_bounds__(256) void window_prep_kernel(PrepArgs a) {
   };
   T* q = pr + a.q_col;
   T* k = pr + a.k_col;
-  const float rq = a.q_norm ? rstd_of(q, a.H * a.D) : 1.f;
-  const float rk = a.k_norm ? rstd_of(k, a.G * a.D) : 1.f;
+  float rq = 1.f, rk = 1.f;
+  if (a.q_norm || a.k_norm) {
+    float sq = squares(q, a.H * a.D), sk = squares(k, a.G * a.D);
+    sq = wave_sum(sq);
+    sk = wave_sum(sk);
+    if ((tid & 63) == 0) {
+      sbuf[tid >> 6] = sq;
+      sbuf[4 + (tid >> 6)] = sk;
+    }
+    __syncthreads();
+    if (a.q_norm) rq = 1.f / sqrtf((sbuf[0] + sbuf[1] + sbuf[2] + sbuf[3]) / (a.H * a.D) + a.eps);
+    if (a.k_norm) rk = 1.f / sqrtf((sbuf[4] + sbuf[5] + sbuf[6] + sbuf[7]) / (a.G * a.D) + a.eps);
+  }
   turn(q, (const T*)a.q_norm, a.H, rq, false);
   turn(k, (const T*)a.k_norm, a.G, rk, true);
   if (append) {
