@@ -23,7 +23,8 @@ Secondary modes (not the headline; each prints its own JSON line):
   --mode sft       BASELINE config 3: RAFT-style LoRA r=16 SFT with distractor docs, tokens/s
   --mode pipeline  BASELINE config 5: RAG index -> LoRA SFT -> PPO on one policy (default
                    --model llama2-13b; --fp8 runs rollouts / reference scoring on e4m3fn weights)
-  --mode layered   prefill and decode throughput of a layered model (Vezatar) beside the closest
+  --mode layered   prefill and decode throughput of a layered model (Vezatar; Pafolorn with
+                   --layered-sizes pafolorn-7b/mistral-7b,pafolorn-2k/mistral-2k) beside the closest
                    existing decoder at equal width and depth (random weights)
 """
 from __future__ import annotations

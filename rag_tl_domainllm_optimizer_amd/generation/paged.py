@@ -1,10 +1,12 @@
 """Paged cache: per layer a pool of pages of 64 tokens, and one page table row per request.
 
 The pool is sized for the tokens that live requests hold at any time (each rounded up to whole pages), not
-for rows x longest sequence. Layers with recurrent state have one slot per row beside it: tensors
-[rows, ...] that belong to the row's request and count as zero at its position 0. Page 0 belongs to nobody: table entries without a page point at it, so a
+for rows x longest sequence. Page 0 belongs to nobody: table entries without a page point at it, so a
 decode graph's idle rows write there. Pools start as zeros and only ever hold finite values, so masked
-keys of a reused page are harmless. Allocation is host bookkeeping; ``sync`` uploads the table."""
+keys of a reused page are harmless. Allocation is host bookkeeping; ``sync`` uploads the table.
+
+Layers with recurrent state have one slot per row beside it: tensors [rows, ...] that belong to the row's
+request and count as zero at its position 0, so a slot that is used again needs no clearing."""
 from __future__ import annotations
 
 import contextlib

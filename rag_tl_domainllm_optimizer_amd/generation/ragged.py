@@ -12,7 +12,7 @@ from typing import List, Sequence, Tuple
 import numpy as np
 import torch
 
-SHORT_TOKENS = 32   # portions up to this many tokens attend in the absorbed form, token by token
+SHORT_TOKENS = 32   # portions up to this many tokens attend token by token, like decoded ones
 QUERY_TILE = 128    # query rows per workgroup of the portions' attention kernel
 CHUNK = 16          # tokens per chunk of a recurrent layer's portions (csrc/kernels/delta_rule.hip)
 
