@@ -258,7 +258,7 @@ def test_needle_at_every_edge(size, keep):
             seen = a - at < size or at < keep
             e = pc.err(moved[a:a + 1], want[a:a + 1])
             assert e > 0.2 if seen else e < 1e-6, (at, a)
-        for sizes in ((n,), (n - 1, 1), (64, 40, 1), (7, 2)):
+        for sizes in ((n - 1, 1), (64, 40, 7)):
             assert pc.err(pc.run(StepEngine(m, 1, 256), t, sizes), want) < TOL, (at, sizes)
 
 
